@@ -149,6 +149,19 @@ PROTOTYPES = {
     "exl2_gated_scan_cols_supported": (ci, [ci, ci]),
     "exl2_gated_scan_cols": (ci, [ci, vp, ci, vp, ci, vp, ci, vp, ci, vp, ci, vp, ci, vp, vp, vp, vp, vp, ci, ci, vp, vp, vp, ci, vp, vp, ci, vp,
                                   ci, ci, ci, ci, cf, cf, vp]),
+    # layers whose mixer and feed-forward read one norm: gated residual step, grouped router (csrc/rowops.hip); latent attention with a sink
+    # per head and either rotary layout (csrc/latent_attn.hip); minimal gated recurrence (csrc/mingru.hip); head-mixing attention
+    # (csrc/talk_attn.hip)
+    "exl2_gated_residual": (ci, [vp, vp, vp, vp, vp, cf, cf, vp, vp, ci, vp, vp, ci, vp, vp, ci, ci, vp, vp, ci, vp, ci, ci, ci, cf, vp]),
+    "exl2_moe_route_grouped": (ci, [vp, ci, vp, vp, ci, ci, ci, cf, ci, ci, vp, vp, vp, vp]),
+    "exl2_latent_append_ex": (ci, [vp, ci, vp, cf, ci, ci, ci, ci, ci, ci, vp, vp, vp, vp, ci, ci, vp, vp]),
+    "exl2_latent_attn_ex": (ci, [vp, ci, ci, ci, vp, vp, ci, vp, vp, vp, ci, vp, ci, ci, ci, ci, ci, ci, ci, vp, cf, ci, vp, vp]),
+    "exl2_latent_attn_tiles_ex": (ci, [vp, ci, ci, ci, vp, vp, ci, vp, vp, vp, ci, vp, vp, vp, ci, ci, vp, vp, ci, ci, ci, ci, ci, ci, vp, cf, ci,
+                                       vp, vp]),
+    "exl2_mingru_scan": (ci, [vp, vp, vp, ci, vp, ci, vp, vp, vp, ci, vp, vp, vp, ci, ci, vp, ci, ci, vp]),
+    "exl2_talk_attn": (ci, [vp, vp, vp, vp, vp, vp, vp, vp, ci, ci, vp, vp, ci, vp, vp, ci, ci, ci, ci, ci, ci, ci, cf, vp]),
+    "exl2_talk_attn_tiles_supported": (ci, [ci, ci, ci]),
+    "exl2_talk_attn_tiles": (ci, [vp, vp, vp, vp, vp, vp, vp, vp, ci, ci, vp, vp, vp, ci, ci, ci, ci, ci, ci, cf, vp]),
     # graphs
     "exl2_graph_begin_capture": (ci, [vp]),
     "exl2_graph_end_capture": (ci, [vp, C.POINTER(vp)]),

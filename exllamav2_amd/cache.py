@@ -172,28 +172,42 @@ class LatentCache:
     def layer(self, layer_idx: int) -> torch.Tensor:
         return self.rows[self.owner[layer_idx]]
 
+    latent_rows = layer
+
     def footprint(self) -> int:
         return sum(t.numel() * t.element_size() for t in self.rows.values())
+
+
+class PagedLatent:
+    """One latent-attention layer's share of a PagePool in a stack of unlike mixers: rows [pages, page, kv_rank + rot_dim]"""
+
+    def __init__(self, pool: PagePool, width: int, dtype):
+        self.rows = torch.zeros((pool.num_pages, pool.page_size, width), dtype=dtype, device=pool.device)
+
+    def tensors(self):
+        return [self.rows]
 
 
 class PagedKV:
     """One attention layer's share of a PagePool: keys [pages, page, kv_heads, dim] and values [pages, page, kv_heads, vdim], and --
     for layers that see pooled blocks behind their window -- one mean key / mean value row per block of `block` tokens, kept with
-    the page of the block's first token: [pages, ceil(page / block), kv_heads, dim | vdim]."""
+    the page of the block's first token: [pages, ceil(page / block), kv_heads, dim | vdim].  `tail` = (rows, channels): also that many fp32
+    rows per sequence slot (the history of a short convolution in front of the attention)."""
 
-    def __init__(self, pool: PagePool, kv_heads: int, dim: int, vdim: int, block: int, dtype):
+    def __init__(self, pool: PagePool, kv_heads: int, dim: int, vdim: int, block: int, dtype, tail=None):
         dev, P, n = pool.device, pool.page_size, pool.num_pages
         self.block = int(block)
         self.k = torch.zeros((n, P, kv_heads, dim), dtype=dtype, device=dev)
         self.v = torch.zeros((n, P, kv_heads, vdim), dtype=dtype, device=dev)
         self.k_pool = self.v_pool = None
+        self.tail = torch.zeros((pool.max_seqs,) + tuple(tail), dtype=torch.float32, device=dev) if tail is not None else None
         if self.block > 0:
             per_page = -(-P // self.block)
             self.k_pool = torch.zeros((n, per_page, kv_heads, dim), dtype=dtype, device=dev)
             self.v_pool = torch.zeros((n, per_page, kv_heads, vdim), dtype=dtype, device=dev)
 
     def tensors(self):
-        return [t for t in (self.k, self.v, self.k_pool, self.v_pool) if t is not None]
+        return [t for t in (self.k, self.v, self.k_pool, self.v_pool, self.tail) if t is not None]
 
 
 class SlotState:
@@ -217,8 +231,10 @@ class LayerStates:
     attention, SlotState for recurrent mixers, None for a layer that reads another layer's rows), all over ONE PagePool, so a request's pages and its slot are handed out and taken
     back together."""
 
-    def __init__(self, pool: PagePool, per_layer: dict, norm_states: dict | None = None):
+    def __init__(self, pool: PagePool, per_layer: dict, norm_states: dict | None = None, later_passes=()):
         self.pool, self.per_layer = pool, dict(per_layer)
+        # a stack that goes through some of its layers several times: what those layers keep for their second, third, .. pass
+        self.later_passes = list(later_passes)
         # what the row-wise steps keep per slot: layer -> the norm in front of its mixer (token shift, input convolution),
         # (layer, "ff") -> the norm in front of its feed-forward, "embed" -> the embedding (previous token)
         self.norm_states = dict(norm_states or {})
@@ -227,9 +243,16 @@ class LayerStates:
         """key: a layer's index, or whatever a mixer that keeps several states names them by"""
         return self.per_layer[key]
 
+    def latent_rows(self, key) -> torch.Tensor:
+        return self.per_layer[key].rows
+
+    def at_pass(self, p: int) -> "LayerStates":
+        return self if p == 0 else self.later_passes[p - 1]
+
     def norm_state(self, key):
         return self.norm_states.get(key)
 
     def footprint(self) -> int:
         states = list(self.per_layer.values()) + list(self.norm_states.values())
-        return sum(t.numel() * t.element_size() for st in states if st is not None for t in st.tensors())
+        return sum(t.numel() * t.element_size() for st in states if st is not None for t in st.tensors()) \
+            + sum(p.footprint() for p in self.later_passes)

@@ -156,6 +156,10 @@ DEV f32x4 mfma_16x16x32_bf16(u32x4 a, u32x4 b, f32x4 c) {
     return __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8_t, a), __builtin_bit_cast(bf16x8_t, b), c, 0, 0, 0);
 }
 
+// sixteen independent 4 x 4 products of depth one, fp32: lane 4 b + x holds row x of A and column x of B of block b and gets column x
+// of D_b += A_b B_b in its four registers -- with the same A in every block, each lane's own scalar times a vector of four
+DEV f32x4 mfma_4x4x1_f32(float a, float b, f32x4 c) { return __builtin_amdgcn_mfma_f32_4x4x1f32(a, b, c, 0, 0, 0); }
+
 // fp32 += dot(half2, half2): v_dot2_f32_f16
 DEV float dot2_f32_f16(f16x2 a, f16x2 b, float c) { return __builtin_amdgcn_fdot2(a, b, c, false); }
 

@@ -11,7 +11,9 @@
 // portions of several requests and single decoded tokens go through the same launch, and a row's result depends only on its own
 // (sequence, position).  Scores, softmax and the weighted sum are fp32; positions and angles are fp32 with the inverse
 // frequencies passed in as a table (made in double precision on the host).
-// Interleaved rotary layout: dimension 2i is paired with 2i + 1, angle p * inv_freq[i]; dimensions past rot_dims pass unchanged.
+// Rotary layouts: interleaved (dimension 2i is paired with 2i + 1) or halves (i with i + rot_dims / 2), angle p * inv_freq[i];
+// dimensions past rot_dims pass unchanged.  The softmax denominator may also hold exp(sink[head]), a score without key and value (the
+// running maximum starts at the sink, the sum at 1; with split keys it counts in the first split).
 #include "hw.h"
 #include "errors.h"
 
@@ -39,13 +41,19 @@ DEV float la_block_max(float v, float* part)
     return fmaxf(fmaxf(part[0], part[1]), fmaxf(part[2], part[3]));
 }
 
+// element indices (ia, ib) of pair i among n rotated values
+DEV void la_pair(int i, int n, int halves, int& ia, int& ib)
+{
+    if (halves) { ia = i; ib = i + n / 2; } else { ia = 2 * i; ib = 2 * i + 1; }
+}
+
 // ---- new rows into the cache: RMS norm of the latent, rotation of the shared key part ----------------------------------------
 
 struct LatAppendArgs
 {
     const float* dkv; int ld;                // [rows, ld]: kv_rank latent values then rot key values
     const void* norm_w; float eps;
-    int R, rot, rot_dims;
+    int R, rot, rot_dims, halves;
     const float* inv_freq;
     const int* row_seq; const int* row_pos; const int* block_table; int bt_stride, page;
     void* cache;
@@ -70,9 +78,11 @@ KERNEL void __launch_bounds__(256) latent_append_kernel(const LatAppendArgs a)
     {
         const float ang = (float)pos * a.inv_freq[i];
         const float c = cosf(ang), s = sinf(ang);
-        const float u = ks[2 * i], v = ks[2 * i + 1];
-        la_st<T>(dst + a.R + 2 * i, u * c - v * s);
-        la_st<T>(dst + a.R + 2 * i + 1, v * c + u * s);
+        int ia, ib;
+        la_pair(i, a.rot_dims, a.halves, ia, ib);
+        const float u = ks[ia], v = ks[ib];
+        la_st<T>(dst + a.R + ia, u * c - v * s);
+        la_st<T>(dst + a.R + ib, v * c + u * s);
     }
     for (int i = a.rot_dims + tid(); i < a.rot; i += 256) la_st<T>(dst + a.R + i, ks[i]);
 }
@@ -86,9 +96,10 @@ struct LatAttnArgs
     const void* cache; int page;
     const int* row_seq; const int* row_pos; const int* block_table; int bt_stride;
     void* out;                                              // [rows, H, R]
-    int H, R, rot, rot_dims;
+    int H, R, rot, rot_dims, halves;
     const float* inv_freq;
     float scale; int window;
+    const float* sink;                                      // [H] (nullable: none)
 };
 
 #define LA_MAX_R_PER_THREAD 4
@@ -115,16 +126,18 @@ KERNEL void __launch_bounds__(256) latent_attn_kernel(const LatAttnArgs a)
     {
         const float ang = (float)pos * a.inv_freq[i];
         const float c = cosf(ang), s = sinf(ang);
-        const float u = la_ld<T>(qr + 2 * i), v = la_ld<T>(qr + 2 * i + 1);
-        qv[a.R + 2 * i] = u * c - v * s;
-        qv[a.R + 2 * i + 1] = v * c + u * s;
+        int ia, ib;
+        la_pair(i, a.rot_dims, a.halves, ia, ib);
+        const float u = la_ld<T>(qr + ia), v = la_ld<T>(qr + ib);
+        qv[a.R + ia] = u * c - v * s;
+        qv[a.R + ib] = v * c + u * s;
     }
     for (int i = a.rot_dims + t; i < a.rot; i += 256) qv[a.R + i] = la_ld<T>(qr + i);
     block_sync();
 
     const int j_lo = max(0, pos - a.window + 1);
     const int nkeys = pos - j_lo + 1;
-    float m_run = -INFINITY, l_run = 0.0f;
+    float m_run = a.sink ? a.sink[h] : -INFINITY, l_run = a.sink ? 1.0f : 0.0f;
     float acc[LA_MAX_R_PER_THREAD];
     #pragma unroll
     for (int e = 0; e < LA_MAX_R_PER_THREAD; e++) acc[e] = 0.0f;
@@ -189,9 +202,10 @@ struct LatMfmaArgs
     const int* tile_row0; const int* tile_rows;
     u16* out;
     float* part_o; float* part_ml; int nsplit;
-    int H, R, rot, rot_dims;
+    int H, R, rot, rot_dims, halves;
     const float* inv_freq;
     float scale; int window;
+    const float* sink;                                       // [H] (nullable: none)
     int DP;                                                  // kv_rank + rot rounded up to a multiple of 32
 };
 
@@ -220,7 +234,7 @@ KERNEL void __launch_bounds__(256) latent_attn_mfma_kernel(const LatMfmaArgs a)
     const int R = RS > 0 ? NT * 16 : a.R, rot = RS > 0 ? RS * 32 : a.rot;
     const int D = R + rot, DP = RS > 0 ? D : a.DP, CS = DP + 8;
     u16* Cs = (u16*)smem;                                    // [32][CS]
-    u16* Ct = Cs + LA_KT * CS;                               // [R][LA_TS]
+    u16* Ct = Cs + max(LA_KT * CS, 4 * 16 * LA_TS);          // [R][LA_TS] (narrow rows: the probability tiles are the larger part)
     u16* Ps = Cs + w * 16 * LA_TS;                           // [16][LA_TS], this wave's: OVER the row-major copy, once every wave is done with it
 
     // the query vector this lane feeds as A-operand row li
@@ -273,7 +287,25 @@ KERNEL void __launch_bounds__(256) latent_attn_mfma_kernel(const LatMfmaArgs a)
                     if (i0 < rot)
                     {
                         x0 = bf16_to_f32(qr[i0]); x1 = bf16_to_f32(qr[i0 + 1]);
-                        if (i0 < a.rot_dims)
+                        if (i0 < a.rot_dims && a.halves)
+                        {
+                            // each of the two values turns with its own partner half the rotated part away
+                            const int hd = a.rot_dims / 2;
+                            #pragma unroll
+                            for (int e = 0; e < 2; e++)
+                            {
+                                const int i = i0 + e, fi = i < hd ? i : i - hd;
+                                const float part = bf16_to_f32(qr[i < hd ? i + hd : i - hd]);
+                                const float ang = (float)qpos * a.inv_freq[fi];
+                                const float nrev = rintf(ang * 0.15915494309189535f);
+                                const float red = fmaf(-nrev, -1.7484555e-07f, fmaf(-nrev, 6.2831855f, ang));
+                                const float c = fast_cos(red), sn = fast_sin(red);
+                                const float own = e == 0 ? x0 : x1;
+                                const float turned = i < hd ? own * c - part * sn : own * c + part * sn;
+                                if (e == 0) x0 = turned; else x1 = turned;
+                            }
+                        }
+                        else if (i0 < a.rot_dims)
                         {
                             // (bfloat16 path: two-term reduction of the fp32 angle to [-pi, pi], then the hardware sine / cosine -- the
                             // library functions' large-argument path costs microseconds per call in a prologue that runs once per key split)
@@ -297,7 +329,13 @@ KERNEL void __launch_bounds__(256) latent_attn_mfma_kernel(const LatMfmaArgs a)
     for (int nt = 0; nt < NT; nt++) acc[nt] = (f32x4){0.0f, 0.0f, 0.0f, 0.0f};
     float m_run[4], l_run[4];
     #pragma unroll
-    for (int r = 0; r < 4; r++) { m_run[r] = -INFINITY; l_run[r] = 0.0f; }
+    for (int r = 0; r < 4; r++)
+    {
+        // accumulator row r of this lane: query 4 g + r (TR == 16: the wave's head; TR == 1: head .. + 4 g + r)
+        const int hd = min(TR == 16 ? hb * 4 + w : (hb * 4 + w) * 16 + 4 * g + r, H - 1);
+        const bool with_sink = a.sink && split == 0;
+        m_run[r] = with_sink ? a.sink[hd] : -INFINITY; l_run[r] = with_sink ? 1.0f : 0.0f;
+    }
 
     const int k_lo = max(0, p0 - a.window + 1), k_hi = p0 + n - 1;
     const int steps = (k_hi - k_lo + 1 + LA_KT - 1) / LA_KT;
@@ -546,9 +584,30 @@ static void launch_lat_mfma(const LatMfmaArgs& a, int tiles, int tile_rows, size
 
 // ---- C ABI --------------------------------------------------------------------------------------------------------------------
 
+extern "C" int exl2_latent_append_ex(const float* dkv, int ld, const void* norm_w, float eps, int dtype, int rows, int kv_rank, int rot,
+                                     int rot_dims, int halves, const float* inv_freq, const int* row_seq, const int* row_pos,
+                                     const int* block_table, int bt_stride, int page, void* cache, void* stream);
+extern "C" int exl2_latent_attn_ex(const void* q, int ldq, int q_head_stride, int q_rot_off, const float* q_abs, const void* cache, int page,
+                                   const int* row_seq, const int* row_pos, const int* block_table, int bt_stride, void* out, int dtype,
+                                   int rows, int heads, int kv_rank, int rot, int rot_dims, int halves, const float* inv_freq, float scale,
+                                   int window, const float* sink, void* stream);
+extern "C" int exl2_latent_attn_tiles_ex(const void* q, int ldq, int q_head_stride, int q_rot_off, const float* q_abs, const void* cache,
+                                         int page, const int* row_seq, const int* row_pos, const int* block_table, int bt_stride, void* out,
+                                         const int* tile_row0, const int* tile_rows, int tiles, int tile_mode, float* part_o, float* part_ml,
+                                         int nsplit, int heads, int kv_rank, int rot, int rot_dims, int halves, const float* inv_freq,
+                                         float scale, int window, const float* sink, void* stream);
+
 extern "C" int exl2_latent_append(const float* dkv, int ld, const void* norm_w, float eps, int dtype, int rows, int kv_rank, int rot,
                                   int rot_dims, const float* inv_freq, const int* row_seq, const int* row_pos, const int* block_table,
                                   int bt_stride, int page, void* cache, void* stream)
+{
+    return exl2_latent_append_ex(dkv, ld, norm_w, eps, dtype, rows, kv_rank, rot, rot_dims, 0, inv_freq, row_seq, row_pos, block_table,
+                                 bt_stride, page, cache, stream);
+}
+
+extern "C" int exl2_latent_append_ex(const float* dkv, int ld, const void* norm_w, float eps, int dtype, int rows, int kv_rank, int rot,
+                                     int rot_dims, int halves, const float* inv_freq, const int* row_seq, const int* row_pos,
+                                     const int* block_table, int bt_stride, int page, void* cache, void* stream)
 {
     EXL2_REQUIRE(dkv && norm_w && inv_freq && row_seq && row_pos && block_table && cache, "latent_append: null operand");
     EXL2_REQUIRE(dtype == 0 || dtype == 1, "latent_append: dtype must be 0 (bfloat16) or 1 (float32)");
@@ -556,7 +615,7 @@ extern "C" int exl2_latent_append(const float* dkv, int ld, const void* norm_w, 
                  "latent_append: bad shape (kv_rank %d, rot %d, rot_dims %d, ld %d, page %d)", kv_rank, rot, rot_dims, ld, page);
     if (rows <= 0) return EXL2_OK;
     LatAppendArgs a;
-    a.dkv = dkv; a.ld = ld; a.norm_w = norm_w; a.eps = eps; a.R = kv_rank; a.rot = rot; a.rot_dims = rot_dims; a.inv_freq = inv_freq;
+    a.dkv = dkv; a.ld = ld; a.norm_w = norm_w; a.eps = eps; a.R = kv_rank; a.rot = rot; a.rot_dims = rot_dims; a.halves = halves; a.inv_freq = inv_freq;
     a.row_seq = row_seq; a.row_pos = row_pos; a.block_table = block_table; a.bt_stride = bt_stride; a.page = page; a.cache = cache;
     if (dtype == 0) LAUNCH(latent_append_kernel<u16>, dim3(rows), dim3(256), 0, stream, a);
     else LAUNCH(latent_append_kernel<float>, dim3(rows), dim3(256), 0, stream, a);
@@ -569,6 +628,15 @@ extern "C" int exl2_latent_attn(const void* q, int ldq, int q_head_stride, int q
                                 int rows, int heads, int kv_rank, int rot, int rot_dims, const float* inv_freq, float scale, int window,
                                 void* stream)
 {
+    return exl2_latent_attn_ex(q, ldq, q_head_stride, q_rot_off, q_abs, cache, page, row_seq, row_pos, block_table, bt_stride, out, dtype,
+                               rows, heads, kv_rank, rot, rot_dims, 0, inv_freq, scale, window, nullptr, stream);
+}
+
+extern "C" int exl2_latent_attn_ex(const void* q, int ldq, int q_head_stride, int q_rot_off, const float* q_abs, const void* cache, int page,
+                                   const int* row_seq, const int* row_pos, const int* block_table, int bt_stride, void* out, int dtype,
+                                   int rows, int heads, int kv_rank, int rot, int rot_dims, int halves, const float* inv_freq, float scale,
+                                   int window, const float* sink, void* stream)
+{
     EXL2_REQUIRE(q && q_abs && cache && row_seq && row_pos && block_table && out && inv_freq, "latent_attn: null operand");
     EXL2_REQUIRE(dtype == 0 || dtype == 1, "latent_attn: dtype must be 0 (bfloat16) or 1 (float32)");
     EXL2_REQUIRE(heads > 0 && kv_rank > 0 && kv_rank <= 256 * LA_MAX_R_PER_THREAD, "latent_attn: kv_rank %d (at most %d)", kv_rank, 256 * LA_MAX_R_PER_THREAD);
@@ -578,7 +646,7 @@ extern "C" int exl2_latent_attn(const void* q, int ldq, int q_head_stride, int q
     LatAttnArgs a;
     a.q = q; a.ldq = ldq; a.q_head_stride = q_head_stride; a.q_rot_off = q_rot_off; a.q_abs = q_abs; a.cache = cache; a.page = page;
     a.row_seq = row_seq; a.row_pos = row_pos; a.block_table = block_table; a.bt_stride = bt_stride; a.out = out;
-    a.H = heads; a.R = kv_rank; a.rot = rot; a.rot_dims = rot_dims; a.inv_freq = inv_freq; a.scale = scale; a.window = window;
+    a.H = heads; a.R = kv_rank; a.rot = rot; a.rot_dims = rot_dims; a.halves = halves; a.inv_freq = inv_freq; a.scale = scale; a.window = window; a.sink = sink;
     const size_t smem = (size_t)(kv_rank + rot) * 4;
     if (dtype == 0) LAUNCH(latent_attn_kernel<u16>, dim3(rows, heads), dim3(256), smem, stream, a);
     else LAUNCH(latent_attn_kernel<float>, dim3(rows, heads), dim3(256), smem, stream, a);
@@ -597,6 +665,17 @@ extern "C" int exl2_latent_attn_tiles(const void* q, int ldq, int q_head_stride,
                                       int nsplit, int heads, int kv_rank, int rot, int rot_dims, const float* inv_freq, float scale,
                                       int window, void* stream)
 {
+    return exl2_latent_attn_tiles_ex(q, ldq, q_head_stride, q_rot_off, q_abs, cache, page, row_seq, row_pos, block_table, bt_stride, out,
+                                     tile_row0, tile_rows, tiles, tile_mode, part_o, part_ml, nsplit, heads, kv_rank, rot, rot_dims, 0,
+                                     inv_freq, scale, window, nullptr, stream);
+}
+
+extern "C" int exl2_latent_attn_tiles_ex(const void* q, int ldq, int q_head_stride, int q_rot_off, const float* q_abs, const void* cache,
+                                         int page, const int* row_seq, const int* row_pos, const int* block_table, int bt_stride, void* out,
+                                         const int* tile_row0, const int* tile_rows, int tiles, int tile_mode, float* part_o, float* part_ml,
+                                         int nsplit, int heads, int kv_rank, int rot, int rot_dims, int halves, const float* inv_freq,
+                                         float scale, int window, const float* sink, void* stream)
+{
     EXL2_REQUIRE(q && q_abs && cache && row_seq && row_pos && block_table && out && inv_freq && tile_row0, "latent_attn_tiles: null operand");
     EXL2_REQUIRE(tile_mode == 16 || tile_mode == 1, "latent_attn_tiles: tile_mode is 16 or 1");
     EXL2_REQUIRE(tile_mode == 1 || tile_rows, "latent_attn_tiles: tile_rows missing");
@@ -610,9 +689,10 @@ extern "C" int exl2_latent_attn_tiles(const void* q, int ldq, int q_head_stride,
     a.q = (const u16*)q; a.ldq = ldq; a.q_head_stride = q_head_stride; a.q_rot_off = q_rot_off; a.q_abs = q_abs;
     a.cache = (const u16*)cache; a.page = page; a.row_seq = row_seq; a.row_pos = row_pos; a.block_table = block_table; a.bt_stride = bt_stride;
     a.tile_row0 = tile_row0; a.tile_rows = tile_rows; a.out = (u16*)out; a.part_o = part_o; a.part_ml = part_ml; a.nsplit = nsplit;
-    a.H = heads; a.R = kv_rank; a.rot = rot; a.rot_dims = rot_dims; a.inv_freq = inv_freq; a.scale = scale; a.window = window;
+    a.H = heads; a.R = kv_rank; a.rot = rot; a.rot_dims = rot_dims; a.halves = halves; a.inv_freq = inv_freq; a.scale = scale; a.window = window; a.sink = sink;
     a.DP = (kv_rank + rot + 31) / 32 * 32;
-    const size_t smem = ((size_t)LA_KT * (a.DP + 8) + (size_t)kv_rank * LA_TS) * 2;      // (<= 78 KB: two workgroups per CU)
+    const size_t cs = (size_t)LA_KT * (a.DP + 8), ps = (size_t)4 * 16 * LA_TS;
+    const size_t smem = ((cs > ps ? cs : ps) + (size_t)kv_rank * LA_TS) * 2;      // (<= 78 KB: two workgroups per CU)
     hipStream_t s = (hipStream_t)stream;
     if (kv_rank <= 128) launch_lat_mfma<8>(a, tiles, tile_mode, smem, s);
     else if (kv_rank <= 256) launch_lat_mfma<16>(a, tiles, tile_mode, smem, s);

@@ -8,9 +8,11 @@
 //     a token shift  h + (h' - h) * shift  towards the previous token's normed row (kept per sequence slot),
 //   * the sandwich-normed residual step  x <- x + mult n_g(sublayer) w_out  with the grouped RMS norm  n_g(x) w_in  that feeds the next
 //     sublayer (and, for single-token steps, the short convolution over the last normed rows of the sequence),
+//   * the residual step of a layer whose mixer and feed-forward read ONE norm and pass gates of their own,
+//     x <- x + t sigmoid(g1) + (weighted expert sum) sigmoid(g2), with the RMS norm that feeds the next layer,
 //   * a token embedding plus a hashed (previous token, token) embedding under a grouped RMS norm (the previous token kept per slot),
 //   * the sparse-MoE router (softmax over all experts, selection by score + correction, weights from the uncorrected scores; or
-//     sigmoid scores, selection and weights by the scores themselves) and the per-expert row lists the grouped linear reads.
+//     sigmoid scores, selection and weights by the scores themselves, maybe among the experts of the best groups only) and the per-expert row lists the grouped linear reads.
 // Element type T of weights / operand copies: u16 = bfloat16 bits, float.
 #include "hw.h"
 #include "errors.h"
@@ -557,6 +559,197 @@ KERNEL void __launch_bounds__(256) sandwich_norm_vec_kernel(const SandwichArgs a
     }
 }
 
+// ---- gated residual step of a parallel layer --------------------------------------------------------------------------------------
+// n(v) = v / sqrt(mean(v^2) + eps).  One launch per row does
+//     x <- x + t sigmoid(g1) + sigmoid(g2) sum_k moe_w[k] moe_row[k],   t = y, or ya n(y) w_y + yb n(y2) w_y2 (two mixers side by side)
+//     x <- x + embed[id]  (ids nullable; `init`: x starts as embed[id], nothing is read from the stream)
+//     out = n(x) w_in                                                    (out nullable: only the additions)
+// Either addition may be absent (y, moe_y nullable) and so may the gates (nullable: 1).
+
+struct GatedResArgs
+{
+    float* x;
+    const float* y; const float* y2; const void* wy; const void* wy2; float ya, yb;      // wy nullable: y as it is
+    const float* g1; const float* g2; int ldg;               // gates in front of the sigmoid: [rows, ldg]
+    const float* moe_y; const float* moe_w; int top;         // [rows * top, width], [rows, top]
+    const void* table; const int* ids; int vocab, init;
+    const void* w_in; void* out; int out_f32;
+    const int* row_idx;                                      // nullable: output row r is made from stream row row_idx[r] (no addition then)
+    int width; float eps;
+};
+
+DEV float ro_sigmoid(float z) { return 1.0f / (1.0f + expf(-z)); }
+
+template <typename T>
+KERNEL void __launch_bounds__(256) gated_residual_kernel(const GatedResArgs a)
+{
+    DYN_SMEM(smem);
+    SHARED float part[4];
+    float* v = (float*)smem;
+    const int r = bid_x();
+    const long long src = a.row_idx ? a.row_idx[r] : r;
+    float* xr = a.x + src * a.width;
+    float my = 1.0f, my2 = 0.0f;
+    if (a.wy)
+    {
+        float s1 = 0.0f, s2 = 0.0f;
+        for (int i = tid(); i < a.width; i += 256)
+        {
+            const float p = a.y[src * a.width + i], q = a.y2[src * a.width + i];
+            s1 = fmaf(p, p, s1); s2 = fmaf(q, q, s2);
+        }
+        s1 = block_sum_256(s1, part);
+        s2 = block_sum_256(s2, part);
+        my = a.ya / sqrtf(s1 / (float)a.width + a.eps);
+        my2 = a.yb / sqrtf(s2 / (float)a.width + a.eps);
+    }
+    const T* er = nullptr;
+    if (a.ids) er = (const T*)a.table + (long long)min(max(a.ids[src], 0), a.vocab - 1) * a.width;
+    const bool adds = a.y || a.moe_y || er;
+    float ss = 0.0f;
+    for (int i = tid(); i < a.width; i += 256)
+    {
+        float xv = a.init ? 0.0f : xr[i];
+        if (a.y)
+        {
+            float t = a.y[src * a.width + i];
+            if (a.wy) t = t * my * ro_ld<T>((const T*)a.wy + i) + a.y2[src * a.width + i] * my2 * ro_ld<T>((const T*)a.wy2 + i);
+            xv = fmaf(t, a.g1 ? ro_sigmoid(a.g1[src * a.ldg + i]) : 1.0f, xv);
+        }
+        if (a.moe_y)
+        {
+            float t = 0.0f;
+            for (int k = 0; k < a.top; k++) t = fmaf(a.moe_w[src * a.top + k], a.moe_y[(src * a.top + k) * a.width + i], t);
+            xv = fmaf(t, a.g2 ? ro_sigmoid(a.g2[src * a.ldg + i]) : 1.0f, xv);
+        }
+        if (er) xv += ro_ld<T>(er + i);
+        if (adds) xr[i] = xv;
+        v[i] = xv;                                               // (a thread reads back only what it wrote)
+        ss = fmaf(xv, xv, ss);
+    }
+    if (!a.out) return;
+    ss = block_sum_256(ss, part);
+    const float rinv = 1.0f / sqrtf(ss / (float)a.width + a.eps);
+    for (int i = tid(); i < a.width; i += 256)
+    {
+        const float o = v[i] * rinv * ro_ld<T>((const T*)a.w_in + i);
+        if (a.out_f32) ((float*)a.out)[(long long)r * a.width + i] = o; else ro_st<T>((T*)a.out + (long long)r * a.width + i, o);
+    }
+}
+
+// The same step for rows of up to 256 * 4 * NC values in fours: a thread keeps its values in registers, every operand is requested
+// before the first is used (up to GR_MAX_TOP expert rows), the sums of y and y2 close in ONE exchange through LDS.
+#define GR_MAX_TOP 8
+
+template <typename T, int NC>
+KERNEL void __launch_bounds__(256) gated_residual_vec_kernel(const GatedResArgs a)
+{
+    SHARED float part[8];
+    SHARED float part2[4];
+    const int r = bid_x();
+    const long long src = a.row_idx ? a.row_idx[r] : r;
+    float* xr = a.x + src * a.width;
+    const f32x4 zero4 = {0.0f, 0.0f, 0.0f, 0.0f};
+    const T* er = nullptr;
+    if (a.ids) er = (const T*)a.table + (long long)min(max(a.ids[src], 0), a.vocab - 1) * a.width;
+    float mw[GR_MAX_TOP];
+    #pragma unroll
+    for (int k = 0; k < GR_MAX_TOP; k++) mw[k] = a.moe_y && k < a.top ? a.moe_w[src * a.top + k] : 0.0f;
+    f32x4 xv[NC], yv[NC], y2v[NC], wy[NC], wy2[NC], g1[NC], g2[NC], ev[NC], wi[NC], mv[NC][GR_MAX_TOP];
+    bool live[NC];
+    #pragma unroll
+    for (int e = 0; e < NC; e++)
+    {
+        const int i = 4 * (tid() + 256 * e);
+        live[e] = i < a.width;
+        xv[e] = yv[e] = y2v[e] = wy[e] = wy2[e] = g1[e] = g2[e] = ev[e] = wi[e] = zero4;
+        #pragma unroll
+        for (int k = 0; k < GR_MAX_TOP; k++) mv[e][k] = zero4;
+        if (!live[e]) continue;
+        if (!a.init) xv[e] = *(const f32x4*)(xr + i);
+        if (a.y)
+        {
+            yv[e] = *(const f32x4*)(a.y + src * a.width + i);
+            if (a.wy)
+            {
+                y2v[e] = *(const f32x4*)(a.y2 + src * a.width + i);
+                wy[e] = ro_ld4<T>((const T*)a.wy + i);
+                wy2[e] = ro_ld4<T>((const T*)a.wy2 + i);
+            }
+            if (a.g1) g1[e] = *(const f32x4*)(a.g1 + src * a.ldg + i);
+        }
+        if (a.moe_y)
+        {
+            #pragma unroll
+            for (int k = 0; k < GR_MAX_TOP; k++)
+                if (k < a.top) mv[e][k] = *(const f32x4*)(a.moe_y + (src * a.top + k) * a.width + i);
+            if (a.g2) g2[e] = *(const f32x4*)(a.g2 + src * a.ldg + i);
+        }
+        if (er) ev[e] = ro_ld4<T>(er + i);
+        if (a.out) wi[e] = ro_ld4<T>((const T*)a.w_in + i);
+    }
+    float my = 1.0f, my2 = 0.0f;
+    if (a.wy)
+    {
+        float s1 = 0.0f, s2 = 0.0f;
+        #pragma unroll
+        for (int e = 0; e < NC; e++)
+            #pragma unroll
+            for (int k = 0; k < 4; k++) { s1 = fmaf(yv[e][k], yv[e][k], s1); s2 = fmaf(y2v[e][k], y2v[e][k], s2); }
+        s1 = wave_allreduce_add(s1);
+        s2 = wave_allreduce_add(s2);
+        if (lane_id() == 0) { part[wave_id()] = s1; part[4 + wave_id()] = s2; }
+        block_sync();
+        my = a.ya / sqrtf((part[0] + part[1] + part[2] + part[3]) / (float)a.width + a.eps);
+        my2 = a.yb / sqrtf((part[4] + part[5] + part[6] + part[7]) / (float)a.width + a.eps);
+    }
+    const bool adds = a.y || a.moe_y || er;
+    float ss = 0.0f;
+    #pragma unroll
+    for (int e = 0; e < NC; e++)
+    {
+        if (!live[e]) continue;
+        #pragma unroll
+        for (int k = 0; k < 4; k++)
+        {
+            float x = xv[e][k];
+            if (a.y)
+            {
+                const float t = a.wy ? yv[e][k] * my * wy[e][k] + y2v[e][k] * my2 * wy2[e][k] : yv[e][k];
+                x = fmaf(t, a.g1 ? ro_sigmoid(g1[e][k]) : 1.0f, x);
+            }
+            if (a.moe_y)
+            {
+                float t = 0.0f;
+                #pragma unroll
+                for (int j = 0; j < GR_MAX_TOP; j++) t = fmaf(mw[j], mv[e][j][k], t);
+                x = fmaf(t, a.g2 ? ro_sigmoid(g2[e][k]) : 1.0f, x);
+            }
+            x += ev[e][k];
+            xv[e][k] = x;
+            ss = fmaf(x, x, ss);
+        }
+        if (adds) *(f32x4*)(xr + 4 * (tid() + 256 * e)) = xv[e];
+    }
+    if (!a.out) return;
+    ss = wave_allreduce_add(ss);
+    if (lane_id() == 0) part2[wave_id()] = ss;
+    block_sync();
+    const float rinv = 1.0f / sqrtf((part2[0] + part2[1] + part2[2] + part2[3]) / (float)a.width + a.eps);
+    #pragma unroll
+    for (int e = 0; e < NC; e++)
+    {
+        if (!live[e]) continue;
+        const int i = 4 * (tid() + 256 * e);
+        f32x4 o;
+        #pragma unroll
+        for (int k = 0; k < 4; k++) o[k] = xv[e][k] * rinv * wi[e][k];
+        if (a.out_f32) *(f32x4*)((float*)a.out + (long long)r * a.width + i) = o;
+        else *(u32x2*)((u16*)a.out + (long long)r * a.width + i) =
+                 (u32x2){(u32)f32_to_bf16(o[0]) | ((u32)f32_to_bf16(o[1]) << 16), (u32)f32_to_bf16(o[2]) | ((u32)f32_to_bf16(o[3]) << 16)};
+    }
+}
+
 // ---- token embedding + hashed token-pair embedding + norm ------------------------------------------------------------------------
 // x = n_g(table[t] * scale + pair[(t' mul_prev + t mul_cur) mod buckets]) w, t' = the sequence's previous token: the row in front
 // when that belongs to the same sequence, else what the slot keeps (prev_tok int32 [slots]); row `buckets` of the pair table at
@@ -625,13 +818,18 @@ KERNEL void __launch_bounds__(64) token_state_kernel(const int* ids, int* prev_t
 // One wave per token.  logits fp32 [rows, n_total]; scores = softmax over all n_total; the `top` largest (score + correction) win
 // (first index on a tie); weight = score / (sum of the chosen scores + 1e-20) * scale.  sigmoid_scores: scores = sigmoid(logits),
 // each on its own, and the weights are the chosen scores times scale (no renormalisation).  Rows of ids / wts are `ld` values apart;
+// group_keep < group_count: the experts stand in group_count equal groups of neighbours, a group scores the sum of its two largest
+// selection scores, and only the experts of the group_keep best groups can be chosen.  Rows of logits are ldl values apart.
 // extra_id >= 0: column `top` of every row names that expert with weight 1 (an expert every token uses, run with the chosen ones).
 
 #define ROUTE_MAX_PER_LANE 8
 
-KERNEL void __launch_bounds__(64) moe_route_kernel(const float* logits, const float* correction, int* ids, float* wts,
-                                                    int n_total, int top, float scale, int sigmoid_scores, int ld, int extra_id)
+KERNEL void __launch_bounds__(64) moe_route_kernel(const float* logits, int ldl, const float* correction, int* ids, float* wts,
+                                                    int n_total, int top, float scale, int sigmoid_scores, int ld, int extra_id,
+                                                    int group_count, int group_keep)
 {
+    SHARED float g_s[64 * ROUTE_MAX_PER_LANE];           // scores, when experts form groups
+    SHARED float g_sum[64 * ROUTE_MAX_PER_LANE];         // group scores
     const int r = bid_x();
     const int lane = lane_id();
     float s[ROUTE_MAX_PER_LANE], c[ROUTE_MAX_PER_LANE];
@@ -640,7 +838,7 @@ KERNEL void __launch_bounds__(64) moe_route_kernel(const float* logits, const fl
     for (int i = 0; i < ROUTE_MAX_PER_LANE; i++)
     {
         const int e = lane + 64 * i;
-        s[i] = e < n_total ? logits[(long long)r * n_total + e] : -INFINITY;
+        s[i] = e < n_total ? logits[(long long)r * ldl + e] : -INFINITY;
         mx = fmaxf(mx, s[i]);
     }
     mx = wave_allreduce_max(mx);
@@ -660,6 +858,36 @@ KERNEL void __launch_bounds__(64) moe_route_kernel(const float* logits, const fl
         const int e = lane + 64 * i;
         s[i] = s[i] / sum;
         c[i] = e < n_total ? s[i] + (correction ? correction[e] : 0.0f) : -INFINITY;
+    }
+    if (group_keep < group_count)
+    {
+        const int gs = n_total / group_count;
+        #pragma unroll
+        for (int i = 0; i < ROUTE_MAX_PER_LANE; i++)
+            if (lane + 64 * i < n_total) g_s[lane + 64 * i] = c[i];
+        block_sync();
+        for (int g = lane; g < group_count; g += 64)
+        {
+            float m1 = -INFINITY, m2 = -INFINITY;        // the two largest of the group
+            for (int j = 0; j < gs; j++)
+            {
+                const float v = g_s[g * gs + j];
+                if (v > m1) { m2 = m1; m1 = v; } else m2 = fmaxf(m2, v);
+            }
+            g_sum[g] = gs > 1 ? m1 + m2 : m1;
+        }
+        block_sync();
+        #pragma unroll
+        for (int i = 0; i < ROUTE_MAX_PER_LANE; i++)
+        {
+            const int e = lane + 64 * i;
+            if (e >= n_total) continue;
+            const int mine = e / gs;
+            const float my_sum = g_sum[mine];
+            int ahead = 0;                               // groups that come before this expert's (the first of equals does)
+            for (int g = 0; g < group_count; g++) ahead += (g_sum[g] > my_sum || (g_sum[g] == my_sum && g < mine)) ? 1 : 0;
+            if (ahead >= group_keep) c[i] = -INFINITY;
+        }
     }
     float chosen_sum = 0.0f;
     float my_w = 0.0f; int my_id = 0;                    // lane k keeps the k-th choice (top <= 64)
@@ -821,33 +1049,38 @@ extern "C" int exl2_add_layer_norm(float* x, const float* y, const void* w, cons
 
 static int moe_route_any(const float* logits, const float* correction, int* ids, float* wts, int rows, int n_total, int top,
                          float scale, int n_real, int* grp_count, int* grp_offset, int* grp_rows, int sigmoid_scores, int shared_slot,
-                         void* stream);
+                         int ldl, int group_count, int group_keep, void* stream);
 
 extern "C" int exl2_moe_route_scored(const float* logits, const float* correction, int* ids, float* wts, int rows, int n_total, int top,
                                      float scale, int n_real, int* grp_count, int* grp_offset, int* grp_rows, void* stream)
 {
-    return moe_route_any(logits, correction, ids, wts, rows, n_total, top, scale, n_real, grp_count, grp_offset, grp_rows, 0, 0, stream);
+    return moe_route_any(logits, correction, ids, wts, rows, n_total, top, scale, n_real, grp_count, grp_offset, grp_rows, 0, 0,
+                         n_total, 1, 1, stream);
 }
 
 extern "C" int exl2_moe_route_sigmoid(const float* logits, int* ids, float* wts, int rows, int n_total, int top, float scale,
                                       int shared_slot, int* grp_count, int* grp_offset, int* grp_rows, void* stream)
 {
     return moe_route_any(logits, nullptr, ids, wts, rows, n_total, top, scale, n_total + (shared_slot ? 1 : 0), grp_count, grp_offset,
-                         grp_rows, 1, shared_slot, stream);
+                         grp_rows, 1, shared_slot, n_total, 1, 1, stream);
 }
 
 static int moe_route_any(const float* logits, const float* correction, int* ids, float* wts, int rows, int n_total, int top,
                          float scale, int n_real, int* grp_count, int* grp_offset, int* grp_rows, int sigmoid_scores, int shared_slot,
-                         void* stream)
+                         int ldl, int group_count, int group_keep, void* stream)
 {
     const int ld = top + (shared_slot ? 1 : 0);                  // values per row of ids / wts
     EXL2_REQUIRE(logits && ids && wts, "moe_route_scored: null operand");
     EXL2_REQUIRE(n_total > 0 && n_total <= 64 * ROUTE_MAX_PER_LANE, "moe_route_scored: %d experts (at most %d)", n_total, 64 * ROUTE_MAX_PER_LANE);
     EXL2_REQUIRE(top > 0 && top <= 64 && top <= n_total, "moe_route_scored: top %d of %d", top, n_total);
+    EXL2_REQUIRE(ldl >= n_total, "moe_route: rows of %d logits %d apart", n_total, ldl);
+    EXL2_REQUIRE(group_count > 0 && group_keep > 0 && group_keep <= group_count && n_total % group_count == 0
+                     && top <= group_keep * (n_total / group_count),
+                 "moe_route: top %d of %d experts in %d groups, %d kept", top, n_total, group_count, group_keep);
     EXL2_REQUIRE(n_real >= 0 && n_real <= n_total + (shared_slot ? 1 : 0), "moe_route_scored: %d experts with weights of %d", n_real, n_total);
     if (rows <= 0) return EXL2_OK;
-    LAUNCH(moe_route_kernel, dim3(rows), dim3(64), 0, stream, logits, correction, ids, wts, n_total, top, scale, sigmoid_scores, ld,
-           shared_slot ? n_total : -1);
+    LAUNCH(moe_route_kernel, dim3(rows), dim3(64), 0, stream, logits, ldl, correction, ids, wts, n_total, top, scale, sigmoid_scores, ld,
+           shared_slot ? n_total : -1, group_count, group_keep);
     if (grp_count)
     {
         EXL2_REQUIRE(grp_offset && grp_rows, "moe_route_scored: grouped lists need offsets and rows");
@@ -859,6 +1092,13 @@ static int moe_route_any(const float* logits, const float* correction, int* ids,
     }
     HIP_TRY(hipGetLastError());
     return EXL2_OK;
+}
+
+extern "C" int exl2_moe_route_grouped(const float* logits, int ldl, int* ids, float* wts, int rows, int n_total, int top, float scale,
+                                      int group_count, int group_keep, int* grp_count, int* grp_offset, int* grp_rows, void* stream)
+{
+    return moe_route_any(logits, nullptr, ids, wts, rows, n_total, top, scale, n_total, grp_count, grp_offset, grp_rows, 1, 0, ldl,
+                         group_count, group_keep, stream);
 }
 
 extern "C" int exl2_add_rms_shift(float* x, const float* y, const float* moe_y, int top, float gain, float eps, const void* shift,
@@ -968,6 +1208,66 @@ extern "C" int exl2_sandwich_norm(float* x, const float* y, float ya, const floa
     }
     if (dtype == 0) LAUNCH(sandwich_norm_kernel<u16>, dim3(rows), dim3(256), smem, stream, a);
     else LAUNCH(sandwich_norm_kernel<float>, dim3(rows), dim3(256), smem, stream, a);
+    HIP_TRY(hipGetLastError());
+    return EXL2_OK;
+}
+
+extern "C" int exl2_gated_residual(float* x, const float* y, const float* y2, const void* wy, const void* wy2, float ya, float yb,
+                                   const float* g1, const float* g2, int ldg, const float* moe_y, const float* moe_w, int top,
+                                   const void* table, const int* ids, int vocab, int init, const void* w_in, void* out, int out_f32,
+                                   const int* row_idx, int dtype, int rows, int width, float eps, void* stream)
+{
+    EXL2_REQUIRE(x, "gated_residual: null stream");
+    EXL2_REQUIRE(dtype == 0 || dtype == 1, "gated_residual: dtype must be 0 (bfloat16) or 1 (float32)");
+    const bool adds = y || moe_y || ids;
+    EXL2_REQUIRE(adds || out, "gated_residual: neither an addition nor a norm");
+    EXL2_REQUIRE(!out || w_in, "gated_residual: an output needs the weight of its norm");
+    EXL2_REQUIRE((wy == nullptr) == (y2 == nullptr) && (wy == nullptr) == (wy2 == nullptr) && (!wy || y),
+                 "gated_residual: two normed results come with both weights");
+    EXL2_REQUIRE(!moe_y || (moe_w && top > 0), "gated_residual: expert outputs need their weights and their count per row");
+    EXL2_REQUIRE(!ids || (table && vocab > 0), "gated_residual: token ids need the table");
+    EXL2_REQUIRE(!init || (ids && !y && !moe_y), "gated_residual: the stream starts from the table alone");
+    EXL2_REQUIRE(!(row_idx && adds), "gated_residual: gathered rows take no addition");
+    EXL2_REQUIRE((!g1 && !g2) || ldg >= width, "gated_residual: gates of %d values %d apart", width, ldg);
+    EXL2_REQUIRE(width > 0 && (size_t)width * 4 <= 160 * 1024 - 64, "gated_residual: row of %d values does not fit the LDS", width);
+    if (rows <= 0) return EXL2_OK;
+    GatedResArgs a;
+    a.x = x; a.y = y; a.y2 = y2; a.wy = wy; a.wy2 = wy2; a.ya = ya; a.yb = yb; a.g1 = g1; a.g2 = g2; a.ldg = ldg; a.moe_y = moe_y;
+    a.moe_w = moe_w; a.top = top; a.table = table; a.ids = ids; a.vocab = vocab; a.init = init; a.w_in = w_in; a.out = out;
+    a.out_f32 = out_f32 || dtype == 1; a.row_idx = row_idx; a.width = width; a.eps = eps;
+    const auto al16 = [](const void* p) { return ((uintptr_t)p % 16) == 0; };
+    const bool vec = width % 4 == 0 && width <= 256 * 4 * 4 && (!moe_y || top <= GR_MAX_TOP) && ldg % 4 == 0 && al16(x) && al16(y) && al16(y2)
+                     && al16(wy) && al16(wy2) && al16(g1) && al16(g2) && al16(moe_y) && al16(table) && al16(w_in) && al16(out);
+    if (vec)
+    {
+        const int nc = width <= 1024 ? 1 : width <= 2048 ? 2 : 4;
+        if (dtype == 0)
+        {
+            if (nc == 1) LAUNCH((gated_residual_vec_kernel<u16, 1>), dim3(rows), dim3(256), 0, stream, a);
+            else if (nc == 2) LAUNCH((gated_residual_vec_kernel<u16, 2>), dim3(rows), dim3(256), 0, stream, a);
+            else LAUNCH((gated_residual_vec_kernel<u16, 4>), dim3(rows), dim3(256), 0, stream, a);
+        }
+        else
+        {
+            if (nc == 1) LAUNCH((gated_residual_vec_kernel<float, 1>), dim3(rows), dim3(256), 0, stream, a);
+            else if (nc == 2) LAUNCH((gated_residual_vec_kernel<float, 2>), dim3(rows), dim3(256), 0, stream, a);
+            else LAUNCH((gated_residual_vec_kernel<float, 4>), dim3(rows), dim3(256), 0, stream, a);
+        }
+        HIP_TRY(hipGetLastError());
+        return EXL2_OK;
+    }
+    const size_t smem = (size_t)width * 4;
+    if (smem > 48 * 1024)
+    {
+        static bool attr_done[EXL2_MAX_DEVICES];
+        if (exl2_first_on_device(attr_done))
+        {
+            (void)hipFuncSetAttribute((const void*)gated_residual_kernel<u16>, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024);
+            (void)hipFuncSetAttribute((const void*)gated_residual_kernel<float>, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024);
+        }
+    }
+    if (dtype == 0) LAUNCH(gated_residual_kernel<u16>, dim3(rows), dim3(256), smem, stream, a);
+    else LAUNCH(gated_residual_kernel<float>, dim3(rows), dim3(256), smem, stream, a);
     HIP_TRY(hipGetLastError());
     return EXL2_OK;
 }

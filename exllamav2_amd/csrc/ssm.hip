@@ -33,7 +33,7 @@ struct ConvArgs
     const void* w; const void* bias;         // [channels, taps], [channels]
     void* out; int ldo;                      // [rows, ldo] fp32, or the operand dtype (out_f32 == 0)
     int out_f32;
-    int residual;                            // 0: out = silu(conv + bias);  1: out = in + conv + bias (no activation)
+    int residual;                            // 0: out = silu(conv + bias);  1: out = in + conv + bias;  2: out = conv + bias (no activation)
     float* tail;                             // [slots, taps - 1, channels]: inputs of the last taps - 1 positions of every sequence
     const int* span_row0; const int* span_rows; const int* row_seq; const int* row_pos;
     int channels, taps;
@@ -89,7 +89,7 @@ KERNEL void __launch_bounds__(256) conv_silu_kernel(const ConvArgs a)
             if (k == a.taps - 1) win[k] = xin[i];                // after the shift the newest value belongs at index taps - 1
             if (k < a.taps) acc = fmaf(w[k], win[k], acc);
         }
-        const float o = a.residual ? xin[i] + acc : ss_silu(acc);
+        const float o = a.residual == 0 ? ss_silu(acc) : a.residual == 1 ? xin[i] + acc : acc;
         if (a.out_f32) ((float*)a.out)[(long long)(r0 + t0 + i) * a.ldo + c] = o;
         else ss_st<T>((T*)a.out + (long long)(r0 + t0 + i) * a.ldo + c, o);
     }
@@ -580,12 +580,13 @@ extern "C" int exl2_conv_silu_rows(const float* in, int ld, const void* w, const
 }
 
 /* The same convolution with a choice of output: residual = 0: silu(conv + bias); 1: in + conv + bias, no activation (what a
-   sublayer reads when its input passes a short convolution beside the identity).  out fp32, or the operand dtype with out_f32 = 0. */
+   sublayer reads when its input passes a short convolution beside the identity); 2: conv + bias, no activation.  out fp32, or the operand dtype with out_f32 = 0. */
 extern "C" int exl2_conv_rows_ex(const float* in, int ld, const void* w, const void* bias, void* out, int ldo, int out_f32, int residual,
                                  float* tail, const int* span_row0, const int* span_rows, int spans, int max_span_rows,
                                  const int* row_seq, const int* row_pos, int dtype, int channels, int taps, void* stream)
 {
     EXL2_REQUIRE(in && w && out && tail && span_row0 && span_rows && row_seq && row_pos, "conv_silu_rows: null operand");
+    EXL2_REQUIRE(residual >= 0 && residual <= 2, "conv_rows: unknown form %d", residual);
     EXL2_REQUIRE(dtype == 0 || dtype == 1, "conv_silu_rows: dtype must be 0 (bfloat16) or 1 (float32)");
     EXL2_REQUIRE(taps >= 1 && taps <= CONV_MAX_TAPS, "conv_silu_rows: %d taps (1 .. %d)", taps, CONV_MAX_TAPS);
     EXL2_REQUIRE(channels > 0 && ld >= channels && ldo >= channels, "conv_silu_rows: bad shape");

@@ -1,0 +1,591 @@
+// talk_attn.hip -- grouped-head softmax attention over a paged cache whose heads exchange their scores before the softmax, for
+// gfx950, + its C ABI.
+//
+// For a position p of a sequence and the keys j it sees (0 <= p - j < window):
+//     a_g,j = c tanh(q_g . k_j / c)  (q rotated and scaled; c = softcap, 0: none),    s_h,j = sum_g T[h, g] a_g,j  over ALL heads,
+//     o_h = sum_j exp(s_h,j) v_j / (exp(sink_h) + sum_j exp(s_h,j))                   (sink nullable: no such term)
+// Query head h reads key / value head h / (heads / kv_heads).  The cache holds rotated keys [pages, page, kv_heads, dim] and values
+// [pages, page, kv_heads, vdim] (window_attn.hip: exl2_kv_rot_append_ex writes them).  Rows of a step are a flat list (row r = position
+// row_pos[r] of sequence row_seq[r]); a row's result depends only on its own (sequence, position).  Scores, their exchange, the
+// softmax and the sums are fp32.
+#include "hw.h"
+#include "errors.h"
+#include <stdint.h>
+
+template <typename T> DEV float ta_ld(const T* p);
+template <> DEV float ta_ld<u16>(const u16* p) { return bf16_to_f32(*p); }
+template <> DEV float ta_ld<float>(const float* p) { return *p; }
+template <typename T> DEV void ta_st(T* p, float v);
+template <> DEV void ta_st<u16>(u16* p, float v) { *p = f32_to_bf16(v); }
+template <> DEV void ta_st<float>(float* p, float v) { *p = v; }
+// 16 bytes of T as floats
+template <typename T> struct TaVec;
+template <> struct TaVec<u16>
+{
+    static constexpr int N = 8;
+    static DEV void load(const u16* p, float* f)
+    {
+        const u32x4 v = *(const u32x4*)p;
+        #pragma unroll
+        for (int i = 0; i < 4; i++) { f[2 * i] = as_f32(v[i] << 16); f[2 * i + 1] = as_f32(v[i] & 0xffff0000u); }
+    }
+};
+template <> struct TaVec<float>
+{
+    static constexpr int N = 4;
+    static DEV void load(const float* p, float* f)
+    {
+        const f32x4 v = *(const f32x4*)p;
+        #pragma unroll
+        for (int i = 0; i < 4; i++) f[i] = v[i];
+    }
+};
+template <typename T> DEV void ta_ld2(const T* p, float& a, float& b);
+template <> DEV void ta_ld2<u16>(const u16* p, float& a, float& b) { const u32 v = *(const u32*)p; a = as_f32(v << 16); b = as_f32(v & 0xffff0000u); }
+template <> DEV void ta_ld2<float>(const float* p, float& a, float& b) { const f32x2 v = *(const f32x2*)p; a = v[0]; b = v[1]; }
+
+#define TA_NEG_BIG (-1.0e30f)
+#define TA_KEYS 64                           // keys per step of the row kernel
+#define TA_MAX_SPLIT 64
+
+struct TalkArgs
+{
+    const void* q;                           // [rows, H, dim] rotated, scaled
+    const void* k_cache; const void* v_cache;
+    const float* talk;                       // [H, H]
+    const float* sink;                       // [H] (nullable)
+    const int* row_seq; const int* row_pos; const int* block_table; int bt_stride, page, page_shift;
+    void* out;                               // [rows, H, vdim]
+    int H, G, dim, vdim, window; float softcap;
+    const int* row_list;                     // row kernel: the rows (nullable: 0, 1, ..)
+    const int* tile_row0; const int* tile_rows;      // tile kernel: runs of <= 16 consecutive positions of one sequence
+    // nsplit > 1 (row kernel): the key steps are dealt to nsplit workgroups; part_o fp32 [rows, H, nsplit, vdim] (sums relative to the
+    // partial maximum), part_ml fp32 [rows, H, nsplit, 2] (maximum, sum)
+    float* part_o; float* part_ml; int nsplit;
+};
+
+DEV float ta_soft_cap(float s, float cap) { return cap > 0.0f ? cap * tanhf(s / cap) : s; }
+DEV long long ta_cache_row(const TalkArgs& a, const int* bt, int j)
+{
+    const int pg = a.page_shift >= 0 ? j >> a.page_shift : j / a.page;
+    const int in = a.page_shift >= 0 ? j & (a.page - 1) : j % a.page;
+    return (long long)bt[pg] * a.page + in;
+}
+
+// ---- one row per workgroup (decoded tokens; every shape and dtype) ---------------------------------------------------------------
+// Keys go by TA_KEYS at a time: (kv head, up to four of its query heads, key) tasks make the capped scores, (head, key) tasks mix
+// them over all heads, a wave per head joins the step to the head's running softmax, and (kv head, up to four of its query heads,
+// pair of values) tasks add the step's weighted values to sums kept in LDS.
+
+// q [H, dim], o [H, vdim] (both rounded up to whole 16-byte pieces), scores a and mixed s [H, TA_KEYS], running maximum / sum / correction [H]
+HD size_t ta_row_smem(int H, int dim, int vdim)
+{
+    return sizeof(float) * ((size_t)((H * dim + 3) & ~3) + ((H * vdim + 3) & ~3) + 2 * (size_t)H * TA_KEYS + 3 * (size_t)H);
+}
+
+template <typename T, bool VEC>
+KERNEL void __launch_bounds__(256) talk_attn_row_kernel(const TalkArgs a)
+{
+    DYN_SMEM(smem);
+    SHARED long long krow[TA_KEYS];
+    const int H = a.H, G = a.G, dim = a.dim, vd = a.vdim, hpg = H / G, quads = (hpg + 3) / 4;
+    float* s_q = (float*)smem;
+    float* s_o = s_q + ((H * dim + 3) & ~3);
+    float* s_a = s_o + ((H * vd + 3) & ~3);
+    float* s_p = s_a + H * TA_KEYS;
+    float* s_m = s_p + H * TA_KEYS;
+    float* s_l = s_m + H;
+    float* s_c = s_l + H;
+    const int t = tid(), lane = lane_id(), wv = wave_id();
+    const int r = a.row_list ? a.row_list[bid_x()] : bid_x();
+    const int split = bid_y();
+    const int pos = a.row_pos[r];
+    const int* bt = a.block_table + (long long)a.row_seq[r] * a.bt_stride;
+    const int j_lo = max(0, pos - a.window + 1);
+    const int total = pos - j_lo + 1;
+    const int all_steps = (total + TA_KEYS - 1) / TA_KEYS;
+    const int per_split = (all_steps + a.nsplit - 1) / a.nsplit;
+    const int step0 = split * per_split, step1 = min(all_steps, step0 + per_split);
+    const T* qr = (const T*)a.q + (long long)r * H * dim;
+    for (int i = t; i < H * dim; i += 256) s_q[i] = ta_ld<T>(qr + i);
+    for (int i = t; i < H * vd; i += 256) s_o[i] = 0.0f;
+    const bool with_sink = a.sink && split == 0;                 // the sink counts once
+    for (int i = t; i < H; i += 256) { s_m[i] = with_sink ? a.sink[i] : TA_NEG_BIG; s_l[i] = with_sink ? 1.0f : 0.0f; }
+    for (int step = step0; step < step1; step++)
+    {
+        const int k0 = step * TA_KEYS, nc = min(TA_KEYS, total - k0);
+        if (t < TA_KEYS) krow[t] = ta_cache_row(a, bt, j_lo + k0 + min(t, nc - 1));
+        block_sync();
+        for (int i = t; i < G * quads * TA_KEYS; i += 256)
+        {
+            const int key = i % TA_KEYS, gq = i / TA_KEYS, g = gq / quads, h0 = g * hpg + (gq % quads) * 4, nh = min(4, g * hpg + hpg - h0);
+            const T* kr = (const T*)a.k_cache + (krow[key] * G + g) * dim;
+            float d[4] = {0.0f, 0.0f, 0.0f, 0.0f};
+            if (VEC)
+            {
+                constexpr int N = TaVec<T>::N;
+                #pragma unroll 4
+                for (int e = 0; e < dim; e += N)
+                {
+                    float kv[N];
+                    TaVec<T>::load(kr + e, kv);
+                    #pragma unroll
+                    for (int n = 0; n < 4; n++)
+                    {
+                        const float* qh = s_q + (h0 + min(n, nh - 1)) * dim + e;
+                        #pragma unroll
+                        for (int x = 0; x < N; x++) d[n] = fmaf(qh[x], kv[x], d[n]);
+                    }
+                }
+            }
+            else
+                for (int e = 0; e < dim; e++)
+                {
+                    const float kv = ta_ld<T>(kr + e);
+                    #pragma unroll
+                    for (int n = 0; n < 4; n++) d[n] = fmaf(s_q[(h0 + min(n, nh - 1)) * dim + e], kv, d[n]);
+                }
+            #pragma unroll
+            for (int n = 0; n < 4; n++)
+                if (n < nh) s_a[(h0 + n) * TA_KEYS + key] = ta_soft_cap(d[n], a.softcap);
+        }
+        block_sync();
+        for (int i = t; i < H * TA_KEYS; i += 256)
+        {
+            const int key = i % TA_KEYS, h = i / TA_KEYS;
+            const float* tr = a.talk + h * H;
+            float s = 0.0f;
+            for (int g = 0; g < H; g++) s = fmaf(tr[g], s_a[g * TA_KEYS + key], s);
+            s_p[i] = key < nc ? s : TA_NEG_BIG;
+        }
+        block_sync();
+        for (int h = wv; h < H; h += 4)
+        {
+            const float s = s_p[h * TA_KEYS + lane];
+            const float m0 = s_m[h], m1 = fmaxf(m0, wave_allreduce_max(s));
+            const float p = lane < nc ? expf(s - m1) : 0.0f;
+            const float ps = wave_allreduce_add(p);
+            s_p[h * TA_KEYS + lane] = p;
+            if (lane == 0)
+            {
+                const float c = expf(m0 - m1);
+                s_c[h] = c; s_m[h] = m1; s_l[h] = s_l[h] * c + ps;
+            }
+        }
+        block_sync();
+        const int vw = VEC ? 2 : 1;
+        for (int i = t; i < G * quads * (vd / vw); i += 256)
+        {
+            const int e = (i % (vd / vw)) * vw, gq = i / (vd / vw), g = gq / quads, h0 = g * hpg + (gq % quads) * 4, nh = min(4, g * hpg + hpg - h0);
+            float o0[4], o1[4];
+            #pragma unroll
+            for (int n = 0; n < 4; n++)
+            {
+                const int h = h0 + min(n, nh - 1);
+                o0[n] = s_o[h * vd + e] * s_c[h];
+                o1[n] = VEC ? s_o[h * vd + e + 1] * s_c[h] : 0.0f;
+            }
+            #pragma unroll 8
+            for (int key = 0; key < nc; key++)
+            {
+                const T* vr = (const T*)a.v_cache + (krow[key] * G + g) * vd + e;
+                float v0, v1 = 0.0f;
+                if (VEC) ta_ld2<T>(vr, v0, v1); else v0 = ta_ld<T>(vr);
+                #pragma unroll
+                for (int n = 0; n < 4; n++)
+                {
+                    const float p = s_p[(h0 + min(n, nh - 1)) * TA_KEYS + key];
+                    o0[n] = fmaf(p, v0, o0[n]);
+                    if (VEC) o1[n] = fmaf(p, v1, o1[n]);
+                }
+            }
+            #pragma unroll
+            for (int n = 0; n < 4; n++)
+                if (n < nh) { s_o[(h0 + n) * vd + e] = o0[n]; if (VEC) s_o[(h0 + n) * vd + e + 1] = o1[n]; }
+        }
+        block_sync();                                            // krow and the probabilities are rewritten by the next step
+    }
+    block_sync();
+    for (int i = t; i < H * vd; i += 256)
+    {
+        const int h = i / vd;
+        if (a.nsplit == 1) { ta_st<T>((T*)a.out + (long long)r * H * vd + i, s_l[h] > 0.0f ? s_o[i] / s_l[h] : 0.0f); continue; }
+        const long long pi = ((long long)r * H + h) * a.nsplit + split;
+        a.part_o[pi * vd + i % vd] = s_o[i];
+        if (i % vd == 0) { a.part_ml[pi * 2] = s_m[h]; a.part_ml[pi * 2 + 1] = s_l[h]; }
+    }
+}
+
+// grid (rows, heads): joins the nsplit partial results of a row's head
+template <typename T>
+KERNEL void __launch_bounds__(64) talk_attn_merge_kernel(const TalkArgs a)
+{
+    const int r = a.row_list ? a.row_list[bid_x()] : bid_x(), h = bid_y();
+    const long long p0 = ((long long)r * a.H + h) * a.nsplit;
+    const int lane = lane_id();
+    const float m = lane < a.nsplit ? a.part_ml[(p0 + lane) * 2] : TA_NEG_BIG;       // (nsplit <= 64: a lane per split)
+    const float l = lane < a.nsplit ? a.part_ml[(p0 + lane) * 2 + 1] : 0.0f;
+    const float mx = wave_allreduce_max(m);
+    const float c = m > 0.5f * TA_NEG_BIG ? expf(m - mx) : 0.0f;
+    const float lsum = wave_allreduce_add(l * c);
+    const float inv = lsum > 0.0f ? 1.0f / lsum : 0.0f;
+    for (int e0 = 0; e0 < a.vdim; e0 += 64)
+    {
+        const int e = e0 + lane;
+        float o = 0.0f;
+        #pragma unroll 8
+        for (int sp = 0; sp < a.nsplit; sp++)
+            o = fmaf(e < a.vdim ? a.part_o[(p0 + sp) * a.vdim + e] : 0.0f, shfl_idx_f32(c, sp), o);
+        if (e < a.vdim) ta_st<T>((T*)a.out + ((long long)r * a.H + h) * a.vdim + e, o * inv);
+    }
+}
+
+// ---- bfloat16 on the matrix cores: portions of prompts -----------------------------------------------------------------------------
+// Workgroup = one tile of <= 16 consecutive positions of one sequence x ALL heads; wave w owns query heads 4 w .. 4 w + 3 (their query
+// rows as operands and their output accumulators in registers).  Keys go by BK at a time in three stages:
+//   1. scores of the wave's heads, S^T = K Q^T (A = key rows straight from the cache: a lane's 8 values are one 16-byte load; the next
+//      step's are requested before stage 2), capped, to LDS as fp32 [head][query][key];
+//   2. the exchange: a lane takes KPL consecutive keys of one query for all heads, s_h = sum_g T[h, g] a_g -- on the fp32 matrix cores in
+//      their 16-block form, where every lane's own column goes through a 4 x 1 product per (four heads out, one head in) without any
+//      lane movement -- and puts the mixed scores back in place;
+//   3. the wave's heads again: online softmax (columns = queries), probabilities to bfloat16 in registers (the accumulator layout of
+//      S^T is the operand layout of O^T += V^T P^T with the keys of a product taken in the order {4 g .. + 3 of block 0, of block 1}),
+//      values through a wave-private LDS tile and transposing reads.
+// Two barriers per step: stage 1 of the next step writes only what its own wave read in stage 3.
+
+#define TM_Q 16
+
+template <int DIM, int VDIM, int NW, int BK>
+struct TalkTile
+{
+    static constexpr int HMAX = 4 * NW, SS = BK + 4, TS = HMAX + 4, VSTR = VDIM + 16, NBLK = BK / 16;
+    static constexpr size_t smem = sizeof(float) * ((size_t)HMAX * TM_Q * SS + (size_t)HMAX * TS) + sizeof(u16) * (size_t)NW * BK * VSTR;
+};
+
+DEV u32 tm_pack2(float lo, float hi) { return (u32)f32_to_bf16(lo) | ((u32)f32_to_bf16(hi) << 16); }
+
+template <int DIM, int VDIM, int NW, int BK>
+KERNEL void __launch_bounds__(64 * NW, 1) talk_attn_tile_kernel(const TalkArgs a)
+{
+    DYN_SMEM(smem);
+    typedef TalkTile<DIM, VDIM, NW, BK> TT;
+    constexpr int SS = TT::SS, TS = TT::TS, VSTR = TT::VSTR, NBLK = TT::NBLK, KK = DIM / 32, DB = VDIM / 16;
+    constexpr int KPL = TM_Q * BK / (64 * NW);                   // stage 2: keys per lane
+    constexpr int VP = BK * VDIM / 8 / 64;                       // stage 3: 16-byte value pieces per lane
+    constexpr int VPR = VDIM / 8;                                // pieces of a value row
+    constexpr int NT = NW;                                       // output tiles of four heads
+    float* s_s = (float*)smem;                                   // [HMAX][TM_Q][SS]
+    float* s_t = s_s + TT::HMAX * TM_Q * SS;                     // [HMAX][TS]: T, zero past H
+    u16* s_v = (u16*)(s_t + TT::HMAX * TS);                      // [NW][BK][VSTR]
+
+    const int t = tid(), lane = lane_id(), wv = wave_id();
+    const int qi = lane & 15, g = lane >> 4;
+    const int H = a.H, G = a.G, hpg = H / G;
+    const int tile_i = gdim_x() - 1 - bid_x();                   // the longest key lists first
+    const int r0 = a.tile_row0[tile_i], n_rows = a.tile_rows[tile_i];
+    const int p0 = a.row_pos[r0], p_last = p0 + n_rows - 1;
+    const int* bt = a.block_table + (long long)a.row_seq[r0] * a.bt_stride;
+    const int j_lo = max(0, p0 - a.window + 1);
+    const int total = p_last - j_lo + 1;
+    const int n_steps = (total + BK - 1) / BK;
+    const u16* kc = (const u16*)a.k_cache; const u16* vc = (const u16*)a.v_cache;
+    u16* my_v = s_v + wv * BK * VSTR;
+
+    for (int i = t; i < TT::HMAX * TT::HMAX; i += 64 * NW)
+    {
+        const int h = i / TT::HMAX, c = i % TT::HMAX;
+        s_t[h * TS + c] = h < H && c < H ? a.talk[h * H + c] : 0.0f;
+    }
+    const int nh = max(0, min(4, H - 4 * wv));                   // heads of this wave
+    const int h0 = min(4 * wv, H - 1);
+    int kvh[4];
+    #pragma unroll
+    for (int n = 0; n < 4; n++) kvh[n] = min(h0 + n, H - 1) / hpg;
+
+    const int qrow = r0 + min(qi, n_rows - 1), qpos = p0 + min(qi, n_rows - 1), q_lo = qpos - a.window + 1;
+    u32x4 qb[4][KK];
+    f32x4 ot[4][DB];
+    float m_run[4], l_run[4];
+    #pragma unroll
+    for (int n = 0; n < 4; n++)
+    {
+        const int h = min(h0 + n, H - 1);
+        const u16* qp = (const u16*)a.q + ((long long)qrow * H + h) * DIM + 8 * g;
+        #pragma unroll
+        for (int kk = 0; kk < KK; kk++) qb[n][kk] = *(const u32x4*)(qp + 32 * kk);
+        #pragma unroll
+        for (int d = 0; d < DB; d++) ot[n][d] = (f32x4){0.0f, 0.0f, 0.0f, 0.0f};
+        m_run[n] = a.sink ? a.sink[h] : TA_NEG_BIG;
+        l_run[n] = a.sink ? 1.0f : 0.0f;
+    }
+
+    // rows in the cache of what this lane loads in a step: its key of every 16-key block, and the rows of its value pieces
+    long long krow[NBLK], vrow[VP];
+    u32x4 kf[NBLK][KK], vreg[VP];
+    auto lookup = [&](int step) {
+        #pragma unroll
+        for (int b = 0; b < NBLK; b++) krow[b] = ta_cache_row(a, bt, j_lo + min(step * BK + 16 * b + qi, total - 1));
+    };
+    auto lookup_v = [&](int step) {
+        #pragma unroll
+        for (int i = 0; i < VP; i++) vrow[i] = ta_cache_row(a, bt, j_lo + min(step * BK + (lane + 64 * i) / VPR, total - 1));
+    };
+    auto load_k = [&](int kv) {
+        #pragma unroll
+        for (int b = 0; b < NBLK; b++)
+            #pragma unroll
+            for (int kk = 0; kk < KK; kk++) kf[b][kk] = *(const u32x4*)(kc + (krow[b] * G + kv) * DIM + 32 * kk + 8 * g);
+    };
+    auto load_v = [&](int kv) {
+        #pragma unroll
+        for (int i = 0; i < VP; i++) vreg[i] = *(const u32x4*)(vc + (vrow[i] * G + kv) * VDIM + ((lane + 64 * i) % VPR) * 8);
+    };
+    if (nh > 0) { lookup(0); load_k(kvh[0]); lookup_v(0); load_v(kvh[0]); }
+    block_sync();
+
+    for (int step = 0; step < n_steps; step++)
+    {
+        const int k0 = step * BK;
+        // ---- 1: scores of this wave's heads
+        #pragma unroll
+        for (int n = 0; n < 4; n++)
+        {
+            if (n >= nh) break;
+            if (n > 0 && kvh[n] != kvh[n - 1]) load_k(kvh[n]);
+            float* sr = s_s + ((h0 + n) * TM_Q + qi) * SS + 4 * g;
+            #pragma unroll
+            for (int b = 0; b < NBLK; b++)
+            {
+                f32x4 st = {0.0f, 0.0f, 0.0f, 0.0f};
+                #pragma unroll
+                for (int kk = 0; kk < KK; kk++) st = mfma_16x16x32_bf16(kf[b][kk], qb[n][kk], st);
+                #pragma unroll
+                for (int r = 0; r < 4; r++) st[r] = ta_soft_cap(st[r], a.softcap);
+                *(f32x4*)(sr + 16 * b) = st;
+            }
+        }
+        block_sync_lds();
+        if (nh > 0 && step + 1 < n_steps) { lookup(step + 1); load_k(kvh[0]); }
+        // ---- 2: the exchange between the heads, in place
+        {
+            const int task = t * KPL, q2 = task / BK, c2 = task % BK;
+            float* sp = s_s + q2 * SS + c2;
+            f32x4 mx[NT][KPL];
+            #pragma unroll
+            for (int i = 0; i < NT; i++)
+                #pragma unroll
+                for (int e = 0; e < KPL; e++) mx[i][e] = (f32x4){0.0f, 0.0f, 0.0f, 0.0f};
+            for (int c4 = 0; c4 < H; c4 += 4)
+            {
+                f32x4 tv[NT];
+                #pragma unroll
+                for (int i = 0; i < NT; i++) tv[i] = *(const f32x4*)(s_t + (4 * i + (lane & 3)) * TS + c4);
+                #pragma unroll
+                for (int k = 0; k < 4; k++)
+                {
+                    const int c = min(c4 + k, H - 1);            // (past the last head T is zero)
+                    float sv[KPL];
+                    #pragma unroll
+                    for (int e = 0; e < KPL; e++) sv[e] = sp[c * TM_Q * SS + e];
+                    #pragma unroll
+                    for (int i = 0; i < NT; i++)
+                        #pragma unroll
+                        for (int e = 0; e < KPL; e++) mx[i][e] = mfma_4x4x1_f32(tv[i][k], sv[e], mx[i][e]);
+                }
+            }
+            wave_sync();
+            #pragma unroll
+            for (int i = 0; i < NT; i++)
+                #pragma unroll
+                for (int r = 0; r < 4; r++)
+                    if (4 * i + r < H)
+                    {
+                        #pragma unroll
+                        for (int e = 0; e < KPL; e++) sp[(4 * i + r) * TM_Q * SS + e] = mx[i][e][r];
+                    }
+        }
+        block_sync_lds();
+        // ---- 3: softmax and values of this wave's heads
+        #pragma unroll
+        for (int n = 0; n < 4; n++)
+        {
+            if (n >= nh) break;
+            if (n == 0 || kvh[n] != kvh[n - 1])
+            {
+                if (n > 0) { load_v(kvh[n]); wave_sync(); }
+                #pragma unroll
+                for (int i = 0; i < VP; i++) *(u32x4*)(my_v + ((lane + 64 * i) / VPR) * VSTR + ((lane + 64 * i) % VPR) * 8) = vreg[i];
+                wave_sync();
+            }
+            const float* sr = s_s + ((h0 + n) * TM_Q + qi) * SS + 4 * g;
+            float sc[4 * NBLK];
+            float m_loc = TA_NEG_BIG;
+            #pragma unroll
+            for (int b = 0; b < NBLK; b++)
+            {
+                const f32x4 v = *(const f32x4*)(sr + 16 * b);
+                #pragma unroll
+                for (int r = 0; r < 4; r++)
+                {
+                    const int j = j_lo + k0 + 16 * b + 4 * g + r;
+                    sc[4 * b + r] = j <= qpos && j >= q_lo ? v[r] : TA_NEG_BIG;
+                    m_loc = fmaxf(m_loc, sc[4 * b + r]);
+                }
+            }
+            m_loc = fmaxf(m_loc, shfl_xor_f32(m_loc, 16));
+            m_loc = fmaxf(m_loc, shfl_xor_f32(m_loc, 32));
+            const float m_new = fmaxf(m_run[n], m_loc);
+            const float alpha = fast_exp(m_run[n] - m_new);
+            float p_sum = 0.0f;
+            u32x4 pb[NBLK / 2];
+            #pragma unroll
+            for (int e2 = 0; e2 < 2 * NBLK; e2++)
+            {
+                const float pa = sc[2 * e2] > 0.5f * TA_NEG_BIG ? fast_exp(sc[2 * e2] - m_new) : 0.0f;
+                const float pc = sc[2 * e2 + 1] > 0.5f * TA_NEG_BIG ? fast_exp(sc[2 * e2 + 1] - m_new) : 0.0f;
+                p_sum += pa + pc;
+                pb[e2 / 4][e2 % 4] = tm_pack2(pa, pc);
+            }
+            p_sum += shfl_xor_f32(p_sum, 16);
+            p_sum += shfl_xor_f32(p_sum, 32);
+            l_run[n] = l_run[n] * alpha + p_sum;
+            m_run[n] = m_new;
+            const u16* vbase = my_v + (4 * g + (qi >> 2)) * VSTR + 4 * (qi & 3);
+            #pragma unroll
+            for (int d = 0; d < DB; d++)
+            {
+                ot[n][d][0] *= alpha; ot[n][d][1] *= alpha; ot[n][d][2] *= alpha; ot[n][d][3] *= alpha;
+                #pragma unroll
+                for (int m2 = 0; m2 < NBLK / 2; m2++)
+                {
+                    const f16x4 lo = lds_read_tr16_b64((const f16*)(vbase + (32 * m2) * VSTR + 16 * d));
+                    const f16x4 hi = lds_read_tr16_b64((const f16*)(vbase + (32 * m2 + 16) * VSTR + 16 * d));
+                    const u32x2 l2 = __builtin_bit_cast(u32x2, lo), h2 = __builtin_bit_cast(u32x2, hi);
+                    ot[n][d] = mfma_16x16x32_bf16((u32x4){l2[0], l2[1], h2[0], h2[1]}, pb[m2], ot[n][d]);
+                }
+            }
+        }
+        wave_sync();                                             // the wave is done with its value tile
+        if (nh > 0 && step + 1 < n_steps) { lookup_v(step + 1); load_v(kvh[0]); }
+    }
+
+    if (qi >= n_rows) return;
+    #pragma unroll
+    for (int n = 0; n < 4; n++)
+    {
+        if (n >= nh) break;
+        const float inv = l_run[n] > 0.0f ? 1.0f / l_run[n] : 0.0f;
+        u16* op = (u16*)a.out + ((long long)qrow * H + h0 + n) * VDIM + 4 * g;
+        #pragma unroll
+        for (int d = 0; d < DB; d++)
+            *(u32x2*)(op + 16 * d) = (u32x2){tm_pack2(ot[n][d][0] * inv, ot[n][d][1] * inv), tm_pack2(ot[n][d][2] * inv, ot[n][d][3] * inv)};
+    }
+}
+
+template <int DIM, int VDIM, int NW, int BK>
+static void tm_launch_one(const TalkArgs& a, int tiles, hipStream_t s)
+{
+    static bool attr_done[EXL2_MAX_DEVICES];
+    static_assert(TalkTile<DIM, VDIM, NW, BK>::smem <= 160 * 1024, "the tile fits the LDS");
+    if (exl2_first_on_device(attr_done))
+        (void)hipFuncSetAttribute((const void*)talk_attn_tile_kernel<DIM, VDIM, NW, BK>, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024);
+    LAUNCH((talk_attn_tile_kernel<DIM, VDIM, NW, BK>), dim3(tiles), dim3(64 * NW), (TalkTile<DIM, VDIM, NW, BK>::smem), s, a);
+}
+
+template <int DIM, int VDIM>
+static void tm_launch(const TalkArgs& a, int tiles, hipStream_t s)
+{
+    if (a.H <= 16) tm_launch_one<DIM, VDIM, 4, 64>(a, tiles, s);
+    else tm_launch_one<DIM, VDIM, 8, 32>(a, tiles, s);
+}
+
+// ---- C ABI ----------------------------------------------------------------------------------------------------------------------
+
+static int ta_log2_exact(int x) { int sh = 0; while ((1 << sh) < x) sh++; return x > 0 && (1 << sh) == x ? sh : -1; }
+
+/* 1 if exl2_talk_attn_tiles takes these sizes (bfloat16) */
+extern "C" int exl2_talk_attn_tiles_supported(int heads, int dim, int vdim)
+{
+    return heads <= 32 && ((dim == 32 && vdim == 32) || ((dim == 64 || dim == 128) && (vdim == 64 || vdim == 128)));
+}
+
+static int ta_fill(TalkArgs& a, const void* q, const void* k_cache, const void* v_cache, const float* talk, const float* sink,
+                   const int* row_seq, const int* row_pos, const int* block_table, int bt_stride, int page, void* out, int heads,
+                   int kv_heads, int dim, int vdim, int window, float softcap)
+{
+    EXL2_REQUIRE(q && k_cache && v_cache && talk && row_seq && row_pos && block_table && out, "talk_attn: null operand");
+    EXL2_REQUIRE(heads > 0 && kv_heads > 0 && heads % kv_heads == 0 && dim > 0 && vdim > 0, "talk_attn: bad head shape");
+    EXL2_REQUIRE(page > 0 && window > 0 && softcap >= 0.0f, "talk_attn: bad window / paging / soft cap");
+    a.q = q; a.k_cache = k_cache; a.v_cache = v_cache; a.talk = talk; a.sink = sink; a.row_seq = row_seq; a.row_pos = row_pos;
+    a.block_table = block_table; a.bt_stride = bt_stride; a.page = page; a.page_shift = ta_log2_exact(page); a.out = out; a.H = heads;
+    a.G = kv_heads; a.dim = dim; a.vdim = vdim; a.window = window; a.softcap = softcap; a.row_list = nullptr; a.tile_row0 = nullptr;
+    a.tile_rows = nullptr; a.part_o = nullptr; a.part_ml = nullptr; a.nsplit = 1;
+    return EXL2_OK;
+}
+
+extern "C" int exl2_talk_attn(const void* q, const void* k_cache, const void* v_cache, const float* talk, const float* sink,
+                              const int* row_seq, const int* row_pos, const int* block_table, int bt_stride, int page, void* out,
+                              const int* row_list, int rows, float* part_o, float* part_ml, int nsplit, int dtype, int heads, int kv_heads,
+                              int dim, int vdim, int window, float softcap, void* stream)
+{
+    TalkArgs a;
+    const int rc = ta_fill(a, q, k_cache, v_cache, talk, sink, row_seq, row_pos, block_table, bt_stride, page, out, heads, kv_heads, dim,
+                           vdim, window, softcap);
+    if (rc != EXL2_OK) return rc;
+    EXL2_REQUIRE(dtype == 0 || dtype == 1, "talk_attn: dtype must be 0 (bfloat16) or 1 (float32)");
+    EXL2_REQUIRE(nsplit >= 1 && nsplit <= TA_MAX_SPLIT && (nsplit == 1 || (part_o && part_ml)), "talk_attn: key splits (1 .. %d) need scratch", TA_MAX_SPLIT);
+    const size_t smem = ta_row_smem(heads, dim, vdim);
+    if (smem + 1024 > 160 * 1024)
+        EXL2_FAIL(EXL2_E_UNSUPPORTED, "talk_attn: %d heads of %d / %d values do not fit the LDS", heads, dim, vdim);
+    if (rows <= 0) return EXL2_OK;
+    a.row_list = row_list; a.part_o = part_o; a.part_ml = part_ml; a.nsplit = nsplit;
+    const int vn = dtype == 0 ? 8 : 4;
+    const bool vec = dim % vn == 0 && vdim % 2 == 0 && ((uintptr_t)k_cache % 16) == 0 && ((uintptr_t)v_cache % 8) == 0;
+    static bool attr_done[EXL2_MAX_DEVICES];
+    if (exl2_first_on_device(attr_done))
+    {
+        (void)hipFuncSetAttribute((const void*)talk_attn_row_kernel<u16, true>, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024 - 1024);
+        (void)hipFuncSetAttribute((const void*)talk_attn_row_kernel<u16, false>, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024 - 1024);
+        (void)hipFuncSetAttribute((const void*)talk_attn_row_kernel<float, true>, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024 - 1024);
+        (void)hipFuncSetAttribute((const void*)talk_attn_row_kernel<float, false>, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024 - 1024);
+    }
+    const dim3 grid(rows, nsplit);
+    if (dtype == 0)
+    {
+        if (vec) LAUNCH((talk_attn_row_kernel<u16, true>), grid, dim3(256), smem, stream, a);
+        else LAUNCH((talk_attn_row_kernel<u16, false>), grid, dim3(256), smem, stream, a);
+        if (nsplit > 1) LAUNCH(talk_attn_merge_kernel<u16>, dim3(rows, heads), dim3(64), 0, stream, a);
+    }
+    else
+    {
+        if (vec) LAUNCH((talk_attn_row_kernel<float, true>), grid, dim3(256), smem, stream, a);
+        else LAUNCH((talk_attn_row_kernel<float, false>), grid, dim3(256), smem, stream, a);
+        if (nsplit > 1) LAUNCH(talk_attn_merge_kernel<float>, dim3(rows, heads), dim3(64), 0, stream, a);
+    }
+    HIP_TRY(hipGetLastError());
+    return EXL2_OK;
+}
+
+extern "C" int exl2_talk_attn_tiles(const void* q, const void* k_cache, const void* v_cache, const float* talk, const float* sink,
+                                    const int* row_seq, const int* row_pos, const int* block_table, int bt_stride, int page, void* out,
+                                    const int* tile_row0, const int* tile_rows, int tiles, int heads, int kv_heads, int dim, int vdim,
+                                    int window, float softcap, void* stream)
+{
+    TalkArgs a;
+    const int rc = ta_fill(a, q, k_cache, v_cache, talk, sink, row_seq, row_pos, block_table, bt_stride, page, out, heads, kv_heads, dim,
+                           vdim, window, softcap);
+    if (rc != EXL2_OK) return rc;
+    EXL2_REQUIRE(tile_row0 && tile_rows, "talk_attn_tiles: tiles missing");
+    if (!exl2_talk_attn_tiles_supported(heads, dim, vdim))
+        EXL2_FAIL(EXL2_E_UNSUPPORTED, "talk_attn_tiles: %d heads of %d / %d values outside the matrix-core form", heads, dim, vdim);
+    if (tiles <= 0) return EXL2_OK;
+    a.tile_row0 = tile_row0; a.tile_rows = tile_rows;
+    hipStream_t s = (hipStream_t)stream;
+    if (dim == 32) tm_launch<32, 32>(a, tiles, s);
+    else if (dim == 64 && vdim == 64) tm_launch<64, 64>(a, tiles, s);
+    else if (dim == 64) tm_launch<64, 128>(a, tiles, s);
+    else if (vdim == 64) tm_launch<128, 64>(a, tiles, s);
+    else tm_launch<128, 128>(a, tiles, s);
+    HIP_TRY(hipGetLastError());
+    return EXL2_OK;
+}

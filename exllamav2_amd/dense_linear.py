@@ -33,3 +33,44 @@ class DenseLinear:
 
     def weight_bytes(self) -> int:
         return self.weight.numel() * self.weight.element_size()
+
+
+class JoinedFront:
+    """ONE linear for everything that reads a layer's input: the members' projections (`member.front_part` = (weight [n, width], bias
+    fp32 [n] | None), left by a module built with `joined=True`) stacked behind each other, every part starting at a multiple of four
+    columns; a member learns where its columns start (`front_base`).  Plain (weight, bias) pairs may join; `bases` lists every
+    member's first column in order."""
+
+    def __init__(self, ext, key: str, members):
+        weights, biases, self.bases, at = [], [], [], 0
+        for m in members:
+            w, b = m if isinstance(m, tuple) else m.front_part
+            self.bases.append(at)
+            if not isinstance(m, tuple):
+                m.front_base, m.front_part = at, None
+            pad = -w.shape[0] % 4
+            weights += [w] + ([w.new_zeros((pad, w.shape[1]))] if pad else [])
+            bias = torch.zeros((w.shape[0] + pad,), dtype=torch.float32, device=w.device)
+            if b is not None:
+                bias[:w.shape[0]] = b.to(torch.float32)
+            biases.append(bias)
+            at += w.shape[0] + pad
+        self.linear = DenseLinear(ext, key, torch.cat(weights, 0))
+        self.bias = torch.cat(biases, 0).contiguous()
+
+    def weight_bytes(self) -> int:
+        return self.linear.weight_bytes()
+
+    def forward(self, xh: torch.Tensor, rows: int, model):
+        """(fp32 rows of all members' projections, their leading dimension)"""
+        n = self.linear.out_features
+        return self.linear.forward(xh, rows, out=model.buf("layer.f", (rows, n), torch.float32), bias=self.bias), n
+
+
+def front_rows(module, xh: torch.Tensor, rows: int, front):
+    """(projections, leading dimension, first column) of a module that has a linear of its own or a share of a joined one"""
+    if front is not None:
+        return front[0], front[1], module.front_base
+    n = module.front.out_features
+    f = module.front.forward(xh, rows, out=module.model.buf("mix.f", (rows, n), torch.float32), bias=getattr(module, "front_bias", None))
+    return f, n, 0

@@ -780,6 +780,7 @@ class ExtC:
     EPI_NONE, EPI_MUL_SIGMOID_AUX, EPI_SILU_AUX_MUL, EPI_CLAMPED_GLU, EPI_RELU_SQUARED, EPI_SOFT_CAP = 0, 1, 2, 3, 4, 5
     EPI_SCALE, EPI_TANH, EPI_ROW_SCALED_RELU_SQUARED = 6, 7, 8        # acc * limit; tanh(acc); relu(aux[row] * acc)^2
     EPI_ROW_SCALED_SILU_SCALED, EPI_AUX_MUL = 9, 10                   # silu(aux[row] * acc) * aux[row]; acc * aux
+    EPI_GELU_ERF, EPI_MUL_SIGMOID_ROW_AUX = 11, 12                    # exact gelu; acc * sigmoid(aux[row])
 
     @staticmethod
     def _dense_code(dtype) -> int:
@@ -853,23 +854,24 @@ class ExtC:
                                                       self._ptr(gr, torch.int32, "grp_rows"), self._stream(logits)))
 
     def latent_append(self, dkv, ld: int, norm_w, eps: float, rows: int, kv_rank: int, rot: int, rot_dims: int, inv_freq, row_seq,
-                      row_pos, block_table, page: int, cache, dkv_off: int = 0) -> None:
-        self.lib.check(self.lib.exl2_latent_append(self._ptr(dkv, torch.float32, "dkv") + dkv_off * 4, int(ld), self._ptr(norm_w, cache.dtype, "norm_w"),
+                      row_pos, block_table, page: int, cache, dkv_off: int = 0, halves: bool = False) -> None:
+        self.lib.check(self.lib.exl2_latent_append_ex(self._ptr(dkv, torch.float32, "dkv") + dkv_off * 4, int(ld), self._ptr(norm_w, cache.dtype, "norm_w"),
                                                    float(eps), self._dense_code(cache.dtype), int(rows), int(kv_rank), int(rot),
-                                                   int(rot_dims), self._ptr(inv_freq, torch.float32, "inv_freq"),
+                                                   int(rot_dims), int(halves), self._ptr(inv_freq, torch.float32, "inv_freq"),
                                                    self._ptr(row_seq, torch.int32, "row_seq"), self._ptr(row_pos, torch.int32, "row_pos"),
                                                    self._ptr(block_table, torch.int32, "block_table"), block_table.shape[-1], int(page),
                                                    self._ptr(cache, None, "cache"), self._stream(cache)))
 
     def latent_attn(self, q, ldq: int, q_head_stride: int, q_rot_off: int, q_abs, cache, page: int, row_seq, row_pos, block_table, out,
-                    rows: int, heads: int, kv_rank: int, rot: int, rot_dims: int, inv_freq, scale: float, window: int) -> None:
-        self.lib.check(self.lib.exl2_latent_attn(self._ptr(q, cache.dtype, "q"), int(ldq), int(q_head_stride), int(q_rot_off),
+                    rows: int, heads: int, kv_rank: int, rot: int, rot_dims: int, inv_freq, scale: float, window: int, halves: bool = False,
+                    sink=None) -> None:
+        self.lib.check(self.lib.exl2_latent_attn_ex(self._ptr(q, cache.dtype, "q"), int(ldq), int(q_head_stride), int(q_rot_off),
                                                  self._ptr(q_abs, torch.float32, "q_abs"), self._ptr(cache, None, "cache"), int(page),
                                                  self._ptr(row_seq, torch.int32, "row_seq"), self._ptr(row_pos, torch.int32, "row_pos"),
                                                  self._ptr(block_table, torch.int32, "block_table"), block_table.shape[-1],
                                                  self._ptr(out, cache.dtype, "out"), self._dense_code(cache.dtype), int(rows), int(heads),
-                                                 int(kv_rank), int(rot), int(rot_dims), self._ptr(inv_freq, torch.float32, "inv_freq"),
-                                                 float(scale), int(window), self._stream(out)))
+                                                 int(kv_rank), int(rot), int(rot_dims), int(halves), self._ptr(inv_freq, torch.float32, "inv_freq"),
+                                                 float(scale), int(window), self._ptr(sink, torch.float32, "sink"), self._stream(out)))
 
     @staticmethod
     def latent_attn_tiles_supported(dtype, kv_rank: int, rot: int) -> bool:
@@ -878,15 +880,16 @@ class ExtC:
 
     def latent_attn_tiles(self, q, ldq: int, q_head_stride: int, q_rot_off: int, q_abs, cache, page: int, row_seq, row_pos, block_table, out,
                           tile_row0, tile_rows, tiles: int, tile_mode: int, heads: int, kv_rank: int, rot: int, rot_dims: int, inv_freq,
-                          scale: float, window: int, nsplit: int = 1, part_o=None, part_ml=None) -> None:
-        self.lib.check(self.lib.exl2_latent_attn_tiles(
+                          scale: float, window: int, nsplit: int = 1, part_o=None, part_ml=None, halves: bool = False, sink=None) -> None:
+        self.lib.check(self.lib.exl2_latent_attn_tiles_ex(
             self._ptr(q, torch.bfloat16, "q"), int(ldq), int(q_head_stride), int(q_rot_off), self._ptr(q_abs, torch.float32, "q_abs"),
             self._ptr(cache, torch.bfloat16, "cache"), int(page), self._ptr(row_seq, torch.int32, "row_seq"),
             self._ptr(row_pos, torch.int32, "row_pos"), self._ptr(block_table, torch.int32, "block_table"), block_table.shape[-1],
             self._ptr(out, torch.bfloat16, "out"), self._ptr(tile_row0, torch.int32, "tile_row0"),
             self._ptr(tile_rows, torch.int32, "tile_rows"), int(tiles), int(tile_mode), self._ptr(part_o, torch.float32, "part_o"),
             self._ptr(part_ml, torch.float32, "part_ml"), int(nsplit), int(heads), int(kv_rank), int(rot), int(rot_dims),
-            self._ptr(inv_freq, torch.float32, "inv_freq"), float(scale), int(window), self._stream(out)))
+            int(halves), self._ptr(inv_freq, torch.float32, "inv_freq"), float(scale), int(window), self._ptr(sink, torch.float32, "sink"),
+            self._stream(out)))
 
     def add_layer_norm(self, x32, y, w, b, out, rows: int, eps: float, row_idx=None) -> None:
         """x32[r] += y[r] (y may be None), then out[r] = layer_norm(x32[r]) * w + b (w None: only the addition); with row_idx output
@@ -1103,8 +1106,9 @@ class ExtC:
             table.shape[0], int(buckets), int(mul_prev), int(mul_cur), float(scale), int(groups), float(eps), self._stream(x32)))
 
     def conv_rows(self, f, ld: int, f_off: int, w, bias, out, tail, spans, row_seq, row_pos, channels: int, taps: int,
-                  residual: bool = False) -> None:
-        """conv_silu_rows with a choice of output: residual -> out = in + conv (+ bias), no activation; out fp32 or w's dtype"""
+                  residual: int = 0) -> None:
+        """conv_silu_rows with a choice of output: residual 1 -> out = in + conv (+ bias), 2 -> conv (+ bias), no activation; out fp32 or
+        w's dtype"""
         row0, nrows, n, longest = spans
         self.lib.check(self.lib.exl2_conv_rows_ex(
             self._ptr(f, torch.float32, "f") + f_off * 4, int(ld), self._ptr(w, None, "w"), self._ptr(bias, w.dtype, "bias"),
@@ -1145,6 +1149,82 @@ class ExtC:
 
     def gated_scan_cols_supported(self, n_key: int, n_val: int) -> bool:
         return bool(self.lib.exl2_gated_scan_cols_supported(int(n_key), int(n_val)))
+
+    # ---- layers with one norm: gated residual step, grouped router (csrc/rowops.hip); minimal gated recurrence (csrc/mingru.hip);
+    # head-mixing attention (csrc/talk_attn.hip) -----------------------------------------------------------------------------------
+
+    def gated_residual(self, x32, out, rows: int, eps: float, w_in=None, y=None, y2=None, wy=None, wy2=None, ya: float = 1.0, yb: float = 1.0,
+                       gates=None, ldg: int = 0, g1_off: int | None = None, g2_off: int | None = None, moe_y=None, moe_w=None, top: int = 0,
+                       table=None, ids=None, init: bool = False, row_idx=None, dtype=None) -> None:
+        """x32 += t sigmoid(g1) + sigmoid(g2) sum_k moe_w moe_y (+ table[ids]; init: x32 = table[ids]), t = y or ya n(y) wy + yb n(y2) wy2;
+        out = n(x32) w_in (out may be None).  The gates are columns g1_off / g2_off of fp32 rows ldg apart."""
+        width = x32.shape[-1]
+        wt = w_in if w_in is not None else table if table is not None else wy
+        dt = dtype if dtype is not None else wt.dtype
+        gp = self._ptr(gates, torch.float32, "gates") if gates is not None else None
+        g1 = gp + 4 * g1_off if gp is not None and g1_off is not None else None
+        g2 = gp + 4 * g2_off if gp is not None and g2_off is not None else None
+        self.lib.check(self.lib.exl2_gated_residual(
+            self._ptr(x32, torch.float32, "x32"), self._ptr(y, torch.float32, "y"), self._ptr(y2, torch.float32, "y2"), self._ptr(wy, dt, "wy"),
+            self._ptr(wy2, dt, "wy2"), float(ya), float(yb), g1, g2, int(ldg), self._ptr(moe_y, torch.float32, "moe_y"),
+            self._ptr(moe_w, torch.float32, "moe_w"), int(top), self._ptr(table, dt, "table"), self._ptr(ids, torch.int32, "ids"),
+            table.shape[0] if table is not None else 0, int(init), self._ptr(w_in, dt, "w_in"), self._ptr(out, None, "out"),
+            int(out is not None and out.dtype is torch.float32), self._ptr(row_idx, torch.int32, "row_idx"), self._dense_code(dt), int(rows),
+            int(width), float(eps), self._stream(x32)))
+
+    def moe_route_grouped(self, logits, ldl: int, logits_off: int, ids, wts, rows: int, n_total: int, top: int, scale: float = 1.0,
+                          group_count: int = 1, group_keep: int = 1, groups=None) -> None:
+        """sigmoid router over columns logits_off .. + n_total of fp32 rows ldl apart, experts of the best group_keep groups only"""
+        gc, go, gr = groups if groups is not None else (None, None, None)
+        if ids.numel() < rows * top or wts.numel() < rows * top:
+            raise RuntimeError("moe_route_grouped: ids / wts smaller than rows x choices")
+        self.lib.check(self.lib.exl2_moe_route_grouped(
+            self._ptr(logits, torch.float32, "logits") + 4 * logits_off, int(ldl), self._ptr(ids, torch.int32, "ids"),
+            self._ptr(wts, torch.float32, "wts"), int(rows), int(n_total), int(top), float(scale), int(group_count), int(group_keep),
+            self._ptr(gc, torch.int32, "grp_count"), self._ptr(go, torch.int32, "grp_offset"), self._ptr(gr, torch.int32, "grp_rows"),
+            self._stream(logits)))
+
+    def mingru_scan(self, f, ld: int, z_off: int, u_off: int, g_off: int, out, state, spans, row_seq, row_pos, width: int, chunks=None,
+                    scratch=None) -> None:
+        """f fp32 [rows, ld]: gate, candidate and output-gate projections at z_off / u_off / g_off.  chunks = (span_chunk0 int32 [n], chunk size,
+        chunks in all) with scratch fp32: the form for long spans"""
+        row0, nrows, n, _longest = spans
+        chunk0, chunk, total = chunks if chunks is not None else (None, 0, 0)
+        if scratch is not None and scratch.numel() < (2 * total + n) * width:
+            raise RuntimeError("mingru_scan: scratch smaller than the step's chunks")
+        p = self._ptr(f, torch.float32, "f")
+        self.lib.check(self.lib.exl2_mingru_scan(
+            p + 4 * z_off, p + 4 * u_off, p + 4 * g_off, int(ld), self._ptr(out, None, "out"), out.shape[-1], self._ptr(state, torch.float32, "state"),
+            self._ptr(row0, torch.int32, "span_row0"), self._ptr(nrows, torch.int32, "span_rows"), int(n), self._ptr(row_seq, torch.int32, "row_seq"),
+            self._ptr(row_pos, torch.int32, "row_pos"), self._ptr(chunk0, torch.int32, "span_chunk0"), int(chunk), int(total),
+            self._ptr(scratch, torch.float32, "scratch"), self._dense_code(out.dtype), int(width), self._stream(out)))
+
+    def talk_attn(self, q, k_cache, v_cache, talk, sink, row_seq, row_pos, block_table, page: int, out, row_list, rows: int, heads: int,
+                  kv_heads: int, dim: int, vdim: int, window: int, softcap: float, nsplit: int = 1, part_o=None, part_ml=None) -> None:
+        """rows `row_list` int32 (None: rows 0 .. rows - 1), one workgroup per row and key split"""
+        dt = k_cache.dtype
+        self.lib.check(self.lib.exl2_talk_attn(
+            self._ptr(q, dt, "q"), self._ptr(k_cache, dt, "k_cache"), self._ptr(v_cache, dt, "v_cache"), self._ptr(talk, torch.float32, "talk"),
+            self._ptr(sink, torch.float32, "sink"), self._ptr(row_seq, torch.int32, "row_seq"), self._ptr(row_pos, torch.int32, "row_pos"),
+            self._ptr(block_table, torch.int32, "block_table"), block_table.shape[-1], int(page), self._ptr(out, dt, "out"),
+            self._ptr(row_list, torch.int32, "row_list"), int(rows), self._ptr(part_o, torch.float32, "part_o"),
+            self._ptr(part_ml, torch.float32, "part_ml"), int(nsplit), self._dense_code(dt), int(heads), int(kv_heads), int(dim), int(vdim),
+            int(window), float(softcap), self._stream(out)))
+
+    def talk_attn_tiles_supported(self, dtype, heads: int, dim: int, vdim: int) -> bool:
+        return dtype is torch.bfloat16 and bool(self.lib.exl2_talk_attn_tiles_supported(int(heads), int(dim), int(vdim)))
+
+    def talk_attn_tiles(self, q, k_cache, v_cache, talk, sink, row_seq, row_pos, block_table, page: int, out, tiles, heads: int, kv_heads: int,
+                        dim: int, vdim: int, window: int, softcap: float) -> None:
+        """tiles = (tile_row0 int32 [n], tile_rows int32 [n], n): runs of <= 16 consecutive positions of one sequence"""
+        row0, nrows, n = tiles
+        bf = torch.bfloat16
+        self.lib.check(self.lib.exl2_talk_attn_tiles(
+            self._ptr(q, bf, "q"), self._ptr(k_cache, bf, "k_cache"), self._ptr(v_cache, bf, "v_cache"), self._ptr(talk, torch.float32, "talk"),
+            self._ptr(sink, torch.float32, "sink"), self._ptr(row_seq, torch.int32, "row_seq"), self._ptr(row_pos, torch.int32, "row_pos"),
+            self._ptr(block_table, torch.int32, "block_table"), block_table.shape[-1], int(page), self._ptr(out, bf, "out"),
+            self._ptr(row0, torch.int32, "tile_row0"), self._ptr(nrows, torch.int32, "tile_rows"), int(n), int(heads), int(kv_heads), int(dim),
+            int(vdim), int(window), float(softcap), self._stream(out)))
 
     def graph_begin_capture(self, stream: int | None) -> None:
         self.lib.check(self.lib.exl2_graph_begin_capture(stream))

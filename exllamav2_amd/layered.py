@@ -3,9 +3,11 @@ registries, on an fp32 residual stream.  The residual style is the configuration
 x <- norm(alpha x + sublayer(x)) (1 + w)  (RMS norm, a `head` matrix), or pre-norm steps  x <- x + sublayer(layer_norm(x))  (weight and
 bias, logits from the embedding table, optional soft cap), or pre-norm steps with scalar-gain RMS norms and a token shift in front
 of every mixer (a `head` matrix, scaled logits), or sandwich-normed steps  x <- x + mult n_g(sublayer(conv_in(n_g(x) w))) w'  with
-grouped RMS norms, a short input convolution and a token-pair table beside the embedding.  Mixers: latent attention, windowed /
+grouped RMS norms, a short input convolution and a token-pair table beside the embedding, or layers with ONE RMS norm whose mixer and
+feed-forward stand side by side behind gates, x <- x + mixer(h) sigmoid(W_1 h + b_1) + ff(h) sigmoid(W_2 h + b_2), some of them gone
+through several times.  Mixers: latent attention, windowed /
 chunked / plain causal attention (pooled blocks, sinks, shared keys and values), state-space scan, decaying linear attention, linear
-attention whose forget gate writes, gated delta rule, two mixers side by side; a stack may mix them -- each keeps what it needs between steps (pages
+attention whose forget gate writes, gated delta rule, minimal gated recurrence, two mixers side by side; a stack may mix them -- each keeps what it needs between steps (pages
 of keys and values, per-slot recurrent state) under one page pool.
 
 The model has ONE forward, `step(batch, cache)`: the rows of a step are a flat list of tokens, each with its sequence slot and
@@ -20,25 +22,27 @@ import torch
 
 from .cache import LatentCache, LayerStates, PagePool
 from .config import LayeredConfig
-from .dense_linear import DenseLinear
+from .dense_linear import DenseLinear, JoinedFront
 from .ext import ext_c
 from .latent_attn import LatentAttention
 from .linear_attn import ForgetGateLinearAttention, GatedDeltaRule
+from .mingru import MinimalGRU
 from .mlp import DenseActMLP, DenseGatedMLP
 from .moe_mlp import ScoredMoEMLP, SigmoidMoEMLP
 from .parallel_mixer import ParallelMixer
-from .rmsnorm import PostNorm, PreLayerNorm, PreShiftRMSNorm, SandwichNorm
+from .rmsnorm import GatedResidualNorm, PostNorm, PreLayerNorm, PreShiftRMSNorm, SandwichNorm
 from .ssm import StateSpaceMixer
 from .window_attn import WindowAttention
 from .wkv import DecayLinearAttention
 
 
 def _latent_attention(model, key, idx, spec):
-    m = spec["mixer"]
+    m, gated = spec["mixer"], model.config.residual == "parallel_gated"
     return LatentAttention(model, key, idx, heads=int(m["heads"]), dim=int(m["dim"]), rot_dim=int(m["rot_dim"]), vdim=int(m["vdim"]),
-                           kv_rank=int(m["kv_rank"]), q_rank=int(m["q_rank"]), window=int(m["mask"]["size"]),
+                           kv_rank=int(m["kv_rank"]), q_rank=int(m["q_rank"]), window=int((m.get("mask") or {}).get("size") or (1 << 30)),
                            rot_base=float(m["rot"]["base"]), rot_dims=int(m["rot"]["dims"]), scale=float(m["scale"]),
-                           kv_from=(int(m["kv_from"]) if m.get("kv_from") is not None else None))
+                           kv_from=(int(m["kv_from"]) if m.get("kv_from") is not None else None),
+                           interleaved=not gated, joined=gated)
 
 
 def _window_attention(model, key, idx, spec):
@@ -51,6 +55,11 @@ def _window_attention(model, key, idx, spec):
         # chunks from position 0, capped scores, a constant 1 in the softmax denominator, values as they are, maybe another layer's rows
         return WindowAttention(model, key, idx, window=1 << 30, pool=0, chunk=int(mask.get("size") or 0), softcap=float(m.get("softcap") or 0.0),
                                sink_one=True, rotate_values=False, kv_from=(int(m["kv_from"]) if m.get("kv_from") is not None else None),
+                               **common)
+    if model.config.residual == "parallel_gated":
+        # convolved projections, capped scores that the heads exchange, a constant 1 in the softmax denominator, neighbouring rotary pairs
+        return WindowAttention(model, key, idx, window=int(mask.get("size") or (1 << 30)), pool=0, softcap=float(m.get("softcap") or 0.0),
+                               sink_one=True, rotate_values=False, interleaved=True, conv_taps=int(m.get("conv") or 0), talk=True, joined=True,
                                **common)
     return WindowAttention(model, key, idx, window=int(mask.get("size") or (1 << 30)), pool=int(mask.get("pool") or 0), **common)
 
@@ -66,19 +75,24 @@ def _state_space(model, key, idx, spec):
                            groups=int(m.get("groups", 1)), norm_groups=int(m.get("norm_groups", 1)), taps=int(m["conv"]))
 
 
-def _causal_attention(model, key, idx, m, out_tag="mix.y"):
-    """plain causal softmax attention: every earlier token is visible, no sink, no gate, values as they are"""
-    rot = m.get("rot") or {}
+def _causal_attention(model, key, idx, m, out_tag="mix.y", **kw):
+    """plain softmax attention over every earlier token (or the window the config gives), no sink, values as they are"""
+    rot, window = m.get("rot") or {}, int((m.get("mask") or {}).get("size") or (1 << 30))
     return WindowAttention(model, key, idx, heads=int(m["heads"]), kv_heads=int(m.get("kv_heads") or m["heads"]), dim=int(m["dim"]),
-                           vdim=int(m.get("vdim") or m["dim"]), window=1 << 30, pool=0, rot_base=float(rot.get("base", 10000.0)),
+                           vdim=int(m.get("vdim") or m["dim"]), window=window, pool=0, rot_base=float(rot.get("base", 10000.0)),
                            rot_dims=int(rot.get("dims", 0)), rot_scaling=rot.get("scaling"), scale=float(m["scale"]), rotate_values=False,
-                           out_tag=out_tag)
+                           out_tag=out_tag, **kw)
 
 
 def _parallel(model, key, idx, spec):
-    """softmax attention (left) beside a state-space scan (right) on the same input"""
+    """softmax attention (left) beside a recurrence (right: a state-space scan, or a minimal gated recurrence) on the same input"""
     m = spec["mixer"]
     r = m["right"]
+    if model.config.residual == "parallel_gated":
+        # half the sum of both results, each normed over the model width
+        left = _causal_attention(model, key + ".left", (idx, "left"), m["left"], out_tag="mix.y.left", interleaved=True, joined=True)
+        right = MinimalGRU(model, key + ".right", (idx, "right"), width=int(r["width"]), out_tag="mix.y.right", joined=True)
+        return ParallelMixer(model, key, idx, left, right, 0.5, 0.5, out_norms=True)
     left = _causal_attention(model, key + ".left", (idx, "left"), m["left"], out_tag="mix.y.left")
     right = StateSpaceMixer(model, key + ".right", (idx, "right"), heads=int(r["heads"]), vdim=int(r["vdim"]), state=int(r["state"]),
                             groups=int(r.get("groups", 1)), norm_groups=int(r.get("norm_groups", 1)), taps=int(r["conv"]),
@@ -105,6 +119,10 @@ def _dense_mlp(model, key, idx, spec):
 
 def _moe_mlp(model, key, idx, spec):
     r, e = spec["router"], spec["expert"]
+    if model.config.residual == "parallel_gated":             # sigmoid scores among the best groups weigh the experts' outputs
+        gr = r.get("groups")
+        return SigmoidMoEMLP(model, key, idx, experts=int(r["experts"]), top=int(r["top"]), ff=int(e["ff"]), shared_ff=None, act="gelu",
+                             groups=(int(gr["count"]), int(gr["keep"])) if gr else None, joined=True)
     if model.config.residual in ("pre_rms_shift", "sandwich"):        # sigmoid scores weigh the experts' inputs; a shared expert beside them
         shared = spec.get("shared")
         return SigmoidMoEMLP(model, key, idx, experts=int(r["experts"]), top=int(r["top"]), ff=int(e["ff"]),
@@ -198,7 +216,8 @@ class LayeredModel:
         self.embed = need("embed")
         if tuple(self.embed.shape) != (cfg.vocab, cfg.width):
             raise RuntimeError(f"embed is {tuple(self.embed.shape)}, config says {(cfg.vocab, cfg.width)}")
-        pre = cfg.residual in ("pre_ln", "pre_rms_shift", "sandwich")
+        gated = cfg.residual == "parallel_gated"
+        pre = cfg.residual in ("pre_ln", "pre_rms_shift", "sandwich") or gated
 
         def make_norm(name, shift=None):
             if cfg.residual == "sandwich":
@@ -207,6 +226,8 @@ class LayeredModel:
                 conv = need(name.replace("norm", "canon"), optional=cfg.input_conv_taps <= 0) if inner else None
                 return SandwichNorm(self.ext, name, need(name), need(name + "b") if inner else None, conv,
                                     cfg.norm_groups, cfg.norm_eps, cfg.residual_mult)
+            if gated:
+                return GatedResidualNorm(self.ext, name, need(name), cfg.norm_eps)
             if cfg.residual == "pre_rms_shift":
                 return PreShiftRMSNorm(self.ext, name, need(name), cfg.norm_eps, shift=need(shift) if shift else None)
             if pre:
@@ -214,6 +235,7 @@ class LayeredModel:
             return PostNorm(self.ext, name, need(name), cfg.norm_eps, cfg.postln_alpha)
 
         self.layers = []
+        self.fronts = []                                      # per layer: (joined linear, column of the mixer's gate, of the feed-forward's)
         for i, spec in enumerate(cfg.layers):
             key = f"l{i}"
             if spec["type"] not in MIXERS:
@@ -226,9 +248,11 @@ class LayeredModel:
                 if ms["kind"] not in FEED_FORWARDS:
                     raise RuntimeError(f"layer {i}: unknown feed-forward kind '{ms['kind']}' (known: {sorted(FEED_FORWARDS)})")
                 ff = FEED_FORWARDS[ms["kind"]](self, key + ".mlp", i, ms).load(lambda n, k=key: need(f"{k}.mlp.{n}"))
-            if ff is not None or (not pre and key + ".norm2" in tensors):
+            if (ff is not None and not gated) or (not pre and key + ".norm2" in tensors):
                 norm2 = make_norm(key + ".norm2")
             self.layers.append((mixer, norm1, ff, norm2))
+            if gated:
+                self.fronts.append(self._join_front(key, mixer, ff, need))
         for i, (mixer, *_rest) in enumerate(self.layers):
             j = getattr(mixer, "kv_from", None)
             if j is not None:
@@ -262,30 +286,41 @@ class LayeredModel:
         self.loaded = True
         return self
 
+    def _join_front(self, key, mixer, ff, need):
+        """everything that reads the layer's input in one linear: the mixer's projections, the router, the residual gates"""
+        members = list(getattr(mixer, "front_members", [mixer]))
+        gates = [(need(key + ".rg1"), need(key + ".rg1.b"))]
+        if ff is not None:
+            members.append(ff)
+            gates.append((need(key + ".rg2"), need(key + ".rg2.b")))
+        if any(tuple(w.shape) != (self.width, self.width) or b.numel() != self.width for w, b in gates):
+            raise RuntimeError(f"{key}: the residual gates are over the model width")
+        front = JoinedFront(self.ext, key + ".front", members + gates)
+        n = len(members)
+        return front, front.bases[n], front.bases[n + 1] if ff is not None else None
+
     def weight_bytes(self) -> int:
         """bytes a decoded token streams (a tied output table counts once: the embedding reads one row of it)"""
         n = self.head.weight_bytes()
-        for mixer, _n1, ff, _n2 in self.layers:
-            n += mixer.weight_bytes() + (ff.weight_bytes() if ff is not None else 0)
+        for i, _pass, _embed in self.config.layer_runs():
+            mixer, _n1, ff, _n2 = self.layers[i]
+            n += mixer.weight_bytes() + (ff.weight_bytes() if ff is not None else 0) + (self.fronts[i][0].weight_bytes() if self.fronts else 0)
         return n
 
     # ---- cache ----------------------------------------------------------------------------------------------------------------
 
     def make_cache(self, pool: PagePool):
-        if any(hasattr(mixer, "make_state") or hasattr(mixer, "make_states") for mixer, *_rest in self.layers):
+        looped = self.config.loop is not None and self.config.loop[2] > 1
+        if looped or not all(hasattr(mixer, "cache_row_width") for mixer, *_rest in self.layers):
             norm_states = {i: norm1.make_state(pool, self.width) for i, (_m, norm1, *_r) in enumerate(self.layers) if hasattr(norm1, "make_state")}
             norm_states.update({(i, "ff"): norm2.make_state(pool, self.width) for i, (_m, _n1, _ff, norm2) in enumerate(self.layers)
                                 if norm2 is not None and hasattr(norm2, "make_state")})
             if getattr(self, "pair_table", None) is not None:
                 from .cache import SlotState
                 norm_states["embed"] = SlotState(pool, {"prev_token": ()}, dtype=torch.int32)
-            per_layer = {}
-            for i, (mixer, *_rest) in enumerate(self.layers):
-                if hasattr(mixer, "make_states"):                 # several states under keys of the mixer's own ((layer, "left"), ...)
-                    per_layer.update(mixer.make_states(pool, self.dtype))
-                else:
-                    per_layer[i] = mixer.make_state(pool, self.dtype)
-            return LayerStates(pool, per_layer, norm_states=norm_states)
+            start, stop, times = self.config.loop or (0, 0, 1)
+            later = [LayerStates(pool, self._mixer_states(pool, range(start, stop))) for _ in range(1, times)]
+            return LayerStates(pool, self._mixer_states(pool, range(len(self.layers))), norm_states=norm_states, later_passes=later)
         widths, owner = {}, {}
         for i, (mixer, *_rest) in enumerate(self.layers):
             if mixer.kv_from is None:
@@ -294,6 +329,16 @@ class LayeredModel:
             else:
                 owner[i] = mixer.kv_from
         return LatentCache(pool, widths, owner, self.dtype)
+
+    def _mixer_states(self, pool: PagePool, layers) -> dict:
+        per_layer = {}
+        for i in layers:
+            mixer = self.layers[i][0]
+            if hasattr(mixer, "make_states"):                     # several states under keys of the mixer's own ((layer, "left"), ...)
+                per_layer.update(mixer.make_states(pool, self.dtype))
+            else:
+                per_layer[i] = mixer.make_state(pool, self.dtype)
+        return per_layer
 
     # ---- forward ----------------------------------------------------------------------------------------------------------------
 
@@ -307,6 +352,8 @@ class LayeredModel:
             return self._step_pre_rms_shift(batch, cache)
         if cfg.residual == "sandwich":
             return self._step_sandwich(batch, cache)
+        if cfg.residual == "parallel_gated":
+            return self._step_parallel_gated(batch, cache)
         x32 = self.buf("x32", (rows, self.width), torch.float32)
         xh = x32 if self.dtype is torch.float32 else self.buf("xh", (rows, self.width), self.dtype)
         ext.embed_scale(self.embed, batch.ids, x32, xh, cfg.embedding_scale)
@@ -412,6 +459,35 @@ class LayeredModel:
         else:
             if pending is not None:
                 self.final_norm.forward(x32, pending, None, rows, dtype=self.dtype)
+            if batch.n_logits == 0:
+                return None
+            self.final_norm.forward(x32, None, xn, batch.n_logits, row_idx=batch.logit_rows, dtype=self.dtype)
+        return self.head.forward(xn, batch.n_logits, out=self.buf("logits", (batch.n_logits, self.vocab), f32))
+
+    def _step_parallel_gated(self, batch: StepBatch, cache) -> torch.Tensor | None:
+        """x <- x + mixer(h) sigmoid(W_1 h + b_1) + ff(h) sigmoid(W_2 h + b_2), h = n(x) w: per layer ONE linear brings everything that
+        reads h (the mixer's projections, the router's logits, both gates), and what lies between two layers -- the norms behind two
+        mixers side by side, the gates, the experts' weighted sum, the additions, at the start of a later pass the embeddings, and the next
+        layer's norm -- is one launch.  A looped layer finds the memory of its pass in `cache.at_pass`.  Logits: head(n(x) w) for the
+        wanted rows."""
+        cfg, rows, f32 = self.config, batch.rows, torch.float32
+        x32 = self.buf("x32", (rows, self.width), f32)
+        xh = self.buf("xh", (rows, self.width), self.dtype)
+        pending = None
+        for n, (i, loop_pass, add_embedding) in enumerate(cfg.layer_runs()):
+            mixer, norm, ff, _ = self.layers[i]
+            joined, g1, g2 = self.fronts[i]
+            norm.forward(x32, pending, xh, rows, table=self.embed, ids=batch.ids if n == 0 or add_embedding else None, init=n == 0,
+                         dtype=self.dtype)
+            front = joined.forward(xh, rows, self)
+            y = mixer.forward(xh, rows, batch, cache.at_pass(loop_pass) if loop_pass else cache, front=front)
+            mix = ff.forward(xh, rows, front=front)[1] if ff is not None else None
+            pending = (y, getattr(mixer, "out_norms", None), front, g1, g2, mix)
+        xn = self.buf("xn", (max(batch.n_logits, 1), self.width), self.dtype)
+        if batch.logits_all_rows and batch.n_logits == rows:
+            self.final_norm.forward(x32, pending, xn, rows, dtype=self.dtype)       # the last addition and the final norm in one launch
+        else:
+            self.final_norm.forward(x32, pending, None, rows, dtype=self.dtype)
             if batch.n_logits == 0:
                 return None
             self.final_norm.forward(x32, None, xn, batch.n_logits, row_idx=batch.logit_rows, dtype=self.dtype)

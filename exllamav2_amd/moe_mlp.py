@@ -129,20 +129,28 @@ class SigmoidMoEMLP:
     the same form (its own width) runs for every token: as wide as the routed ones it is stacked behind them and rides their
     launches as one more pair per token, otherwise it runs as a feed-forward of its own.  `act="silu_glu"`: experts are gated units
     W_down (silu(W_gate z) * W_up z); with z = s h the gate launch leaves silu(s g) s and the up launch multiplies by it, so both
-    matrices still run on h.  Few rows: every (token, choice) pair names its expert's slab; many rows:
+    matrices still run on h.  `act="gelu"`: experts W_down gelu(W_up z) (exact gelu) whose OUTPUTS carry the weights -- the weighted
+    sum is the residual step's (rmsnorm.GatedResidualNorm).  `groups` = (count, keep): the experts stand in `count` equal groups and only those of
+    the `keep` groups with the largest sums of two scores can be chosen.  `joined`: the router is part of a linear the layer shares
+    (dense_linear.JoinedFront).  Few rows: every (token, choice) pair names its expert's slab; many rows:
     one grouped launch per projection.  forward returns (y | None, mixture): y is the shared expert's output, the chosen experts'
     rows are added by the residual step's launch (rmsnorm.PreShiftRMSNorm)."""
 
     PAIR_ROWS_MAX = 64
 
     def __init__(self, model, key: str, layer_idx: int, *, experts: int, top: int, ff: int, shared_ff: int | None, route_scale: float = 1.0,
-                 act: str = "relu2"):
+                 act: str = "relu2", groups: tuple | None = None, joined: bool = False):
         self.model, self.ext, self.key, self.layer_idx = model, model.ext, key, layer_idx
         self.experts, self.top, self.ff, self.shared_ff, self.route_scale = experts, top, ff, shared_ff, route_scale
-        self.glu = act == "silu_glu"
+        self.glu, self.gelu = act == "silu_glu", act == "gelu"
+        self.groups = groups or (1, 1)
+        self.grouped_router = self.gelu or groups is not None or joined
+        self.joined, self.front_base = joined, 0
+        if self.grouped_router and shared_ff:
+            raise ValueError(f"{key}: a shared expert does not go with this router")
         if not 0 < top <= experts:
             raise ValueError(f"{key}: top {top} of {experts} experts")
-        if act not in ("relu2", "silu_glu"):
+        if act not in ("relu2", "silu_glu", "gelu"):
             raise ValueError(f"{key}: unknown expert form '{act}'")
 
     def load(self, get):
@@ -150,6 +158,8 @@ class SigmoidMoEMLP:
         from .mlp import DenseActMLP, DenseGatedMLP
         E, width = self.experts, self.model.width
         self.router = DenseLinear(self.ext, self.key + ".router", get("router"))
+        if self.joined:
+            self.front_part = (self.router.weight, None)
         # a shared expert as wide as the routed ones is stacked behind them as expert E: the router's launch names it for every token
         # with weight 1 and the two expert launches run it with the chosen ones
         self.merged = bool(self.shared_ff) and self.shared_ff == self.ff
@@ -163,6 +173,8 @@ class SigmoidMoEMLP:
                 or tuple(self.down.weight.shape) != (self.slabs, width, self.ff) \
                 or (self.glu and tuple(self.gate.weight.shape) != (self.slabs, self.ff, width)):
             raise RuntimeError(f"{self.key}: tensor shapes do not match the feed-forward's sizes")
+        if self.joined:
+            self.router = None
         self.shared = None
         if self.shared_ff and not self.merged:
             form = DenseGatedMLP if self.glu else DenseActMLP
@@ -173,13 +185,16 @@ class SigmoidMoEMLP:
 
     def weight_bytes(self) -> int:
         per_slab = (self.up.weight_bytes() + self.down.weight_bytes() + (self.gate.weight_bytes() if self.glu else 0)) // self.slabs
-        n = self.router.weight_bytes() + per_slab * (self.top + int(self.merged))
+        n = (self.router.weight_bytes() if self.router is not None else 0) + per_slab * (self.top + int(self.merged))
         return n + (self.shared.weight_bytes() if self.shared is not None else 0)
 
-    def forward(self, xh: torch.Tensor, rows: int):
+    def forward(self, xh: torch.Tensor, rows: int, front=None):
         ext, m = self.ext, self.model
         E, top, ff, width, dt = self.experts, self.top, self.ff, m.width, m.dtype
-        logits = self.router.forward(xh, rows, out=m.buf("moe.logits", (rows, E), torch.float32))
+        if front is None:
+            logits, ldl, at = self.router.forward(xh, rows, out=m.buf("moe.logits", (rows, E), torch.float32)), E, 0
+        else:
+            logits, ldl, at = front[0], front[1], self.front_base
         per_row, S = top + int(self.merged), self.slabs          # (token, expert) pairs per row; weight slabs
         ids = m.buf("moe.ids", (rows, per_row), torch.int32)
         wts = m.buf("moe.wts", (rows, per_row), torch.float32)
@@ -188,7 +203,10 @@ class SigmoidMoEMLP:
         groups = None
         if grouped:
             groups = (m.buf("moe.count", (S,), torch.int32), m.buf("moe.offset", (S,), torch.int32), m.buf("moe.rows", (pairs,), torch.int32))
-        ext.moe_route_sigmoid(logits, ids, wts, rows, E, top, self.route_scale, groups=groups, shared_slot=self.merged)
+        if self.grouped_router:
+            ext.moe_route_grouped(logits, ldl, at, ids, wts, rows, E, top, self.route_scale, *self.groups, groups=groups)
+        else:
+            ext.moe_route_sigmoid(logits, ids, wts, rows, E, top, self.route_scale, groups=groups, shared_slot=self.merged)
         a = m.buf("moe.a", (pairs, ff), dt)
         y = m.buf("moe.y", (pairs, width), torch.float32)
         kw = dict(batch=S, groups=groups) if grouped else dict(w_sel=ids.view(-1), n_sel=S)
@@ -198,6 +216,8 @@ class SigmoidMoEMLP:
                              aux=wts, ldaux=1, epi=ext.EPI_ROW_SCALED_SILU_SCALED, **kw)
             ext.dense_linear(xh, self.up.weight, a, pairs, ff, width, width, width, ff, swb=ff * width, x_div=per_row,
                              aux=g, ldaux=ff, epi=ext.EPI_AUX_MUL, **kw)
+        elif self.gelu:
+            ext.dense_linear(xh, self.up.weight, a, pairs, ff, width, width, width, ff, swb=ff * width, x_div=per_row, epi=ext.EPI_GELU_ERF, **kw)
         else:
             ext.dense_linear(xh, self.up.weight, a, pairs, ff, width, width, width, ff, swb=ff * width, x_div=per_row,
                              aux=wts, ldaux=1, epi=ext.EPI_ROW_SCALED_RELU_SQUARED, **kw)

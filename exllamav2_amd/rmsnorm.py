@@ -137,3 +137,31 @@ class SandwichNorm:
             ext.sandwich_norm(x32, w_out, mult, self.w_in, hn, rows, self.groups, self.eps, dtype=dtype, **pa)
             ext.conv_rows(hn, width, 0, self.conv_w, None, out, state["tail"], batch.spans_dev, batch.row_seq, batch.row_pos, width,
                           self.taps, residual=True)
+
+
+class GatedResidualNorm:
+    """The norm in front of a layer whose mixer and feed-forward both read it, n(x) w with n(v) = v / sqrt(mean(v^2) + eps), fused with the
+    residual step of the layer BEFORE it (csrc/rowops.hip: gated_residual_vec_kernel): x <- x + mixer * sigmoid(g1) + ff * sigmoid(g2), where
+    the mixer's result is one linear's output or the weighted sum of two separately normed ones (ParallelMixer with `out_norms`), the
+    feed-forward's the weighted rows of the chosen experts, and both gates are columns of the layer's joined linear."""
+
+    def __init__(self, ext, key: str, weight: torch.Tensor, eps: float):
+        self.ext, self.key, self.weight, self.eps = ext, key, weight.contiguous(), float(eps)
+
+    def forward(self, x32: torch.Tensor, pending, out: torch.Tensor | None, rows: int, table=None, ids=None, init: bool = False, row_idx=None,
+                dtype=None) -> None:
+        """pending: None or (mixer result(s), norms behind the two halves | None, (gate rows, leading dimension), first gate column, second
+        gate column, mixture | None); ids: the rows' embeddings are added too (init: the stream starts from them).  out None: only the
+        additions."""
+        kw = {}
+        if pending is not None:
+            y, norms, (f, ld), g1, g2, mix = pending
+            if norms is not None:
+                kw.update(y=y[0], ya=y[1], y2=y[2], yb=y[3], wy=norms[0], wy2=norms[1])
+            else:
+                kw.update(y=y)
+            kw.update(gates=f, ldg=ld, g1_off=g1, g2_off=g2)
+            if mix is not None:
+                kw.update(moe_y=mix[0], moe_w=mix[2], top=mix[2].shape[-1])
+        self.ext.gated_residual(x32, out, rows, self.eps, w_in=self.weight if out is not None else None, table=table if ids is not None else None,
+                                ids=ids, init=init, row_idx=row_idx, dtype=dtype, **kw)

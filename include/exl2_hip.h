@@ -607,7 +607,7 @@ int exl2_embed_pair(const void* table, const void* pair, const void* w, const in
                     const int* row_pos, const int* span_row0, const int* span_rows, int spans, int max_span_rows, float* x,
                     int dtype, int rows, int width, int vocab, int buckets, int mul_prev, int mul_cur, float scale, int groups,
                     float eps, void* stream);
-/* exl2_conv_silu_rows with a choice of output: residual 0: silu(conv + bias); 1: in + conv + bias without activation.  out fp32
+/* exl2_conv_silu_rows with a choice of output: residual 0: silu(conv + bias); 1: in + conv + bias; 2: conv + bias (no activation).  out fp32
    (out_f32 = 1) or the operand dtype. */
 int exl2_conv_rows_ex(const float* in, int ld, const void* w, const void* bias, void* out, int ldo, int out_f32, int residual,
                       float* tail, const int* span_row0, const int* span_rows, int spans, int max_span_rows,
@@ -636,6 +636,58 @@ int exl2_gated_scan_cols(int mode, const float* q, int ldq, const float* k, int 
                          float* state, const int* span_row0, const int* span_rows, int spans, const int* row_seq,
                          const int* row_pos, int rows, float* o_raw, int heads, int qk_heads, int n_key, int n_val,
                          float q_scale, float eps, void* stream);
+
+/* ---- layers whose mixer and feed-forward read ONE norm and pass gates of their own (csrc/rowops.hip), a minimal gated recurrence
+   (csrc/mingru.hip), attention whose heads exchange their scores (csrc/talk_attn.hip), latent attention with a sink per head and either
+   rotary layout (csrc/latent_attn.hip) */
+
+/* x[r] <- x[r] + t sigmoid(g1[r]) + sigmoid(g2[r]) sum_k moe_w[r, k] moe_y[r * top + k],  t = y[r], or ya n(y[r]) wy + yb n(y2[r]) wy2 when
+   wy / wy2 are given;  x[r] <- x[r] + table[ids[r]] (ids nullable; init: x[r] = table[ids[r]], nothing is read);  then
+   out[r] = n(x[r]) w_in (out nullable), n(v) = v / sqrt(mean(v^2) + eps).  y, moe_y and the gates (fp32 rows ldg apart) are nullable.
+   row_idx: output row r reads stream row row_idx[r] (no addition then).  Weights and table in the operand dtype. */
+int exl2_gated_residual(float* x, const float* y, const float* y2, const void* wy, const void* wy2, float ya, float yb,
+                        const float* g1, const float* g2, int ldg, const float* moe_y, const float* moe_w, int top,
+                        const void* table, const int* ids, int vocab, int init, const void* w_in, void* out, int out_f32,
+                        const int* row_idx, int dtype, int rows, int width, float eps, void* stream);
+/* exl2_moe_route_sigmoid with logits ldl apart and experts in group_count equal groups of neighbours: a group scores the sum of its two
+   largest scores, only experts of the group_keep best groups can be chosen (the first of equals wins) */
+int exl2_moe_route_grouped(const float* logits, int ldl, int* ids, float* wts, int rows, int n_total, int top, float scale,
+                           int group_count, int group_keep, int* grp_count, int* grp_offset, int* grp_rows, void* stream);
+/* exl2_latent_append / _attn / _attn_tiles with a choice of rotary layout (halves 0: pairs (2i, 2i + 1); 1: (i, i + rot_dims / 2)) and,
+   nullable, a learned score per head (sink fp32 [heads]) that joins the softmax denominator without key or value */
+int exl2_latent_append_ex(const float* dkv, int ld, const void* norm_w, float eps, int dtype, int rows, int kv_rank, int rot,
+                          int rot_dims, int halves, const float* inv_freq, const int* row_seq, const int* row_pos,
+                          const int* block_table, int bt_stride, int page, void* cache, void* stream);
+int exl2_latent_attn_ex(const void* q, int ldq, int q_head_stride, int q_rot_off, const float* q_abs, const void* cache, int page,
+                        const int* row_seq, const int* row_pos, const int* block_table, int bt_stride, void* out, int dtype,
+                        int rows, int heads, int kv_rank, int rot, int rot_dims, int halves, const float* inv_freq, float scale,
+                        int window, const float* sink, void* stream);
+int exl2_latent_attn_tiles_ex(const void* q, int ldq, int q_head_stride, int q_rot_off, const float* q_abs, const void* cache,
+                              int page, const int* row_seq, const int* row_pos, const int* block_table, int bt_stride, void* out,
+                              const int* tile_row0, const int* tile_rows, int tiles, int tile_mode, float* part_o, float* part_ml,
+                              int nsplit, int heads, int kv_rank, int rot, int rot_dims, int halves, const float* inv_freq,
+                              float scale, int window, const float* sink, void* stream);
+/* per channel: k = 1 - sigmoid(z), c = u + 1/2 where u >= 0 else sigmoid(u), S <- k S + (1 - k) c, out = S silu(g); z, u, g fp32 rows ld
+   apart, out operand dtype, state fp32 [slots, width].  Spans as in exl2_ssm_scan.  scratch (nullable; fp32 [(2 chunks + spans) width]):
+   the form for long spans, cut into chunks of `chunk` tokens (span_chunk0 = chunks in front of each span). */
+int exl2_mingru_scan(const float* z, const float* u, const float* g, int ld, void* out, int ldo, float* state,
+                     const int* span_row0, const int* span_rows, int spans, const int* row_seq, const int* row_pos,
+                     const int* span_chunk0, int chunk, int total_chunks, float* scratch, int dtype, int width, void* stream);
+/* softmax attention over 0 <= p - j < window whose heads exchange their (soft-capped; softcap 0: none) scores before the softmax:
+   s_h = sum_g talk[h, g] cap(q_g . k), talk fp32 [heads, heads]; sink fp32 [heads] nullable.  q, cache and out as in exl2_window_attn.
+   row_list (nullable: rows 0 .. rows - 1): the rows to compute; nsplit > 1 (<= 64): the keys of a row are dealt to nsplit workgroups, part_o
+   fp32 [rows, heads, nsplit, vdim] and part_ml fp32 [rows, heads, nsplit, 2] (indexed by row) are scratch. */
+int exl2_talk_attn(const void* q, const void* k_cache, const void* v_cache, const float* talk, const float* sink,
+                   const int* row_seq, const int* row_pos, const int* block_table, int bt_stride, int page, void* out,
+                   const int* row_list, int rows, float* part_o, float* part_ml, int nsplit, int dtype, int heads, int kv_heads,
+                   int dim, int vdim, int window, float softcap, void* stream);
+/* the same for portions of prompts on the matrix cores (bfloat16): tile i = rows tile_row0[i] .. + tile_rows[i], <= 16 consecutive positions
+   of ONE sequence.  Sizes: exl2_talk_attn_tiles_supported. */
+int exl2_talk_attn_tiles_supported(int heads, int dim, int vdim);
+int exl2_talk_attn_tiles(const void* q, const void* k_cache, const void* v_cache, const float* talk, const float* sink,
+                         const int* row_seq, const int* row_pos, const int* block_table, int bt_stride, int page, void* out,
+                         const int* tile_row0, const int* tile_rows, int tiles, int heads, int kv_heads, int dim, int vdim,
+                         int window, float softcap, void* stream);
 
 #ifdef __cplusplus
 }

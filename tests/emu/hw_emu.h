@@ -248,6 +248,22 @@ DEV u16 f32_to_bf16(float f)
     u += 0x7fffu + ((u >> 16) & 1u);
     return (u16)(u >> 16);
 }
+DEV f32x4 mfma_4x4x1_f32(float a, float b, f32x4 c)
+{
+    EmuWave& w = emu_ctx_->wave[wave_id()];
+    const int l = lane_id();
+    memcpy(w.slot[l], &a, 4);
+    w.bar.wait();
+    f32x4 d = c;
+    for (int r = 0; r < 4; r++)
+    {
+        float av;
+        memcpy(&av, w.slot[(l & ~3) + r], 4);
+        d[r] += av * b;
+    }
+    w.bar.wait();
+    return d;
+}
 DEV f32x4 mfma_16x16x32_bf16(u32x4 a, u32x4 b, f32x4 c)
 {
     EmuWave& w = emu_ctx_->wave[wave_id()];
