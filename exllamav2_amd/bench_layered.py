@@ -2,8 +2,8 @@
 other model of the package at equal size: the latent-attention / scored-MoE stack beside a Mixtral-style EXL2 stack (same width,
 expert width, expert count, depth), the state-space / windowed-attention stack beside a latent-attention stack (same width, depth,
 heads, window, feed-forward parameters), the token-shifted chunked-attention / linear-attention stack beside a state-space /
-windowed-attention stack (same width, depth, heads, reach, streamed feed-forward parameters).  Used by
-`bench.py --design benolix | tibalorn | negilorn`; one JSON object per size and model."""
+windowed-attention stack (same width, depth, heads, reach, streamed feed-forward parameters), and so on for each later design.  Used by
+`bench.py --design benolix | tibalorn | negilorn | kilurax | zevilorn`; one JSON object per size and model."""
 from __future__ import annotations
 
 import json
@@ -350,7 +350,8 @@ def shift_random_tensors(cfg: dict, s: dict, device, seed: int = 0) -> dict:
                 mat(k + ".mlp.router", ms["router"]["experts"], w)
                 for e in range(ms["router"]["experts"]):
                     mat(f"{k}.mlp.e{e}.up", ms["expert"]["ff"], w); mat(f"{k}.mlp.e{e}.down", w, ms["expert"]["ff"])
-                mat(k + ".mlp.shared.up", ms["shared"]["ff"], w); mat(k + ".mlp.shared.down", w, ms["shared"]["ff"])
+                if ms.get("shared"):
+                    mat(k + ".mlp.shared.up", ms["shared"]["ff"], w); mat(k + ".mlp.shared.down", w, ms["shared"]["ff"])
     return T
 
 
@@ -508,8 +509,129 @@ def bench_sandwich_peer(size: str, device="cuda:0", prompt: int = 2048, ctx: int
     return _bench_engine(model, out, s["vocab"], prompt, ctx, decode_steps, batches)
 
 
+GATED_SIZES = {
+    # pattern: p = window attention beside a minimal gated recurrence, a = head-mixing attention, l = latent attention; every layer has a
+    # sparse feed-forward of two-matrix experts; loop: those layers are gone through twice
+    "w2048": dict(width=2048, heads=16, kv_heads=4, dim=128, vdim=128, window=4096, rot=64, kv_rank=512, q_rank=768, gru=2048, experts=8, top=2,
+                  groups=(4, 2), expert_ff=4224, pattern="palp", loop=None, vocab=32000),
+    "w4096": dict(width=4096, heads=32, kv_heads=8, dim=128, vdim=128, window=4096, rot=64, kv_rank=512, q_rank=1536, gru=4096, experts=8, top=2,
+                  groups=(4, 2), expert_ff=10752, pattern="pal", loop=None, vocab=32000),
+    "w2048-loop": dict(width=2048, heads=16, kv_heads=4, dim=128, vdim=128, window=4096, rot=64, kv_rank=512, q_rank=768, gru=2048, experts=8,
+                       top=2, groups=(4, 2), expert_ff=4224, pattern="palp", loop={"start": 0, "stop": 3, "times": 2}, vocab=32000),
+}
+
+
+def gated_config(s: dict) -> dict:
+    layers = []
+    ff = {"expert": {"ff": s["expert_ff"]}, "kind": "moe",
+          "router": {"experts": s["experts"], "groups": {"count": s["groups"][0], "keep": s["groups"][1]}, "top": s["top"]}}
+    for ch in s["pattern"]:
+        attn = {"dim": s["dim"], "heads": s["heads"], "kv_heads": s["kv_heads"], "vdim": s["vdim"], "mask": {"size": s["window"]},
+                "scale": s["dim"] ** -0.5}
+        if ch == "p":
+            m = {"left": dict(attn, rot={"base": 500000.0, "dims": s["dim"], "scaling": {"factor": 4.0}}), "right": {"width": s["gru"]}}
+            layers.append({"type": "parallel", "mixer": m, "mlp": ff})
+        elif ch == "a":
+            rot = {"base": 500000.0, "dims": s["dim"], "scaling": {"factor": 8.0, "original": 8192, "low": 1.0, "high": 4.0}}
+            layers.append({"type": "attention", "mixer": dict(attn, conv=4, softcap=30.0, rot=rot), "mlp": ff})
+        else:
+            layers.append({"type": "latent_attention", "mlp": ff,
+                           "mixer": {"dim": s["dim"], "heads": s["heads"], "kv_rank": s["kv_rank"], "q_rank": s["q_rank"],
+                                     "rot": {"base": 10000.0, "dims": s["rot"]}, "rot_dim": s["rot"], "scale": (s["dim"] + s["rot"]) ** -0.5,
+                                     "vdim": s["vdim"]}})
+    return {"architecture": "Zevilorn", "layers": layers, "loop": s["loop"], "norm": {"eps": 1e-5}, "vocab": s["vocab"], "width": s["width"]}
+
+
+def gated_random_tensors(cfg: dict, device, seed: int = 0) -> dict:
+    g = torch.Generator(device=device).manual_seed(seed)
+    T = {}
+
+    def mat(name, out, inp, gain=1.0):
+        T[name] = (torch.randn((out, inp), device=device, generator=g) * gain / inp ** 0.5).to(torch.bfloat16)
+
+    def vec(name, n, centre, spread=0.1):
+        T[name] = (centre + spread * torch.randn((n,), device=device, generator=g)).to(torch.bfloat16)
+
+    w = cfg["width"]
+    T["embed"] = (torch.randn((cfg["vocab"], w), device=device, generator=g) * 0.5).to(torch.bfloat16)
+    vec("final.norm", w, 1.0); mat("head", cfg["vocab"], w)
+    for i, L in enumerate(cfg["layers"]):
+        m, k = L["mixer"], f"l{i}"
+        x = k + ".mix"
+        vec(k + ".norm1", w, 1.0)
+        for n in ("rg1", "rg2"):
+            mat(f"{k}.{n}", w, w); vec(f"{k}.{n}.b", w, 0.0)
+        if L["type"] == "attention":
+            H, G, dim, vd = m["heads"], m["kv_heads"], m["dim"], m["vdim"]
+            for n, c in (("q", H * dim), ("k", G * dim), ("v", G * vd)):
+                mat(f"{x}.{n}", c, w); vec(f"{x}.{n}.b", c, 0.0)
+                T[f"{x}.{n}.conv"] = (0.5 * torch.randn((c, m["conv"]), device=device, generator=g)).to(torch.bfloat16)
+            T[x + ".talk"] = (torch.eye(H, device=device) + 0.2 * torch.randn((H, H), device=device, generator=g)).to(torch.bfloat16)
+            mat(x + ".o", w, H * vd); vec(x + ".o.b", w, 0.0)
+        elif L["type"] == "latent_attention":
+            H, dim, rd, vd, R, Q = m["heads"], m["dim"], m["rot_dim"], m["vdim"], m["kv_rank"], m["q_rank"]
+            mat(x + ".dq", Q, w); vec(x + ".dq.norm", Q, 1.0); mat(x + ".uq", H * (dim + rd), Q); mat(x + ".dkv", R + rd, w)
+            vec(x + ".dkv.norm", R, 1.0); mat(x + ".uk", H * dim, R); mat(x + ".uv", H * vd, R); vec(x + ".sink", H, 0.0, 1.0)
+            mat(x + ".g", H, w); mat(x + ".o", w, H * vd)
+        else:
+            a, n = m["left"], m["right"]["width"]
+            H, G, dim, vd = a["heads"], a["kv_heads"], a["dim"], a["vdim"]
+            mat(x + ".left.q", H * dim, w); mat(x + ".left.k", G * dim, w); mat(x + ".left.v", G * vd, w); mat(x + ".left.g", H, w)
+            mat(x + ".left.o", w, H * vd)
+            for c in "zxg":
+                mat(f"{x}.right.{c}", n, w)
+            vec(x + ".right.z.b", n, -2.0, 1.0); vec(x + ".right.x.b", n, 0.0); mat(x + ".right.o", w, n)
+            vec(x + ".left.out", w, 1.0); vec(x + ".right.out", w, 1.0)
+        ms = L["mlp"]
+        mat(k + ".mlp.router", ms["router"]["experts"], w)
+        for e in range(ms["router"]["experts"]):
+            mat(f"{k}.mlp.e{e}.up", ms["expert"]["ff"], w); mat(f"{k}.mlp.e{e}.down", w, ms["expert"]["ff"])
+    return T
+
+
+def bench_gated(size: str, device="cuda:0", prompt: int = 2048, ctx: int = 1024, decode_steps: int = 64, batches=(1, 4)) -> dict:
+    from .config import LayeredConfig
+    from .layered import LayeredModel
+    s = GATED_SIZES[size]
+    cfg = gated_config(s)
+    lc = LayeredConfig.from_dict_parallel_gated(cfg)
+    model = LayeredModel(lc, device=device, dtype=torch.bfloat16).load(gated_random_tensors(cfg, device))
+    out = {"design": "zevilorn", "size": size, "layers": len(cfg["layers"]), "layer_runs": len(lc.layer_runs()), "pattern": s["pattern"],
+           "weight_bytes_per_token": model.weight_bytes()}
+    return _bench_engine(model, out, s["vocab"], prompt, ctx, decode_steps, batches)
+
+
+def bench_gated_peer(size: str, device="cuda:0", prompt: int = 2048, ctx: int = 1024, decode_steps: int = 64, batches=(1, 4)) -> dict:
+    """the closest model of the package: a token-shifted stack of chunked attention (bfloat16, the same engine) of the same width with one
+    layer per layer run -- attention of the same heads and reach with capped scores and the constant in the softmax for every mixer, the
+    same number of two-matrix experts, as much wider as it takes for a token to stream the same bytes"""
+    from .config import LayeredConfig
+    from .layered import LayeredModel
+    s = GATED_SIZES[size]
+    runs = LayeredConfig.from_dict_parallel_gated(gated_config(s)).layer_runs()
+    w, H, G, dim, vd = s["width"], s["heads"], s["kv_heads"], s["dim"], s["vdim"]
+    attn = w * (H * dim + G * (dim + vd) + H) + w * H * vd
+    mixer = {"p": attn + 4 * w * s["gru"], "a": attn - w * H,
+             "l": w * (s["q_rank"] + s["kv_rank"] + s["rot"] + H) + s["q_rank"] * H * (dim + s["rot"]) + s["kv_rank"] * H * (dim + vd) + w * H * vd}
+    extra = sum(mixer[s["pattern"][i]] + 2 * w * w - attn for i, _p, _e in runs) / len(runs)
+    ff = s["expert_ff"] + int(extra / (2 * w * s["top"])) // 64 * 64
+    layers = [{"type": "attention", "mlp": {"expert": {"ff": ff}, "kind": "moe", "router": {"experts": s["experts"], "top": s["top"]}},
+               "mixer": {"dim": dim, "heads": H, "kv_heads": G, "vdim": vd, "mask": {"size": s["window"]}, "scale": dim ** -0.5, "softcap": 30.0,
+                         "rot": {"base": 500000.0, "dims": dim}}} for _ in runs]
+    cfg = {"architecture": "Negilorn", "layers": layers, "logit_scale": 0.5, "norm": {"eps": 1e-5}, "vocab": s["vocab"], "width": w}
+    model = LayeredModel(LayeredConfig.from_dict_prerms_shift(cfg), device=device, dtype=torch.bfloat16).load(
+        shift_random_tensors(cfg, dict(rank=64), device))
+    out = {"design": "negilorn-peer", "size": size, "layers": len(layers), "weight_bytes_per_token": model.weight_bytes()}
+    return _bench_engine(model, out, s["vocab"], prompt, ctx, decode_steps, batches)
+
+
 def run(sizes, device="cuda:0", peer: bool = True, design: str = "benolix"):
     for size in sizes:
+        if design == "zevilorn":
+            print(json.dumps(bench_gated(size, device)), flush=True)
+            if peer:
+                print(json.dumps(bench_gated_peer(size, device)), flush=True)
+            continue
         if design == "kilurax":
             print(json.dumps(bench_sandwich(size, device)), flush=True)
             if peer:
