@@ -413,6 +413,7 @@ DEV float fast_rsqrt(float x) { return rsqrtf(x); }
 DEV float fast_sin(float x) { return __sinf(x); }
 DEV float fast_cos(float x) { return __cosf(x); }
 DEV float fast_rcp(float x) { return __frcp_rn(x); }
+DEV float fast_rcp_approx(float x) { return __builtin_amdgcn_rcpf(x); }        // within 1 ulp
 
 // shader-clock timestamp (s_memtime): used only by the EXL2_TRACE profiling build
 DEV u64 cycle_stamp() { return __builtin_amdgcn_s_memtime(); }

@@ -223,60 +223,317 @@ KERNEL void __launch_bounds__(64) talk_attn_merge_kernel(const TalkArgs a)
     const int r = a.row_list ? a.row_list[bid_x()] : bid_x(), h = bid_y();
     const long long p0 = ((long long)r * a.H + h) * a.nsplit;
     const int lane = lane_id();
-    const float m = lane < a.nsplit ? a.part_ml[(p0 + lane) * 2] : TA_NEG_BIG;       // (nsplit <= 64: a lane per split)
+    // (nsplit <= 64: a lane per split; the sums of the first values are requested before the weights are known)
+    const float m = lane < a.nsplit ? a.part_ml[(p0 + lane) * 2] : TA_NEG_BIG;
     const float l = lane < a.nsplit ? a.part_ml[(p0 + lane) * 2 + 1] : 0.0f;
+    float pv[16];
+    #pragma unroll
+    for (int i = 0; i < 16; i++) pv[i] = a.part_o[(p0 + min(i, a.nsplit - 1)) * a.vdim + min(lane, a.vdim - 1)];
     const float mx = wave_allreduce_max(m);
     const float c = m > 0.5f * TA_NEG_BIG ? expf(m - mx) : 0.0f;
     const float lsum = wave_allreduce_add(l * c);
     const float inv = lsum > 0.0f ? 1.0f / lsum : 0.0f;
     for (int e0 = 0; e0 < a.vdim; e0 += 64)
     {
-        const int e = e0 + lane;
+        const int e = e0 + lane, ec = min(e, a.vdim - 1);
         float o = 0.0f;
-        #pragma unroll 8
-        for (int sp = 0; sp < a.nsplit; sp++)
-            o = fmaf(e < a.vdim ? a.part_o[(p0 + sp) * a.vdim + e] : 0.0f, shfl_idx_f32(c, sp), o);
+        for (int s0 = 0; s0 < a.nsplit; s0 += 16)
+        {
+            if (e0 + s0 > 0)
+            {
+                #pragma unroll
+                for (int i = 0; i < 16; i++) pv[i] = a.part_o[(p0 + min(s0 + i, a.nsplit - 1)) * a.vdim + ec];
+            }
+            #pragma unroll
+            for (int i = 0; i < 16; i++)
+            {
+                const float ci = shfl_idx_f32(c, min(s0 + i, 63));
+                if (s0 + i < a.nsplit && ci > 0.0f) o = fmaf(pv[i], ci, o);
+            }
+        }
         if (e < a.vdim) ta_st<T>((T*)a.out + ((long long)r * a.H + h) * a.vdim + e, o * inv);
     }
 }
 
-// ---- bfloat16 on the matrix cores: portions of prompts -----------------------------------------------------------------------------
-// Workgroup = one tile of <= 16 consecutive positions of one sequence x ALL heads; wave w owns query heads 4 w .. 4 w + 3 (their query
-// rows as operands and their output accumulators in registers).  Keys go by BK at a time in three stages:
-//   1. scores of the wave's heads, S^T = K Q^T (A = key rows straight from the cache: a lane's 8 values are one 16-byte load; the next
-//      step's are requested before stage 2), capped, to LDS as fp32 [head][query][key];
-//   2. the exchange: a lane takes KPL consecutive keys of one query for all heads, s_h = sum_g T[h, g] a_g -- on the fp32 matrix cores in
-//      their 16-block form, where every lane's own column goes through a 4 x 1 product per (four heads out, one head in) without any
-//      lane movement -- and puts the mixed scores back in place;
-//   3. the wave's heads again: online softmax (columns = queries), probabilities to bfloat16 in registers (the accumulator layout of
-//      S^T is the operand layout of O^T += V^T P^T with the keys of a product taken in the order {4 g .. + 3 of block 0, of block 1}),
-//      values through a wave-private LDS tile and transposing reads.
-// Two barriers per step: stage 1 of the next step writes only what its own wave read in stage 3.
-
-#define TM_Q 16
-
-template <int DIM, int VDIM, int NW, int BK>
-struct TalkTile
+// c tanh(s / c) by the hardware exponential and reciprocal (bfloat16 forms): 1 - 2 / (e^(2 s / c) + 1), absolute error a few 1e-7 c
+DEV float tm_soft_cap(float s, float cap, float two_over_cap)
 {
-    static constexpr int HMAX = 4 * NW, SS = BK + 4, TS = HMAX + 4, VSTR = VDIM + 16, NBLK = BK / 16;
-    static constexpr size_t smem = sizeof(float) * ((size_t)HMAX * TM_Q * SS + (size_t)HMAX * TS) + sizeof(u16) * (size_t)NW * BK * VSTR;
-};
+    return cap > 0.0f ? fmaf(-2.0f * cap, fast_rcp_approx(fast_exp(s * two_over_cap) + 1.0f), cap) : s;
+}
 
 DEV u32 tm_pack2(float lo, float hi) { return (u32)f32_to_bf16(lo) | ((u32)f32_to_bf16(hi) << 16); }
 
-template <int DIM, int VDIM, int NW, int BK>
-KERNEL void __launch_bounds__(64 * NW, 1) talk_attn_tile_kernel(const TalkArgs a)
+extern "C" int exl2_talk_attn_tiles_supported(int heads, int dim, int vdim);
+
+// ---- bfloat16 on the matrix cores: decoded tokens -----------------------------------------------------------------------------------
+// Workgroup = one row x all heads x one share of the keys, 64 keys at a time: wave w scores keys 16 w .. + 15 for one key / value head
+// after the other (A = key rows from the cache, B = the query heads that share them), the scores go to LDS as [head][key]; a wave then
+// takes HQ heads with a key per lane, mixes (T in LDS, transposed, read as broadcasts), joins the running softmax with lane
+// exchanges and leaves the probabilities in LDS; last a wave takes key / value heads w, w + 4, .. and adds V^T P^T (values through a
+// wave-private LDS tile and transposing reads).  Keys and values of a step are all requested before its first product.
+
+#define TD_STR 68                            // floats between two heads' scores
+
+template <int VDIM> HD size_t td_smem(int H)
+{
+    return sizeof(float) * ((size_t)2 * H * TD_STR + (size_t)H * 36 + ((3 * (size_t)H + 3) & ~(size_t)3)) + sizeof(u16) * (size_t)4 * 64 * (VDIM + 16);
+}
+
+template <int DIM, int VDIM, int KVW>
+KERNEL void __launch_bounds__(256, 1) talk_attn_decode_kernel(const TalkArgs a)
 {
     DYN_SMEM(smem);
-    typedef TalkTile<DIM, VDIM, NW, BK> TT;
-    constexpr int SS = TT::SS, TS = TT::TS, VSTR = TT::VSTR, NBLK = TT::NBLK, KK = DIM / 32, DB = VDIM / 16;
-    constexpr int KPL = TM_Q * BK / (64 * NW);                   // stage 2: keys per lane
-    constexpr int VP = BK * VDIM / 8 / 64;                       // stage 3: 16-byte value pieces per lane
-    constexpr int VPR = VDIM / 8;                                // pieces of a value row
-    constexpr int NT = NW;                                       // output tiles of four heads
+    SHARED long long s_row[64];
+    constexpr int KK = DIM / 32, DB = VDIM / 16, VSTR = VDIM + 16, VPR = VDIM / 8, VP = 64 * VPR / 64, HQ = 4 * KVW;
+    const int H = a.H, G = a.G, hpg = H / G;
+    float* s_a = (float*)smem;                                   // [H][TD_STR] capped scores
+    float* s_p = s_a + H * TD_STR;                               // [H][TD_STR] probabilities
+    float* s_t = s_p + H * TD_STR;                               // [H (head in)][36]: T transposed, head out along the row
+    float* s_c = s_t + H * 36;                                   // [H] correction of the step, [H] final maximum, [H] final sum
+    u16* s_v = (u16*)(s_c + ((3 * H + 3) & ~3));                 // [4][64][VSTR], 16-byte aligned
+    const int t = tid(), lane = lane_id(), wv = wave_id();
+    const int qi = lane & 15, g = lane >> 4;
+    const int r = a.row_list ? a.row_list[bid_x()] : bid_x();
+    const int split = bid_y();
+    const int pos = a.row_pos[r];
+    const int* bt = a.block_table + (long long)a.row_seq[r] * a.bt_stride;
+    const int j_lo = max(0, pos - a.window + 1);
+    const int total = pos - j_lo + 1;
+    const int all_steps = (total + 63) / 64;
+    const int per_split = (all_steps + a.nsplit - 1) / a.nsplit;
+    const int step0 = split * per_split, step1 = min(all_steps, step0 + per_split);
+    const u16* kc = (const u16*)a.k_cache; const u16* vc = (const u16*)a.v_cache;
+    u16* my_v = s_v + wv * 64 * VSTR;
+    for (int i = t; i < H * 36; i += 256)
+    {
+        const int in = i / 36, out = i % 36;
+        s_t[i] = out < H ? a.talk[out * H + in] : 0.0f;
+    }
+    // this wave's heads in the mixing stage: HQ wv .. + HQ - 1 (uniform over the lanes)
+    float m_run[HQ], l_run[HQ];
+    const bool with_sink = a.sink && split == 0;                 // the sink counts once
+    #pragma unroll
+    for (int i = 0; i < HQ; i++)
+    {
+        const int h = min(wv * HQ + i, H - 1);
+        m_run[i] = with_sink ? a.sink[h] : TA_NEG_BIG;
+        l_run[i] = with_sink ? 1.0f : 0.0f;
+    }
+    f32x4 ot[KVW][DB];
+    #pragma unroll
+    for (int k = 0; k < KVW; k++)
+        #pragma unroll
+        for (int d = 0; d < DB; d++) ot[k][d] = (f32x4){0.0f, 0.0f, 0.0f, 0.0f};
+    const float cap2 = a.softcap > 0.0f ? 2.0f / a.softcap : 0.0f;
+
+    for (int step = step0; step < step1; step++)
+    {
+        const int k0 = step * 64, nc = min(64, total - k0);
+        if (t < 64) s_row[t] = ta_cache_row(a, bt, j_lo + k0 + min(t, nc - 1));
+        block_sync();                                            // (also: everybody is done with the previous step)
+        const long long krow = s_row[16 * wv + qi];
+        u32x4 vreg[KVW][VP];
+        // ---- scores: four key / value heads' rows in flight
+        for (int g0 = 0; g0 < G; g0 += 4)
+        {
+            u32x4 kf[4][KK], qf[4][KK];
+            #pragma unroll
+            for (int k = 0; k < 4; k++)
+            {
+                const int kv = min(g0 + k, G - 1);
+                const u16* kp = kc + (krow * G + kv) * DIM + 8 * g;
+                const u16* qp = (const u16*)a.q + ((long long)r * H + kv * hpg + min(qi, hpg - 1)) * DIM + 8 * g;
+                #pragma unroll
+                for (int kk = 0; kk < KK; kk++) { kf[k][kk] = *(const u32x4*)(kp + 32 * kk); qf[k][kk] = *(const u32x4*)(qp + 32 * kk); }
+            }
+            if (g0 == 0)
+            {
+                #pragma unroll
+                for (int k = 0; k < KVW; k++)
+                    #pragma unroll
+                    for (int i = 0; i < VP; i++)
+                        vreg[k][i] = *(const u32x4*)(vc + (s_row[(lane + 64 * i) / VPR] * G + min(wv + 4 * k, G - 1)) * VDIM + ((lane + 64 * i) % VPR) * 8);
+            }
+            #pragma unroll
+            for (int k = 0; k < 4; k++)
+            {
+                if (g0 + k >= G) break;
+                f32x4 st = {0.0f, 0.0f, 0.0f, 0.0f};
+                #pragma unroll
+                for (int kk = 0; kk < KK; kk++) st = mfma_16x16x32_bf16(kf[k][kk], qf[k][kk], st);
+                #pragma unroll
+                for (int e = 0; e < 4; e++) st[e] = tm_soft_cap(st[e], a.softcap, cap2);
+                if (qi < hpg) *(f32x4*)(s_a + ((g0 + k) * hpg + qi) * TD_STR + 16 * wv + 4 * g) = st;
+            }
+        }
+        block_sync_lds();
+        // ---- the exchange between the heads and the softmax: lane = key
+        if (wv * HQ < H)
+        {
+            float mx[HQ];
+            #pragma unroll
+            for (int i = 0; i < HQ; i++) mx[i] = 0.0f;
+            for (int c = 0; c < H; c++)
+            {
+                const float sv = s_a[c * TD_STR + lane];
+                #pragma unroll
+                for (int i4 = 0; i4 < HQ; i4 += 4)
+                {
+                    const f32x4 tv = *(const f32x4*)(s_t + c * 36 + wv * HQ + i4);
+                    #pragma unroll
+                    for (int e = 0; e < 4; e++) mx[i4 + e] = fmaf(tv[e], sv, mx[i4 + e]);
+                }
+            }
+            #pragma unroll
+            for (int i = 0; i < HQ; i++)
+            {
+                const int h = wv * HQ + i;
+                if (h >= H) break;
+                const float s = lane < nc ? mx[i] : TA_NEG_BIG;
+                const float m_new = fmaxf(m_run[i], wave_allreduce_max(s));
+                const float p = lane < nc ? fast_exp(s - m_new) : 0.0f;
+                const float c = fast_exp(m_run[i] - m_new);
+                l_run[i] = l_run[i] * c + wave_allreduce_add(p);
+                m_run[i] = m_new;
+                s_p[h * TD_STR + lane] = p;
+                if (lane == 0) s_c[h] = c;
+            }
+        }
+        block_sync_lds();
+        // ---- values: this wave's key / value heads
+        #pragma unroll
+        for (int k = 0; k < KVW; k++)
+        {
+            const int kv = wv + 4 * k;
+            if (kv >= G) break;
+            wave_sync();
+            #pragma unroll
+            for (int i = 0; i < VP; i++) *(u32x4*)(my_v + ((lane + 64 * i) / VPR) * VSTR + ((lane + 64 * i) % VPR) * 8) = vreg[k][i];
+            wave_sync();
+            const int h = kv * hpg + min(qi, hpg - 1);
+            const float alpha = s_c[h];
+            u32x4 pb[2];
+            #pragma unroll
+            for (int b = 0; b < 4; b++)
+            {
+                const f32x4 p = *(const f32x4*)(s_p + h * TD_STR + 16 * b + 4 * g);
+                pb[b / 2][2 * (b % 2)] = tm_pack2(p[0], p[1]);
+                pb[b / 2][2 * (b % 2) + 1] = tm_pack2(p[2], p[3]);
+            }
+            const u16* vbase = my_v + (4 * g + (qi >> 2)) * VSTR + 4 * (qi & 3);
+            #pragma unroll
+            for (int d = 0; d < DB; d++)
+            {
+                #pragma unroll
+                for (int e = 0; e < 4; e++) ot[k][d][e] *= alpha;
+                #pragma unroll
+                for (int m2 = 0; m2 < 2; m2++)
+                {
+                    const f16x4 lo = lds_read_tr16_b64((const f16*)(vbase + (32 * m2) * VSTR + 16 * d));
+                    const f16x4 hi = lds_read_tr16_b64((const f16*)(vbase + (32 * m2 + 16) * VSTR + 16 * d));
+                    const u32x2 l2 = __builtin_bit_cast(u32x2, lo), h2 = __builtin_bit_cast(u32x2, hi);
+                    ot[k][d] = mfma_16x16x32_bf16((u32x4){l2[0], l2[1], h2[0], h2[1]}, pb[m2], ot[k][d]);
+                }
+            }
+        }
+    }
+    #pragma unroll
+    for (int i = 0; i < HQ; i++)
+    {
+        const int h = wv * HQ + i;
+        if (h < H && lane == 0)
+        {
+            s_c[H + h] = m_run[i];
+            s_c[2 * H + h] = l_run[i];
+            if (a.nsplit > 1)
+            {
+                const long long pi = ((long long)r * H + h) * a.nsplit + split;
+                a.part_ml[pi * 2] = m_run[i]; a.part_ml[pi * 2 + 1] = l_run[i];
+            }
+        }
+    }
+    block_sync();
+    #pragma unroll
+    for (int k = 0; k < KVW; k++)
+    {
+        const int kv = wv + 4 * k;
+        if (kv >= G || qi >= hpg) continue;
+        const int h = kv * hpg + qi;
+        if (a.nsplit > 1)
+        {
+            float* po = a.part_o + (((long long)r * H + h) * a.nsplit + split) * VDIM + 4 * g;
+            #pragma unroll
+            for (int d = 0; d < DB; d++) *(f32x4*)(po + 16 * d) = ot[k][d];
+        }
+        else
+        {
+            const float l = s_c[2 * H + h], inv = l > 0.0f ? 1.0f / l : 0.0f;
+            u16* op = (u16*)a.out + ((long long)r * H + h) * VDIM + 4 * g;
+            #pragma unroll
+            for (int d = 0; d < DB; d++)
+                *(u32x2*)(op + 16 * d) = (u32x2){tm_pack2(ot[k][d][0] * inv, ot[k][d][1] * inv), tm_pack2(ot[k][d][2] * inv, ot[k][d][3] * inv)};
+        }
+    }
+}
+
+template <int DIM, int VDIM, int KVW>
+static void td_launch_one(const TalkArgs& a, int rows, hipStream_t s)
+{
+    static bool attr_done[EXL2_MAX_DEVICES];
+    if (exl2_first_on_device(attr_done))
+        (void)hipFuncSetAttribute((const void*)talk_attn_decode_kernel<DIM, VDIM, KVW>, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024 - 1024);
+    LAUNCH((talk_attn_decode_kernel<DIM, VDIM, KVW>), dim3(rows, a.nsplit), dim3(256), td_smem<VDIM>(a.H), s, a);
+}
+
+template <int DIM, int VDIM>
+static void td_launch(const TalkArgs& a, int rows, hipStream_t s)
+{
+    if (a.H <= 16 && a.G <= 4) td_launch_one<DIM, VDIM, 1>(a, rows, s);
+    else td_launch_one<DIM, VDIM, 2>(a, rows, s);
+}
+
+// ---- bfloat16 on the matrix cores: portions of prompts -----------------------------------------------------------------------------
+// Workgroup = one tile of <= 16 consecutive positions of one sequence x ALL heads, eight waves; wave w owns query heads HPW w .. + HPW - 1
+// (their query rows as operands and their output accumulators in registers).  Keys go by 32 at a time in three stages:
+//   1. scores of the wave's heads, S^T = K Q^T (A = key rows straight from the cache: a lane's 8 values are one 16-byte load), capped, to
+//      LDS as fp32 [head][query][key];
+//   2. the exchange: a lane takes one (query, key) for all heads, s_h = sum_g T[h, g] a_g -- on the fp32 matrix cores in their 16-block
+//      form, where every lane's own scalar goes through a 4 x 1 product per (four heads out, one head in) without any lane
+//      movement -- and puts the mixed scores back in place;
+//   3. the wave's heads again: online softmax (columns = queries), probabilities to bfloat16 in registers (the accumulator layout of
+//      S^T is the operand layout of O^T += V^T P^T with the keys of a product taken in the order {4 g .. + 3 of block 0, of block 1}),
+//      values through a wave-private LDS tile and transposing reads.
+// The step's value rows are requested before stage 2, the next step's key rows before stage 3 (they take turns in the same registers);
+// the rows' places in the cache are looked up by one wave a step ahead.  Two barriers per step: stage 1 of the next step writes only
+// what its own wave read in stage 3.
+
+#define TM_Q 16
+#define TM_NW 8
+#define TM_BK 32
+
+template <int DIM, int VDIM, int HPW>
+struct TalkTile
+{
+    static constexpr int HMAX = TM_NW * HPW, SS = TM_BK + 4, TS = HMAX + 4, VSTR = VDIM + 16;
+    static constexpr size_t smem = sizeof(float) * ((size_t)HMAX * TM_Q * SS + (size_t)HMAX * TS) + sizeof(u16) * (size_t)TM_NW * TM_BK * VSTR;
+};
+
+template <int DIM, int VDIM, int HPW>
+KERNEL void __launch_bounds__(64 * TM_NW, 1) talk_attn_tile_kernel(const TalkArgs a)
+{
+    DYN_SMEM(smem);
+    SHARED int s_row[2][TM_BK];
+    typedef TalkTile<DIM, VDIM, HPW> TT;
+    constexpr int SS = TT::SS, TS = TT::TS, VSTR = TT::VSTR, NBLK = TM_BK / 16, KK = DIM / 32, DB = VDIM / 16;
+    constexpr int VPR = VDIM / 8, VP = TM_BK * VPR / 64;         // 16-byte pieces of a value row; value pieces per lane
+    constexpr int NT = TT::HMAX / 4;                             // groups of four heads out
+    // registers are short where a wave holds four wide heads: its query rows are read again every step (they stay in the caches) and the
+    // next step's key rows are not requested ahead
+    constexpr bool LEAN = HPW * 4 * (KK + DB) > 128;
+    constexpr int QN = LEAN ? 1 : HPW;
     float* s_s = (float*)smem;                                   // [HMAX][TM_Q][SS]
     float* s_t = s_s + TT::HMAX * TM_Q * SS;                     // [HMAX][TS]: T, zero past H
-    u16* s_v = (u16*)(s_t + TT::HMAX * TS);                      // [NW][BK][VSTR]
+    u16* s_v = (u16*)(s_t + TT::HMAX * TS);                      // [TM_NW][TM_BK][VSTR]
 
     const int t = tid(), lane = lane_id(), wv = wave_id();
     const int qi = lane & 15, g = lane >> 4;
@@ -287,191 +544,198 @@ KERNEL void __launch_bounds__(64 * NW, 1) talk_attn_tile_kernel(const TalkArgs a
     const int* bt = a.block_table + (long long)a.row_seq[r0] * a.bt_stride;
     const int j_lo = max(0, p0 - a.window + 1);
     const int total = p_last - j_lo + 1;
-    const int n_steps = (total + BK - 1) / BK;
+    const int n_steps = (total + TM_BK - 1) / TM_BK;
     const u16* kc = (const u16*)a.k_cache; const u16* vc = (const u16*)a.v_cache;
-    u16* my_v = s_v + wv * BK * VSTR;
+    u16* my_v = s_v + wv * TM_BK * VSTR;
+    const float cap2 = a.softcap > 0.0f ? 2.0f / a.softcap : 0.0f;
 
-    for (int i = t; i < TT::HMAX * TT::HMAX; i += 64 * NW)
+    for (int i = t; i < TT::HMAX * TT::HMAX; i += 64 * TM_NW)
     {
         const int h = i / TT::HMAX, c = i % TT::HMAX;
         s_t[h * TS + c] = h < H && c < H ? a.talk[h * H + c] : 0.0f;
     }
-    const int nh = max(0, min(4, H - 4 * wv));                   // heads of this wave
-    const int h0 = min(4 * wv, H - 1);
-    int kvh[4];
+    if (t < TM_BK) s_row[0][t] = (int)ta_cache_row(a, bt, j_lo + min(t, total - 1));
+    const int nh = max(0, min(HPW, H - HPW * wv));               // heads of this wave
+    const int h0 = min(HPW * wv, H - 1);
+    int kvh[HPW];
     #pragma unroll
-    for (int n = 0; n < 4; n++) kvh[n] = min(h0 + n, H - 1) / hpg;
+    for (int n = 0; n < HPW; n++) kvh[n] = uniform(min(h0 + n, H - 1) / hpg);
 
     const int qrow = r0 + min(qi, n_rows - 1), qpos = p0 + min(qi, n_rows - 1), q_lo = qpos - a.window + 1;
-    u32x4 qb[4][KK];
-    f32x4 ot[4][DB];
-    float m_run[4], l_run[4];
+    u32x4 qb[QN][KK];
+    auto load_q = [&](int n) {
+        const u16* qp = (const u16*)a.q + ((long long)qrow * H + min(h0 + n, H - 1)) * DIM + 8 * g;
+        #pragma unroll
+        for (int kk = 0; kk < KK; kk++) qb[LEAN ? 0 : n][kk] = *(const u32x4*)(qp + 32 * kk);
+    };
+    f32x4 ot[HPW][DB];
+    float m_run[HPW], l_run[HPW];
     #pragma unroll
-    for (int n = 0; n < 4; n++)
+    for (int n = 0; n < HPW; n++)
     {
         const int h = min(h0 + n, H - 1);
-        const u16* qp = (const u16*)a.q + ((long long)qrow * H + h) * DIM + 8 * g;
-        #pragma unroll
-        for (int kk = 0; kk < KK; kk++) qb[n][kk] = *(const u32x4*)(qp + 32 * kk);
+        if (!LEAN) load_q(n);
         #pragma unroll
         for (int d = 0; d < DB; d++) ot[n][d] = (f32x4){0.0f, 0.0f, 0.0f, 0.0f};
         m_run[n] = a.sink ? a.sink[h] : TA_NEG_BIG;
         l_run[n] = a.sink ? 1.0f : 0.0f;
     }
-
-    // rows in the cache of what this lane loads in a step: its key of every 16-key block, and the rows of its value pieces
-    long long krow[NBLK], vrow[VP];
     u32x4 kf[NBLK][KK], vreg[VP];
-    auto lookup = [&](int step) {
-        #pragma unroll
-        for (int b = 0; b < NBLK; b++) krow[b] = ta_cache_row(a, bt, j_lo + min(step * BK + 16 * b + qi, total - 1));
-    };
-    auto lookup_v = [&](int step) {
-        #pragma unroll
-        for (int i = 0; i < VP; i++) vrow[i] = ta_cache_row(a, bt, j_lo + min(step * BK + (lane + 64 * i) / VPR, total - 1));
-    };
-    auto load_k = [&](int kv) {
+    auto load_k = [&](int step, int kv) {
         #pragma unroll
         for (int b = 0; b < NBLK; b++)
+        {
+            const u16* kp = kc + ((long long)s_row[step & 1][16 * b + qi] * G + kv) * DIM + 8 * g;
             #pragma unroll
-            for (int kk = 0; kk < KK; kk++) kf[b][kk] = *(const u32x4*)(kc + (krow[b] * G + kv) * DIM + 32 * kk + 8 * g);
+            for (int kk = 0; kk < KK; kk++) kf[b][kk] = *(const u32x4*)(kp + 32 * kk);
+        }
     };
-    auto load_v = [&](int kv) {
+    auto load_v = [&](int step, int kv) {
         #pragma unroll
-        for (int i = 0; i < VP; i++) vreg[i] = *(const u32x4*)(vc + (vrow[i] * G + kv) * VDIM + ((lane + 64 * i) % VPR) * 8);
+        for (int i = 0; i < VP; i++)
+            vreg[i] = *(const u32x4*)(vc + ((long long)s_row[step & 1][(lane + 64 * i) / VPR] * G + kv) * VDIM + ((lane + 64 * i) % VPR) * 8);
     };
-    if (nh > 0) { lookup(0); load_k(kvh[0]); lookup_v(0); load_v(kvh[0]); }
     block_sync();
+    if (nh > 0 && !LEAN) load_k(0, kvh[0]);
 
     for (int step = 0; step < n_steps; step++)
     {
-        const int k0 = step * BK;
+        const int k0 = step * TM_BK;
+        int next_row = 0;
+        if (t < TM_BK) next_row = (int)ta_cache_row(a, bt, j_lo + min(k0 + TM_BK + t, total - 1));
         // ---- 1: scores of this wave's heads
         #pragma unroll
-        for (int n = 0; n < 4; n++)
+        for (int n = 0; n < HPW; n++)
         {
             if (n >= nh) break;
-            if (n > 0 && kvh[n] != kvh[n - 1]) load_k(kvh[n]);
+            if (n > 0 ? kvh[n] != kvh[n - 1] : LEAN) load_k(step, kvh[n]);
+            if (LEAN) load_q(n);
             float* sr = s_s + ((h0 + n) * TM_Q + qi) * SS + 4 * g;
             #pragma unroll
             for (int b = 0; b < NBLK; b++)
             {
                 f32x4 st = {0.0f, 0.0f, 0.0f, 0.0f};
                 #pragma unroll
-                for (int kk = 0; kk < KK; kk++) st = mfma_16x16x32_bf16(kf[b][kk], qb[n][kk], st);
+                for (int kk = 0; kk < KK; kk++) st = mfma_16x16x32_bf16(kf[b][kk], qb[LEAN ? 0 : n][kk], st);
                 #pragma unroll
-                for (int r = 0; r < 4; r++) st[r] = ta_soft_cap(st[r], a.softcap);
+                for (int r = 0; r < 4; r++) st[r] = tm_soft_cap(st[r], a.softcap, cap2);
                 *(f32x4*)(sr + 16 * b) = st;
             }
         }
         block_sync_lds();
-        if (nh > 0 && step + 1 < n_steps) { lookup(step + 1); load_k(kvh[0]); }
+        if (nh > 0) load_v(step, kvh[0]);
+        // (the other half of the table held the step before this one: every wave is past it)
+        if (t < TM_BK) s_row[(step + 1) & 1][t] = next_row;
         // ---- 2: the exchange between the heads, in place
         {
-            const int task = t * KPL, q2 = task / BK, c2 = task % BK;
-            float* sp = s_s + q2 * SS + c2;
-            f32x4 mx[NT][KPL];
+            float* sp = s_s + (t / TM_BK) * SS + t % TM_BK;
+            f32x4 mx[NT];
             #pragma unroll
-            for (int i = 0; i < NT; i++)
-                #pragma unroll
-                for (int e = 0; e < KPL; e++) mx[i][e] = (f32x4){0.0f, 0.0f, 0.0f, 0.0f};
+            for (int i = 0; i < NT; i++) mx[i] = (f32x4){0.0f, 0.0f, 0.0f, 0.0f};
             for (int c4 = 0; c4 < H; c4 += 4)
             {
                 f32x4 tv[NT];
+                float sv[4];
+                #pragma unroll
+                for (int k = 0; k < 4; k++) sv[k] = sp[min(c4 + k, H - 1) * TM_Q * SS];         // (past the last head T is zero)
                 #pragma unroll
                 for (int i = 0; i < NT; i++) tv[i] = *(const f32x4*)(s_t + (4 * i + (lane & 3)) * TS + c4);
                 #pragma unroll
                 for (int k = 0; k < 4; k++)
-                {
-                    const int c = min(c4 + k, H - 1);            // (past the last head T is zero)
-                    float sv[KPL];
                     #pragma unroll
-                    for (int e = 0; e < KPL; e++) sv[e] = sp[c * TM_Q * SS + e];
-                    #pragma unroll
-                    for (int i = 0; i < NT; i++)
-                        #pragma unroll
-                        for (int e = 0; e < KPL; e++) mx[i][e] = mfma_4x4x1_f32(tv[i][k], sv[e], mx[i][e]);
-                }
+                    for (int i = 0; i < NT; i++) mx[i] = mfma_4x4x1_f32(tv[i][k], sv[k], mx[i]);
             }
-            wave_sync();
             #pragma unroll
             for (int i = 0; i < NT; i++)
                 #pragma unroll
                 for (int r = 0; r < 4; r++)
-                    if (4 * i + r < H)
-                    {
-                        #pragma unroll
-                        for (int e = 0; e < KPL; e++) sp[(4 * i + r) * TM_Q * SS + e] = mx[i][e][r];
-                    }
+                    if (4 * i + r < H) sp[(4 * i + r) * TM_Q * SS] = mx[i][r];
         }
         block_sync_lds();
         // ---- 3: softmax and values of this wave's heads
-        #pragma unroll
-        for (int n = 0; n < 4; n++)
+        if (nh > 0)
         {
-            if (n >= nh) break;
-            if (n == 0 || kvh[n] != kvh[n - 1])
+            u32x4 pb[HPW];
+            float alpha[HPW];
+            bool moved = false;
+            #pragma unroll
+            for (int n = 0; n < HPW; n++)
             {
-                if (n > 0) { load_v(kvh[n]); wave_sync(); }
+                alpha[n] = 1.0f;
+                if (n >= nh) break;
+                const float* sr = s_s + ((h0 + n) * TM_Q + qi) * SS + 4 * g;
+                float sc[8];
+                float m_loc = TA_NEG_BIG;
+                #pragma unroll
+                for (int b = 0; b < NBLK; b++)
+                {
+                    const f32x4 v = *(const f32x4*)(sr + 16 * b);
+                    #pragma unroll
+                    for (int r = 0; r < 4; r++)
+                    {
+                        const int j = j_lo + k0 + 16 * b + 4 * g + r;
+                        sc[4 * b + r] = j <= qpos && j >= q_lo ? v[r] : TA_NEG_BIG;
+                        m_loc = fmaxf(m_loc, sc[4 * b + r]);
+                    }
+                }
+                m_loc = fmaxf(m_loc, shfl_xor_f32(m_loc, 16));
+                m_loc = fmaxf(m_loc, shfl_xor_f32(m_loc, 32));
+                const float m_new = fmaxf(m_run[n], m_loc);
+                alpha[n] = fast_exp(m_run[n] - m_new);
+                moved = moved || alpha[n] != 1.0f;
+                float p_sum = 0.0f;
+                #pragma unroll
+                for (int e2 = 0; e2 < 4; e2++)
+                {
+                    const float pa = sc[2 * e2] > 0.5f * TA_NEG_BIG ? fast_exp(sc[2 * e2] - m_new) : 0.0f;
+                    const float pc = sc[2 * e2 + 1] > 0.5f * TA_NEG_BIG ? fast_exp(sc[2 * e2 + 1] - m_new) : 0.0f;
+                    p_sum += pa + pc;
+                    pb[n][e2] = tm_pack2(pa, pc);
+                }
+                p_sum += shfl_xor_f32(p_sum, 16);
+                p_sum += shfl_xor_f32(p_sum, 32);
+                l_run[n] = l_run[n] * alpha[n] + p_sum;
+                m_run[n] = m_new;
+            }
+            if (wave_ballot(moved) != 0ull)                      // the running maxima rarely move once a few steps have gone by
+            {
+                #pragma unroll
+                for (int n = 0; n < HPW; n++)
+                    #pragma unroll
+                    for (int d = 0; d < DB; d++)
+                        #pragma unroll
+                        for (int e = 0; e < 4; e++) ot[n][d][e] *= alpha[n];
+            }
+            // runs of heads that read the same key / value head: its values once through LDS, every fragment feeds all of the run
+            #pragma unroll
+            for (int n0 = 0; n0 < HPW; n0++)
+            {
+                if (n0 >= nh) break;
+                if (n0 > 0 && kvh[n0] == kvh[n0 - 1]) continue;
+                if (n0 > 0) load_v(step, kvh[n0]);
+                wave_sync();
                 #pragma unroll
                 for (int i = 0; i < VP; i++) *(u32x4*)(my_v + ((lane + 64 * i) / VPR) * VSTR + ((lane + 64 * i) % VPR) * 8) = vreg[i];
                 wave_sync();
-            }
-            const float* sr = s_s + ((h0 + n) * TM_Q + qi) * SS + 4 * g;
-            float sc[4 * NBLK];
-            float m_loc = TA_NEG_BIG;
-            #pragma unroll
-            for (int b = 0; b < NBLK; b++)
-            {
-                const f32x4 v = *(const f32x4*)(sr + 16 * b);
+                const u16* vbase = my_v + (4 * g + (qi >> 2)) * VSTR + 4 * (qi & 3);
                 #pragma unroll
-                for (int r = 0; r < 4; r++)
+                for (int d = 0; d < DB; d++)
                 {
-                    const int j = j_lo + k0 + 16 * b + 4 * g + r;
-                    sc[4 * b + r] = j <= qpos && j >= q_lo ? v[r] : TA_NEG_BIG;
-                    m_loc = fmaxf(m_loc, sc[4 * b + r]);
-                }
-            }
-            m_loc = fmaxf(m_loc, shfl_xor_f32(m_loc, 16));
-            m_loc = fmaxf(m_loc, shfl_xor_f32(m_loc, 32));
-            const float m_new = fmaxf(m_run[n], m_loc);
-            const float alpha = fast_exp(m_run[n] - m_new);
-            float p_sum = 0.0f;
-            u32x4 pb[NBLK / 2];
-            #pragma unroll
-            for (int e2 = 0; e2 < 2 * NBLK; e2++)
-            {
-                const float pa = sc[2 * e2] > 0.5f * TA_NEG_BIG ? fast_exp(sc[2 * e2] - m_new) : 0.0f;
-                const float pc = sc[2 * e2 + 1] > 0.5f * TA_NEG_BIG ? fast_exp(sc[2 * e2 + 1] - m_new) : 0.0f;
-                p_sum += pa + pc;
-                pb[e2 / 4][e2 % 4] = tm_pack2(pa, pc);
-            }
-            p_sum += shfl_xor_f32(p_sum, 16);
-            p_sum += shfl_xor_f32(p_sum, 32);
-            l_run[n] = l_run[n] * alpha + p_sum;
-            m_run[n] = m_new;
-            const u16* vbase = my_v + (4 * g + (qi >> 2)) * VSTR + 4 * (qi & 3);
-            #pragma unroll
-            for (int d = 0; d < DB; d++)
-            {
-                ot[n][d][0] *= alpha; ot[n][d][1] *= alpha; ot[n][d][2] *= alpha; ot[n][d][3] *= alpha;
-                #pragma unroll
-                for (int m2 = 0; m2 < NBLK / 2; m2++)
-                {
-                    const f16x4 lo = lds_read_tr16_b64((const f16*)(vbase + (32 * m2) * VSTR + 16 * d));
-                    const f16x4 hi = lds_read_tr16_b64((const f16*)(vbase + (32 * m2 + 16) * VSTR + 16 * d));
+                    const f16x4 lo = lds_read_tr16_b64((const f16*)(vbase + 16 * d));
+                    const f16x4 hi = lds_read_tr16_b64((const f16*)(vbase + 16 * VSTR + 16 * d));
                     const u32x2 l2 = __builtin_bit_cast(u32x2, lo), h2 = __builtin_bit_cast(u32x2, hi);
-                    ot[n][d] = mfma_16x16x32_bf16((u32x4){l2[0], l2[1], h2[0], h2[1]}, pb[m2], ot[n][d]);
+                    #pragma unroll
+                    for (int n = n0; n < HPW; n++)
+                        if (n < nh && kvh[n] == kvh[n0]) ot[n][d] = mfma_16x16x32_bf16((u32x4){l2[0], l2[1], h2[0], h2[1]}, pb[n], ot[n][d]);
                 }
             }
+            if (!LEAN && step + 1 < n_steps) load_k(step + 1, kvh[0]);
         }
-        wave_sync();                                             // the wave is done with its value tile
-        if (nh > 0 && step + 1 < n_steps) { lookup_v(step + 1); load_v(kvh[0]); }
     }
 
     if (qi >= n_rows) return;
     #pragma unroll
-    for (int n = 0; n < 4; n++)
+    for (int n = 0; n < HPW; n++)
     {
         if (n >= nh) break;
         const float inv = l_run[n] > 0.0f ? 1.0f / l_run[n] : 0.0f;
@@ -482,21 +746,21 @@ KERNEL void __launch_bounds__(64 * NW, 1) talk_attn_tile_kernel(const TalkArgs a
     }
 }
 
-template <int DIM, int VDIM, int NW, int BK>
+template <int DIM, int VDIM, int HPW>
 static void tm_launch_one(const TalkArgs& a, int tiles, hipStream_t s)
 {
     static bool attr_done[EXL2_MAX_DEVICES];
-    static_assert(TalkTile<DIM, VDIM, NW, BK>::smem <= 160 * 1024, "the tile fits the LDS");
+    static_assert(TalkTile<DIM, VDIM, HPW>::smem <= 159 * 1024, "the tile fits the LDS");
     if (exl2_first_on_device(attr_done))
-        (void)hipFuncSetAttribute((const void*)talk_attn_tile_kernel<DIM, VDIM, NW, BK>, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024);
-    LAUNCH((talk_attn_tile_kernel<DIM, VDIM, NW, BK>), dim3(tiles), dim3(64 * NW), (TalkTile<DIM, VDIM, NW, BK>::smem), s, a);
+        (void)hipFuncSetAttribute((const void*)talk_attn_tile_kernel<DIM, VDIM, HPW>, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024 - 1024);
+    LAUNCH((talk_attn_tile_kernel<DIM, VDIM, HPW>), dim3(tiles), dim3(64 * TM_NW), (TalkTile<DIM, VDIM, HPW>::smem), s, a);
 }
 
 template <int DIM, int VDIM>
 static void tm_launch(const TalkArgs& a, int tiles, hipStream_t s)
 {
-    if (a.H <= 16) tm_launch_one<DIM, VDIM, 4, 64>(a, tiles, s);
-    else tm_launch_one<DIM, VDIM, 8, 32>(a, tiles, s);
+    if (a.H <= 2 * TM_NW) tm_launch_one<DIM, VDIM, 2>(a, tiles, s);
+    else tm_launch_one<DIM, VDIM, 4>(a, tiles, s);
 }
 
 // ---- C ABI ----------------------------------------------------------------------------------------------------------------------
@@ -541,6 +805,20 @@ extern "C" int exl2_talk_attn(const void* q, const void* k_cache, const void* v_
     a.row_list = row_list; a.part_o = part_o; a.part_ml = part_ml; a.nsplit = nsplit;
     const int vn = dtype == 0 ? 8 : 4;
     const bool vec = dim % vn == 0 && vdim % 2 == 0 && ((uintptr_t)k_cache % 16) == 0 && ((uintptr_t)v_cache % 8) == 0;
+    hipStream_t s = (hipStream_t)stream;
+    if (dtype == 0 && vec && row_list && exl2_talk_attn_tiles_supported(heads, dim, vdim) && kv_heads <= 8 && heads / kv_heads <= 16
+        && ((uintptr_t)q % 16) == 0 && ((uintptr_t)v_cache % 16) == 0 && ((uintptr_t)part_o % 16) == 0 && ((uintptr_t)out % 8) == 0)
+    {
+        // listed rows (decoded tokens) at the sizes of the matrix-core form
+        if (dim == 32) td_launch<32, 32>(a, rows, s);
+        else if (dim == 64 && vdim == 64) td_launch<64, 64>(a, rows, s);
+        else if (dim == 64) td_launch<64, 128>(a, rows, s);
+        else if (vdim == 64) td_launch<128, 64>(a, rows, s);
+        else td_launch<128, 128>(a, rows, s);
+        if (nsplit > 1) LAUNCH(talk_attn_merge_kernel<u16>, dim3(rows, heads), dim3(64), 0, stream, a);
+        HIP_TRY(hipGetLastError());
+        return EXL2_OK;
+    }
     static bool attr_done[EXL2_MAX_DEVICES];
     if (exl2_first_on_device(attr_done))
     {

@@ -135,6 +135,7 @@ DEV float fast_rsqrt(float x) { return 1.0f / sqrtf(x); }
 DEV float fast_sin(float x) { return sinf(x); }
 DEV float fast_cos(float x) { return cosf(x); }
 DEV float fast_rcp(float x) { return 1.0f / x; }
+DEV float fast_rcp_approx(float x) { return 1.0f / x; }
 
 template <typename T> DEV void pin_scalar(T&) { }
 template <typename T> DEV void pin_vector(T&) { }
