@@ -44,6 +44,10 @@ template <typename T> DEV void ta_ld2(const T* p, float& a, float& b);
 template <> DEV void ta_ld2<u16>(const u16* p, float& a, float& b) { const u32 v = *(const u32*)p; a = as_f32(v << 16); b = as_f32(v & 0xffff0000u); }
 template <> DEV void ta_ld2<float>(const float* p, float& a, float& b) { const f32x2 v = *(const f32x2*)p; a = v[0]; b = v[1]; }
 
+// the wave's lanes meet around a tile of LDS that only they share: neither the hardware nor the compiler (whose alias analysis sees one
+// lane's own addresses only) moves LDS accesses across it
+DEV void ta_wave_lds() { wave_sync(); wait_lds_reads(); }
+
 #define TA_NEG_BIG (-1.0e30f)
 #define TA_KEYS 64                           // keys per step of the row kernel
 #define TA_MAX_SPLIT 64
@@ -291,7 +295,8 @@ KERNEL void __launch_bounds__(256, 1) talk_attn_decode_kernel(const TalkArgs a)
     float* s_t = s_p + H * TD_STR;                               // [H (head in)][36]: T transposed, head out along the row
     float* s_c = s_t + H * 36;                                   // [H] correction of the step, [H] final maximum, [H] final sum
     u16* s_v = (u16*)(s_c + ((3 * H + 3) & ~3));                 // [4][64][VSTR], 16-byte aligned
-    const int t = tid(), lane = lane_id(), wv = wave_id();
+    const int t = tid(), lane = lane_id();
+    const int wv = uniform(wave_id());                           // (scalar branches around the matrix products: they ignore the lane mask)
     const int qi = lane & 15, g = lane >> 4;
     const int r = a.row_list ? a.row_list[bid_x()] : bid_x();
     const int split = bid_y();
@@ -406,10 +411,10 @@ KERNEL void __launch_bounds__(256, 1) talk_attn_decode_kernel(const TalkArgs a)
         {
             const int kv = wv + 4 * k;
             if (kv >= G) break;
-            wave_sync();
+            ta_wave_lds();
             #pragma unroll
             for (int i = 0; i < VP; i++) *(u32x4*)(my_v + ((lane + 64 * i) / VPR) * VSTR + ((lane + 64 * i) % VPR) * 8) = vreg[k][i];
-            wave_sync();
+            ta_wave_lds();
             const int h = kv * hpg + min(qi, hpg - 1);
             const float alpha = s_c[h];
             u32x4 pb[2];
@@ -535,7 +540,8 @@ KERNEL void __launch_bounds__(64 * TM_NW, 1) talk_attn_tile_kernel(const TalkArg
     float* s_t = s_s + TT::HMAX * TM_Q * SS;                     // [HMAX][TS]: T, zero past H
     u16* s_v = (u16*)(s_t + TT::HMAX * TS);                      // [TM_NW][TM_BK][VSTR]
 
-    const int t = tid(), lane = lane_id(), wv = wave_id();
+    const int t = tid(), lane = lane_id();
+    const int wv = uniform(wave_id());                           // (scalar branches around the matrix products: they ignore the lane mask)
     const int qi = lane & 15, g = lane >> 4;
     const int H = a.H, G = a.G, hpg = H / G;
     const int tile_i = gdim_x() - 1 - bid_x();                   // the longest key lists first
@@ -713,10 +719,10 @@ KERNEL void __launch_bounds__(64 * TM_NW, 1) talk_attn_tile_kernel(const TalkArg
                 if (n0 >= nh) break;
                 if (n0 > 0 && kvh[n0] == kvh[n0 - 1]) continue;
                 if (n0 > 0) load_v(step, kvh[n0]);
-                wave_sync();
+                ta_wave_lds();
                 #pragma unroll
                 for (int i = 0; i < VP; i++) *(u32x4*)(my_v + ((lane + 64 * i) / VPR) * VSTR + ((lane + 64 * i) % VPR) * 8) = vreg[i];
-                wave_sync();
+                ta_wave_lds();
                 const u16* vbase = my_v + (4 * g + (qi >> 2)) * VSTR + 4 * (qi & 3);
                 #pragma unroll
                 for (int d = 0; d < DB; d++)
