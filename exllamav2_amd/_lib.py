@@ -161,7 +161,7 @@ PROTOTYPES = {
     "exl2_mingru_scan": (ci, [vp, vp, vp, ci, vp, ci, vp, vp, vp, ci, vp, vp, vp, ci, ci, vp, ci, ci, vp]),
     "exl2_talk_attn": (ci, [vp, vp, vp, vp, vp, vp, vp, vp, ci, ci, vp, vp, ci, vp, vp, ci, ci, ci, ci, ci, ci, ci, cf, vp]),
     "exl2_talk_attn_tiles_supported": (ci, [ci, ci, ci]),
-    "exl2_talk_attn_tiles": (ci, [vp, vp, vp, vp, vp, vp, vp, vp, ci, ci, vp, vp, vp, ci, ci, ci, ci, ci, ci, cf, vp]),
+    "exl2_talk_attn_tiles": (ci, [vp, vp, vp, vp, vp, vp, vp, vp, ci, ci, vp, vp, vp, ci, vp, vp, ci, ci, ci, ci, ci, ci, cf, vp]),
     # graphs
     "exl2_graph_begin_capture": (ci, [vp]),
     "exl2_graph_end_capture": (ci, [vp, C.POINTER(vp)]),

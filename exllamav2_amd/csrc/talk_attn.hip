@@ -498,100 +498,94 @@ static void td_launch(const TalkArgs& a, int rows, hipStream_t s)
 }
 
 // ---- bfloat16 on the matrix cores: portions of prompts -----------------------------------------------------------------------------
-// Workgroup = one tile of <= 16 consecutive positions of one sequence x ALL heads, eight waves; wave w owns query heads HPW w .. + HPW - 1
-// (their query rows as operands and their output accumulators in registers).  Keys go by 32 at a time in three stages:
-//   1. scores of the wave's heads, S^T = K Q^T (A = key rows straight from the cache: a lane's 8 values are one 16-byte load), capped, to
-//      LDS as fp32 [head][query][key];
-//   2. the exchange: a lane takes one (query, key) for all heads, s_h = sum_g T[h, g] a_g -- on the fp32 matrix cores in their 16-block
-//      form, where every lane's own scalar goes through a 4 x 1 product per (four heads out, one head in) without any lane
-//      movement -- and puts the mixed scores back in place;
-//   3. the wave's heads again: online softmax (columns = queries), probabilities to bfloat16 in registers (the accumulator layout of
-//      S^T is the operand layout of O^T += V^T P^T with the keys of a product taken in the order {4 g .. + 3 of block 0, of block 1}),
-//      values through a wave-private LDS tile and transposing reads.
-// The step's value rows are requested before stage 2, the next step's key rows before stage 3 (they take turns in the same registers);
-// the rows' places in the cache are looked up by one wave a step ahead.  Two barriers per step: stage 1 of the next step writes only
-// what its own wave read in stage 3.
+// Workgroup = one tile of <= 16 consecutive positions of one sequence x 16 output heads x one share of the key steps, eight waves.  Keys
+// go by 32 at a time in three stages (heads in quads of four consecutive ones; HB = 1: up to 16 heads, 2: up to 32, two workgroups):
+//   1. scores of ALL heads, S^T = K Q^T: a wave takes a quad and all 32 keys (HB = 2) or half of them (A = key rows straight from the
+//      cache: a lane's 8 values are one 16-byte load that feeds every head of the quad with the same key / value head), capped, to LDS
+//      as fp32 [head][query][key];
+//   2. the exchange: a lane takes one (query, key), s_h = sum_g T[h, g] a_g -- on the fp32 matrix cores in their 16-block form, where
+//      every lane's own scalar goes through a 4 x 1 product per (four heads out, one head in) without any lane movement -- and puts the
+//      mixed scores of the 16 output heads back in place;
+//   3. the output heads, two waves per quad: online softmax (columns = queries), probabilities to bfloat16 in registers (the accumulator layout of S^T is the
+//      operand layout of O^T += V^T P^T with the keys of a product taken in the order {4 g .. + 3 of block 0, of block 1}); the two waves
+//      take half of the value columns each, through a wave-private LDS tile and transposing reads.
+// The step's value rows are requested before stage 2, the next step's key rows before stage 3; the rows' places in the cache are looked
+// up by one wave a step ahead.
 
 #define TM_Q 16
 #define TM_NW 8
 #define TM_BK 32
+#define TM_MAX_SPLIT 8
 
-template <int DIM, int VDIM, int HPW>
+template <int DIM, int VDIM, int HB>
 struct TalkTile
 {
-    static constexpr int HMAX = TM_NW * HPW, SS = TM_BK + 4, TS = HMAX + 4, VSTR = VDIM + 16;
-    static constexpr size_t smem = sizeof(float) * ((size_t)HMAX * TM_Q * SS + (size_t)HMAX * TS) + sizeof(u16) * (size_t)TM_NW * TM_BK * VSTR;
+    static constexpr int HMAX = 16 * HB, SS = TM_BK + 4, TS = HMAX + 4, VW = VDIM / 2, VSTR = VW + 16;
+    static constexpr size_t smem = sizeof(float) * ((size_t)HMAX * TM_Q * SS + (size_t)16 * TS) + sizeof(u16) * (size_t)TM_NW * TM_BK * VSTR;
 };
 
-template <int DIM, int VDIM, int HPW>
+template <int DIM, int VDIM, int HB>
 KERNEL void __launch_bounds__(64 * TM_NW, 1) talk_attn_tile_kernel(const TalkArgs a)
 {
     DYN_SMEM(smem);
     SHARED int s_row[2][TM_BK];
-    typedef TalkTile<DIM, VDIM, HPW> TT;
-    constexpr int SS = TT::SS, TS = TT::TS, VSTR = TT::VSTR, NBLK = TM_BK / 16, KK = DIM / 32, DB = VDIM / 16;
-    constexpr int VPR = VDIM / 8, VP = TM_BK * VPR / 64;         // 16-byte pieces of a value row; value pieces per lane
-    constexpr int NT = TT::HMAX / 4;                             // groups of four heads out
-    // registers are short where a wave holds four wide heads: its query rows are read again every step (they stay in the caches) and the
-    // next step's key rows are not requested ahead
-    constexpr bool LEAN = HPW * 4 * (KK + DB) > 128;
-    constexpr int QN = LEAN ? 1 : HPW;
+    typedef TalkTile<DIM, VDIM, HB> TT;
+    constexpr int SS = TT::SS, TS = TT::TS, VSTR = TT::VSTR, VW = TT::VW, KB = HB, KK = DIM / 32, DB = VW / 16;
+    constexpr int VPR = VW / 8, VP = TM_BK * VPR / 64;           // 16-byte pieces of a wave's part of a value row; pieces per lane
+    constexpr int NT = 4;                                        // groups of four heads out
     float* s_s = (float*)smem;                                   // [HMAX][TM_Q][SS]
-    float* s_t = s_s + TT::HMAX * TM_Q * SS;                     // [HMAX][TS]: T, zero past H
-    u16* s_v = (u16*)(s_t + TT::HMAX * TS);                      // [TM_NW][TM_BK][VSTR]
+    float* s_t = s_s + TT::HMAX * TM_Q * SS;                     // [16][TS]: T's rows of the output heads, zero past H
+    u16* s_v = (u16*)(s_t + 16 * TS);                            // [TM_NW][TM_BK][VSTR]
 
     const int t = tid(), lane = lane_id();
     const int wv = uniform(wave_id());                           // (scalar branches around the matrix products: they ignore the lane mask)
+    const int og = bid_z() * 16;                                 // first output head of the workgroup
+    const int quad1 = HB == 1 ? wv / 2 : wv, kpart = HB == 1 ? wv % 2 : 0;       // stage 1: quad of heads, first 16-key block
+    const int part = wv % 2;                                     // stage 3: half of the value columns
     const int qi = lane & 15, g = lane >> 4;
     const int H = a.H, G = a.G, hpg = H / G;
-    const int tile_i = gdim_x() - 1 - bid_x();                   // the longest key lists first
+    const int tile_i = gdim_x() - 1 - bid_x(), split = bid_y();  // the longest key lists first
     const int r0 = a.tile_row0[tile_i], n_rows = a.tile_rows[tile_i];
     const int p0 = a.row_pos[r0], p_last = p0 + n_rows - 1;
     const int* bt = a.block_table + (long long)a.row_seq[r0] * a.bt_stride;
     const int j_lo = max(0, p0 - a.window + 1);
     const int total = p_last - j_lo + 1;
-    const int n_steps = (total + TM_BK - 1) / TM_BK;
+    const int all_steps = (total + TM_BK - 1) / TM_BK;
+    const int per_split = (all_steps + a.nsplit - 1) / a.nsplit;
+    const int step0 = split * per_split, step1 = min(all_steps, step0 + per_split);
     const u16* kc = (const u16*)a.k_cache; const u16* vc = (const u16*)a.v_cache;
     u16* my_v = s_v + wv * TM_BK * VSTR;
     const float cap2 = a.softcap > 0.0f ? 2.0f / a.softcap : 0.0f;
 
-    for (int i = t; i < TT::HMAX * TT::HMAX; i += 64 * TM_NW)
-    {
-        const int h = i / TT::HMAX, c = i % TT::HMAX;
-        s_t[h * TS + c] = h < H && c < H ? a.talk[h * H + c] : 0.0f;
-    }
-    if (t < TM_BK) s_row[0][t] = (int)ta_cache_row(a, bt, j_lo + min(t, total - 1));
-    const int nh = max(0, min(HPW, H - HPW * wv));               // heads of this wave
-    const int h0 = min(HPW * wv, H - 1);
-    int kvh[HPW];
+    const int nq = max(0, min(4, H - 4 * quad1)), q0 = min(4 * quad1, H - 1);                        // stage 1: heads of this wave
+    const int nh = max(0, min(4, H - og - 4 * (wv / 2))), h0 = min(og + 4 * (wv / 2), H - 1);        // stage 3
+    int kvq[4], kvh[4];
     #pragma unroll
-    for (int n = 0; n < HPW; n++) kvh[n] = uniform(min(h0 + n, H - 1) / hpg);
+    for (int n = 0; n < 4; n++) { kvq[n] = uniform(min(q0 + n, H - 1) / hpg); kvh[n] = uniform(min(h0 + n, H - 1) / hpg); }
 
     const int qrow = r0 + min(qi, n_rows - 1), qpos = p0 + min(qi, n_rows - 1), q_lo = qpos - a.window + 1;
-    u32x4 qb[QN][KK];
-    auto load_q = [&](int n) {
-        const u16* qp = (const u16*)a.q + ((long long)qrow * H + min(h0 + n, H - 1)) * DIM + 8 * g;
-        #pragma unroll
-        for (int kk = 0; kk < KK; kk++) qb[LEAN ? 0 : n][kk] = *(const u32x4*)(qp + 32 * kk);
-    };
-    f32x4 ot[HPW][DB];
-    float m_run[HPW], l_run[HPW];
+    u32x4 qb[4][KK];
+    f32x4 ot[4][DB];
+    float m_run[4], l_run[4];
+    const bool with_sink = a.sink && split == 0;                 // the sink counts once
     #pragma unroll
-    for (int n = 0; n < HPW; n++)
+    for (int n = 0; n < 4; n++)
     {
         const int h = min(h0 + n, H - 1);
-        if (!LEAN) load_q(n);
+        const u16* qp = (const u16*)a.q + ((long long)qrow * H + min(q0 + n, H - 1)) * DIM + 8 * g;
+        #pragma unroll
+        for (int kk = 0; kk < KK; kk++) qb[n][kk] = *(const u32x4*)(qp + 32 * kk);
         #pragma unroll
         for (int d = 0; d < DB; d++) ot[n][d] = (f32x4){0.0f, 0.0f, 0.0f, 0.0f};
-        m_run[n] = a.sink ? a.sink[h] : TA_NEG_BIG;
-        l_run[n] = a.sink ? 1.0f : 0.0f;
+        m_run[n] = with_sink ? a.sink[h] : TA_NEG_BIG;
+        l_run[n] = with_sink && g == 0 ? 1.0f : 0.0f;            // (a lane's own share: the four lanes of a query add theirs up at the end)
     }
-    u32x4 kf[NBLK][KK], vreg[VP];
+    u32x4 kf[KB][KK], vreg[VP];
     auto load_k = [&](int step, int kv) {
         #pragma unroll
-        for (int b = 0; b < NBLK; b++)
+        for (int b = 0; b < KB; b++)
         {
-            const u16* kp = kc + ((long long)s_row[step & 1][16 * b + qi] * G + kv) * DIM + 8 * g;
+            const u16* kp = kc + ((long long)s_row[step & 1][16 * (kpart + b) + qi] * G + kv) * DIM + 8 * g;
             #pragma unroll
             for (int kk = 0; kk < KK; kk++) kf[b][kk] = *(const u32x4*)(kp + 32 * kk);
         }
@@ -599,30 +593,38 @@ KERNEL void __launch_bounds__(64 * TM_NW, 1) talk_attn_tile_kernel(const TalkArg
     auto load_v = [&](int step, int kv) {
         #pragma unroll
         for (int i = 0; i < VP; i++)
-            vreg[i] = *(const u32x4*)(vc + ((long long)s_row[step & 1][(lane + 64 * i) / VPR] * G + kv) * VDIM + ((lane + 64 * i) % VPR) * 8);
+            vreg[i] = *(const u32x4*)(vc + ((long long)s_row[step & 1][(lane + 64 * i) / VPR] * G + kv) * VDIM + part * VW + ((lane + 64 * i) % VPR) * 8);
     };
-    block_sync();
-    if (nh > 0 && !LEAN) load_k(0, kvh[0]);
+    if (step0 < step1)
+    {
+        for (int i = t; i < 16 * TT::HMAX; i += 64 * TM_NW)
+        {
+            const int h = i / TT::HMAX, c = i % TT::HMAX;
+            s_t[h * TS + c] = og + h < H && c < H ? a.talk[(og + h) * H + c] : 0.0f;
+        }
+        if (t < TM_BK) s_row[step0 & 1][t] = (int)ta_cache_row(a, bt, j_lo + min(step0 * TM_BK + t, total - 1));
+        block_sync();
+        if (nq > 0) load_k(step0, kvq[0]);
+    }
 
-    for (int step = 0; step < n_steps; step++)
+    for (int step = step0; step < step1; step++)
     {
         const int k0 = step * TM_BK;
         int next_row = 0;
         if (t < TM_BK) next_row = (int)ta_cache_row(a, bt, j_lo + min(k0 + TM_BK + t, total - 1));
-        // ---- 1: scores of this wave's heads
+        // ---- 1: scores of the quad's heads
         #pragma unroll
-        for (int n = 0; n < HPW; n++)
+        for (int n = 0; n < 4; n++)
         {
-            if (n >= nh) break;
-            if (n > 0 ? kvh[n] != kvh[n - 1] : LEAN) load_k(step, kvh[n]);
-            if (LEAN) load_q(n);
-            float* sr = s_s + ((h0 + n) * TM_Q + qi) * SS + 4 * g;
+            if (n >= nq) break;
+            if (n > 0 && kvq[n] != kvq[n - 1]) load_k(step, kvq[n]);
+            float* sr = s_s + ((q0 + n) * TM_Q + qi) * SS + 16 * kpart + 4 * g;
             #pragma unroll
-            for (int b = 0; b < NBLK; b++)
+            for (int b = 0; b < KB; b++)
             {
                 f32x4 st = {0.0f, 0.0f, 0.0f, 0.0f};
                 #pragma unroll
-                for (int kk = 0; kk < KK; kk++) st = mfma_16x16x32_bf16(kf[b][kk], qb[LEAN ? 0 : n][kk], st);
+                for (int kk = 0; kk < KK; kk++) st = mfma_16x16x32_bf16(kf[b][kk], qb[n][kk], st);
                 #pragma unroll
                 for (int r = 0; r < 4; r++) st[r] = tm_soft_cap(st[r], a.softcap, cap2);
                 *(f32x4*)(sr + 16 * b) = st;
@@ -638,14 +640,15 @@ KERNEL void __launch_bounds__(64 * TM_NW, 1) talk_attn_tile_kernel(const TalkArg
             f32x4 mx[NT];
             #pragma unroll
             for (int i = 0; i < NT; i++) mx[i] = (f32x4){0.0f, 0.0f, 0.0f, 0.0f};
-            for (int c4 = 0; c4 < H; c4 += 4)
+            #pragma unroll 2
+            for (int c = 0; c < H; c += 4)
             {
                 f32x4 tv[NT];
                 float sv[4];
                 #pragma unroll
-                for (int k = 0; k < 4; k++) sv[k] = sp[min(c4 + k, H - 1) * TM_Q * SS];         // (past the last head T is zero)
+                for (int k = 0; k < 4; k++) sv[k] = sp[min(c + k, H - 1) * TM_Q * SS];          // (past the last head T is zero)
                 #pragma unroll
-                for (int i = 0; i < NT; i++) tv[i] = *(const f32x4*)(s_t + (4 * i + (lane & 3)) * TS + c4);
+                for (int i = 0; i < NT; i++) tv[i] = *(const f32x4*)(s_t + (4 * i + (lane & 3)) * TS + c);
                 #pragma unroll
                 for (int k = 0; k < 4; k++)
                     #pragma unroll
@@ -655,25 +658,26 @@ KERNEL void __launch_bounds__(64 * TM_NW, 1) talk_attn_tile_kernel(const TalkArg
             for (int i = 0; i < NT; i++)
                 #pragma unroll
                 for (int r = 0; r < 4; r++)
-                    if (4 * i + r < H) sp[(4 * i + r) * TM_Q * SS] = mx[i][r];
+                    if (4 * i + r < H - og) sp[(4 * i + r) * TM_Q * SS] = mx[i][r];
         }
         block_sync_lds();
-        // ---- 3: softmax and values of this wave's heads
+        // ---- 3: softmax and values of the quad's heads
+        if (nq > 0 && step + 1 < step1) load_k(step + 1, kvq[0]);
         if (nh > 0)
         {
-            u32x4 pb[HPW];
-            float alpha[HPW];
+            u32x4 pb[4];
+            float alpha[4];
             bool moved = false;
             #pragma unroll
-            for (int n = 0; n < HPW; n++)
+            for (int n = 0; n < 4; n++)
             {
                 alpha[n] = 1.0f;
                 if (n >= nh) break;
-                const float* sr = s_s + ((h0 + n) * TM_Q + qi) * SS + 4 * g;
+                const float* sr = s_s + ((h0 - og + n) * TM_Q + qi) * SS + 4 * g;
                 float sc[8];
                 float m_loc = TA_NEG_BIG;
                 #pragma unroll
-                for (int b = 0; b < NBLK; b++)
+                for (int b = 0; b < 2; b++)
                 {
                     const f32x4 v = *(const f32x4*)(sr + 16 * b);
                     #pragma unroll
@@ -698,15 +702,13 @@ KERNEL void __launch_bounds__(64 * TM_NW, 1) talk_attn_tile_kernel(const TalkArg
                     p_sum += pa + pc;
                     pb[n][e2] = tm_pack2(pa, pc);
                 }
-                p_sum += shfl_xor_f32(p_sum, 16);
-                p_sum += shfl_xor_f32(p_sum, 32);
                 l_run[n] = l_run[n] * alpha[n] + p_sum;
                 m_run[n] = m_new;
             }
             if (wave_ballot(moved) != 0ull)                      // the running maxima rarely move once a few steps have gone by
             {
                 #pragma unroll
-                for (int n = 0; n < HPW; n++)
+                for (int n = 0; n < 4; n++)
                     #pragma unroll
                     for (int d = 0; d < DB; d++)
                         #pragma unroll
@@ -714,7 +716,7 @@ KERNEL void __launch_bounds__(64 * TM_NW, 1) talk_attn_tile_kernel(const TalkArg
             }
             // runs of heads that read the same key / value head: its values once through LDS, every fragment feeds all of the run
             #pragma unroll
-            for (int n0 = 0; n0 < HPW; n0++)
+            for (int n0 = 0; n0 < 4; n0++)
             {
                 if (n0 >= nh) break;
                 if (n0 > 0 && kvh[n0] == kvh[n0 - 1]) continue;
@@ -731,42 +733,95 @@ KERNEL void __launch_bounds__(64 * TM_NW, 1) talk_attn_tile_kernel(const TalkArg
                     const f16x4 hi = lds_read_tr16_b64((const f16*)(vbase + 16 * VSTR + 16 * d));
                     const u32x2 l2 = __builtin_bit_cast(u32x2, lo), h2 = __builtin_bit_cast(u32x2, hi);
                     #pragma unroll
-                    for (int n = n0; n < HPW; n++)
+                    for (int n = n0; n < 4; n++)
                         if (n < nh && kvh[n] == kvh[n0]) ot[n][d] = mfma_16x16x32_bf16((u32x4){l2[0], l2[1], h2[0], h2[1]}, pb[n], ot[n][d]);
                 }
             }
-            if (!LEAN && step + 1 < n_steps) load_k(step + 1, kvh[0]);
         }
+        block_sync_lds();                                        // stage 1 of the next step overwrites the scores
     }
 
+    #pragma unroll
+    for (int n = 0; n < 4; n++)
+    {
+        l_run[n] += shfl_xor_f32(l_run[n], 16);
+        l_run[n] += shfl_xor_f32(l_run[n], 32);
+    }
     if (qi >= n_rows) return;
     #pragma unroll
-    for (int n = 0; n < HPW; n++)
+    for (int n = 0; n < 4; n++)
     {
         if (n >= nh) break;
+        if (a.nsplit > 1)
+        {
+            const long long pi = ((long long)qrow * H + h0 + n) * a.nsplit + split;
+            float* po = a.part_o + pi * VDIM + part * VW + 4 * g;
+            #pragma unroll
+            for (int d = 0; d < DB; d++) *(f32x4*)(po + 16 * d) = ot[n][d];
+            if (part == 0 && g == 0) { a.part_ml[pi * 2] = m_run[n]; a.part_ml[pi * 2 + 1] = l_run[n]; }
+            continue;
+        }
         const float inv = l_run[n] > 0.0f ? 1.0f / l_run[n] : 0.0f;
-        u16* op = (u16*)a.out + ((long long)qrow * H + h0 + n) * VDIM + 4 * g;
+        u16* op = (u16*)a.out + ((long long)qrow * H + h0 + n) * VDIM + part * VW + 4 * g;
         #pragma unroll
         for (int d = 0; d < DB; d++)
             *(u32x2*)(op + 16 * d) = (u32x2){tm_pack2(ot[n][d][0] * inv, ot[n][d][1] * inv), tm_pack2(ot[n][d][2] * inv, ot[n][d][3] * inv)};
     }
 }
 
-template <int DIM, int VDIM, int HPW>
+// grid (tiles, heads): joins the key splits of a tile's rows; thread = (row, four values)
+KERNEL void __launch_bounds__(256) talk_attn_tile_merge_kernel(const TalkArgs a)
+{
+    const int r0 = a.tile_row0[bid_x()], n_rows = a.tile_rows[bid_x()], h = bid_y(), per = a.vdim / 4;
+    for (int i = tid(); i < n_rows * per; i += 256)
+    {
+        const int row = r0 + i / per, e = (i % per) * 4;
+        const long long p0 = ((long long)row * a.H + h) * a.nsplit;
+        float m[TM_MAX_SPLIT], l[TM_MAX_SPLIT];
+        f32x4 o[TM_MAX_SPLIT];
+        float mx = TA_NEG_BIG;
+        #pragma unroll
+        for (int s = 0; s < TM_MAX_SPLIT; s++)
+        {
+            const long long p = p0 + min(s, a.nsplit - 1);
+            m[s] = a.part_ml[p * 2];
+            l[s] = a.part_ml[p * 2 + 1];
+            o[s] = *(const f32x4*)(a.part_o + p * a.vdim + e);
+        }
+        #pragma unroll
+        for (int s = 0; s < TM_MAX_SPLIT; s++) mx = fmaxf(mx, m[s]);
+        float lsum = 0.0f;
+        f32x4 acc = {0.0f, 0.0f, 0.0f, 0.0f};
+        #pragma unroll
+        for (int s = 0; s < TM_MAX_SPLIT; s++)
+        {
+            if (s >= a.nsplit || m[s] <= 0.5f * TA_NEG_BIG) continue;
+            const float c = fast_exp(m[s] - mx);
+            lsum = fmaf(l[s], c, lsum);
+            #pragma unroll
+            for (int k = 0; k < 4; k++) acc[k] = fmaf(o[s][k], c, acc[k]);
+        }
+        const float inv = lsum > 0.0f ? 1.0f / lsum : 0.0f;
+        *(u32x2*)((u16*)a.out + ((long long)row * a.H + h) * a.vdim + e) = (u32x2){tm_pack2(acc[0] * inv, acc[1] * inv), tm_pack2(acc[2] * inv, acc[3] * inv)};
+    }
+}
+
+template <int DIM, int VDIM, int HB>
 static void tm_launch_one(const TalkArgs& a, int tiles, hipStream_t s)
 {
     static bool attr_done[EXL2_MAX_DEVICES];
-    static_assert(TalkTile<DIM, VDIM, HPW>::smem <= 159 * 1024, "the tile fits the LDS");
+    static_assert(TalkTile<DIM, VDIM, HB>::smem <= 159 * 1024, "the tile fits the LDS");
     if (exl2_first_on_device(attr_done))
-        (void)hipFuncSetAttribute((const void*)talk_attn_tile_kernel<DIM, VDIM, HPW>, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024 - 1024);
-    LAUNCH((talk_attn_tile_kernel<DIM, VDIM, HPW>), dim3(tiles), dim3(64 * TM_NW), (TalkTile<DIM, VDIM, HPW>::smem), s, a);
+        (void)hipFuncSetAttribute((const void*)talk_attn_tile_kernel<DIM, VDIM, HB>, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024 - 1024);
+    LAUNCH((talk_attn_tile_kernel<DIM, VDIM, HB>), dim3(tiles, a.nsplit, HB), dim3(64 * TM_NW), (TalkTile<DIM, VDIM, HB>::smem), s, a);
+    if (a.nsplit > 1) LAUNCH(talk_attn_tile_merge_kernel, dim3(tiles, a.H), dim3(256), 0, s, a);
 }
 
 template <int DIM, int VDIM>
 static void tm_launch(const TalkArgs& a, int tiles, hipStream_t s)
 {
-    if (a.H <= 2 * TM_NW) tm_launch_one<DIM, VDIM, 2>(a, tiles, s);
-    else tm_launch_one<DIM, VDIM, 4>(a, tiles, s);
+    if (a.H <= 16) tm_launch_one<DIM, VDIM, 1>(a, tiles, s);
+    else tm_launch_one<DIM, VDIM, 2>(a, tiles, s);
 }
 
 // ---- C ABI ----------------------------------------------------------------------------------------------------------------------
@@ -852,8 +907,8 @@ extern "C" int exl2_talk_attn(const void* q, const void* k_cache, const void* v_
 
 extern "C" int exl2_talk_attn_tiles(const void* q, const void* k_cache, const void* v_cache, const float* talk, const float* sink,
                                     const int* row_seq, const int* row_pos, const int* block_table, int bt_stride, int page, void* out,
-                                    const int* tile_row0, const int* tile_rows, int tiles, int heads, int kv_heads, int dim, int vdim,
-                                    int window, float softcap, void* stream)
+                                    const int* tile_row0, const int* tile_rows, int tiles, float* part_o, float* part_ml, int nsplit,
+                                    int heads, int kv_heads, int dim, int vdim, int window, float softcap, void* stream)
 {
     TalkArgs a;
     const int rc = ta_fill(a, q, k_cache, v_cache, talk, sink, row_seq, row_pos, block_table, bt_stride, page, out, heads, kv_heads, dim,
@@ -862,8 +917,10 @@ extern "C" int exl2_talk_attn_tiles(const void* q, const void* k_cache, const vo
     EXL2_REQUIRE(tile_row0 && tile_rows, "talk_attn_tiles: tiles missing");
     if (!exl2_talk_attn_tiles_supported(heads, dim, vdim))
         EXL2_FAIL(EXL2_E_UNSUPPORTED, "talk_attn_tiles: %d heads of %d / %d values outside the matrix-core form", heads, dim, vdim);
+    EXL2_REQUIRE(nsplit >= 1 && nsplit <= TM_MAX_SPLIT && (nsplit == 1 || (part_o && part_ml && ((uintptr_t)part_o % 16) == 0)),
+                 "talk_attn_tiles: key splits (1 .. %d) need scratch", TM_MAX_SPLIT);
     if (tiles <= 0) return EXL2_OK;
-    a.tile_row0 = tile_row0; a.tile_rows = tile_rows;
+    a.tile_row0 = tile_row0; a.tile_rows = tile_rows; a.part_o = part_o; a.part_ml = part_ml; a.nsplit = nsplit;
     hipStream_t s = (hipStream_t)stream;
     if (dim == 32) tm_launch<32, 32>(a, tiles, s);
     else if (dim == 64 && vdim == 64) tm_launch<64, 64>(a, tiles, s);

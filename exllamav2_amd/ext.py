@@ -1215,7 +1215,7 @@ class ExtC:
         return dtype is torch.bfloat16 and bool(self.lib.exl2_talk_attn_tiles_supported(int(heads), int(dim), int(vdim)))
 
     def talk_attn_tiles(self, q, k_cache, v_cache, talk, sink, row_seq, row_pos, block_table, page: int, out, tiles, heads: int, kv_heads: int,
-                        dim: int, vdim: int, window: int, softcap: float) -> None:
+                        dim: int, vdim: int, window: int, softcap: float, nsplit: int = 1, part_o=None, part_ml=None) -> None:
         """tiles = (tile_row0 int32 [n], tile_rows int32 [n], n): runs of <= 16 consecutive positions of one sequence"""
         row0, nrows, n = tiles
         bf = torch.bfloat16
@@ -1223,8 +1223,9 @@ class ExtC:
             self._ptr(q, bf, "q"), self._ptr(k_cache, bf, "k_cache"), self._ptr(v_cache, bf, "v_cache"), self._ptr(talk, torch.float32, "talk"),
             self._ptr(sink, torch.float32, "sink"), self._ptr(row_seq, torch.int32, "row_seq"), self._ptr(row_pos, torch.int32, "row_pos"),
             self._ptr(block_table, torch.int32, "block_table"), block_table.shape[-1], int(page), self._ptr(out, bf, "out"),
-            self._ptr(row0, torch.int32, "tile_row0"), self._ptr(nrows, torch.int32, "tile_rows"), int(n), int(heads), int(kv_heads), int(dim),
-            int(vdim), int(window), float(softcap), self._stream(out)))
+            self._ptr(row0, torch.int32, "tile_row0"), self._ptr(nrows, torch.int32, "tile_rows"), int(n), self._ptr(part_o, torch.float32, "part_o"),
+            self._ptr(part_ml, torch.float32, "part_ml"), int(nsplit), int(heads), int(kv_heads), int(dim), int(vdim), int(window), float(softcap),
+            self._stream(out)))
 
     def graph_begin_capture(self, stream: int | None) -> None:
         self.lib.check(self.lib.exl2_graph_begin_capture(stream))

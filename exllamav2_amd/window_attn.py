@@ -67,6 +67,7 @@ def rotary_tables(base: float, dims: int, scaling: dict | None, device):
 
 
 class WindowAttention:
+    TILE_SPLIT, TILE_WORKGROUPS = 8, 512                      # head mixing, prompts: most workgroups that share a tile's keys; workgroups aimed at
     MAX_SPLIT = 16                                            # decoded tokens: workgroups that share one row's key list
 
     def __init__(self, model, key: str, layer_idx: int, *, heads: int, kv_heads: int, dim: int, vdim: int, window: int, pool: int,
@@ -222,20 +223,25 @@ class WindowAttention:
     def _talk(self, q, st, batch, page, o, rows: int) -> None:
         """attention with the heads' score exchange: portions of prompts as tiles of 16 positions x all heads on the matrix cores where the
         sizes allow, decoded tokens (and every other shape) one row per workgroup with the keys split over workgroups"""
-        ext, m, f32 = self.ext, self.model, torch.float32
-        H, vd = self.heads, self.vdim
+        ext, H, vd = self.ext, self.heads, self.vdim
         common = (q, st.k, st.v, self.talk_w, self.sink, batch.row_seq, batch.row_pos, batch.block_table, page, o)
         shape = (H, self.kv_heads, self.dim, vd, self.window, self.softcap)
         if batch.tiles16 is not None and not self.talk_tiles:
             ext.talk_attn(*common, None, rows, *shape)
             return
         if batch.tiles16 is not None:
-            ext.talk_attn_tiles(*common, batch.tiles16, *shape)
+            # few tiles fill the chip only when several workgroups share one's keys (at least four steps of 32 keys each)
+            tiles = batch.tiles16[2]
+            longest = max((s[3] + s[1] for s in batch.spans), default=1) if batch.spans is not None else 1
+            nsplit = max(1, min(self.TILE_SPLIT, -(-self.TILE_WORKGROUPS // tiles), min(self.window + 15, longest) // 128))
+            ext.talk_attn_tiles(*common, batch.tiles16, *shape, nsplit=nsplit, **self._parts(rows, nsplit))
         if batch.tiles1 is not None:
             row0, n, max_pos = batch.tiles1
             nsplit = max(1, min(self.MAX_SPLIT, -(-min(self.window, max_pos + 1) // 64)))
-            part_o = part_ml = None
-            if nsplit > 1:
-                part_o = m.buf("attn.part_o", (rows, H, nsplit, vd), f32)
-                part_ml = m.buf("attn.part_ml", (rows, H, nsplit, 2), f32)
-            ext.talk_attn(*common, row0, n, *shape, nsplit=nsplit, part_o=part_o, part_ml=part_ml)
+            ext.talk_attn(*common, row0, n, *shape, nsplit=nsplit, **self._parts(rows, nsplit))
+
+    def _parts(self, rows: int, nsplit: int) -> dict:
+        if nsplit == 1:
+            return {}
+        return dict(part_o=self.model.buf("attn.part_o", (rows, self.heads, nsplit, self.vdim), torch.float32),
+                    part_ml=self.model.buf("attn.part_ml", (rows, self.heads, nsplit, 2), torch.float32))

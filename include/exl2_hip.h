@@ -682,12 +682,12 @@ int exl2_talk_attn(const void* q, const void* k_cache, const void* v_cache, cons
                    const int* row_list, int rows, float* part_o, float* part_ml, int nsplit, int dtype, int heads, int kv_heads,
                    int dim, int vdim, int window, float softcap, void* stream);
 /* the same for portions of prompts on the matrix cores (bfloat16): tile i = rows tile_row0[i] .. + tile_rows[i], <= 16 consecutive positions
-   of ONE sequence.  Sizes: exl2_talk_attn_tiles_supported. */
+   of ONE sequence; nsplit (<= 8) and its scratch as above.  Sizes: exl2_talk_attn_tiles_supported. */
 int exl2_talk_attn_tiles_supported(int heads, int dim, int vdim);
 int exl2_talk_attn_tiles(const void* q, const void* k_cache, const void* v_cache, const float* talk, const float* sink,
                          const int* row_seq, const int* row_pos, const int* block_table, int bt_stride, int page, void* out,
-                         const int* tile_row0, const int* tile_rows, int tiles, int heads, int kv_heads, int dim, int vdim,
-                         int window, float softcap, void* stream);
+                         const int* tile_row0, const int* tile_rows, int tiles, float* part_o, float* part_ml, int nsplit,
+                         int heads, int kv_heads, int dim, int vdim, int window, float softcap, void* stream);
 
 #ifdef __cplusplus
 }

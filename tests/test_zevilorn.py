@@ -296,10 +296,13 @@ def test_head_mixing_attention(be, dtype, heads, kv_heads, dim, vdim, window, ca
     if be.ext.talk_attn_tiles_supported(dtype, heads, dim, vdim):
         base = rows - sum(n for *_x, n in tiles)
         row0 = base + np.cumsum([0] + [n for *_x, n in tiles[:-1]])
-        out = torch.full((rows, heads * vdim), 3.0, dtype=dtype, device=be.device)
-        be.ext.talk_attn_tiles(*args, out, (ints(be, row0), ints(be, [n for *_x, n in tiles]), len(tiles)), *shape)
-        got = be.n(out.float())
-        assert close(got[base:], want[base:], 1e-2) and (got[:base] == 3.0).all()
+        for nsplit in (1, 2, 5):
+            out = torch.full((rows, heads * vdim), 3.0, dtype=dtype, device=be.device)
+            part = dict(part_o=torch.full((rows, heads, nsplit, vdim), float("nan"), dtype=F32, device=be.device),
+                        part_ml=torch.full((rows, heads, nsplit, 2), float("nan"), dtype=F32, device=be.device)) if nsplit > 1 else {}
+            be.ext.talk_attn_tiles(*args, out, (ints(be, row0), ints(be, [n for *_x, n in tiles]), len(tiles)), *shape, nsplit=nsplit, **part)
+            got = be.n(out.float())
+            assert close(got[base:], want[base:], 1e-2) and (got[:base] == 3.0).all(), nsplit
 
 
 @pytest.mark.parametrize("dtype,heads,R,rot,rot_dims,halves,sink", [
