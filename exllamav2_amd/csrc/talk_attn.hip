@@ -270,31 +270,32 @@ DEV u32 tm_pack2(float lo, float hi) { return (u32)f32_to_bf16(lo) | ((u32)f32_t
 extern "C" int exl2_talk_attn_tiles_supported(int heads, int dim, int vdim);
 
 // ---- bfloat16 on the matrix cores: decoded tokens -----------------------------------------------------------------------------------
-// Workgroup = one row x all heads x one share of the keys, 64 keys at a time: wave w scores keys 16 w .. + 15 for one key / value head
-// after the other (A = key rows from the cache, B = the query heads that share them), the scores go to LDS as [head][key]; a wave then
-// takes HQ heads with a key per lane, mixes (T in LDS, transposed, read as broadcasts), joins the running softmax with lane
-// exchanges and leaves the probabilities in LDS; last a wave takes key / value heads w, w + 4, .. and adds V^T P^T (values through a
-// wave-private LDS tile and transposing reads).  Keys and values of a step are all requested before its first product.
+// Workgroup = one row x all heads x one share of the keys, 64 keys at a time, NW = 4 or 8 waves (up to 4 NW heads and NW key / value
+// heads): wave w scores keys 16 (w % 4) .. + 15 for four key / value heads (A = key rows from the cache, B = the query heads that share
+// them), the scores go to LDS as [head][key]; a wave then takes four heads with a key per lane, mixes (T in LDS, transposed, read as
+// broadcasts), joins the running softmax with lane exchanges and leaves the probabilities in LDS; last wave w adds V^T P^T of
+// key / value head w (values through a wave-private LDS tile, 32 keys at a time, and transposing reads).  Keys and values of a step are
+// all requested before its first product.
 
 #define TD_STR 68                            // floats between two heads' scores
 
-template <int VDIM> HD size_t td_smem(int H)
+template <int VDIM, int NW> HD size_t td_smem(int H)
 {
-    return sizeof(float) * ((size_t)2 * H * TD_STR + (size_t)H * 36 + ((3 * (size_t)H + 3) & ~(size_t)3)) + sizeof(u16) * (size_t)4 * 64 * (VDIM + 16);
+    return sizeof(float) * ((size_t)2 * H * TD_STR + (size_t)H * 36 + ((3 * (size_t)H + 3) & ~(size_t)3)) + sizeof(u16) * (size_t)NW * 32 * (VDIM + 16);
 }
 
-template <int DIM, int VDIM, int KVW>
-KERNEL void __launch_bounds__(256, 1) talk_attn_decode_kernel(const TalkArgs a)
+template <int DIM, int VDIM, int NW>
+KERNEL void __launch_bounds__(64 * NW, 1) talk_attn_decode_kernel(const TalkArgs a)
 {
     DYN_SMEM(smem);
     SHARED long long s_row[64];
-    constexpr int KK = DIM / 32, DB = VDIM / 16, VSTR = VDIM + 16, VPR = VDIM / 8, VP = 64 * VPR / 64, HQ = 4 * KVW;
+    constexpr int KK = DIM / 32, DB = VDIM / 16, VSTR = VDIM + 16, VPR = VDIM / 8, VP = 64 * VPR / 64, HQ = 4;
     const int H = a.H, G = a.G, hpg = H / G;
     float* s_a = (float*)smem;                                   // [H][TD_STR] capped scores
     float* s_p = s_a + H * TD_STR;                               // [H][TD_STR] probabilities
     float* s_t = s_p + H * TD_STR;                               // [H (head in)][36]: T transposed, head out along the row
     float* s_c = s_t + H * 36;                                   // [H] correction of the step, [H] final maximum, [H] final sum
-    u16* s_v = (u16*)(s_c + ((3 * H + 3) & ~3));                 // [4][64][VSTR], 16-byte aligned
+    u16* s_v = (u16*)(s_c + ((3 * H + 3) & ~3));                 // [NW][32][VSTR], 16-byte aligned
     const int t = tid(), lane = lane_id();
     const int wv = uniform(wave_id());                           // (scalar branches around the matrix products: they ignore the lane mask)
     const int qi = lane & 15, g = lane >> 4;
@@ -308,8 +309,8 @@ KERNEL void __launch_bounds__(256, 1) talk_attn_decode_kernel(const TalkArgs a)
     const int per_split = (all_steps + a.nsplit - 1) / a.nsplit;
     const int step0 = split * per_split, step1 = min(all_steps, step0 + per_split);
     const u16* kc = (const u16*)a.k_cache; const u16* vc = (const u16*)a.v_cache;
-    u16* my_v = s_v + wv * 64 * VSTR;
-    for (int i = t; i < H * 36; i += 256)
+    u16* my_v = s_v + wv * 32 * VSTR;
+    for (int i = t; i < H * 36; i += 64 * NW)
     {
         const int in = i / 36, out = i % 36;
         s_t[i] = out < H ? a.talk[out * H + in] : 0.0f;
@@ -324,11 +325,9 @@ KERNEL void __launch_bounds__(256, 1) talk_attn_decode_kernel(const TalkArgs a)
         m_run[i] = with_sink ? a.sink[h] : TA_NEG_BIG;
         l_run[i] = with_sink ? 1.0f : 0.0f;
     }
-    f32x4 ot[KVW][DB];
+    f32x4 ot[DB];
     #pragma unroll
-    for (int k = 0; k < KVW; k++)
-        #pragma unroll
-        for (int d = 0; d < DB; d++) ot[k][d] = (f32x4){0.0f, 0.0f, 0.0f, 0.0f};
+    for (int d = 0; d < DB; d++) ot[d] = (f32x4){0.0f, 0.0f, 0.0f, 0.0f};
     const float cap2 = a.softcap > 0.0f ? 2.0f / a.softcap : 0.0f;
 
     for (int step = step0; step < step1; step++)
@@ -336,11 +335,11 @@ KERNEL void __launch_bounds__(256, 1) talk_attn_decode_kernel(const TalkArgs a)
         const int k0 = step * 64, nc = min(64, total - k0);
         if (t < 64) s_row[t] = ta_cache_row(a, bt, j_lo + k0 + min(t, nc - 1));
         block_sync();                                            // (also: everybody is done with the previous step)
-        const long long krow = s_row[16 * wv + qi];
-        u32x4 vreg[KVW][VP];
+        const long long krow = s_row[16 * (wv % 4) + qi];
+        u32x4 vreg[VP];
         // ---- scores: four key / value heads' rows in flight
-        for (int g0 = 0; g0 < G; g0 += 4)
         {
+            const int g0 = 4 * (wv / 4);
             u32x4 kf[4][KK], qf[4][KK];
             #pragma unroll
             for (int k = 0; k < 4; k++)
@@ -351,14 +350,9 @@ KERNEL void __launch_bounds__(256, 1) talk_attn_decode_kernel(const TalkArgs a)
                 #pragma unroll
                 for (int kk = 0; kk < KK; kk++) { kf[k][kk] = *(const u32x4*)(kp + 32 * kk); qf[k][kk] = *(const u32x4*)(qp + 32 * kk); }
             }
-            if (g0 == 0)
-            {
-                #pragma unroll
-                for (int k = 0; k < KVW; k++)
-                    #pragma unroll
-                    for (int i = 0; i < VP; i++)
-                        vreg[k][i] = *(const u32x4*)(vc + (s_row[(lane + 64 * i) / VPR] * G + min(wv + 4 * k, G - 1)) * VDIM + ((lane + 64 * i) % VPR) * 8);
-            }
+            #pragma unroll
+            for (int i = 0; i < VP; i++)
+                vreg[i] = *(const u32x4*)(vc + (s_row[(lane + 64 * i) / VPR] * G + min(wv, G - 1)) * VDIM + ((lane + 64 * i) % VPR) * 8);
             #pragma unroll
             for (int k = 0; k < 4; k++)
             {
@@ -368,7 +362,7 @@ KERNEL void __launch_bounds__(256, 1) talk_attn_decode_kernel(const TalkArgs a)
                 for (int kk = 0; kk < KK; kk++) st = mfma_16x16x32_bf16(kf[k][kk], qf[k][kk], st);
                 #pragma unroll
                 for (int e = 0; e < 4; e++) st[e] = tm_soft_cap(st[e], a.softcap, cap2);
-                if (qi < hpg) *(f32x4*)(s_a + ((g0 + k) * hpg + qi) * TD_STR + 16 * wv + 4 * g) = st;
+                if (qi < hpg) *(f32x4*)(s_a + ((g0 + k) * hpg + qi) * TD_STR + 16 * (wv % 4) + 4 * g) = st;
             }
         }
         block_sync_lds();
@@ -405,39 +399,33 @@ KERNEL void __launch_bounds__(256, 1) talk_attn_decode_kernel(const TalkArgs a)
             }
         }
         block_sync_lds();
-        // ---- values: this wave's key / value heads
-        #pragma unroll
-        for (int k = 0; k < KVW; k++)
+        // ---- values: this wave's key / value head
+        if (wv < G)
         {
-            const int kv = wv + 4 * k;
-            if (kv >= G) break;
-            ta_wave_lds();
-            #pragma unroll
-            for (int i = 0; i < VP; i++) *(u32x4*)(my_v + ((lane + 64 * i) / VPR) * VSTR + ((lane + 64 * i) % VPR) * 8) = vreg[k][i];
-            ta_wave_lds();
-            const int h = kv * hpg + min(qi, hpg - 1);
+            const int h = wv * hpg + min(qi, hpg - 1);
             const float alpha = s_c[h];
-            u32x4 pb[2];
-            #pragma unroll
-            for (int b = 0; b < 4; b++)
-            {
-                const f32x4 p = *(const f32x4*)(s_p + h * TD_STR + 16 * b + 4 * g);
-                pb[b / 2][2 * (b % 2)] = tm_pack2(p[0], p[1]);
-                pb[b / 2][2 * (b % 2) + 1] = tm_pack2(p[2], p[3]);
-            }
-            const u16* vbase = my_v + (4 * g + (qi >> 2)) * VSTR + 4 * (qi & 3);
             #pragma unroll
             for (int d = 0; d < DB; d++)
+                #pragma unroll
+                for (int e = 0; e < 4; e++) ot[d][e] *= alpha;
+            const u16* vbase = my_v + (4 * g + (qi >> 2)) * VSTR + 4 * (qi & 3);
+            #pragma unroll
+            for (int m2 = 0; m2 < 2; m2++)
             {
+                ta_wave_lds();
                 #pragma unroll
-                for (int e = 0; e < 4; e++) ot[k][d][e] *= alpha;
+                for (int i = 0; i < VP / 2; i++)
+                    *(u32x4*)(my_v + ((lane + 64 * i) / VPR) * VSTR + ((lane + 64 * i) % VPR) * 8) = vreg[m2 * (VP / 2) + i];
+                ta_wave_lds();
+                const f32x4 pa = *(const f32x4*)(s_p + h * TD_STR + 32 * m2 + 4 * g), pc = *(const f32x4*)(s_p + h * TD_STR + 32 * m2 + 16 + 4 * g);
+                const u32x4 pb = {tm_pack2(pa[0], pa[1]), tm_pack2(pa[2], pa[3]), tm_pack2(pc[0], pc[1]), tm_pack2(pc[2], pc[3])};
                 #pragma unroll
-                for (int m2 = 0; m2 < 2; m2++)
+                for (int d = 0; d < DB; d++)
                 {
-                    const f16x4 lo = lds_read_tr16_b64((const f16*)(vbase + (32 * m2) * VSTR + 16 * d));
-                    const f16x4 hi = lds_read_tr16_b64((const f16*)(vbase + (32 * m2 + 16) * VSTR + 16 * d));
+                    const f16x4 lo = lds_read_tr16_b64((const f16*)(vbase + 16 * d));
+                    const f16x4 hi = lds_read_tr16_b64((const f16*)(vbase + 16 * VSTR + 16 * d));
                     const u32x2 l2 = __builtin_bit_cast(u32x2, lo), h2 = __builtin_bit_cast(u32x2, hi);
-                    ot[k][d] = mfma_16x16x32_bf16((u32x4){l2[0], l2[1], h2[0], h2[1]}, pb[m2], ot[k][d]);
+                    ot[d] = mfma_16x16x32_bf16((u32x4){l2[0], l2[1], h2[0], h2[1]}, pb, ot[d]);
                 }
             }
         }
@@ -458,43 +446,38 @@ KERNEL void __launch_bounds__(256, 1) talk_attn_decode_kernel(const TalkArgs a)
         }
     }
     block_sync();
-    #pragma unroll
-    for (int k = 0; k < KVW; k++)
+    if (wv >= G || qi >= hpg) return;
+    const int h = wv * hpg + qi;
+    if (a.nsplit > 1)
     {
-        const int kv = wv + 4 * k;
-        if (kv >= G || qi >= hpg) continue;
-        const int h = kv * hpg + qi;
-        if (a.nsplit > 1)
-        {
-            float* po = a.part_o + (((long long)r * H + h) * a.nsplit + split) * VDIM + 4 * g;
-            #pragma unroll
-            for (int d = 0; d < DB; d++) *(f32x4*)(po + 16 * d) = ot[k][d];
-        }
-        else
-        {
-            const float l = s_c[2 * H + h], inv = l > 0.0f ? 1.0f / l : 0.0f;
-            u16* op = (u16*)a.out + ((long long)r * H + h) * VDIM + 4 * g;
-            #pragma unroll
-            for (int d = 0; d < DB; d++)
-                *(u32x2*)(op + 16 * d) = (u32x2){tm_pack2(ot[k][d][0] * inv, ot[k][d][1] * inv), tm_pack2(ot[k][d][2] * inv, ot[k][d][3] * inv)};
-        }
+        float* po = a.part_o + (((long long)r * H + h) * a.nsplit + split) * VDIM + 4 * g;
+        #pragma unroll
+        for (int d = 0; d < DB; d++) *(f32x4*)(po + 16 * d) = ot[d];
+    }
+    else
+    {
+        const float l = s_c[2 * H + h], inv = l > 0.0f ? 1.0f / l : 0.0f;
+        u16* op = (u16*)a.out + ((long long)r * H + h) * VDIM + 4 * g;
+        #pragma unroll
+        for (int d = 0; d < DB; d++)
+            *(u32x2*)(op + 16 * d) = (u32x2){tm_pack2(ot[d][0] * inv, ot[d][1] * inv), tm_pack2(ot[d][2] * inv, ot[d][3] * inv)};
     }
 }
 
-template <int DIM, int VDIM, int KVW>
+template <int DIM, int VDIM, int NW>
 static void td_launch_one(const TalkArgs& a, int rows, hipStream_t s)
 {
     static bool attr_done[EXL2_MAX_DEVICES];
     if (exl2_first_on_device(attr_done))
-        (void)hipFuncSetAttribute((const void*)talk_attn_decode_kernel<DIM, VDIM, KVW>, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024 - 1024);
-    LAUNCH((talk_attn_decode_kernel<DIM, VDIM, KVW>), dim3(rows, a.nsplit), dim3(256), td_smem<VDIM>(a.H), s, a);
+        (void)hipFuncSetAttribute((const void*)talk_attn_decode_kernel<DIM, VDIM, NW>, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024 - 1024);
+    LAUNCH((talk_attn_decode_kernel<DIM, VDIM, NW>), dim3(rows, a.nsplit), dim3(64 * NW), (td_smem<VDIM, NW>(a.H)), s, a);
 }
 
 template <int DIM, int VDIM>
 static void td_launch(const TalkArgs& a, int rows, hipStream_t s)
 {
-    if (a.H <= 16 && a.G <= 4) td_launch_one<DIM, VDIM, 1>(a, rows, s);
-    else td_launch_one<DIM, VDIM, 2>(a, rows, s);
+    if (a.H <= 16 && a.G <= 4) td_launch_one<DIM, VDIM, 4>(a, rows, s);
+    else td_launch_one<DIM, VDIM, 8>(a, rows, s);
 }
 
 // ---- bfloat16 on the matrix cores: portions of prompts -----------------------------------------------------------------------------
