@@ -310,11 +310,11 @@ KERNEL void __launch_bounds__(64 * NW, 1) talk_attn_decode_kernel(const TalkArgs
     const int step0 = split * per_split, step1 = min(all_steps, step0 + per_split);
     const u16* kc = (const u16*)a.k_cache; const u16* vc = (const u16*)a.v_cache;
     u16* my_v = s_v + wv * 32 * VSTR;
-    for (int i = t; i < H * 36; i += 64 * NW)
-    {
-        const int in = i / 36, out = i % 36;
-        s_t[i] = out < H ? a.talk[out * H + in] : 0.0f;
-    }
+    // T is requested first and put down behind the look-ups of the first step's rows (which take longer)
+    constexpr int TL = (16 * NW * NW + 64 * NW - 1) / (64 * NW);
+    float tv0[TL];
+    #pragma unroll
+    for (int i = 0; i < TL; i++) tv0[i] = a.talk[min(t + i * 64 * NW, H * H - 1)];
     // this wave's heads in the mixing stage: HQ wv .. + HQ - 1 (uniform over the lanes)
     float m_run[HQ], l_run[HQ];
     const bool with_sink = a.sink && split == 0;                 // the sink counts once
@@ -333,9 +333,18 @@ KERNEL void __launch_bounds__(64 * NW, 1) talk_attn_decode_kernel(const TalkArgs
     for (int step = step0; step < step1; step++)
     {
         const int k0 = step * 64, nc = min(64, total - k0);
+        const long long krow = ta_cache_row(a, bt, j_lo + k0 + min(16 * (wv % 4) + qi, nc - 1));
         if (t < 64) s_row[t] = ta_cache_row(a, bt, j_lo + k0 + min(t, nc - 1));
+        if (step == step0)
+        {
+            #pragma unroll
+            for (int i = 0; i < TL; i++)
+            {
+                const int at = t + i * 64 * NW;
+                if (at < H * H) s_t[(at % H) * 36 + at / H] = tv0[i];
+            }
+        }
         block_sync();                                            // (also: everybody is done with the previous step)
-        const long long krow = s_row[16 * (wv % 4) + qi];
         u32x4 vreg[VP];
         // ---- scores: four key / value heads' rows in flight
         {
@@ -372,6 +381,7 @@ KERNEL void __launch_bounds__(64 * NW, 1) talk_attn_decode_kernel(const TalkArgs
             float mx[HQ];
             #pragma unroll
             for (int i = 0; i < HQ; i++) mx[i] = 0.0f;
+            #pragma unroll 8
             for (int c = 0; c < H; c++)
             {
                 const float sv = s_a[c * TD_STR + lane];
