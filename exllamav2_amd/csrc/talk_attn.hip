@@ -270,32 +270,40 @@ DEV u32 tm_pack2(float lo, float hi) { return (u32)f32_to_bf16(lo) | ((u32)f32_t
 extern "C" int exl2_talk_attn_tiles_supported(int heads, int dim, int vdim);
 
 // ---- bfloat16 on the matrix cores: decoded tokens -----------------------------------------------------------------------------------
-// Workgroup = one row x all heads x one share of the keys, 64 keys at a time, NW = 4 or 8 waves (up to 4 NW heads and NW key / value
-// heads): wave w scores keys 16 (w % 4) .. + 15 for four key / value heads (A = key rows from the cache, B = the query heads that share
-// them), the scores go to LDS as [head][key]; a wave then takes four heads with a key per lane, mixes (T in LDS, transposed, read as
-// broadcasts), joins the running softmax with lane exchanges and leaves the probabilities in LDS; last wave w adds V^T P^T of
-// key / value head w (values through a wave-private LDS tile, 32 keys at a time, and transposing reads).  Keys and values of a step are
-// all requested before its first product.
+// Workgroup = one row x all heads x one share of the keys, 32 keys at a time (one workgroup draws only so much from memory at once: few
+// keys each, many workgroups), eight waves, up to 16 GPW heads over up to 4 GPW key / value heads.  Wave w scores keys 16 (w % 2) .. + 15
+// for GPW key / value heads (A = key rows from the cache, B = the query heads that share them), the scores go to LDS as [head][key];
+// then a half of a wave takes GPW heads with a key per lane: it mixes (T in LDS, transposed, read as broadcasts), joins the running
+// softmax with lane exchanges and leaves the probabilities in LDS; last wave w adds V^T P^T of key / value head w (values through a
+// wave-private LDS tile and transposing reads).  Keys and values of a step are all requested before its first product.
 
-#define TD_STR 68                            // floats between two heads' scores
+#define TD_NW 8
+#define TD_BK 32
+#define TD_STR 36                            // floats between two heads' scores
+#define TD_TS 36                             // floats between two rows of T
 
-template <int VDIM, int NW> HD size_t td_smem(int H)
+// H <= 16 GPW heads, G <= 4 GPW key / value heads
+template <int VDIM> HD size_t td_smem(int H)
 {
-    return sizeof(float) * ((size_t)2 * H * TD_STR + (size_t)H * 36 + ((3 * (size_t)H + 3) & ~(size_t)3)) + sizeof(u16) * (size_t)NW * 32 * (VDIM + 16);
+    return sizeof(float) * ((size_t)2 * H * TD_STR + (size_t)H * TD_TS + ((3 * (size_t)H + 3) & ~(size_t)3)) + sizeof(u16) * (size_t)TD_NW * TD_BK * (VDIM + 16);
 }
 
-template <int DIM, int VDIM, int NW>
-KERNEL void __launch_bounds__(64 * NW, 1) talk_attn_decode_kernel(const TalkArgs a)
+DEV float td_half_max(float v) { v = row16_allreduce_max(v); return fmaxf(v, shfl_xor_f32(v, 16)); }
+DEV float td_half_sum(float v) { v = row16_allreduce_add(v); return v + shfl_xor_f32(v, 16); }
+
+template <int DIM, int VDIM, int GPW>
+KERNEL void __launch_bounds__(64 * TD_NW, 1) talk_attn_decode_kernel(const TalkArgs a)
 {
     DYN_SMEM(smem);
-    SHARED long long s_row[64];
-    constexpr int KK = DIM / 32, DB = VDIM / 16, VSTR = VDIM + 16, VPR = VDIM / 8, VP = 64 * VPR / 64, HQ = 4;
+    SHARED long long s_row[TD_BK];
+    constexpr int KK = DIM / 32, DB = VDIM / 16, VSTR = VDIM + 16, VPR = VDIM / 8, VP = TD_BK * VPR / 64;
+    constexpr int HQ = GPW;                                      // heads per half of a wave
     const int H = a.H, G = a.G, hpg = H / G;
     float* s_a = (float*)smem;                                   // [H][TD_STR] capped scores
     float* s_p = s_a + H * TD_STR;                               // [H][TD_STR] probabilities
-    float* s_t = s_p + H * TD_STR;                               // [H (head in)][36]: T transposed, head out along the row
-    float* s_c = s_t + H * 36;                                   // [H] correction of the step, [H] final maximum, [H] final sum
-    u16* s_v = (u16*)(s_c + ((3 * H + 3) & ~3));                 // [NW][32][VSTR], 16-byte aligned
+    float* s_t = s_p + H * TD_STR;                               // [H (head in)][TD_TS]: T transposed, head out along the row
+    float* s_c = s_t + H * TD_TS;                                // [H] correction of the step, [H] final maximum, [H] final sum
+    u16* s_v = (u16*)(s_c + ((3 * H + 3) & ~3));                 // [TD_NW][TD_BK][VSTR], 16-byte aligned
     const int t = tid(), lane = lane_id();
     const int wv = uniform(wave_id());                           // (scalar branches around the matrix products: they ignore the lane mask)
     const int qi = lane & 15, g = lane >> 4;
@@ -305,24 +313,24 @@ KERNEL void __launch_bounds__(64 * NW, 1) talk_attn_decode_kernel(const TalkArgs
     const int* bt = a.block_table + (long long)a.row_seq[r] * a.bt_stride;
     const int j_lo = max(0, pos - a.window + 1);
     const int total = pos - j_lo + 1;
-    const int all_steps = (total + 63) / 64;
+    const int all_steps = (total + TD_BK - 1) / TD_BK;
     const int per_split = (all_steps + a.nsplit - 1) / a.nsplit;
     const int step0 = split * per_split, step1 = min(all_steps, step0 + per_split);
     const u16* kc = (const u16*)a.k_cache; const u16* vc = (const u16*)a.v_cache;
-    u16* my_v = s_v + wv * 32 * VSTR;
+    u16* my_v = s_v + wv * TD_BK * VSTR;
     // T is requested first and put down behind the look-ups of the first step's rows (which take longer)
-    constexpr int TL = (16 * NW * NW + 64 * NW - 1) / (64 * NW);
+    constexpr int TL = (16 * GPW * 16 * GPW + 64 * TD_NW - 1) / (64 * TD_NW);
     float tv0[TL];
     #pragma unroll
-    for (int i = 0; i < TL; i++) tv0[i] = a.talk[min(t + i * 64 * NW, H * H - 1)];
-    // this wave's heads in the mixing stage: HQ wv .. + HQ - 1 (uniform over the lanes)
+    for (int i = 0; i < TL; i++) tv0[i] = a.talk[min(t + i * 64 * TD_NW, H * H - 1)];
+    // the heads of this half wave in the mixing stage: hm .. + HQ - 1, key = lane % 32
+    const int hm = (2 * wv + lane / 32) * HQ, key = lane % 32;
     float m_run[HQ], l_run[HQ];
     const bool with_sink = a.sink && split == 0;                 // the sink counts once
     #pragma unroll
     for (int i = 0; i < HQ; i++)
     {
-        const int h = min(wv * HQ + i, H - 1);
-        m_run[i] = with_sink ? a.sink[h] : TA_NEG_BIG;
+        m_run[i] = with_sink ? a.sink[min(hm + i, H - 1)] : TA_NEG_BIG;
         l_run[i] = with_sink ? 1.0f : 0.0f;
     }
     f32x4 ot[DB];
@@ -332,51 +340,48 @@ KERNEL void __launch_bounds__(64 * NW, 1) talk_attn_decode_kernel(const TalkArgs
 
     for (int step = step0; step < step1; step++)
     {
-        const int k0 = step * 64, nc = min(64, total - k0);
-        const long long krow = ta_cache_row(a, bt, j_lo + k0 + min(16 * (wv % 4) + qi, nc - 1));
-        if (t < 64) s_row[t] = ta_cache_row(a, bt, j_lo + k0 + min(t, nc - 1));
+        const int k0 = step * TD_BK, nc = min(TD_BK, total - k0);
+        const long long krow = ta_cache_row(a, bt, j_lo + k0 + min(16 * (wv % 2) + qi, nc - 1));
+        if (t < TD_BK) s_row[t] = ta_cache_row(a, bt, j_lo + k0 + min(t, nc - 1));
         if (step == step0)
         {
             #pragma unroll
             for (int i = 0; i < TL; i++)
             {
-                const int at = t + i * 64 * NW;
-                if (at < H * H) s_t[(at % H) * 36 + at / H] = tv0[i];
+                const int at = t + i * 64 * TD_NW;
+                if (at < H * H) s_t[(at % H) * TD_TS + at / H] = tv0[i];
             }
         }
-        block_sync();                                            // (also: everybody is done with the previous step)
-        u32x4 vreg[VP];
-        // ---- scores: four key / value heads' rows in flight
+        u32x4 kf[GPW][KK], qf[GPW][KK], vreg[VP];
+        const int g0 = (wv / 2) * GPW;
+        #pragma unroll
+        for (int k = 0; k < GPW; k++)
         {
-            const int g0 = 4 * (wv / 4);
-            u32x4 kf[4][KK], qf[4][KK];
+            const int kv = min(g0 + k, G - 1);
+            const u16* kp = kc + (krow * G + kv) * DIM + 8 * g;
+            const u16* qp = (const u16*)a.q + ((long long)r * H + kv * hpg + min(qi, hpg - 1)) * DIM + 8 * g;
             #pragma unroll
-            for (int k = 0; k < 4; k++)
-            {
-                const int kv = min(g0 + k, G - 1);
-                const u16* kp = kc + (krow * G + kv) * DIM + 8 * g;
-                const u16* qp = (const u16*)a.q + ((long long)r * H + kv * hpg + min(qi, hpg - 1)) * DIM + 8 * g;
-                #pragma unroll
-                for (int kk = 0; kk < KK; kk++) { kf[k][kk] = *(const u32x4*)(kp + 32 * kk); qf[k][kk] = *(const u32x4*)(qp + 32 * kk); }
-            }
+            for (int kk = 0; kk < KK; kk++) { kf[k][kk] = *(const u32x4*)(kp + 32 * kk); qf[k][kk] = *(const u32x4*)(qp + 32 * kk); }
+        }
+        block_sync();                                            // (also: everybody is done with the previous step)
+        #pragma unroll
+        for (int i = 0; i < VP; i++)
+            vreg[i] = *(const u32x4*)(vc + (s_row[(lane + 64 * i) / VPR] * G + min(wv, G - 1)) * VDIM + ((lane + 64 * i) % VPR) * 8);
+        // ---- scores
+        #pragma unroll
+        for (int k = 0; k < GPW; k++)
+        {
+            if (g0 + k >= G) break;
+            f32x4 st = {0.0f, 0.0f, 0.0f, 0.0f};
             #pragma unroll
-            for (int i = 0; i < VP; i++)
-                vreg[i] = *(const u32x4*)(vc + (s_row[(lane + 64 * i) / VPR] * G + min(wv, G - 1)) * VDIM + ((lane + 64 * i) % VPR) * 8);
+            for (int kk = 0; kk < KK; kk++) st = mfma_16x16x32_bf16(kf[k][kk], qf[k][kk], st);
             #pragma unroll
-            for (int k = 0; k < 4; k++)
-            {
-                if (g0 + k >= G) break;
-                f32x4 st = {0.0f, 0.0f, 0.0f, 0.0f};
-                #pragma unroll
-                for (int kk = 0; kk < KK; kk++) st = mfma_16x16x32_bf16(kf[k][kk], qf[k][kk], st);
-                #pragma unroll
-                for (int e = 0; e < 4; e++) st[e] = tm_soft_cap(st[e], a.softcap, cap2);
-                if (qi < hpg) *(f32x4*)(s_a + ((g0 + k) * hpg + qi) * TD_STR + 16 * (wv % 4) + 4 * g) = st;
-            }
+            for (int e = 0; e < 4; e++) st[e] = tm_soft_cap(st[e], a.softcap, cap2);
+            if (qi < hpg) *(f32x4*)(s_a + ((g0 + k) * hpg + qi) * TD_STR + 16 * (wv % 2) + 4 * g) = st;
         }
         block_sync_lds();
         // ---- the exchange between the heads and the softmax: lane = key
-        if (wv * HQ < H)
+        if (2 * wv * HQ < H)
         {
             float mx[HQ];
             #pragma unroll
@@ -384,28 +389,24 @@ KERNEL void __launch_bounds__(64 * NW, 1) talk_attn_decode_kernel(const TalkArgs
             #pragma unroll 8
             for (int c = 0; c < H; c++)
             {
-                const float sv = s_a[c * TD_STR + lane];
+                const float sv = s_a[c * TD_STR + key];
                 #pragma unroll
-                for (int i4 = 0; i4 < HQ; i4 += 4)
-                {
-                    const f32x4 tv = *(const f32x4*)(s_t + c * 36 + wv * HQ + i4);
-                    #pragma unroll
-                    for (int e = 0; e < 4; e++) mx[i4 + e] = fmaf(tv[e], sv, mx[i4 + e]);
-                }
+                for (int i = 0; i < HQ; i++) mx[i] = fmaf(s_t[c * TD_TS + hm + i], sv, mx[i]);       // (columns past H are never used)
             }
             #pragma unroll
             for (int i = 0; i < HQ; i++)
             {
-                const int h = wv * HQ + i;
-                if (h >= H) break;
-                const float s = lane < nc ? mx[i] : TA_NEG_BIG;
-                const float m_new = fmaxf(m_run[i], wave_allreduce_max(s));
-                const float p = lane < nc ? fast_exp(s - m_new) : 0.0f;
+                const float s = key < nc ? mx[i] : TA_NEG_BIG;
+                const float m_new = fmaxf(m_run[i], td_half_max(s));
+                const float p = key < nc ? fast_exp(s - m_new) : 0.0f;
                 const float c = fast_exp(m_run[i] - m_new);
-                l_run[i] = l_run[i] * c + wave_allreduce_add(p);
+                l_run[i] = l_run[i] * c + td_half_sum(p);
                 m_run[i] = m_new;
-                s_p[h * TD_STR + lane] = p;
-                if (lane == 0) s_c[h] = c;
+                if (hm + i < H)
+                {
+                    s_p[(hm + i) * TD_STR + key] = p;
+                    if (key == 0) s_c[hm + i] = c;
+                }
             }
         }
         block_sync_lds();
@@ -414,37 +415,30 @@ KERNEL void __launch_bounds__(64 * NW, 1) talk_attn_decode_kernel(const TalkArgs
         {
             const int h = wv * hpg + min(qi, hpg - 1);
             const float alpha = s_c[h];
+            ta_wave_lds();
+            #pragma unroll
+            for (int i = 0; i < VP; i++) *(u32x4*)(my_v + ((lane + 64 * i) / VPR) * VSTR + ((lane + 64 * i) % VPR) * 8) = vreg[i];
+            ta_wave_lds();
+            const u16* vbase = my_v + (4 * g + (qi >> 2)) * VSTR + 4 * (qi & 3);
+            const f32x4 pa = *(const f32x4*)(s_p + h * TD_STR + 4 * g), pc = *(const f32x4*)(s_p + h * TD_STR + 16 + 4 * g);
+            const u32x4 pb = {tm_pack2(pa[0], pa[1]), tm_pack2(pa[2], pa[3]), tm_pack2(pc[0], pc[1]), tm_pack2(pc[2], pc[3])};
             #pragma unroll
             for (int d = 0; d < DB; d++)
+            {
                 #pragma unroll
                 for (int e = 0; e < 4; e++) ot[d][e] *= alpha;
-            const u16* vbase = my_v + (4 * g + (qi >> 2)) * VSTR + 4 * (qi & 3);
-            #pragma unroll
-            for (int m2 = 0; m2 < 2; m2++)
-            {
-                ta_wave_lds();
-                #pragma unroll
-                for (int i = 0; i < VP / 2; i++)
-                    *(u32x4*)(my_v + ((lane + 64 * i) / VPR) * VSTR + ((lane + 64 * i) % VPR) * 8) = vreg[m2 * (VP / 2) + i];
-                ta_wave_lds();
-                const f32x4 pa = *(const f32x4*)(s_p + h * TD_STR + 32 * m2 + 4 * g), pc = *(const f32x4*)(s_p + h * TD_STR + 32 * m2 + 16 + 4 * g);
-                const u32x4 pb = {tm_pack2(pa[0], pa[1]), tm_pack2(pa[2], pa[3]), tm_pack2(pc[0], pc[1]), tm_pack2(pc[2], pc[3])};
-                #pragma unroll
-                for (int d = 0; d < DB; d++)
-                {
-                    const f16x4 lo = lds_read_tr16_b64((const f16*)(vbase + 16 * d));
-                    const f16x4 hi = lds_read_tr16_b64((const f16*)(vbase + 16 * VSTR + 16 * d));
-                    const u32x2 l2 = __builtin_bit_cast(u32x2, lo), h2 = __builtin_bit_cast(u32x2, hi);
-                    ot[d] = mfma_16x16x32_bf16((u32x4){l2[0], l2[1], h2[0], h2[1]}, pb, ot[d]);
-                }
+                const f16x4 lo = lds_read_tr16_b64((const f16*)(vbase + 16 * d));
+                const f16x4 hi = lds_read_tr16_b64((const f16*)(vbase + 16 * VSTR + 16 * d));
+                const u32x2 l2 = __builtin_bit_cast(u32x2, lo), h2 = __builtin_bit_cast(u32x2, hi);
+                ot[d] = mfma_16x16x32_bf16((u32x4){l2[0], l2[1], h2[0], h2[1]}, pb, ot[d]);
             }
         }
     }
     #pragma unroll
     for (int i = 0; i < HQ; i++)
     {
-        const int h = wv * HQ + i;
-        if (h < H && lane == 0)
+        const int h = hm + i;
+        if (h < H && key == 0)
         {
             s_c[H + h] = m_run[i];
             s_c[2 * H + h] = l_run[i];
@@ -474,20 +468,20 @@ KERNEL void __launch_bounds__(64 * NW, 1) talk_attn_decode_kernel(const TalkArgs
     }
 }
 
-template <int DIM, int VDIM, int NW>
+template <int DIM, int VDIM, int GPW>
 static void td_launch_one(const TalkArgs& a, int rows, hipStream_t s)
 {
     static bool attr_done[EXL2_MAX_DEVICES];
     if (exl2_first_on_device(attr_done))
-        (void)hipFuncSetAttribute((const void*)talk_attn_decode_kernel<DIM, VDIM, NW>, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024 - 1024);
-    LAUNCH((talk_attn_decode_kernel<DIM, VDIM, NW>), dim3(rows, a.nsplit), dim3(64 * NW), (td_smem<VDIM, NW>(a.H)), s, a);
+        (void)hipFuncSetAttribute((const void*)talk_attn_decode_kernel<DIM, VDIM, GPW>, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024 - 1024);
+    LAUNCH((talk_attn_decode_kernel<DIM, VDIM, GPW>), dim3(rows, a.nsplit), dim3(64 * TD_NW), td_smem<VDIM>(a.H), s, a);
 }
 
 template <int DIM, int VDIM>
 static void td_launch(const TalkArgs& a, int rows, hipStream_t s)
 {
-    if (a.H <= 16 && a.G <= 4) td_launch_one<DIM, VDIM, 4>(a, rows, s);
-    else td_launch_one<DIM, VDIM, 8>(a, rows, s);
+    if (a.H <= 16 && a.G <= 4) td_launch_one<DIM, VDIM, 1>(a, rows, s);
+    else td_launch_one<DIM, VDIM, 2>(a, rows, s);
 }
 
 // ---- bfloat16 on the matrix cores: portions of prompts -----------------------------------------------------------------------------
@@ -633,7 +627,6 @@ KERNEL void __launch_bounds__(64 * TM_NW, 1) talk_attn_tile_kernel(const TalkArg
             f32x4 mx[NT];
             #pragma unroll
             for (int i = 0; i < NT; i++) mx[i] = (f32x4){0.0f, 0.0f, 0.0f, 0.0f};
-            #pragma unroll 2
             for (int c = 0; c < H; c += 4)
             {
                 f32x4 tv[NT];

@@ -237,7 +237,7 @@ class WindowAttention:
             ext.talk_attn_tiles(*common, batch.tiles16, *shape, nsplit=nsplit, **self._parts(rows, nsplit))
         if batch.tiles1 is not None:
             row0, n, max_pos = batch.tiles1
-            nsplit = max(1, min(self.MAX_SPLIT, -(-min(self.window, max_pos + 1) // 64)))
+            nsplit = max(1, min(2 * self.MAX_SPLIT, -(-min(self.window, max_pos + 1) // 32)))
             ext.talk_attn(*common, row0, n, *shape, nsplit=nsplit, **self._parts(rows, nsplit))
 
     def _parts(self, rows: int, nsplit: int) -> dict:
