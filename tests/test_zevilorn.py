@@ -440,3 +440,405 @@ def test_whole_prompt(be, name, dtype):
     eng = make_engine(be, cfg, W, dtype, 32)
     got = run_cuts(be, eng, "a", toks, [23])
     assert ok(got, want, dtype), pos_errs(got, want)
+
+
+def test_residual_stream_after_every_layer_run(be):
+    """the oracle's stream behind the last layer of a stack against the model's, for stacks of one layer up to all of them, gone through
+    once, twice and three times"""
+    cfg = CONFIGS["mixed"]()
+    cfg["loop"] = {"start": 0, "stop": 5, "times": 1}
+    W = OZ.random_model(cfg, seed=31)
+    toks = [int(t) for t in np.random.default_rng(32).integers(0, cfg["vocab"], size=9)]
+    for times in (1, 2, 3):
+        for depth in range(1, 6):
+            sub = dict(cfg, layers=cfg["layers"][:depth], loop={"start": 0, "stop": depth, "times": times})
+            trail = []
+            OZ.Oracle(sub, W).feed("a", toks, residuals=trail)
+            Ws = dict(W)
+            Ws["final.norm"] = np.ones(cfg["width"], dtype=np.float32)
+            Ws["head"] = np.concatenate([np.eye(cfg["width"], dtype=np.float32),
+                                         np.zeros((cfg["vocab"] - cfg["width"], cfg["width"]), dtype=np.float32)])      # logits = the normed stream
+            eng = make_engine(be, sub, Ws, F32, 16)
+            got = run_cuts(be, eng, "a", toks, [9])[:, :cfg["width"]]
+            want = np.array([OZ.rms_norm(trail[t][-1], np.ones(cfg["width"]), cfg["norm"]["eps"]) for t in range(9)])
+            assert close(got, want, 2e-5), (times, depth)
+
+
+@pytest.mark.parametrize("loop", [None, (0, 1, 1), (0, 3, 2), (2, 3, 4), (1, 2, 3), (1, 1, 2)])
+def test_loops_anywhere(be, loop):
+    """no loop, one pass, the whole stack, the last layer only, one layer in the middle, an empty run: whole prompt and decoding"""
+    cfg = CONFIGS["mixed"]()
+    cfg["layers"] = cfg["layers"][:3]
+    cfg["loop"] = {"start": loop[0], "stop": loop[1], "times": loop[2]} if loop else None
+    W = OZ.random_model(cfg, seed=33)
+    toks = list(np.random.default_rng(34).integers(0, cfg["vocab"], size=17))
+    want = OZ.Oracle(cfg, W).feed("a", toks)
+    for cuts in ([17], [6, 2, 3] + [1] * 6):
+        assert rel_err(run_cuts(be, make_engine(be, cfg, W, F32, 20), "a", toks, cuts), want) <= TOL[F32], cuts
+
+
+@pytest.mark.parametrize("name", sorted(CONFIGS))
+def test_decoding_and_portions(be, name):
+    """the same positions through a whole prompt, token by token from the first token on (the convolutions' tails, every pass's keys and
+    the recurrent states pass over decoded tokens), and in portions down to two tokens that end inside pages"""
+    cfg = CONFIGS[name]()
+    W = OZ.random_model(cfg, seed=3)
+    toks = list(np.random.default_rng(4).integers(0, cfg["vocab"], size=26))
+    want = OZ.Oracle(cfg, W).feed("a", toks)
+    for cuts in ([1] * 26, [2, 3, 2, 5, 2, 1, 1, 4, 2, 2, 2], [9] + [1] * 17, [25, 1], [1, 25]):
+        eng = make_engine(be, cfg, W, F32, 28, page=4)
+        assert rel_err(run_cuts(be, eng, "a", toks, cuts), want) <= TOL[F32], cuts
+
+
+def test_mixed_batches_reuse_pages_and_slots(be):
+    """five unequal requests over four slots and a pool smaller than their sum: portions beside single tokens, a request left out of
+    a step, finished requests' pages and slot (with its tails, every pass's keys and its recurrent state) taken by the next; every
+    position equals the request alone"""
+    cfg = CONFIGS["mixed"]()
+    W = OZ.random_model(cfg, seed=5)
+    rng = np.random.default_rng(6)
+    reqs = {r: list(rng.integers(0, cfg["vocab"], size=n)) for r, n in (("a", 13), ("b", 5), ("c", 9), ("d", 2), ("e", 11))}
+    oracle = OZ.Oracle(cfg, W)
+    want = {r: oracle.feed(r, t) for r, t in reqs.items()}
+    eng = make_engine(be, cfg, W, F32, max_tokens=32, page=4, max_seqs=4)
+    plan = [[("a", 5), ("b", 2)], [("a", 1), ("b", 3), ("c", 4), ("d", 2)], [("a", 2), ("c", 1)], [("c", 2), ("e", 3), ("a", 1)],
+            [("a", 4), ("e", 2), ("c", 2)], [("e", 1)], [("e", 5)]]
+    at, got = {r: 0 for r in reqs}, {r: [] for r in reqs}
+    for step in plan:
+        entries, end = [], []
+        for r, n in step:
+            entries.append((r, reqs[r][at[r]:at[r] + n], list(range(n))))
+            at[r] += n
+            if at[r] == len(reqs[r]):
+                end.append(r)
+        lg = be.n(eng.step(entries, end))
+        k = 0
+        for r, n in step:
+            got[r].append(lg[k:k + n])
+            k += n
+    assert all(at[r] == len(reqs[r]) for r in reqs)
+    assert len(eng.pool.free_pages) == eng.pool.num_pages and len(eng.pool.free_slots) == 4
+    assert sum(-(-len(t) // 4) for t in reqs.values()) > eng.pool.num_pages            # pages were used again
+    for r in reqs:
+        assert rel_err(np.concatenate(got[r], 0), want[r]) <= TOL[F32], r
+
+
+def test_a_reused_slot_starts_from_zeros(be):
+    """one slot, three requests one after the other: the second and third find the first one's tails, recurrent state and cached
+    keys of every pass in their slot and pages and must not see them"""
+    cfg = CONFIGS["mixed"]()
+    W = OZ.random_model(cfg, seed=15)
+    rng = np.random.default_rng(16)
+    eng = make_engine(be, cfg, W, F32, max_tokens=16, page=4, max_seqs=1)
+    for r, n, cuts in (("a", 14, [14]), ("b", 9, [1, 1, 7]), ("c", 12, [2, 10])):
+        toks = list(rng.integers(0, cfg["vocab"], size=n))
+        want = OZ.Oracle(cfg, W).feed(r, toks)
+        assert rel_err(run_cuts(be, eng, r, toks, cuts), want) <= TOL[F32], r
+        eng.finish(r)
+
+
+def drive(be, eng, reqs, plan):
+    """plan: steps of [(request, first, last + 1)] with the requests that end after them; returns logits per request in token order"""
+    got = {r: {} for r in reqs}
+    for parts, end in plan:
+        lg = be.n(eng.step([(r, reqs[r][lo:hi], list(range(hi - lo))) for r, lo, hi in parts], end))
+        k = 0
+        for r, lo, hi in parts:
+            for p in range(lo, hi):
+                got[r][p] = lg[k]; k += 1
+    return {r: np.stack([got[r][p] for p in range(len(reqs[r]))]) for r in reqs}
+
+
+@pytest.mark.parametrize("dtype", [F32, BF16])
+def test_decode_steps_as_graphs(be, dtype):
+    """decoding steps through the engine's persistent-input path (on a GPU: captured once per batch size and replayed; every replay
+    is checked): two requests decode side by side, one ends, the other goes on alone, a third joins"""
+    cfg = CONFIGS["mixed"]()
+    W = OZ.random_model(cfg, seed=21)
+    reqs = {r: clear_tokens(cfg, W, n, 22 + i, gap=0.01) for i, (r, n) in enumerate((("a", 14), ("b", 9), ("c", 8)))}
+    oracle = OZ.Oracle(cfg, W)
+    want = {r: oracle.feed(r, t) for r, t in reqs.items()}
+    eng = make_engine(be, cfg, W, dtype, max_tokens=48, page=4, graphs=True)
+    plan = [([("a", 0, 3), ("b", 0, 2)], [])] + [([("a", 3 + i, 4 + i), ("b", 2 + i, 3 + i)], []) for i in range(6)] + [([("b", 8, 9)], ["b"])]
+    plan += [([("a", 9 + i, 10 + i)], []) for i in range(3)] + [([("c", 0, 4)], [])]
+    plan += [([("c", 4 + i, 5 + i), ("a", 12 + i, 13 + i)], []) for i in range(2)] + [([("c", 6, 8)], ["c", "a"])]
+    got = drive(be, eng, reqs, plan)
+    for r in reqs:
+        assert ok(got[r], want[r], dtype), (r, pos_errs(got[r], want[r]))
+    eng.close()
+
+
+def test_matrix_core_sizes_in_portions_and_decoding_bf16(be):
+    """head sizes of the tile kernels: a prompt of many tiles that crosses page borders and passes every window, then decoding, beside a
+    second request"""
+    cfg = CONFIGS["wide"]()
+    W = OZ.random_model(cfg, seed=41)
+    reqs = {"a": clear_tokens(cfg, W, 12, 42, gap=0.006), "b": clear_tokens(cfg, W, 160, 43, gap=0.006)}
+    oracle = OZ.Oracle(cfg, W)
+    want = {r: oracle.feed(r, t) for r, t in reqs.items()}
+    eng = make_engine(be, cfg, W, BF16, max_tokens=256, page=16, graphs=True)
+    plan = [([("a", i, i + 1)], []) for i in range(5)] + [([("b", 0, 139), ("a", 5, 6)], [])]
+    plan += [([("a", i, i + 1), ("b", 133 + i, 134 + i)], []) for i in range(6, 12)] + [([("b", 145, 160)], [])]
+    got = drive(be, eng, reqs, plan)
+    for r in reqs:
+        assert ok(got[r], want[r], BF16), (r, pos_errs(got[r], want[r]))
+    eng.close()
+
+
+def test_head_sizes_of_a_real_model_bf16_and_f32(be):
+    """sizes at which every tuned kernel path is taken (head-mixing tiles of 128 with 16 and more heads and with split keys, the matrix-core
+    decode kernel, latent tiles of 128 + 64, window tiles of 128, the chunked recurrence, the vector residual step, grouped expert
+    launches): a prompt in portions, then decoding, beside a second request"""
+    if be.is_emu:
+        pytest.skip("minutes on the CPU twin; the small configurations cover its logic")
+    moe = dict(experts=8, top=2, ff=64, count=4, keep=2)
+    cfg = OZ.small_config([
+        OZ.layer(OZ.talking_mixer(heads=16, kv_heads=4, dim=128, vdim=128, dims=128, window=1000, conv=4, softcap=20.0, base=500000.0,
+                                  scaling={"factor": 8.0, "low": 1.0, "high": 4.0, "original": 2048}), OZ.moe_ff_spec(**moe)),
+        OZ.layer(OZ.latent_mixer(heads=8, dim=64, rot_dim=64, vdim=64, kv_rank=128, q_rank=96), OZ.moe_ff_spec(**moe)),
+        OZ.layer(OZ.talking_mixer(heads=24, kv_heads=8, dim=64, vdim=64, dims=32, window=90, conv=3, softcap=20.0), None),
+        OZ.layer(OZ.parallel_mixer(OZ.window_spec(heads=4, kv_heads=2, dim=128, vdim=128, dims=64, window=100, base=500000.0), width=256), OZ.moe_ff_spec(**moe))],
+        width=256, vocab=300, loop=(1, 3, 2))
+    W = OZ.random_model(cfg, seed=61)
+    reqs = {"a": clear_tokens(cfg, W, 420, 62, gap=0.003), "b": clear_tokens(cfg, W, 20, 63, gap=0.003)}
+    oracle = OZ.Oracle(cfg, W)
+    want = {r: oracle.feed(r, t) for r, t in reqs.items()}
+    plan = [([("a", 0, 70)], []), ([("a", 70, 405), ("b", 0, 9)], []), ([("a", 405, 407), ("b", 9, 10)], [])]
+    plan += [([("a", 407 + i, 408 + i), ("b", 10 + i, 11 + i)], []) for i in range(10)] + [([("a", 417, 420)], [])]
+    for dtype in (F32, BF16):
+        eng = make_engine(be, cfg, W, dtype, max_tokens=1024, page=64, graphs=True)
+        got = drive(be, eng, reqs, plan)
+        for r in reqs:
+            assert ok(got[r], want[r], dtype), (r, dtype, np.sort(pos_errs(got[r], want[r]))[-20:])
+        eng.close()
+
+
+def crafted_model(kind, window, seed=31):
+    """one layer whose attention is made so that token 0's query matches token 1's key and nothing else: queries read inputs 0-3, keys
+    inputs 4-7 through the same matrix, values the other inputs; token 0 is marked in inputs 0-3, token 1 in 4-7, all other tokens
+    are zero there; no rotation to speak of.  Wherever a token 1 stands in front of token 0 inside the window, however far, that key
+    takes the softmax among hundreds."""
+    small = dict(base=1e30, dims=2)
+    if kind == "talking":
+        mix = OZ.talking_mixer(heads=2, kv_heads=2, dim=8, vdim=8, window=window, conv=2, softcap=30.0, scale=1.0, scaling=None, **small)
+    elif kind == "parallel":
+        mix = OZ.parallel_mixer(OZ.window_spec(heads=2, kv_heads=2, dim=8, vdim=8, window=window, scale=1.0, factor=1.0, **small), width=4)
+    else:
+        mix = OZ.latent_mixer(heads=2, dim=8, rot_dim=2, vdim=8, kv_rank=16, q_rank=8, base=1e30, scale=1.0)
+    cfg = OZ.small_config([OZ.layer(mix, OZ.moe_ff_spec(experts=4, top=1, ff=8, count=2, keep=1))], width=16, vocab=40, loop=None)
+    W = OZ.random_model(cfg, seed=seed)
+    rng = np.random.default_rng(seed + 1)
+    E = W["embed"]
+    E[:, :8] = 0.0
+    mark = rng.standard_normal(4)
+    mark *= 6.0 / np.linalg.norm(mark)
+    E[0, :4], E[1, 4:8] = mark, mark
+    W["embed"] = OZ.bf16_round(E)
+    W["l0.norm1"][:] = 1.0
+    M = rng.standard_normal((16, 4))
+    M[[0, 1, 8, 9]] = 0.0                                         # (the turned pair of each head stays empty)
+    x = "l0.mix.left" if kind == "parallel" else "l0.mix"
+    if kind == "latent":
+        for n in ("dq", "dkv", "uq", "uk"):
+            W[f"{x}.{n}"][:] = 0.0
+        W[x + ".dq"][:4, :4] = np.eye(4)
+        W[x + ".uq"][2:6, :4] = W[x + ".uq"][12:16, :4] = 2.0 * np.eye(4)
+        W[x + ".dkv"][:4, 4:8] = np.eye(4)
+        W[x + ".dkv"][4:12, 8:16] = np.eye(8)
+        W[x + ".uk"][2:6, :4] = W[x + ".uk"][10:14, :4] = np.eye(4)
+        W[x + ".uv"][:, :4] = 0.0
+        W[x + ".uv"] = OZ.bf16_round(W[x + ".uv"] * 4)
+        W[x + ".dq.norm"][:] = 1.0; W[x + ".dkv.norm"][:] = 1.0; W[x + ".sink"][:] = 0.0
+    else:
+        W[x + ".q"], W[x + ".k"] = np.zeros((16, 16), dtype=np.float32), np.zeros((16, 16), dtype=np.float32)
+        W[x + ".q"][:, :4], W[x + ".k"][:, 4:8] = OZ.bf16_round(M), OZ.bf16_round(M)
+        W[x + ".v"][:, :8] = 0.0
+        W[x + ".v"] = OZ.bf16_round(W[x + ".v"] * 4)
+    if kind == "talking":
+        for s in "qkv":
+            W[f"{x}.{s}.b"][:] = 0.0
+            W[f"{x}.{s}.conv"][:] = 0.0
+            W[f"{x}.{s}.conv"][:, -1] = 1.0
+    return cfg, W
+
+
+@pytest.mark.parametrize("kind", ["talking", "latent", "parallel"])
+@pytest.mark.parametrize("page", [4, 64])
+def test_a_marked_key_far_back_and_at_page_borders(be, kind, page):
+    """whole prompt, portions and decoding: the marked key sits right in front of the query, at the sequence's first token, on both
+    sides of a page border and hundreds of tokens back; where it stands it decides the query's logits"""
+    cfg, W = crafted_model(kind, 400)
+    rng = np.random.default_rng(page)
+    T = 330
+    query = T - 1
+    changes = 0
+    for target in (0, 1, page - 1, page, 2 * page, 200, query - page, query - 1):
+        toks = [int(t) for t in rng.integers(2, cfg["vocab"], size=T)]
+        toks[target], toks[query] = 1, 0                      # the marked pair, nowhere else
+        base = list(toks)
+        base[target] = 2
+        want = OZ.Oracle(cfg, W).feed("t", toks)
+        other = OZ.Oracle(cfg, W).feed("t", base)[-1]
+        changes += rel_err(want[-1:], other[None]) > 0.05
+        plans = [[T], [target + 1, T - target - 2, 1], [T - 3, 2, 1], [T - 20] + [1] * 20]
+        for cuts in plans if target in (0, 200) else plans[2:3]:
+            eng = make_engine(be, cfg, W, F32, max_tokens=T + page, page=page)
+            got = run_cuts(be, eng, "t", toks, [c for c in cuts if c > 0])
+            assert rel_err(got[-4:], want[-4:]) <= TOL[F32], (target, cuts[:3])
+    assert changes >= 7
+
+
+@pytest.mark.parametrize("kind", ["talking", "parallel"])
+@pytest.mark.parametrize("window", [1, 2, 16, 21, 64])
+def test_a_marked_key_at_the_window_edge(be, kind, window):
+    """the marked key at the last place the window reaches and one in front of it, in a prompt, at a portion's start and decoded token by
+    token: inside it decides the logits, outside nothing of it is left"""
+    cfg, W = crafted_model(kind, window)
+    rng = np.random.default_rng(window)
+    T = window + 30
+    query = T - 1
+    for dist in ([window - 1, window] if window > 1 else [1]):
+        toks = [int(t) for t in rng.integers(2, cfg["vocab"], size=T)]
+        toks[query - dist], toks[query] = 1, 0
+        base = list(toks)
+        base[query - dist] = 2
+        want, other = OZ.Oracle(cfg, W).feed("t", toks), OZ.Oracle(cfg, W).feed("t", base)
+        if kind == "talking":                                     # (beside the window attention the recurrence remembers the token either way)
+            assert (rel_err(want[-1:], other[-1:]) > 0.05) == (dist < window), dist
+        for cuts in ([T], [T - 1, 1], [T - dist - 1, dist + 1], [T - 25] + [1] * 25):
+            eng = make_engine(be, cfg, W, F32, max_tokens=T + 8, page=8)
+            assert rel_err(run_cuts(be, eng, "t", toks, [c for c in cuts if c > 0])[-3:], want[-3:]) <= TOL[F32], (dist, cuts[:3])
+
+
+def test_the_state_carries_a_far_token(be):
+    """a token 300 positions back reaches the last position of a layer with a window of three only through the recurrent state: changing
+    it changes the logits, and portions and decoding carry it like the whole prompt does"""
+    cfg = OZ.small_config([OZ.layer(OZ.parallel_mixer(OZ.window_spec(heads=2, kv_heads=1, dim=8, vdim=8, dims=4, window=3), width=24),
+                                    OZ.moe_ff_spec(experts=4, top=1, ff=8, count=2, keep=1))], width=16, vocab=40, loop=None)
+    W = OZ.random_model(cfg, seed=51)
+    W["l0.mix.right.z.b"][:] = -7.0                                                # slow forgetting
+    rng = np.random.default_rng(52)
+    toks = [int(t) for t in rng.integers(0, cfg["vocab"], size=310)]
+    other = list(toks)
+    other[9] = (toks[9] + 1) % cfg["vocab"]
+    want = OZ.Oracle(cfg, W).feed("a", toks)
+    assert rel_err(OZ.Oracle(cfg, W).feed("a", other)[-1:], want[-1:]) > 1e-3
+    for cuts in ([310], [100, 2, 65, 143], [290] + [1] * 20):
+        eng = make_engine(be, cfg, W, F32, max_tokens=320, page=16)
+        assert rel_err(run_cuts(be, eng, "a", toks, cuts)[-8:], want[-8:]) <= 2 * TOL[F32], cuts
+
+
+def test_sinks_take_weight_at_the_first_tokens(be):
+    """with one or two keys the sinks hold much of the softmax: the first tokens' logits differ clearly from the same model with the
+    learned sinks far down, and match the equations"""
+    cfg = OZ.small_config([OZ.layer(OZ.latent_mixer(), None), OZ.layer(OZ.talking_mixer(), None)], loop=None)
+    W = OZ.random_model(cfg, seed=71)
+    W["l0.mix.sink"][:] = 3.0
+    toks = [5, 9, 2, 30, 7]
+    want = OZ.Oracle(cfg, W).feed("a", toks)
+    low = dict(W)
+    low["l0.mix.sink"] = np.full_like(W["l0.mix.sink"], -60.0)
+    assert pos_errs(OZ.Oracle(cfg, low).feed("a", toks), want)[:2].min() > 0.05
+    for dtype in (F32, BF16):
+        for cuts in ([5], [1] * 5, [2, 3]):
+            assert ok(run_cuts(be, make_engine(be, cfg, W, dtype, 16), "a", toks, cuts), want, dtype), (dtype, cuts)
+
+
+def test_long_decoding_bf16(be):
+    cfg = CONFIGS["mixed"]()
+    W = OZ.random_model(cfg, seed=7)
+    toks = clear_tokens(cfg, W, 60, 8, gap=0.008)
+    want = OZ.Oracle(cfg, W).feed("a", toks)
+    eng = make_engine(be, cfg, W, BF16, 64, page=8)
+    got = run_cuts(be, eng, "a", toks, [3] + [1] * 57)
+    assert ok(got, want, BF16), pos_errs(got, want)
+
+
+def test_greedy_generation_through_the_generator(be):
+    from exllamav2_amd.engine import Generator
+    cfg = CONFIGS["mixed"]()
+    W = OZ.random_model(cfg, seed=9)
+    rng = np.random.default_rng(10)
+    prompts = [list(map(int, rng.integers(0, cfg["vocab"], size=n))) for n in (7, 3, 5, 4, 6)]
+    eng = make_engine(be, cfg, W, F32, max_tokens=64, page=4, max_seqs=3)
+    out = Generator(eng, chunk=3).generate(prompts, 6)
+    oracle = OZ.Oracle(cfg, W)
+    checked = 0
+    for i, p in enumerate(prompts):
+        lg = oracle.feed(i, p)[-1]
+        for t in out[i]:
+            top2 = np.sort(lg)[-2:]
+            if top2[1] - top2[0] < 1e-3:
+                break                                             # a near tie: later tokens may differ legitimately
+            assert t == int(np.argmax(lg))
+            checked += 1
+            lg = oracle.feed(i, [t])[-1]
+        assert len(out[i]) == 6
+    assert checked >= 20
+    assert len(eng.pool.free_pages) == eng.pool.num_pages
+
+
+def test_model_directory_registry(be, tmp_path):
+    """config.json + model.safetensors -> architectures.load_model picks the class by the architecture name"""
+    from safetensors.torch import save_file
+    from exllamav2_amd.architectures import load_model, read_config
+    from exllamav2_amd.engine import Engine
+    cfg = CONFIGS["odd"]()
+    W = OZ.random_model(cfg, seed=11)
+    save_file({k: torch.from_numpy(np.asarray(v)).to(BF16) for k, v in W.items()}, str(tmp_path / "model.safetensors"))
+    (tmp_path / "config.json").write_text(json.dumps(cfg))
+    assert read_config(str(tmp_path))[0] == "Zevilorn"
+    model = load_model(str(tmp_path), device=be.device, dtype=F32, ext=be.ext)
+    toks = [1, 5, 9, 2, 2, 7]
+    got = be.n(Engine(model, 16, page_size=4).step([("x", toks, list(range(6)))]))
+    assert rel_err(got, OZ.Oracle(cfg, W).feed("x", toks)) <= TOL[F32]
+
+
+def test_bad_configurations_are_refused(be):
+    from exllamav2_amd.config import LayeredConfig
+    cfg = CONFIGS["mixed"]()
+    with pytest.raises(RuntimeError, match="loop"):
+        LayeredConfig.from_dict_parallel_gated(dict(cfg, loop={"start": 1, "stop": 9, "times": 2}))
+    with pytest.raises(RuntimeError, match="missing key"):
+        LayeredConfig.from_dict_parallel_gated({k: v for k, v in cfg.items() if k != "norm"})
+    W = OZ.random_model(cfg, seed=1)
+    with pytest.raises(RuntimeError, match="unknown mixer"):
+        make_engine(be, dict(cfg, layers=[dict(cfg["layers"][0], type="nonesuch")], loop=None), W, F32, 16)
+    bad = dict(W)
+    bad["l1.mix.talk"] = bad["l1.mix.talk"][:, :-1]
+    with pytest.raises(RuntimeError, match="mixing"):
+        make_engine(be, cfg, bad, F32, 16)
+    bad = dict(W)
+    bad["l0.rg1"] = bad["l0.rg1"][:-1]
+    with pytest.raises(RuntimeError, match="gates"):
+        make_engine(be, cfg, bad, F32, 16)
+
+
+@pytest.mark.gpu
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+def test_trace_command_replays_steps(tmp_path, dtype):
+    """bin/trace_run in a process of its own: steps on standard input, logits files and `done` lines out"""
+    if not torch.cuda.is_available():
+        pytest.skip("no GPU visible")
+    from safetensors.torch import save_file
+    cfg = CONFIGS["mixed"]()
+    W = OZ.random_model(cfg, seed=12)
+    mdir = tmp_path / "model"
+    mdir.mkdir()
+    save_file({k: torch.from_numpy(np.asarray(v)).to(BF16) for k, v in W.items()}, str(mdir / "model.safetensors"))
+    (mdir / "config.json").write_text(json.dumps(cfg))
+    a, b = clear_tokens(cfg, W, 300, 13, gap=0.008), clear_tokens(cfg, W, 9, 14)
+    steps = [{"step": 0, "entries": [{"id": "a", "tokens": a[:290], "want": [0, 289]}], "end": []},
+             {"step": 1, "entries": [{"id": "a", "tokens": a[290:295], "want": []}, {"id": "b", "tokens": b[:8], "want": [7]}], "end": []},
+             {"step": 2, "entries": [{"id": "b", "tokens": b[8:], "want": [0]}, {"id": "a", "tokens": a[295:], "want": [4]}], "end": ["a", "b"]}]
+    out = tmp_path / "out"
+    p = subprocess.run([os.path.join(ROOT, "bin", "trace_run"), "--model", str(mdir), "--dtype", dtype, "--out", str(out), "--max-tokens", "512"],
+                       input="".join(json.dumps(s) + "\n" for s in steps), capture_output=True, text=True, timeout=600, cwd=str(tmp_path))
+    assert p.returncode == 0, p.stderr[-2000:]
+    assert [l for l in p.stdout.splitlines() if l.startswith("done")] == ["done 0", "done 1", "done 2"]
+    oracle = OZ.Oracle(cfg, W)
+    wa, wb = oracle.feed("a", a), oracle.feed("b", b)
+    got = np.concatenate([np.fromfile(out / f"{n}.f32", dtype="<f4").reshape(k, -1) for n, k in ((0, 2), (1, 1), (2, 2))])
+    want = np.stack([wa[0], wa[289], wb[7], wb[8], wa[299]])
+    e = pos_errs(got, want)
+    assert (e.max() <= TOL[F32]) if dtype == "float32" else (np.median(e) <= 2e-2 and e.max() <= 6e-2), e
