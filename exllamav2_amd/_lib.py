@@ -128,9 +128,9 @@ PROTOTYPES = {
     "exl2_window_attn_tiles_supported": (ci, [ci, ci]),
     "exl2_window_attn_tiles": (ci, [vp, vp, vp, vp, vp, vp, vp, ci, vp, ci, ci, vp, vp, vp, ci, ci, ci, vp, vp, vp, ci, ci, vp, vp, ci, ci, ci, ci, ci, ci, vp]),
     # variants of the windowed attention (chunked mask, soft cap, one gate per head, query-only rows)
-    "exl2_kv_rot_append_ex": (ci, [vp, ci, ci, ci, ci, vp, vp, vp, vp, vp, vp, vp, cf, ci, vp, ci, ci, vp, vp, vp, ci, ci, ci, ci, ci, ci, ci, ci, ci, vp]),
-    "exl2_window_attn_ex": (ci, [vp, vp, vp, vp, vp, vp, vp, ci, vp, ci, ci, vp, vp, vp, ci, ci, ci, vp, ci, ci, ci, ci, ci, ci, ci, ci, cf, ci, vp]),
-    "exl2_window_attn_tiles_ex": (ci, [vp, vp, vp, vp, vp, vp, vp, ci, vp, ci, ci, vp, vp, vp, ci, ci, ci, vp, vp, vp, ci, ci, vp, vp, ci, ci, ci, ci, ci, ci, ci, cf, ci, vp]),
+    "exl2_kv_rot_append_ex": (ci, [vp, ci, ci, ci, ci, vp, vp, vp, vp, vp, vp, vp, cf, ci, vp, ci, ci, vp, vp, vp, ci, ci, ci, ci, ci, ci, ci, ci, ci, ci, cf, vp]),
+    "exl2_window_attn_ex": (ci, [vp, vp, vp, vp, vp, vp, vp, ci, vp, ci, ci, vp, vp, vp, ci, ci, ci, vp, ci, ci, ci, ci, ci, ci, ci, ci, ci, cf, ci, vp]),
+    "exl2_window_attn_tiles_ex": (ci, [vp, vp, vp, vp, vp, vp, vp, ci, vp, ci, ci, vp, vp, vp, ci, ci, ci, vp, vp, vp, ci, ci, vp, vp, ci, ci, ci, ci, ci, ci, ci, ci, cf, ci, vp]),
     # scalar-gain RMS norm + token shift, sigmoid router (csrc/rowops.hip); decaying linear attention (csrc/wkv.hip)
     "exl2_add_rms_shift": (ci, [vp, vp, vp, ci, cf, cf, vp, vp, vp, vp, ci, vp, vp, vp, vp, vp, ci, ci, ci, ci, ci, vp]),
     "exl2_span_last_rows": (ci, [vp, ci, vp, ci, vp, vp, ci, vp, vp]),
@@ -142,18 +142,21 @@ PROTOTYPES = {
     # sandwich-normed residual step, token-pair embedding (csrc/rowops.hip); convolution variants (csrc/ssm.hip); matrix-state recurrences
     # (csrc/gated_scan.hip)
     "exl2_sandwich_norm": (ci, [vp, vp, cf, vp, cf, vp, ci, vp, cf, vp, vp, ci, vp, vp, vp, vp, vp, ci, ci, ci, ci, ci, cf, vp]),
-    "exl2_embed_pair": (ci, [vp, vp, vp, vp, vp, vp, vp, vp, vp, ci, ci, vp, ci, ci, ci, ci, ci, ci, ci, cf, ci, cf, vp]),
+    "exl2_embed_pair": (ci, [vp, vp, vp, vp, vp, vp, vp, vp, vp, ci, ci, vp, vp, ci, ci, ci, ci, ci, ci, ci, ci, cf, ci, cf, vp]),
     "exl2_conv_rows_ex": (ci, [vp, ci, vp, vp, vp, ci, ci, ci, vp, vp, vp, ci, ci, vp, vp, ci, ci, ci, vp]),
-    "exl2_gated_scan": (ci, [ci, vp, ci, vp, ci, vp, ci, vp, ci, vp, ci, vp, ci, vp, vp, vp, vp, vp, ci, ci, vp, vp, vp, ci, vp, vp, ci, ci,
+    "exl2_gated_scan": (ci, [ci, vp, ci, vp, ci, vp, ci, vp, ci, ci, vp, ci, vp, ci, vp, vp, vp, vp, vp, ci, ci, vp, vp, vp, ci, vp, vp, ci, ci,
                              ci, ci, cf, cf, vp]),
     "exl2_gated_scan_cols_supported": (ci, [ci, ci]),
-    "exl2_gated_scan_cols": (ci, [ci, vp, ci, vp, ci, vp, ci, vp, ci, vp, ci, vp, ci, vp, vp, vp, vp, vp, ci, ci, vp, vp, vp, ci, vp, vp, ci, vp,
+    "exl2_gated_scan_cols": (ci, [ci, vp, ci, vp, ci, vp, ci, vp, ci, ci, vp, ci, vp, ci, vp, vp, vp, vp, vp, ci, ci, vp, vp, vp, ci, vp, vp, ci, vp,
                                   ci, ci, ci, ci, cf, cf, vp]),
     # layers whose mixer and feed-forward read one norm: gated residual step, grouped router (csrc/rowops.hip); latent attention with a sink
     # per head and either rotary layout (csrc/latent_attn.hip); minimal gated recurrence (csrc/mingru.hip); head-mixing attention
     # (csrc/talk_attn.hip)
-    "exl2_gated_residual": (ci, [vp, vp, vp, vp, vp, cf, cf, vp, vp, ci, vp, vp, ci, vp, vp, ci, ci, vp, vp, ci, vp, ci, ci, ci, cf, vp]),
+    "exl2_gated_residual": (ci, [vp, vp, vp, vp, vp, cf, cf, vp, vp, ci, vp, vp, ci, vp, vp, ci, ci, vp, vp, ci, ci, vp, ci, ci, ci, cf, cf, vp]),
     "exl2_moe_route_grouped": (ci, [vp, ci, vp, vp, ci, ci, ci, cf, ci, ci, vp, vp, vp, vp]),
+    # plain pre-norm stacks: split linear (csrc/dense.hip), softmax-over-the-chosen router (csrc/rowops.hip)
+    "exl2_dense_linear_split": (ci, [vp, vp, vp, vp, ci, vp, ci, ci, ci, ci, ci, ci, ci, ci, ci, vp]),
+    "exl2_moe_route_chosen": (ci, [vp, ci, vp, vp, ci, ci, ci, cf, ci, ci, vp, vp, vp, vp]),
     "exl2_latent_append_ex": (ci, [vp, ci, vp, cf, ci, ci, ci, ci, ci, ci, vp, vp, vp, vp, ci, ci, vp, vp]),
     "exl2_latent_attn_ex": (ci, [vp, ci, ci, ci, vp, vp, ci, vp, vp, vp, ci, vp, ci, ci, ci, ci, ci, ci, ci, vp, cf, ci, vp, vp]),
     "exl2_latent_attn_tiles_ex": (ci, [vp, ci, ci, ci, vp, vp, ci, vp, vp, vp, ci, vp, vp, vp, ci, ci, vp, vp, ci, ci, ci, ci, ci, ci, vp, cf, ci,

@@ -59,6 +59,7 @@ register("Tibalorn", LayeredConfig.from_dict_prenorm, _build_layered)
 register("Negilorn", LayeredConfig.from_dict_prerms_shift, _build_layered)
 register("Kilurax", LayeredConfig.from_dict_sandwich, _build_layered)
 register("Zevilorn", LayeredConfig.from_dict_parallel_gated, _build_layered)
+register("Savenex", LayeredConfig.from_dict_prerms, _build_layered)
 register("LlamaForCausalLM", _read_llama, _build_quantized)
 register("MixtralForCausalLM", _read_llama, _build_quantized)
 

@@ -76,9 +76,11 @@ class LayeredConfig:
     residual_mult: float = 1.0
     input_conv_taps: int = 0
     # "parallel_gated": h = rms_norm(x) w;  x <- x + mixer(h) sigmoid(W_1 h + b_1) + ff(h) sigmoid(W_2 h + b_2), one norm per layer
+    # "pre_rms": x <- x + residual_mult * f(rms_norm(x) w), mixer and feed-forward one after the other
     # (start, stop, times): those layers are gone through `times` times in a row, every pass with state of its own; in front of every pass
-    # but the first the embeddings are added to the stream
+    # but the first the embeddings are added to the stream, or (loop_linear) in front of EVERY pass x <- W [x; embedding output]
     loop: tuple | None = None
+    loop_linear: bool = False
     pair_embedding: dict | None = None   # {"buckets", "mul_prev", "mul_cur"}: a hashed (previous token, token) table added to the embedding
 
     @staticmethod
@@ -148,13 +150,31 @@ class LayeredConfig:
             raise RuntimeError(f"config.json: loop {cfg.loop} does not fit {len(cfg.layers)} layers")
         return cfg
 
+    @staticmethod
+    def from_dict_prerms(d: dict) -> "LayeredConfig":
+        """plain pre-norm stacks with RMS norms, a factor on the residual branch, a normed embedding, a run of layers that may be gone
+        through several times behind a linear of the stream and the embedding, and a `head` matrix"""
+        try:
+            loop = d.get("loop")
+            cfg = LayeredConfig(architecture=str(d["architecture"]), vocab=int(d["vocab"]), width=int(d["width"]),
+                                norm_eps=float(d["norm"]["eps"]), layers=list(d["layers"]), residual="pre_rms",
+                                residual_mult=float(d.get("residual_mult", 1.0)), loop_linear=True,
+                                loop=(int(loop["start"]), int(loop["stop"]), int(loop["times"])) if loop else None)
+        except KeyError as e:
+            raise RuntimeError(f"config.json: missing key {e}") from e
+        if cfg.vocab <= 0 or cfg.width <= 0 or not cfg.layers:
+            raise RuntimeError("config.json: vocab, width and layers must be given")
+        if cfg.loop is not None and not (0 <= cfg.loop[0] <= cfg.loop[1] <= len(cfg.layers) and cfg.loop[2] >= 1):
+            raise RuntimeError(f"config.json: loop {cfg.loop} does not fit {len(cfg.layers)} layers")
+        return cfg
+
     def layer_runs(self) -> list:
-        """[(layer, pass, the embeddings are added in front of it)] in the order the layers are gone through"""
+        """[(layer, pass, the embeddings enter in front of it)] in the order the layers are gone through"""
         n = len(self.layers)
         start, stop, times = self.loop or (0, 0, 1)
         runs = [(i, 0, False) for i in range(start)]
         for p in range(times):
-            runs += [(i, p, p > 0 and i == start) for i in range(start, stop)]
+            runs += [(i, p, (p > 0 or (self.loop_linear and self.loop is not None)) and i == start) for i in range(start, stop)]
         return runs + [(i, 0, False) for i in range(stop, n)]
 
     @staticmethod

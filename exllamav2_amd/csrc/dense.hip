@@ -15,18 +15,21 @@
 // (gated MLP), the clamped gated unit min(aux, L) * sigmoid(1.702 min(aux, L)) * (clamp(acc, -L, L) + 1), relu(acc)^2, the soft
 // cap L tanh(acc / L), a plain scale L acc, tanh(acc), and relu(aux[row] acc)^2 (an expert whose INPUT carries the router's weight:
 // W (s h) = s (W h)), the two halves of a gated unit on such an input -- silu(aux[row] acc) aux[row] from the gate matrix, then
-// aux acc from the up matrix --, the exact (error function) gelu(acc), and acc * sigmoid(aux[row]) (one output gate per row and batch,
-// i.e. per head); a bias vector (fp32, one value per output column) is added to the accumulator first.
+// aux acc from the up matrix --, the exact (error function) gelu(acc), acc * sigmoid(aux[row]) (one output gate per row and batch,
+// i.e. per head), and exp(aux[column] softplus(acc)) (a recurrence's decays; with aux = -1 and the weight's sign turned it is the
+// sigmoid of the product, so decays and gates can share a launch); a bias vector (fp32, one value per output column) is added to the
+// accumulator first.  A call may be SPLIT: the columns from n2 on go to a second buffer in the operand dtype (what a further linear
+// reads), the ones in front of it to y.
 #include "hw.h"
 #include "errors.h"
 
 enum { DENSE_BF16 = 0, DENSE_F32 = 1 };
 enum { EPI_NONE = 0, EPI_MUL_SIGMOID_AUX = 1, EPI_SILU_AUX_MUL = 2, EPI_CLAMPED_GLU = 3, EPI_RELU_SQUARED = 4, EPI_SOFT_CAP = 5,
        EPI_SCALE = 6, EPI_TANH = 7, EPI_ROW_SCALED_RELU_SQUARED = 8, EPI_ROW_SCALED_SILU_SCALED = 9, EPI_AUX_MUL = 10, EPI_GELU_ERF = 11,
-       EPI_MUL_SIGMOID_ROW_AUX = 12, EPI_LAST = 12 };
-// aux holds ONE value per row (ldaux apart), not one per output
+       EPI_MUL_SIGMOID_ROW_AUX = 12, EPI_EXP_SOFTPLUS = 13, EPI_LAST = 13 };
+// aux holds ONE value per row (ldaux apart), not one per output (ldaux 0 with the other forms: one value per column)
 #define EPI_ROW_AUX(e) ((e) == EPI_ROW_SCALED_RELU_SQUARED || (e) == EPI_ROW_SCALED_SILU_SCALED || (e) == EPI_MUL_SIGMOID_ROW_AUX)
-#define EPI_READS_AUX(e) (((e) >= EPI_MUL_SIGMOID_AUX && (e) <= EPI_CLAMPED_GLU) || EPI_ROW_AUX(e) || (e) == EPI_AUX_MUL)
+#define EPI_READS_AUX(e) (((e) >= EPI_MUL_SIGMOID_AUX && (e) <= EPI_CLAMPED_GLU) || EPI_ROW_AUX(e) || (e) == EPI_AUX_MUL || (e) == EPI_EXP_SOFTPLUS)
 #define EPI_AUX_COL(e, n) (EPI_ROW_AUX(e) ? 0 : (n))
 
 struct LinArgs
@@ -40,6 +43,7 @@ struct LinArgs
     const int* grp_count; const int* grp_offset; const int* grp_rows;     // grouped: rows of batch z = grp_rows[grp_offset[z] + i]
     int x_div;                               // x row of logical row p = p / x_div (several output rows per input row)
     int epi; float limit;
+    void* y2; int n2, ldy2;                  // columns n >= n2 go to y2[r, n - n2] in the operand dtype (n2 = N: none)
 };
 
 template <typename T> DEV float ld1(const T* p);
@@ -93,7 +97,19 @@ DEV float lin_epilogue(int epi, float acc, float aux, float limit)
     if (epi == EPI_AUX_MUL) return acc * aux;
     if (epi == EPI_GELU_ERF) return 0.5f * acc * (1.0f + erff(acc * 0.70710678118654752f));
     if (epi == EPI_MUL_SIGMOID_ROW_AUX) return acc * sigmoid_f32(aux);
+    if (epi == EPI_EXP_SOFTPLUS) return expf(aux * (acc > 20.0f ? acc : log1pf(expf(acc))));
     return acc;
+}
+
+// bias, epilogue and store of output (row r, column n) of batch z
+template <typename T, typename TY>
+DEV void lin_store(const LinArgs& a, int z, long long r, int n, float acc)
+{
+    float aux = 0.0f;
+    if (EPI_READS_AUX(a.epi)) aux = a.aux[(long long)z * a.sauxb + r * a.ldaux + EPI_AUX_COL(a.epi, n)];
+    const float v = lin_epilogue(a.epi, acc + (a.bias ? a.bias[n] : 0.0f), aux, a.limit);
+    if (n >= a.n2) { st1<T>((T*)a.y2 + r * a.ldy2 + (n - a.n2), v); return; }
+    st1<TY>((TY*)a.y + (long long)z * a.syb + r * a.ldy + n, v);
 }
 
 // ---- <= 16 rows -------------------------------------------------------------------------------------------------------------
@@ -159,9 +175,7 @@ KERNEL void __launch_bounds__(256) lin_rows_kernel(const LinArgs a)
         {
             const int r = r0 + m;
             if (r >= a.M) break;
-            float aux = 0.0f;
-            if (EPI_READS_AUX(a.epi)) aux = a.aux[(long long)z * a.sauxb + (long long)r * a.ldaux + EPI_AUX_COL(a.epi, n)];
-            st1<TY>((TY*)a.y + (long long)z * a.syb + (long long)r * a.ldy + n, lin_epilogue(a.epi, acc[m] + (a.bias ? a.bias[n] : 0.0f), aux, a.limit));
+            lin_store<T, TY>(a, z, r, n, acc[m]);
         }
     }
 }
@@ -228,9 +242,7 @@ KERNEL void __launch_bounds__(256) lin_tile_kernel(const LinArgs a)
         {
             const int n = n0 + tx * 4 + j;
             if (n >= a.N) continue;
-            float aux = 0.0f;
-            if (EPI_READS_AUX(a.epi)) aux = a.aux[(long long)z * a.sauxb + r * a.ldaux + EPI_AUX_COL(a.epi, n)];
-            st1<TY>((TY*)a.y + (long long)z * a.syb + r * a.ldy + n, lin_epilogue(a.epi, acc[i][j] + (a.bias ? a.bias[n] : 0.0f), aux, a.limit));
+            lin_store<T, TY>(a, z, r, n, acc[i][j]);
         }
     }
 }
@@ -298,9 +310,7 @@ KERNEL void __launch_bounds__(256) lin_mfma_kernel(const LinArgs a)
             {
                 const int n = n0 + 16 * j + li;
                 if (n >= a.N) continue;
-                float aux = 0.0f;
-                if (EPI_READS_AUX(a.epi)) aux = a.aux[(long long)z * a.sauxb + row * a.ldaux + EPI_AUX_COL(a.epi, n)];
-                st1<TY>((TY*)a.y + (long long)z * a.syb + row * a.ldy + n, lin_epilogue(a.epi, acc[i][j][r] + (a.bias ? a.bias[n] : 0.0f), aux, a.limit));
+                lin_store<u16, TY>(a, z, row, n, acc[i][j][r]);
             }
         }
 }
@@ -395,9 +405,7 @@ KERNEL void __launch_bounds__(256) lin_mfma_tile_kernel(const LinArgs a)
             {
                 const int n = n0 + wn + 16 * j + li;
                 if (n >= a.N) continue;
-                float aux = 0.0f;
-                if (EPI_READS_AUX(a.epi)) aux = a.aux[(long long)z * a.sauxb + row * a.ldaux + EPI_AUX_COL(a.epi, n)];
-                st1<TY>((TY*)a.y + (long long)z * a.syb + row * a.ldy + n, lin_epilogue(a.epi, acc[i][j][r] + (a.bias ? a.bias[n] : 0.0f), aux, a.limit));
+                lin_store<u16, TY>(a, z, row, n, acc[i][j][r]);
             }
         }
 }
@@ -435,6 +443,41 @@ static void launch_dense(const LinArgs& a, int batch, bool vec_ok, int max_rows,
     LAUNCH((lin_tile_kernel<T, TY>), dim3((a.N + 63) / 64, (max_rows + 63) / 64, batch), dim3(256), 0, s, a);
 }
 
+static int dense_linear_any(const void* x, const void* w, const float* bias, void* y, void* y2, int n2, int ldy2, const float* aux,
+                            int dtype, int y_f32, int M, int N, int K, int ldx, int ldw, int ldy, int ldaux,
+                            int batch, long long sxb, long long swb, long long syb, long long sauxb,
+                            const int* w_sel, int n_sel, const int* grp_count, const int* grp_offset, const int* grp_rows,
+                            int x_div, int epi, float limit, void* stream)
+{
+    EXL2_REQUIRE(x && w && y, "dense_linear: null operand");
+    EXL2_REQUIRE(dtype == DENSE_BF16 || dtype == DENSE_F32, "dense_linear: dtype must be 0 (bfloat16) or 1 (float32)");
+    EXL2_REQUIRE(M >= 0 && N > 0 && K > 0 && batch > 0 && x_div > 0, "dense_linear: bad shape %d x %d x %d, batch %d", M, N, K, batch);
+    EXL2_REQUIRE(ldx >= K || x_div > 0, "dense_linear: ldx"); EXL2_REQUIRE(ldw >= K && ldy > 0, "dense_linear: leading dimensions");
+    EXL2_REQUIRE(epi >= EPI_NONE && epi <= EPI_LAST, "dense_linear: unknown epilogue %d", epi);
+    EXL2_REQUIRE(!EPI_READS_AUX(epi) || aux, "dense_linear: the epilogue needs aux");
+    EXL2_REQUIRE(epi != EPI_SOFT_CAP || limit > 0.0f, "dense_linear: the soft cap needs a positive limit");
+    EXL2_REQUIRE(!bias || (batch == 1 && !w_sel && !grp_count), "dense_linear: a bias goes with a plain (one-slab) call");
+    EXL2_REQUIRE(!(w_sel && grp_count), "dense_linear: w_sel and groups exclude each other");
+    EXL2_REQUIRE(!grp_count || (grp_offset && grp_rows), "dense_linear: grouped call without offsets / row lists");
+    EXL2_REQUIRE(dtype == DENSE_BF16 || y_f32, "dense_linear: float32 operands give float32 results");
+    if (M == 0) return EXL2_OK;
+    LinArgs a;
+    a.x = x; a.w = w; a.y = y; a.aux = aux; a.bias = bias; a.M = M; a.N = N; a.K = K; a.ldx = ldx; a.ldw = ldw; a.ldy = ldy; a.ldaux = ldaux;
+    a.sxb = sxb; a.swb = swb; a.syb = syb; a.sauxb = sauxb; a.w_sel = w_sel; a.n_sel = n_sel;
+    a.y2 = y2; a.n2 = n2; a.ldy2 = ldy2;
+    a.grp_count = grp_count; a.grp_offset = grp_offset; a.grp_rows = grp_rows; a.x_div = x_div; a.epi = epi; a.limit = limit;
+    const int es = dtype == DENSE_BF16 ? 2 : 4, v = 16 / es;
+    // 16-byte loads: every row start and every step must stay aligned
+    const bool vec_ok = K % v == 0 && ldx % v == 0 && ldw % v == 0 && sxb % v == 0 && swb % v == 0
+                        && ((uintptr_t)x % 16) == 0 && ((uintptr_t)w % 16) == 0;
+    hipStream_t s = (hipStream_t)stream;
+    if (dtype == DENSE_F32) launch_dense<float, float>(a, batch, vec_ok, M, s);
+    else if (y_f32) launch_dense<u16, float>(a, batch, vec_ok, M, s);
+    else launch_dense<u16, u16>(a, batch, vec_ok, M, s);
+    HIP_TRY(hipGetLastError());
+    return EXL2_OK;
+}
+
 extern "C" int exl2_dense_linear_bias(const void* x, const void* w, const float* bias, void* y, const float* aux, int dtype, int y_f32,
                                       int M, int N, int K, int ldx, int ldw, int ldy, int ldaux,
                                       int batch, long long sxb, long long swb, long long syb, long long sauxb,
@@ -457,30 +500,14 @@ extern "C" int exl2_dense_linear_bias(const void* x, const void* w, const float*
                                       const int* w_sel, int n_sel, const int* grp_count, const int* grp_offset, const int* grp_rows,
                                       int x_div, int epi, float limit, void* stream)
 {
-    EXL2_REQUIRE(x && w && y, "dense_linear: null operand");
-    EXL2_REQUIRE(dtype == DENSE_BF16 || dtype == DENSE_F32, "dense_linear: dtype must be 0 (bfloat16) or 1 (float32)");
-    EXL2_REQUIRE(M >= 0 && N > 0 && K > 0 && batch > 0 && x_div > 0, "dense_linear: bad shape %d x %d x %d, batch %d", M, N, K, batch);
-    EXL2_REQUIRE(ldx >= K || x_div > 0, "dense_linear: ldx"); EXL2_REQUIRE(ldw >= K && ldy > 0, "dense_linear: leading dimensions");
-    EXL2_REQUIRE(epi >= EPI_NONE && epi <= EPI_LAST, "dense_linear: unknown epilogue %d", epi);
-    EXL2_REQUIRE(!EPI_READS_AUX(epi) || aux, "dense_linear: the epilogue needs aux");
-    EXL2_REQUIRE(epi != EPI_SOFT_CAP || limit > 0.0f, "dense_linear: the soft cap needs a positive limit");
-    EXL2_REQUIRE(!bias || (batch == 1 && !w_sel && !grp_count), "dense_linear: a bias goes with a plain (one-slab) call");
-    EXL2_REQUIRE(!(w_sel && grp_count), "dense_linear: w_sel and groups exclude each other");
-    EXL2_REQUIRE(!grp_count || (grp_offset && grp_rows), "dense_linear: grouped call without offsets / row lists");
-    EXL2_REQUIRE(dtype == DENSE_BF16 || y_f32, "dense_linear: float32 operands give float32 results");
-    if (M == 0) return EXL2_OK;
-    LinArgs a;
-    a.x = x; a.w = w; a.y = y; a.aux = aux; a.bias = bias; a.M = M; a.N = N; a.K = K; a.ldx = ldx; a.ldw = ldw; a.ldy = ldy; a.ldaux = ldaux;
-    a.sxb = sxb; a.swb = swb; a.syb = syb; a.sauxb = sauxb; a.w_sel = w_sel; a.n_sel = n_sel;
-    a.grp_count = grp_count; a.grp_offset = grp_offset; a.grp_rows = grp_rows; a.x_div = x_div; a.epi = epi; a.limit = limit;
-    const int es = dtype == DENSE_BF16 ? 2 : 4, v = 16 / es;
-    // 16-byte loads: every row start and every step must stay aligned
-    const bool vec_ok = K % v == 0 && ldx % v == 0 && ldw % v == 0 && sxb % v == 0 && swb % v == 0
-                        && ((uintptr_t)x % 16) == 0 && ((uintptr_t)w % 16) == 0;
-    hipStream_t s = (hipStream_t)stream;
-    if (dtype == DENSE_F32) launch_dense<float, float>(a, batch, vec_ok, M, s);
-    else if (y_f32) launch_dense<u16, float>(a, batch, vec_ok, M, s);
-    else launch_dense<u16, u16>(a, batch, vec_ok, M, s);
-    HIP_TRY(hipGetLastError());
-    return EXL2_OK;
+    return dense_linear_any(x, w, bias, y, nullptr, N, 0, aux, dtype, y_f32, M, N, K, ldx, ldw, ldy, ldaux, batch, sxb, swb, syb, sauxb,
+                            w_sel, n_sel, grp_count, grp_offset, grp_rows, x_div, epi, limit, stream);
+}
+
+extern "C" int exl2_dense_linear_split(const void* x, const void* w, const float* bias, void* y, int y_f32, void* y2, int n2, int ldy2,
+                                       int dtype, int M, int N, int K, int ldx, int ldw, int ldy, void* stream)
+{
+    EXL2_REQUIRE(y2 && n2 > 0 && n2 < N && ldy2 >= N - n2 && ldy >= n2, "dense_linear_split: %d of %d columns in front of the split", n2, N);
+    return dense_linear_any(x, w, bias, y, y2, n2, ldy2, nullptr, dtype, y_f32, M, N, K, ldx, ldw, ldy, 0, 1, 0, 0, 0, 0, nullptr, 0,
+                            nullptr, nullptr, nullptr, 1, EPI_NONE, 0.0f, stream);
 }

@@ -6,10 +6,12 @@
 //   mode 1, "gated delta rule":     q, k made unit vectors per head (x / sqrt(sum x^2 + 1e-6)), q also times q_scale,
 //       beta = sigmoid(z_b),  g = exp(-exp(A) softplus(z_a + a_bias))  (one number per head),
 //       S <- g S,   u = beta (v - S^T k),   S <- S + k u^T,   o = S^T q        (the read-out sees the token's own write).
+//   mode 2, "delta rule, decay per key channel":  as mode 1 with g a vector over the head's key channels (row n of S is multiplied by
+//       g[n]) that comes ready made, one value per head and channel (the linear that brings its argument takes the exponential).
 // The head's o is divided by its root mean square over P, multiplied by a weight per value channel (shared by the heads) and, in
-// mode 1, by silu of an output gate, and leaves in the operand dtype for the output projection.  Query / key heads may be fewer than
-// value heads (head h reads q / k head h / (heads / qk_heads)).  Inputs are the fp32 outputs of the mixer's projections (mode 1: of
-// its short convolutions); gates, decays, unit norms and the state are fp32 throughout.
+// modes 1 and 2, by an output gate (silu of it, or the gate as it comes), and leaves in the operand dtype for the output projection.  Query / key heads may be fewer than
+// value heads (head h reads q / k head h / (heads / qk_heads)).  Inputs are the fp32 outputs of the mixer's projections (modes 1, 2:
+// of its short convolutions); gates, decays, unit norms and the state are fp32 throughout.
 //
 // Rows of a step are a flat list; a span is the run of consecutive rows one sequence brings (span i = rows span_row0[i] ..
 // + span_rows[i], slot and first position = row_seq / row_pos of its first row).  A span at position 0 starts from zeros whatever
@@ -29,16 +31,16 @@ DEV float gs_softplus(float z) { return z > 20.0f ? z : log1pf(expf(z)); }
 #define GS_MAX_NPT 256                       // state rows per thread
 #define GS_MAX_N 1024                        // key channels per head (16 per lane while a wave normalises a token's q and k)
 
-enum { GS_FORGET_WRITES = 0, GS_DELTA = 1 };
+enum { GS_FORGET_WRITES = 0, GS_DELTA = 1, GS_DELTA_CHANNELS = 2 };
 
 struct GatedScanArgs
 {
     const float* q; int ldq;                 // [rows, ldq]: q head g at g * N (mode 0: pre-activation)
-    const float* k; int ldk;                 // mode 1: keys, head g at g * N;  mode 0: the forget gate's pre-activation, head h at h * N
+    const float* k; int ldk;                 // modes 1, 2: keys, head g at g * N;  mode 0: the forget gate's pre-activation, head h at h * N
     const float* v; int ldv;                 // head h at h * P
-    const float* gate; int ldg;              // mode 1: output gate pre-activation, head h at h * P (nullable)
-    const float* beta; int ldb;              // mode 1: [rows, ldb], head h at h (pre-sigmoid)
-    const float* dt; int lddt;               // mode 1: [rows, lddt], head h at h
+    const float* gate; int ldg, gate_ready;  // modes 1, 2: output gate, head h at h * P (nullable): silu(gate), or gate itself (gate_ready)
+    const float* beta; int ldb;              // modes 1, 2: [rows, ldb], head h at h (pre-sigmoid)
+    const float* dt; int lddt;               // mode 1: [rows, lddt], head h at h;  mode 2: the decays, head h at h * N
     const float* dt_bias; const float* a_log;        // mode 1: [heads]
     const float* lower;                      // mode 0: [heads * N]
     const float* norm_w;                     // [P]
@@ -58,6 +60,7 @@ template <typename T, int NPT, int MODE>
 KERNEL void __launch_bounds__(256) gated_scan_kernel(const GatedScanArgs a)
 {
     DYN_SMEM(smem);
+    constexpr bool RULE = MODE != GS_FORGET_WRITES, CHANNELS = MODE == GS_DELTA_CHANNELS;
     const int h = bid_x(), sp = bid_y();
     const int n_tok = a.span_rows[sp], r0 = a.span_row0[sp];
     const int pos0 = a.row_pos[r0];
@@ -67,11 +70,11 @@ KERNEL void __launch_bounds__(256) gated_scan_kernel(const GatedScanArgs a)
     const int p = owner ? t / KS : 0, j = t % KS;
     const int hq = h / (a.heads / a.qk_heads);
     float* s_q = (float*)smem;                                   // [CHUNK, N]
-    float* s_k = s_q + GS_CHUNK * N;                             // [CHUNK, N]  mode 1: unit keys; mode 0: forget gates
+    float* s_k = s_q + GS_CHUNK * N;                             // [CHUNK, N]  modes 1, 2: unit keys; mode 0: forget gates
     float* s_v = s_k + GS_CHUNK * N;                             // [CHUNK, P]
     float* s_o = s_v + GS_CHUNK * P;                             // [CHUNK, P]
     float* s_b = s_o + GS_CHUNK * P;                             // [CHUNK] beta
-    float* s_g = s_b + GS_CHUNK;                                 // [CHUNK] decay
+    float* s_g = s_b + GS_CHUNK;                                 // [CHUNK] decay (mode 2: [CHUNK, N])
     float* st = a.state + ((long long)a.row_seq[r0] * a.heads + h) * (long long)N * P;
     float S[NPT];
     #pragma unroll
@@ -87,7 +90,7 @@ KERNEL void __launch_bounds__(256) gated_scan_kernel(const GatedScanArgs a)
         for (int kk = wave_id(); kk < nc; kk += nt / 64)
         {
             const long long row = r0 + c0 + kk;
-            if (MODE == GS_DELTA)
+            if (RULE)
             {
                 float qv[GS_MAX_N / 64], kv[GS_MAX_N / 64];
                 float sq = 0.0f, sk = 0.0f;
@@ -112,8 +115,10 @@ KERNEL void __launch_bounds__(256) gated_scan_kernel(const GatedScanArgs a)
                 if (lane_id() == 0)
                 {
                     s_b[kk] = gs_sigmoid(a.beta[row * a.ldb + h]);
-                    s_g[kk] = expf(-expf(a.a_log[h]) * gs_softplus(a.dt[row * a.lddt + h] + a.dt_bias[h]));
+                    if (!CHANNELS) s_g[kk] = expf(-expf(a.a_log[h]) * gs_softplus(a.dt[row * a.lddt + h] + a.dt_bias[h]));
                 }
+                if (CHANNELS)
+                    for (int n = lane_id(); n < N; n += 64) s_g[kk * N + n] = a.dt[row * a.lddt + h * N + n];
             }
             else
             {
@@ -132,15 +137,15 @@ KERNEL void __launch_bounds__(256) gated_scan_kernel(const GatedScanArgs a)
         {
             const float vv = s_v[kk * P + p];
             float o = 0.0f;
-            if (MODE == GS_DELTA)
+            if (RULE)
             {
-                const float g = s_g[kk];
+                const float g = CHANNELS ? 1.0f : s_g[kk];
                 float kt = 0.0f;
                 #pragma unroll
                 for (int i = 0; i < NPT; i++)
                 {
                     const int n = j + KS * i;
-                    if (n < N) { S[i] *= g; kt = fmaf(S[i], s_k[kk * N + n], kt); }
+                    if (n < N) { S[i] *= CHANNELS ? s_g[kk * N + n] : g; kt = fmaf(S[i], s_k[kk * N + n], kt); }
                 }
                 for (int m = 1; m < KS; m <<= 1) kt += shfl_xor_f32(kt, m);
                 const float u = s_b[kk] * (vv - kt);
@@ -179,7 +184,7 @@ KERNEL void __launch_bounds__(256) gated_scan_kernel(const GatedScanArgs a)
             for (int pp = lane_id(); pp < P; pp += 64)
             {
                 float o = s_o[kk * P + pp] * rinv * a.norm_w[pp];
-                if (a.gate) { const float gv = a.gate[row * a.ldg + h * P + pp]; o *= gv * gs_sigmoid(gv); }
+                if (a.gate) { const float gv = a.gate[row * a.ldg + h * P + pp]; o *= a.gate_ready ? gv : gv * gs_sigmoid(gv); }
                 gs_st<T>((T*)a.out + row * a.ldo + h * P + pp, o);
             }
         }
@@ -214,6 +219,7 @@ template <int NPT, int MODE, bool FULL>
 KERNEL void __launch_bounds__(256) gated_scan_cols_kernel(const GatedScanArgs a, float* o_raw)
 {
     DYN_SMEM(smem);
+    constexpr bool RULE = MODE != GS_FORGET_WRITES, CHANNELS = MODE == GS_DELTA_CHANNELS;
     const int h = bid_x(), sp = bid_y(), cb = bid_z();
     const int n_tok = a.span_rows[sp], r0 = a.span_row0[sp];
     const int pos0 = a.row_pos[r0];
@@ -228,7 +234,7 @@ KERNEL void __launch_bounds__(256) gated_scan_cols_kernel(const GatedScanArgs a,
     float* s_k = s_q + GSC_CHUNK * N;                            // [CHUNK, N]
     float* s_v = s_k + GSC_CHUNK * N;                            // [CHUNK, COLS]
     float* s_b = s_v + GSC_CHUNK * GSC_COLS;                     // [CHUNK]
-    float* s_g = s_b + GSC_CHUNK;                                // [CHUNK]
+    float* s_g = s_b + GSC_CHUNK;                                // [CHUNK] (mode 2: [CHUNK, N])
     float* st = a.state + ((long long)a.row_seq[r0] * a.heads + h) * (long long)N * P;
     float S[NPT];
     #pragma unroll
@@ -239,8 +245,8 @@ KERNEL void __launch_bounds__(256) gated_scan_cols_kernel(const GatedScanArgs a,
     }
     const float a_neg = MODE == GS_DELTA ? -expf(a.a_log[h]) : 0.0f, dtb = MODE == GS_DELTA ? a.dt_bias[h] : 0.0f;
     // what a thread keeps of the next batch of tokens while the current one is stepped through
-    float rq[GSC_TPW][GSC_MAX_N / 64], rk[GSC_TPW][GSC_MAX_N / 64], rv[2], rb = 0.0f, rd = 0.0f;
-    const int qh = MODE == GS_DELTA ? hq : h;
+    float rq[GSC_TPW][GSC_MAX_N / 64], rk[GSC_TPW][GSC_MAX_N / 64], rg[CHANNELS ? GSC_TPW : 1][GSC_MAX_N / 64], rv[2], rb = 0.0f, rd = 0.0f;
+    const int qh = RULE ? hq : h;
 
     auto request = [&](int c0)
     {
@@ -256,6 +262,7 @@ KERNEL void __launch_bounds__(256) gated_scan_cols_kernel(const GatedScanArgs a,
                 const int n = lane + 64 * e;
                 rq[u][e] = n < N ? a.q[row * a.ldq + qh * N + n] : 0.0f;
                 rk[u][e] = n < N ? a.k[row * a.ldk + qh * N + n] : 0.0f;
+                if (CHANNELS) rg[u][e] = n < N ? a.dt[row * a.lddt + h * N + n] : 0.0f;
             }
         }
         #pragma unroll
@@ -264,11 +271,11 @@ KERNEL void __launch_bounds__(256) gated_scan_cols_kernel(const GatedScanArgs a,
             const int kk = t / GSC_COLS + 16 * u, col = cb * GSC_COLS + t % GSC_COLS;
             rv[u] = (kk < nc && col < P) ? a.v[(long long)(r0 + c0 + kk) * a.ldv + h * P + col] : 0.0f;
         }
-        if (MODE == GS_DELTA && t < GSC_CHUNK)
+        if (RULE && t < GSC_CHUNK)
         {
             const long long row = r0 + c0 + min(t, nc - 1);
             rb = a.beta[row * a.ldb + h];
-            rd = a.dt[row * a.lddt + h];
+            if (!CHANNELS) rd = a.dt[row * a.lddt + h];
         }
     };
 
@@ -277,7 +284,7 @@ KERNEL void __launch_bounds__(256) gated_scan_cols_kernel(const GatedScanArgs a,
         // (the sums of squares of all the wave's tokens first, then their reductions side by side: sixteen independent exchanges
         // instead of a chain of them)
         float sq[GSC_TPW], sk[GSC_TPW];
-        if (MODE == GS_DELTA)
+        if (RULE)
         {
             #pragma unroll
             for (int u = 0; u < GSC_TPW; u++)
@@ -293,14 +300,14 @@ KERNEL void __launch_bounds__(256) gated_scan_cols_kernel(const GatedScanArgs a,
         for (int u = 0; u < GSC_TPW; u++)
         {
             const int kk = wv + 4 * u;
-            if (MODE == GS_DELTA)
+            if (RULE)
             {
                 const float mq = a.q_scale / sqrtf(sq[u] + 1e-6f), mk = 1.0f / sqrtf(sk[u] + 1e-6f);
                 #pragma unroll
                 for (int e = 0; e < GSC_MAX_N / 64; e++)
                 {
                     const int n = lane + 64 * e;
-                    if (n < N) { s_q[kk * N + n] = rq[u][e] * mq; s_k[kk * N + n] = rk[u][e] * mk; }
+                    if (n < N) { s_q[kk * N + n] = rq[u][e] * mq; s_k[kk * N + n] = rk[u][e] * mk; if (CHANNELS) s_g[kk * N + n] = rg[u][e]; }
                 }
             }
             else
@@ -320,10 +327,10 @@ KERNEL void __launch_bounds__(256) gated_scan_cols_kernel(const GatedScanArgs a,
         }
         #pragma unroll
         for (int u = 0; u < 2; u++) s_v[(t / GSC_COLS + 16 * u) * GSC_COLS + t % GSC_COLS] = rv[u];
-        if (MODE == GS_DELTA && t < GSC_CHUNK)
+        if (RULE && t < GSC_CHUNK)
         {
             s_b[t] = gs_sigmoid(rb);
-            s_g[t] = expf(a_neg * gs_softplus(rd + dtb));
+            if (!CHANNELS) s_g[t] = expf(a_neg * gs_softplus(rd + dtb));
         }
     };
 
@@ -343,7 +350,7 @@ KERNEL void __launch_bounds__(256) gated_scan_cols_kernel(const GatedScanArgs a,
         {
             const float vv = s_v[kk * GSC_COLS + pl];
             float o = 0.0f;
-            float kr[NPT], qr[NPT];                              // the token's k (or forget gate) and q at this thread's rows
+            float kr[NPT], qr[NPT], gr[NPT];                     // the token's k (or forget gate), q and decays at this thread's rows
             if (FULL)
             {
                 #pragma unroll
@@ -352,6 +359,12 @@ KERNEL void __launch_bounds__(256) gated_scan_cols_kernel(const GatedScanArgs a,
                     const f32x4 k4 = *(const f32x4*)(s_k + kk * N + j * NPT + 4 * c), q4 = *(const f32x4*)(s_q + kk * N + j * NPT + 4 * c);
                     #pragma unroll
                     for (int e = 0; e < 4; e++) { kr[4 * c + e] = k4[e]; qr[4 * c + e] = q4[e]; }
+                    if (CHANNELS)
+                    {
+                        const f32x4 g4 = *(const f32x4*)(s_g + kk * N + j * NPT + 4 * c);
+                        #pragma unroll
+                        for (int e = 0; e < 4; e++) gr[4 * c + e] = g4[e];
+                    }
                 }
             }
             else
@@ -362,14 +375,15 @@ KERNEL void __launch_bounds__(256) gated_scan_cols_kernel(const GatedScanArgs a,
                     const int n = GSC_ROW(i);
                     kr[i] = n < N ? s_k[kk * N + n] : 0.0f;
                     qr[i] = n < N ? s_q[kk * N + n] : 0.0f;
+                    if (CHANNELS) gr[i] = n < N ? s_g[kk * N + n] : 0.0f;
                 }
             }
-            if (MODE == GS_DELTA)
+            if (RULE)
             {
-                const float g = s_g[kk];
+                const float g = CHANNELS ? 1.0f : s_g[kk];
                 float kt[2] = {0.0f, 0.0f}, o2 = 0.0f;
                 #pragma unroll
-                for (int i = 0; i < NPT; i++) { S[i] *= g; kt[i & 1] = fmaf(S[i], kr[i], kt[i & 1]); }
+                for (int i = 0; i < NPT; i++) { S[i] *= CHANNELS ? gr[i] : g; kt[i & 1] = fmaf(S[i], kr[i], kt[i & 1]); }
                 const float u = s_b[kk] * (vv - row16_allreduce_add(kt[0] + kt[1]));
                 #pragma unroll
                 for (int i = 0; i < NPT; i++)
@@ -403,10 +417,10 @@ KERNEL void __launch_bounds__(256) gated_scan_cols_kernel(const GatedScanArgs a,
     (void)pc;
 }
 
-// grid (rows, heads), one wave: out = o / sqrt(mean(o^2) + eps) * norm_w (* silu(gate))
+// grid (rows, heads), one wave: out = o / sqrt(mean(o^2) + eps) * norm_w (* silu(gate), or the gate as it comes)
 template <typename T>
-KERNEL void __launch_bounds__(64) head_norm_gate_kernel(const float* o_raw, const float* norm_w, const float* gate, int ldg, void* out, int ldo,
-                                                         int heads, int P, float eps)
+KERNEL void __launch_bounds__(64) head_norm_gate_kernel(const float* o_raw, const float* norm_w, const float* gate, int ldg, int gate_ready, void* out,
+                                                         int ldo, int heads, int P, float eps)
 {
     const long long row = bid_x();
     const int h = bid_y();
@@ -418,7 +432,7 @@ KERNEL void __launch_bounds__(64) head_norm_gate_kernel(const float* o_raw, cons
     for (int pp = lane_id(); pp < P; pp += 64)
     {
         float v = o[pp] * rinv * norm_w[pp];
-        if (gate) { const float gv = gate[row * ldg + h * P + pp]; v *= gv * gs_sigmoid(gv); }
+        if (gate) { const float gv = gate[row * ldg + h * P + pp]; v *= gate_ready ? gv : gv * gs_sigmoid(gv); }
         gs_st<T>((T*)out + row * ldo + h * P + pp, v);
     }
 }
@@ -433,18 +447,20 @@ static void gated_scan_launch(const GatedScanArgs& a, int npt, dim3 grid, dim3 b
 
 /* The recurrence over the rows of every span, state read from and left in state[slot of the span][head].  mode 0: k is the forget
    gate's pre-activation (heads x n_key), lower its lower bound, qk_heads == heads; gate / beta / dt / dt_bias / a_log unused.
-   mode 1: q / k hold qk_heads heads, beta / dt one value per head, gate nullable; lower unused.  All inputs fp32. */
+   mode 1: q / k hold qk_heads heads, beta / dt one value per head, gate nullable; lower unused.  mode 2: as mode 1 with dt = the decays
+   themselves, one per head and key channel (heads x n_key); dt_bias / a_log unused.  gate_ready: the gate multiplies as it is (0: its
+   silu).  All inputs fp32. */
 extern "C" int exl2_gated_scan(int mode, const float* q, int ldq, const float* k, int ldk, const float* v, int ldv, const float* gate,
-                               int ldg, const float* beta, int ldb, const float* dt, int lddt, const float* dt_bias, const float* a_log,
+                               int ldg, int gate_ready, const float* beta, int ldb, const float* dt, int lddt, const float* dt_bias, const float* a_log,
                                const float* lower, const float* norm_w, void* out, int ldo, int out_f32, float* state,
                                const int* span_row0, const int* span_rows, int spans, const int* row_seq, const int* row_pos, int heads,
                                int qk_heads, int n_key, int n_val, float q_scale, float eps, void* stream)
 {
-    EXL2_REQUIRE(mode == GS_FORGET_WRITES || mode == GS_DELTA, "gated_scan: mode must be 0 (forget gate writes) or 1 (delta rule)");
+    EXL2_REQUIRE(mode >= GS_FORGET_WRITES && mode <= GS_DELTA_CHANNELS, "gated_scan: mode must be 0 (forget gate writes), 1 (delta rule) or 2 (decay per key channel)");
     EXL2_REQUIRE(q && k && v && norm_w && out && state && span_row0 && span_rows && row_seq && row_pos, "gated_scan: null operand");
     EXL2_REQUIRE(mode != GS_FORGET_WRITES || lower, "gated_scan: the forget gate needs its lower bound");
-    EXL2_REQUIRE(mode != GS_DELTA || (beta && dt && dt_bias && a_log), "gated_scan: the delta rule needs beta and the decay's inputs");
-    EXL2_REQUIRE(heads > 0 && qk_heads > 0 && heads % qk_heads == 0 && (mode == GS_DELTA || qk_heads == heads), "gated_scan: %d heads over %d query / key heads", heads, qk_heads);
+    EXL2_REQUIRE(mode == GS_FORGET_WRITES || (beta && dt && (mode == GS_DELTA_CHANNELS || (dt_bias && a_log))), "gated_scan: the delta rule needs beta and the decay's inputs");
+    EXL2_REQUIRE(heads > 0 && qk_heads > 0 && heads % qk_heads == 0 && (mode != GS_FORGET_WRITES || qk_heads == heads), "gated_scan: %d heads over %d query / key heads", heads, qk_heads);
     EXL2_REQUIRE(n_key > 0 && n_key <= GS_MAX_N && n_val > 0 && n_val <= 256, "gated_scan: state %d x %d", n_key, n_val);
     if (spans <= 0) return EXL2_OK;
     int ks = 1;
@@ -452,11 +468,12 @@ extern "C" int exl2_gated_scan(int mode, const float* q, int ldq, const float* k
     const int npt = (n_key + ks - 1) / ks;
     EXL2_REQUIRE(npt <= GS_MAX_NPT, "gated_scan: state %d x %d needs %d rows per thread (at most %d)", n_key, n_val, npt, GS_MAX_NPT);
     GatedScanArgs a;
-    a.q = q; a.ldq = ldq; a.k = k; a.ldk = ldk; a.v = v; a.ldv = ldv; a.gate = gate; a.ldg = ldg; a.beta = beta; a.ldb = ldb; a.dt = dt;
+    a.q = q; a.ldq = ldq; a.k = k; a.ldk = ldk; a.v = v; a.ldv = ldv; a.gate = gate; a.ldg = ldg; a.gate_ready = gate_ready; a.beta = beta; a.ldb = ldb; a.dt = dt;
     a.lddt = lddt; a.dt_bias = dt_bias; a.a_log = a_log; a.lower = lower; a.norm_w = norm_w; a.out = out; a.ldo = ldo; a.state = state;
     a.span_row0 = span_row0; a.span_rows = span_rows; a.row_seq = row_seq; a.row_pos = row_pos;
     a.heads = heads; a.qk_heads = qk_heads; a.N = n_key; a.P = n_val; a.KS = ks; a.q_scale = q_scale; a.eps = eps;
-    const size_t smem = sizeof(float) * ((size_t)GS_CHUNK * (2 * n_key + 2 * n_val + 2));
+    const size_t smem = sizeof(float) * ((size_t)GS_CHUNK * ((mode == GS_DELTA_CHANNELS ? 3 : 2) * n_key + 2 * n_val + 2));
+    EXL2_REQUIRE(smem <= 160 * 1024, "gated_scan: state %d x %d does not fit the LDS", n_key, n_val);
     if (smem > 48 * 1024)
     {
         static bool attr_done[EXL2_MAX_DEVICES];
@@ -464,12 +481,22 @@ extern "C" int exl2_gated_scan(int mode, const float* q, int ldq, const float* k
         {
             (void)hipFuncSetAttribute((const void*)gated_scan_kernel<u16, GS_MAX_NPT, GS_FORGET_WRITES>, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024);
             (void)hipFuncSetAttribute((const void*)gated_scan_kernel<float, GS_MAX_NPT, GS_FORGET_WRITES>, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024);
-            (void)hipFuncSetAttribute((const void*)gated_scan_kernel<u16, GS_MAX_NPT, GS_DELTA>, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024);
-            (void)hipFuncSetAttribute((const void*)gated_scan_kernel<float, GS_MAX_NPT, GS_DELTA>, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024);
             (void)hipFuncSetAttribute((const void*)gated_scan_kernel<u16, 64, GS_FORGET_WRITES>, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024);
             (void)hipFuncSetAttribute((const void*)gated_scan_kernel<float, 64, GS_FORGET_WRITES>, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024);
+            (void)hipFuncSetAttribute((const void*)gated_scan_kernel<u16, 16, GS_FORGET_WRITES>, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024);
+            (void)hipFuncSetAttribute((const void*)gated_scan_kernel<float, 16, GS_FORGET_WRITES>, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024);
+            (void)hipFuncSetAttribute((const void*)gated_scan_kernel<u16, GS_MAX_NPT, GS_DELTA>, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024);
+            (void)hipFuncSetAttribute((const void*)gated_scan_kernel<float, GS_MAX_NPT, GS_DELTA>, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024);
             (void)hipFuncSetAttribute((const void*)gated_scan_kernel<u16, 64, GS_DELTA>, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024);
             (void)hipFuncSetAttribute((const void*)gated_scan_kernel<float, 64, GS_DELTA>, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024);
+            (void)hipFuncSetAttribute((const void*)gated_scan_kernel<u16, 16, GS_DELTA>, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024);
+            (void)hipFuncSetAttribute((const void*)gated_scan_kernel<float, 16, GS_DELTA>, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024);
+            (void)hipFuncSetAttribute((const void*)gated_scan_kernel<u16, GS_MAX_NPT, GS_DELTA_CHANNELS>, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024);
+            (void)hipFuncSetAttribute((const void*)gated_scan_kernel<float, GS_MAX_NPT, GS_DELTA_CHANNELS>, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024);
+            (void)hipFuncSetAttribute((const void*)gated_scan_kernel<u16, 64, GS_DELTA_CHANNELS>, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024);
+            (void)hipFuncSetAttribute((const void*)gated_scan_kernel<float, 64, GS_DELTA_CHANNELS>, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024);
+            (void)hipFuncSetAttribute((const void*)gated_scan_kernel<u16, 16, GS_DELTA_CHANNELS>, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024);
+            (void)hipFuncSetAttribute((const void*)gated_scan_kernel<float, 16, GS_DELTA_CHANNELS>, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024);
         }
     }
     const dim3 grid(heads, spans), block((n_val * ks + 63) / 64 * 64);
@@ -477,6 +504,11 @@ extern "C" int exl2_gated_scan(int mode, const float* q, int ldq, const float* k
     {
         if (out_f32) gated_scan_launch<float, GS_DELTA>(a, npt, grid, block, smem, stream);
         else gated_scan_launch<u16, GS_DELTA>(a, npt, grid, block, smem, stream);
+    }
+    else if (mode == GS_DELTA_CHANNELS)
+    {
+        if (out_f32) gated_scan_launch<float, GS_DELTA_CHANNELS>(a, npt, grid, block, smem, stream);
+        else gated_scan_launch<u16, GS_DELTA_CHANNELS>(a, npt, grid, block, smem, stream);
     }
     else
     {
@@ -497,25 +529,25 @@ extern "C" int exl2_gated_scan_cols_supported(int n_key, int n_val)
    flight behind the current one; the head norm (and gate) as a second launch over o_raw (scratch, fp32 [rows, heads * n_val]).  Same
    operands and results as exl2_gated_scan (sums associate differently: results agree to rounding). */
 extern "C" int exl2_gated_scan_cols(int mode, const float* q, int ldq, const float* k, int ldk, const float* v, int ldv, const float* gate,
-                                    int ldg, const float* beta, int ldb, const float* dt, int lddt, const float* dt_bias,
+                                    int ldg, int gate_ready, const float* beta, int ldb, const float* dt, int lddt, const float* dt_bias,
                                     const float* a_log, const float* lower, const float* norm_w, void* out, int ldo, int out_f32,
                                     float* state, const int* span_row0, const int* span_rows, int spans, const int* row_seq,
                                     const int* row_pos, int rows, float* o_raw, int heads, int qk_heads, int n_key, int n_val,
                                     float q_scale, float eps, void* stream)
 {
-    EXL2_REQUIRE(mode == GS_FORGET_WRITES || mode == GS_DELTA, "gated_scan_cols: mode must be 0 (forget gate writes) or 1 (delta rule)");
+    EXL2_REQUIRE(mode >= GS_FORGET_WRITES && mode <= GS_DELTA_CHANNELS, "gated_scan_cols: mode must be 0 (forget gate writes), 1 (delta rule) or 2 (decay per key channel)");
     EXL2_REQUIRE(q && k && v && norm_w && out && state && o_raw && span_row0 && span_rows && row_seq && row_pos, "gated_scan_cols: null operand");
     EXL2_REQUIRE(mode != GS_FORGET_WRITES || lower, "gated_scan_cols: the forget gate needs its lower bound");
-    EXL2_REQUIRE(mode != GS_DELTA || (beta && dt && dt_bias && a_log), "gated_scan_cols: the delta rule needs beta and the decay's inputs");
-    EXL2_REQUIRE(heads > 0 && qk_heads > 0 && heads % qk_heads == 0 && (mode == GS_DELTA || qk_heads == heads), "gated_scan_cols: %d heads over %d query / key heads", heads, qk_heads);
+    EXL2_REQUIRE(mode == GS_FORGET_WRITES || (beta && dt && (mode == GS_DELTA_CHANNELS || (dt_bias && a_log))), "gated_scan_cols: the delta rule needs beta and the decay's inputs");
+    EXL2_REQUIRE(heads > 0 && qk_heads > 0 && heads % qk_heads == 0 && (mode != GS_FORGET_WRITES || qk_heads == heads), "gated_scan_cols: %d heads over %d query / key heads", heads, qk_heads);
     EXL2_REQUIRE(exl2_gated_scan_cols_supported(n_key, n_val), "gated_scan_cols: state %d x %d", n_key, n_val);
     if (spans <= 0 || rows <= 0) return EXL2_OK;
     GatedScanArgs a;
-    a.q = q; a.ldq = ldq; a.k = k; a.ldk = ldk; a.v = v; a.ldv = ldv; a.gate = gate; a.ldg = ldg; a.beta = beta; a.ldb = ldb; a.dt = dt;
+    a.q = q; a.ldq = ldq; a.k = k; a.ldk = ldk; a.v = v; a.ldv = ldv; a.gate = gate; a.ldg = ldg; a.gate_ready = gate_ready; a.beta = beta; a.ldb = ldb; a.dt = dt;
     a.lddt = lddt; a.dt_bias = dt_bias; a.a_log = a_log; a.lower = lower; a.norm_w = norm_w; a.out = out; a.ldo = ldo; a.state = state;
     a.span_row0 = span_row0; a.span_rows = span_rows; a.row_seq = row_seq; a.row_pos = row_pos;
     a.heads = heads; a.qk_heads = qk_heads; a.N = n_key; a.P = n_val; a.KS = GSC_KS; a.q_scale = q_scale; a.eps = eps;
-    const size_t smem = sizeof(float) * ((size_t)GSC_CHUNK * (2 * n_key + GSC_COLS + 2));
+    const size_t smem = sizeof(float) * ((size_t)GSC_CHUNK * ((mode == GS_DELTA_CHANNELS ? 3 : 2) * n_key + GSC_COLS + 2));
     if (smem > 48 * 1024)
     {
         static bool attr_done[EXL2_MAX_DEVICES];
@@ -525,6 +557,10 @@ extern "C" int exl2_gated_scan_cols(int mode, const float* q, int ldq, const flo
             (void)hipFuncSetAttribute((const void*)gated_scan_cols_kernel<16, GS_DELTA, false>, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024);
             (void)hipFuncSetAttribute((const void*)gated_scan_cols_kernel<16, GS_FORGET_WRITES, true>, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024);
             (void)hipFuncSetAttribute((const void*)gated_scan_cols_kernel<16, GS_DELTA, true>, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024);
+            (void)hipFuncSetAttribute((const void*)gated_scan_cols_kernel<16, GS_DELTA_CHANNELS, false>, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024);
+            (void)hipFuncSetAttribute((const void*)gated_scan_cols_kernel<16, GS_DELTA_CHANNELS, true>, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024);
+            (void)hipFuncSetAttribute((const void*)gated_scan_cols_kernel<8, GS_DELTA_CHANNELS, false>, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024);
+            (void)hipFuncSetAttribute((const void*)gated_scan_cols_kernel<8, GS_DELTA_CHANNELS, true>, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024);
         }
     }
     const dim3 grid(heads, spans, (n_val + GSC_COLS - 1) / GSC_COLS);
@@ -536,14 +572,18 @@ extern "C" int exl2_gated_scan_cols(int mode, const float* q, int ldq, const flo
     {
         if (npt <= 4) GSC_LAUNCH(4, GS_DELTA); else if (npt <= 8) GSC_LAUNCH(8, GS_DELTA); else GSC_LAUNCH(16, GS_DELTA);
     }
+    else if (mode == GS_DELTA_CHANNELS)
+    {
+        if (npt <= 4) GSC_LAUNCH(4, GS_DELTA_CHANNELS); else if (npt <= 8) GSC_LAUNCH(8, GS_DELTA_CHANNELS); else GSC_LAUNCH(16, GS_DELTA_CHANNELS);
+    }
     else
     {
         if (npt <= 4) GSC_LAUNCH(4, GS_FORGET_WRITES); else if (npt <= 8) GSC_LAUNCH(8, GS_FORGET_WRITES); else GSC_LAUNCH(16, GS_FORGET_WRITES);
     }
 #undef GSC_LAUNCH
-    const float* gt = mode == GS_DELTA ? gate : nullptr;
-    if (out_f32) LAUNCH(head_norm_gate_kernel<float>, dim3(rows, heads), dim3(64), 0, stream, (const float*)o_raw, norm_w, gt, ldg, out, ldo, heads, n_val, eps);
-    else LAUNCH(head_norm_gate_kernel<u16>, dim3(rows, heads), dim3(64), 0, stream, (const float*)o_raw, norm_w, gt, ldg, out, ldo, heads, n_val, eps);
+    const float* gt = mode != GS_FORGET_WRITES ? gate : nullptr;
+    if (out_f32) LAUNCH(head_norm_gate_kernel<float>, dim3(rows, heads), dim3(64), 0, stream, (const float*)o_raw, norm_w, gt, ldg, gate_ready, out, ldo, heads, n_val, eps);
+    else LAUNCH(head_norm_gate_kernel<u16>, dim3(rows, heads), dim3(64), 0, stream, (const float*)o_raw, norm_w, gt, ldg, gate_ready, out, ldo, heads, n_val, eps);
     HIP_TRY(hipGetLastError());
     return EXL2_OK;
 }

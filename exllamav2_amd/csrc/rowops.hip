@@ -9,10 +9,12 @@
 //   * the sandwich-normed residual step  x <- x + mult n_g(sublayer) w_out  with the grouped RMS norm  n_g(x) w_in  that feeds the next
 //     sublayer (and, for single-token steps, the short convolution over the last normed rows of the sequence),
 //   * the residual step of a layer whose mixer and feed-forward read ONE norm and pass gates of their own,
-//     x <- x + t sigmoid(g1) + (weighted expert sum) sigmoid(g2), with the RMS norm that feeds the next layer,
+//     x <- x + t sigmoid(g1) + (weighted expert sum) sigmoid(g2), with the RMS norm that feeds the next layer (without gates and with a
+//     factor in front of both terms: the residual step of a plain pre-norm layer),
 //   * a token embedding plus a hashed (previous token, token) embedding under a grouped RMS norm (the previous token kept per slot),
 //   * the sparse-MoE router (softmax over all experts, selection by score + correction, weights from the uncorrected scores; or
-//     sigmoid scores, selection and weights by the scores themselves, maybe among the experts of the best groups only) and the per-expert row lists the grouped linear reads.
+//     sigmoid scores, selection and weights by the scores themselves, maybe among the experts of the best groups only; or selection by the
+//     logits, weights = softmax over the chosen ones) and the per-expert row lists the grouped linear reads.
 // Element type T of weights / operand copies: u16 = bfloat16 bits, float.
 #include "hw.h"
 #include "errors.h"
@@ -561,9 +563,9 @@ KERNEL void __launch_bounds__(256) sandwich_norm_vec_kernel(const SandwichArgs a
 
 // ---- gated residual step of a parallel layer --------------------------------------------------------------------------------------
 // n(v) = v / sqrt(mean(v^2) + eps).  One launch per row does
-//     x <- x + t sigmoid(g1) + sigmoid(g2) sum_k moe_w[k] moe_row[k],   t = y, or ya n(y) w_y + yb n(y2) w_y2 (two mixers side by side)
+//     x <- x + mult (t sigmoid(g1) + sigmoid(g2) sum_k moe_w[k] moe_row[k]),  t = y, or ya n(y) w_y + yb n(y2) w_y2 (two mixers side by side)
 //     x <- x + embed[id]  (ids nullable; `init`: x starts as embed[id], nothing is read from the stream)
-//     out = n(x) w_in                                                    (out nullable: only the additions)
+//     out = n(x) w_in  (out nullable: only the additions; w_in nullable: x itself, what a linear of the stream reads), rows ldo apart
 // Either addition may be absent (y, moe_y nullable) and so may the gates (nullable: 1).
 
 struct GatedResArgs
@@ -573,9 +575,9 @@ struct GatedResArgs
     const float* g1; const float* g2; int ldg;               // gates in front of the sigmoid: [rows, ldg]
     const float* moe_y; const float* moe_w; int top;         // [rows * top, width], [rows, top]
     const void* table; const int* ids; int vocab, init;
-    const void* w_in; void* out; int out_f32;
+    const void* w_in; void* out; int out_f32, ldo;
     const int* row_idx;                                      // nullable: output row r is made from stream row row_idx[r] (no addition then)
-    int width; float eps;
+    int width; float eps, mult;
 };
 
 DEV float ro_sigmoid(float z) { return 1.0f / (1.0f + expf(-z)); }
@@ -614,13 +616,13 @@ KERNEL void __launch_bounds__(256) gated_residual_kernel(const GatedResArgs a)
         {
             float t = a.y[src * a.width + i];
             if (a.wy) t = t * my * ro_ld<T>((const T*)a.wy + i) + a.y2[src * a.width + i] * my2 * ro_ld<T>((const T*)a.wy2 + i);
-            xv = fmaf(t, a.g1 ? ro_sigmoid(a.g1[src * a.ldg + i]) : 1.0f, xv);
+            xv = fmaf(t, a.g1 ? a.mult * ro_sigmoid(a.g1[src * a.ldg + i]) : a.mult, xv);
         }
         if (a.moe_y)
         {
             float t = 0.0f;
             for (int k = 0; k < a.top; k++) t = fmaf(a.moe_w[src * a.top + k], a.moe_y[(src * a.top + k) * a.width + i], t);
-            xv = fmaf(t, a.g2 ? ro_sigmoid(a.g2[src * a.ldg + i]) : 1.0f, xv);
+            xv = fmaf(t, a.g2 ? a.mult * ro_sigmoid(a.g2[src * a.ldg + i]) : a.mult, xv);
         }
         if (er) xv += ro_ld<T>(er + i);
         if (adds) xr[i] = xv;
@@ -632,8 +634,8 @@ KERNEL void __launch_bounds__(256) gated_residual_kernel(const GatedResArgs a)
     const float rinv = 1.0f / sqrtf(ss / (float)a.width + a.eps);
     for (int i = tid(); i < a.width; i += 256)
     {
-        const float o = v[i] * rinv * ro_ld<T>((const T*)a.w_in + i);
-        if (a.out_f32) ((float*)a.out)[(long long)r * a.width + i] = o; else ro_st<T>((T*)a.out + (long long)r * a.width + i, o);
+        const float o = a.w_in ? v[i] * rinv * ro_ld<T>((const T*)a.w_in + i) : v[i];
+        if (a.out_f32) ((float*)a.out)[(long long)r * a.ldo + i] = o; else ro_st<T>((T*)a.out + (long long)r * a.ldo + i, o);
     }
 }
 
@@ -686,7 +688,7 @@ KERNEL void __launch_bounds__(256) gated_residual_vec_kernel(const GatedResArgs 
             if (a.g2) g2[e] = *(const f32x4*)(a.g2 + src * a.ldg + i);
         }
         if (er) ev[e] = ro_ld4<T>(er + i);
-        if (a.out) wi[e] = ro_ld4<T>((const T*)a.w_in + i);
+        if (a.w_in) wi[e] = ro_ld4<T>((const T*)a.w_in + i);
     }
     float my = 1.0f, my2 = 0.0f;
     if (a.wy)
@@ -716,14 +718,14 @@ KERNEL void __launch_bounds__(256) gated_residual_vec_kernel(const GatedResArgs 
             if (a.y)
             {
                 const float t = a.wy ? yv[e][k] * my * wy[e][k] + y2v[e][k] * my2 * wy2[e][k] : yv[e][k];
-                x = fmaf(t, a.g1 ? ro_sigmoid(g1[e][k]) : 1.0f, x);
+                x = fmaf(t, a.g1 ? a.mult * ro_sigmoid(g1[e][k]) : a.mult, x);
             }
             if (a.moe_y)
             {
                 float t = 0.0f;
                 #pragma unroll
                 for (int j = 0; j < GR_MAX_TOP; j++) t = fmaf(mw[j], mv[e][j][k], t);
-                x = fmaf(t, a.g2 ? ro_sigmoid(g2[e][k]) : 1.0f, x);
+                x = fmaf(t, a.g2 ? a.mult * ro_sigmoid(g2[e][k]) : a.mult, x);
             }
             x += ev[e][k];
             xv[e][k] = x;
@@ -743,9 +745,9 @@ KERNEL void __launch_bounds__(256) gated_residual_vec_kernel(const GatedResArgs 
         const int i = 4 * (tid() + 256 * e);
         f32x4 o;
         #pragma unroll
-        for (int k = 0; k < 4; k++) o[k] = xv[e][k] * rinv * wi[e][k];
-        if (a.out_f32) *(f32x4*)((float*)a.out + (long long)r * a.width + i) = o;
-        else *(u32x2*)((u16*)a.out + (long long)r * a.width + i) =
+        for (int k = 0; k < 4; k++) o[k] = a.w_in ? xv[e][k] * rinv * wi[e][k] : xv[e][k];
+        if (a.out_f32) *(f32x4*)((float*)a.out + (long long)r * a.ldo + i) = o;
+        else *(u32x2*)((u16*)a.out + (long long)r * a.ldo + i) =
                  (u32x2){(u32)f32_to_bf16(o[0]) | ((u32)f32_to_bf16(o[1]) << 16), (u32)f32_to_bf16(o[2]) | ((u32)f32_to_bf16(o[3]) << 16)};
     }
 }
@@ -754,12 +756,13 @@ KERNEL void __launch_bounds__(256) gated_residual_vec_kernel(const GatedResArgs 
 // x = n_g(table[t] * scale + pair[(t' mul_prev + t mul_cur) mod buckets]) w, t' = the sequence's previous token: the row in front
 // when that belongs to the same sequence, else what the slot keeps (prev_tok int32 [slots]); row `buckets` of the pair table at
 // position 0.  fused (single-row spans): the slot takes the row's token here, otherwise token_state_kernel does after the launch.
+// xh (nullable): a copy of the row in the operand dtype, rows ldxh apart.
 
 struct EmbedPairArgs
 {
     const void* table; const void* pair; const void* w;         // pair, w nullable
     const int* ids; int* prev_tok; const int* row_seq; const int* row_pos;
-    float* x;
+    float* x; void* xh; int ldxh;
     int width, vocab, buckets, mul_prev, mul_cur, groups, fused; float scale, eps;
 };
 
@@ -787,7 +790,11 @@ KERNEL void __launch_bounds__(256) embed_pair_kernel(const EmbedPairArgs a)
         float t = ro_ld<T>(src + i) * a.scale;
         if (psrc) t += ro_ld<T>(psrc + i);
         v[i] = t;
-        if (!a.w) xr[i] = t;
+        if (!a.w)
+        {
+            xr[i] = t;
+            if (a.xh) ro_st<T>((T*)a.xh + (long long)r * a.ldxh + i, t);
+        }
     }
     if (a.w)
     {
@@ -798,7 +805,12 @@ KERNEL void __launch_bounds__(256) embed_pair_kernel(const EmbedPairArgs a)
             for (int i = g * gs + tid(); i < (g + 1) * gs; i += 256) ss = fmaf(v[i], v[i], ss);
             ss = block_sum_256(ss, part);
             const float rinv = 1.0f / sqrtf(ss / (float)gs + a.eps);
-            for (int i = g * gs + tid(); i < (g + 1) * gs; i += 256) xr[i] = v[i] * rinv * ro_ld<T>((const T*)a.w + i);
+            for (int i = g * gs + tid(); i < (g + 1) * gs; i += 256)
+            {
+                const float o = v[i] * rinv * ro_ld<T>((const T*)a.w + i);
+                xr[i] = o;
+                if (a.xh) ro_st<T>((T*)a.xh + (long long)r * a.ldxh + i, o);
+            }
         }
     }
     else block_sync();
@@ -816,22 +828,25 @@ KERNEL void __launch_bounds__(64) token_state_kernel(const int* ids, int* prev_t
 
 // ---- router -----------------------------------------------------------------------------------------------------------------
 // One wave per token.  logits fp32 [rows, n_total]; scores = softmax over all n_total; the `top` largest (score + correction) win
-// (first index on a tie); weight = score / (sum of the chosen scores + 1e-20) * scale.  sigmoid_scores: scores = sigmoid(logits),
-// each on its own, and the weights are the chosen scores times scale (no renormalisation).  Rows of ids / wts are `ld` values apart;
+// (first index on a tie); weight = score / (sum of the chosen scores + 1e-20) * scale.  mode 1: scores = sigmoid(logits),
+// each on its own, and the weights are the chosen scores times scale (no renormalisation).  mode 2: the `top` largest logits win and
+// their weights are the softmax over the chosen logits times scale.  Rows of ids / wts are `ld` values apart;
 // group_keep < group_count: the experts stand in group_count equal groups of neighbours, a group scores the sum of its two largest
 // selection scores, and only the experts of the group_keep best groups can be chosen.  Rows of logits are ldl values apart.
-// extra_id >= 0: column `top` of every row names that expert with weight 1 (an expert every token uses, run with the chosen ones).
+// extra > 0: columns top .. top + extra - 1 of every row name the experts extra_id .. extra_id + extra - 1 (what every token uses, run
+// with the chosen ones) with weight 1, or sigmoid(column extra_col of the row's logits) where extra_col >= 0.
 
 #define ROUTE_MAX_PER_LANE 8
 
 KERNEL void __launch_bounds__(64) moe_route_kernel(const float* logits, int ldl, const float* correction, int* ids, float* wts,
-                                                    int n_total, int top, float scale, int sigmoid_scores, int ld, int extra_id,
-                                                    int group_count, int group_keep)
+                                                    int n_total, int top, float scale, int mode, int ld, int extra_id, int extra,
+                                                    int extra_col, int group_count, int group_keep)
 {
     SHARED float g_s[64 * ROUTE_MAX_PER_LANE];           // scores, when experts form groups
     SHARED float g_sum[64 * ROUTE_MAX_PER_LANE];         // group scores
     const int r = bid_x();
     const int lane = lane_id();
+    const bool sigmoid_scores = mode == 1;
     float s[ROUTE_MAX_PER_LANE], c[ROUTE_MAX_PER_LANE];
     float mx = -INFINITY;
     #pragma unroll
@@ -847,17 +862,18 @@ KERNEL void __launch_bounds__(64) moe_route_kernel(const float* logits, int ldl,
     for (int i = 0; i < ROUTE_MAX_PER_LANE; i++)
     {
         const int e = lane + 64 * i;
+        c[i] = s[i];                                     // the logit
         if (sigmoid_scores) s[i] = e < n_total ? 1.0f / (1.0f + expf(-s[i])) : 0.0f;
         else s[i] = e < n_total ? expf(s[i] - mx) : 0.0f;
         sum += s[i];
     }
-    sum = sigmoid_scores ? 1.0f : wave_allreduce_add(sum);
+    sum = mode == 0 ? wave_allreduce_add(sum) : 1.0f;
     #pragma unroll
     for (int i = 0; i < ROUTE_MAX_PER_LANE; i++)
     {
         const int e = lane + 64 * i;
         s[i] = s[i] / sum;
-        c[i] = e < n_total ? s[i] + (correction ? correction[e] : 0.0f) : -INFINITY;
+        if (mode != 2) c[i] = e < n_total ? s[i] + (correction ? correction[e] : 0.0f) : -INFINITY;
     }
     if (group_keep < group_count)
     {
@@ -918,7 +934,11 @@ KERNEL void __launch_bounds__(64) moe_route_kernel(const float* logits, int ldl,
         ids[r * ld + lane] = my_id;
         wts[r * ld + lane] = sigmoid_scores ? my_w * scale : my_w / (chosen_sum + 1e-20f) * scale;
     }
-    if (extra_id >= 0 && lane == 0) { ids[r * ld + top] = extra_id; wts[r * ld + top] = 1.0f; }
+    if (lane < extra)
+    {
+        ids[r * ld + top + lane] = extra_id + lane;
+        wts[r * ld + top + lane] = extra_col >= 0 ? 1.0f / (1.0f + expf(-logits[(long long)r * ldl + extra_col])) : 1.0f;
+    }
 }
 
 // per-expert row lists for the grouped linear, in pair order.  Two launches of one workgroup per expert: counts (256 threads, ballot +
@@ -1048,13 +1068,13 @@ extern "C" int exl2_add_layer_norm(float* x, const float* y, const void* w, cons
 }
 
 static int moe_route_any(const float* logits, const float* correction, int* ids, float* wts, int rows, int n_total, int top,
-                         float scale, int n_real, int* grp_count, int* grp_offset, int* grp_rows, int sigmoid_scores, int shared_slot,
+                         float scale, int n_real, int* grp_count, int* grp_offset, int* grp_rows, int mode, int extra, int extra_col,
                          int ldl, int group_count, int group_keep, void* stream);
 
 extern "C" int exl2_moe_route_scored(const float* logits, const float* correction, int* ids, float* wts, int rows, int n_total, int top,
                                      float scale, int n_real, int* grp_count, int* grp_offset, int* grp_rows, void* stream)
 {
-    return moe_route_any(logits, correction, ids, wts, rows, n_total, top, scale, n_real, grp_count, grp_offset, grp_rows, 0, 0,
+    return moe_route_any(logits, correction, ids, wts, rows, n_total, top, scale, n_real, grp_count, grp_offset, grp_rows, 0, 0, -1,
                          n_total, 1, 1, stream);
 }
 
@@ -1062,14 +1082,14 @@ extern "C" int exl2_moe_route_sigmoid(const float* logits, int* ids, float* wts,
                                       int shared_slot, int* grp_count, int* grp_offset, int* grp_rows, void* stream)
 {
     return moe_route_any(logits, nullptr, ids, wts, rows, n_total, top, scale, n_total + (shared_slot ? 1 : 0), grp_count, grp_offset,
-                         grp_rows, 1, shared_slot, n_total, 1, 1, stream);
+                         grp_rows, 1, shared_slot ? 1 : 0, -1, n_total, 1, 1, stream);
 }
 
 static int moe_route_any(const float* logits, const float* correction, int* ids, float* wts, int rows, int n_total, int top,
-                         float scale, int n_real, int* grp_count, int* grp_offset, int* grp_rows, int sigmoid_scores, int shared_slot,
+                         float scale, int n_real, int* grp_count, int* grp_offset, int* grp_rows, int mode, int extra, int extra_col,
                          int ldl, int group_count, int group_keep, void* stream)
 {
-    const int ld = top + (shared_slot ? 1 : 0);                  // values per row of ids / wts
+    const int ld = top + extra;                                  // values per row of ids / wts
     EXL2_REQUIRE(logits && ids && wts, "moe_route_scored: null operand");
     EXL2_REQUIRE(n_total > 0 && n_total <= 64 * ROUTE_MAX_PER_LANE, "moe_route_scored: %d experts (at most %d)", n_total, 64 * ROUTE_MAX_PER_LANE);
     EXL2_REQUIRE(top > 0 && top <= 64 && top <= n_total, "moe_route_scored: top %d of %d", top, n_total);
@@ -1077,10 +1097,11 @@ static int moe_route_any(const float* logits, const float* correction, int* ids,
     EXL2_REQUIRE(group_count > 0 && group_keep > 0 && group_keep <= group_count && n_total % group_count == 0
                      && top <= group_keep * (n_total / group_count),
                  "moe_route: top %d of %d experts in %d groups, %d kept", top, n_total, group_count, group_keep);
-    EXL2_REQUIRE(n_real >= 0 && n_real <= n_total + (shared_slot ? 1 : 0), "moe_route_scored: %d experts with weights of %d", n_real, n_total);
+    EXL2_REQUIRE(extra >= 0 && extra <= 64 && extra_col < ldl, "moe_route: %d experts for every token, gated by column %d of %d", extra, extra_col, ldl);
+    EXL2_REQUIRE(n_real >= 0 && n_real <= n_total + extra, "moe_route_scored: %d experts with weights of %d", n_real, n_total);
     if (rows <= 0) return EXL2_OK;
-    LAUNCH(moe_route_kernel, dim3(rows), dim3(64), 0, stream, logits, ldl, correction, ids, wts, n_total, top, scale, sigmoid_scores, ld,
-           shared_slot ? n_total : -1, group_count, group_keep);
+    LAUNCH(moe_route_kernel, dim3(rows), dim3(64), 0, stream, logits, ldl, correction, ids, wts, n_total, top, scale, mode, ld,
+           n_total, extra, extra_col, group_count, group_keep);
     if (grp_count)
     {
         EXL2_REQUIRE(grp_offset && grp_rows, "moe_route_scored: grouped lists need offsets and rows");
@@ -1097,8 +1118,15 @@ static int moe_route_any(const float* logits, const float* correction, int* ids,
 extern "C" int exl2_moe_route_grouped(const float* logits, int ldl, int* ids, float* wts, int rows, int n_total, int top, float scale,
                                       int group_count, int group_keep, int* grp_count, int* grp_offset, int* grp_rows, void* stream)
 {
-    return moe_route_any(logits, nullptr, ids, wts, rows, n_total, top, scale, n_total, grp_count, grp_offset, grp_rows, 1, 0, ldl,
+    return moe_route_any(logits, nullptr, ids, wts, rows, n_total, top, scale, n_total, grp_count, grp_offset, grp_rows, 1, 0, -1, ldl,
                          group_count, group_keep, stream);
+}
+
+extern "C" int exl2_moe_route_chosen(const float* logits, int ldl, int* ids, float* wts, int rows, int n_total, int top, float scale,
+                                     int extra, int extra_col, int* grp_count, int* grp_offset, int* grp_rows, void* stream)
+{
+    return moe_route_any(logits, nullptr, ids, wts, rows, n_total, top, scale, n_total + extra, grp_count, grp_offset, grp_rows, 2, extra,
+                         extra_col, ldl, 1, 1, stream);
 }
 
 extern "C" int exl2_add_rms_shift(float* x, const float* y, const float* moe_y, int top, float gain, float eps, const void* shift,
@@ -1215,13 +1243,13 @@ extern "C" int exl2_sandwich_norm(float* x, const float* y, float ya, const floa
 extern "C" int exl2_gated_residual(float* x, const float* y, const float* y2, const void* wy, const void* wy2, float ya, float yb,
                                    const float* g1, const float* g2, int ldg, const float* moe_y, const float* moe_w, int top,
                                    const void* table, const int* ids, int vocab, int init, const void* w_in, void* out, int out_f32,
-                                   const int* row_idx, int dtype, int rows, int width, float eps, void* stream)
+                                   int ldo, const int* row_idx, int dtype, int rows, int width, float mult, float eps, void* stream)
 {
     EXL2_REQUIRE(x, "gated_residual: null stream");
     EXL2_REQUIRE(dtype == 0 || dtype == 1, "gated_residual: dtype must be 0 (bfloat16) or 1 (float32)");
     const bool adds = y || moe_y || ids;
     EXL2_REQUIRE(adds || out, "gated_residual: neither an addition nor a norm");
-    EXL2_REQUIRE(!out || w_in, "gated_residual: an output needs the weight of its norm");
+    EXL2_REQUIRE(!out || ldo >= width, "gated_residual: output rows of %d values %d apart", width, ldo);
     EXL2_REQUIRE((wy == nullptr) == (y2 == nullptr) && (wy == nullptr) == (wy2 == nullptr) && (!wy || y),
                  "gated_residual: two normed results come with both weights");
     EXL2_REQUIRE(!moe_y || (moe_w && top > 0), "gated_residual: expert outputs need their weights and their count per row");
@@ -1234,9 +1262,9 @@ extern "C" int exl2_gated_residual(float* x, const float* y, const float* y2, co
     GatedResArgs a;
     a.x = x; a.y = y; a.y2 = y2; a.wy = wy; a.wy2 = wy2; a.ya = ya; a.yb = yb; a.g1 = g1; a.g2 = g2; a.ldg = ldg; a.moe_y = moe_y;
     a.moe_w = moe_w; a.top = top; a.table = table; a.ids = ids; a.vocab = vocab; a.init = init; a.w_in = w_in; a.out = out;
-    a.out_f32 = out_f32 || dtype == 1; a.row_idx = row_idx; a.width = width; a.eps = eps;
+    a.out_f32 = out_f32 || dtype == 1; a.ldo = ldo; a.row_idx = row_idx; a.width = width; a.eps = eps; a.mult = mult;
     const auto al16 = [](const void* p) { return ((uintptr_t)p % 16) == 0; };
-    const bool vec = width % 4 == 0 && width <= 256 * 4 * 4 && (!moe_y || top <= GR_MAX_TOP) && ldg % 4 == 0 && al16(x) && al16(y) && al16(y2)
+    const bool vec = width % 4 == 0 && width <= 256 * 4 * 4 && (!moe_y || top <= GR_MAX_TOP) && ldg % 4 == 0 && (!out || ldo % 4 == 0) && al16(x) && al16(y) && al16(y2)
                      && al16(wy) && al16(wy2) && al16(g1) && al16(g2) && al16(moe_y) && al16(table) && al16(w_in) && al16(out);
     if (vec)
     {
@@ -1274,7 +1302,7 @@ extern "C" int exl2_gated_residual(float* x, const float* y, const float* y2, co
 
 extern "C" int exl2_embed_pair(const void* table, const void* pair, const void* w, const int* ids, int* prev_tok, const int* row_seq,
                                const int* row_pos, const int* span_row0, const int* span_rows, int spans, int max_span_rows, float* x,
-                               int dtype, int rows, int width, int vocab, int buckets, int mul_prev, int mul_cur, float scale, int groups,
+                               void* xh, int ldxh, int dtype, int rows, int width, int vocab, int buckets, int mul_prev, int mul_cur, float scale, int groups,
                                float eps, void* stream)
 {
     EXL2_REQUIRE(table && ids && x && row_seq && row_pos, "embed_pair: null operand");
@@ -1282,10 +1310,12 @@ extern "C" int exl2_embed_pair(const void* table, const void* pair, const void* 
     EXL2_REQUIRE(!pair || (prev_tok && buckets > 0 && span_row0 && span_rows && spans > 0 && max_span_rows > 0),
                  "embed_pair: the pair table needs its size, the slots' tokens and the step's spans");
     EXL2_REQUIRE(width > 0 && vocab > 0 && (!w || (groups > 0 && width % groups == 0)), "embed_pair: bad shape");
+    EXL2_REQUIRE(!xh || ldxh >= width, "embed_pair: copies of %d values %d apart", width, ldxh);
     EXL2_REQUIRE((size_t)width * 4 <= 160 * 1024 - 64, "embed_pair: row of %d values does not fit the LDS", width);
     if (rows <= 0) return EXL2_OK;
     EmbedPairArgs a;
     a.table = table; a.pair = pair; a.w = w; a.ids = ids; a.prev_tok = prev_tok; a.row_seq = row_seq; a.row_pos = row_pos; a.x = x;
+    a.xh = xh; a.ldxh = ldxh;
     a.width = width; a.vocab = vocab; a.buckets = buckets; a.mul_prev = mul_prev; a.mul_cur = mul_cur; a.groups = groups > 0 ? groups : 1;
     a.fused = pair && max_span_rows == 1; a.scale = scale; a.eps = eps;
     const size_t smem = (size_t)width * 4;

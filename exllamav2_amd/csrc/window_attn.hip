@@ -17,8 +17,9 @@
 // Rotary layouts: halves (value i pairs with i + n / 2) or interleaved (2i with 2i + 1); angle p * freq[i], cos and sin times `amp`.
 // Variants a design may ask for (the *_ex entry points): a CHUNKED mask instead of the window -- p sees j <= p with
 // floor(j / chunk) == floor(p / chunk), chunks counted from the sequence's start --, a soft cap  c tanh(s / c)  on the scores, ONE gate
-// value per head instead of one per output value, and rows that bring queries only (a layer that attends over another layer's
-// cached keys and values).
+// value per head instead of one per output value, rows that bring queries only (a layer that attends over another layer's
+// cached keys and values), KEPT first tokens -- p also sees every j < keep, however far back --, and queries and keys divided by
+// their root mean square per head after the rotation.
 #include "hw.h"
 #include "errors.h"
 #include <stdint.h>
@@ -130,6 +131,71 @@ KERNEL void __launch_bounds__(256) rot_append_kernel(const RotAppendArgs a)
             wa_st<T>((T*)a.v_cache + (slot * a.G + g) * a.vdim + a.vdim - 1, src[a.v_off + g * a.vdim + a.vdim - 1]);
 }
 
+// The same with every query and key head divided by sqrt(mean over dim + eps) after its rotation (no weight; the query's scale comes
+// after it).  grid (rows, heads in fours): a wave takes one head -- lane l the pairs / single values l, l + 64, .. --, and the sum of
+// squares closes inside the wave; the waves behind the H + G heads copy one value head each.
+#define RN_ITEMS 8                           // pairs and single values per lane
+
+template <typename T>
+KERNEL void __launch_bounds__(256) rot_norm_append_kernel(const RotAppendArgs a, float eps)
+{
+    const int r = bid_x(), w = bid_y() * 4 + wave_id(), lane = lane_id();
+    const int kv_heads = a.k_cache ? a.G : 0;
+    if (w >= a.H + 2 * kv_heads) return;
+    const float* src = a.f + (long long)r * a.ld;
+    const int pos = a.row_pos[r];
+    const int pg = a.block_table[(long long)a.row_seq[r] * a.bt_stride + pos / a.page];
+    const long long slot = (long long)pg * a.page + pos % a.page;
+    if (w >= a.H + kv_heads)                                     // a value head
+    {
+        const int g = w - a.H - kv_heads;
+        const float* s = src + a.v_off + g * a.vdim;
+        T* d = (T*)a.v_cache + (slot * a.G + g) * a.vdim;
+        for (int i = lane; i < a.vdim; i += 64) wa_st<T>(d + i, s[i]);
+        return;
+    }
+    const float fpos = (float)pos;
+    const int half = a.rot_dims / 2, per = half + (a.dim - a.rot_dims);
+    const bool is_q = w < a.H;
+    const float* s = is_q ? src + a.q_off + w * a.dim : src + a.k_off + (w - a.H) * a.dim;
+    T* d = is_q ? (T*)a.q_out + ((long long)r * a.H + w) * a.dim : (T*)a.k_cache + (slot * a.G + (w - a.H)) * a.dim;
+    float u[RN_ITEMS], v[RN_ITEMS];
+    float ss = 0.0f;
+    #pragma unroll
+    for (int i = 0; i < RN_ITEMS; i++)
+    {
+        const int e = lane + 64 * i;
+        u[i] = v[i] = 0.0f;
+        if (e < half)
+        {
+            int ia, ib;
+            wa_pair(e, a.rot_dims, a.interleaved, ia, ib);
+            const float ang = fpos * a.freq[e];
+            const float c = cosf(ang) * a.amp, sn = sinf(ang) * a.amp;
+            const float p = s[ia], q = s[ib];
+            u[i] = p * c - q * sn;
+            v[i] = q * c + p * sn;
+        }
+        else if (e < per) u[i] = s[a.rot_dims + (e - half)];
+        ss = fmaf(u[i], u[i], fmaf(v[i], v[i], ss));
+    }
+    ss = wave_allreduce_add(ss);
+    const float mul = (is_q ? a.q_scale[w] : 1.0f) / sqrtf(ss / (float)a.dim + eps);
+    #pragma unroll
+    for (int i = 0; i < RN_ITEMS; i++)
+    {
+        const int e = lane + 64 * i;
+        if (e < half)
+        {
+            int ia, ib;
+            wa_pair(e, a.rot_dims, a.interleaved, ia, ib);
+            wa_st<T>(d + ia, u[i] * mul);
+            wa_st<T>(d + ib, v[i] * mul);
+        }
+        else if (e < per) wa_st<T>(d + a.rot_dims + (e - half), u[i] * mul);
+    }
+}
+
 // ---- pooled rows ----------------------------------------------------------------------------------------------------------------
 
 struct PoolArgs
@@ -234,6 +300,7 @@ struct WinAttnArgs
     int page_shift, pool_shift;              // log2 of page / pool where they are powers of two, else -1 (tile kernels: no divisions)
     int chunk;                               // > 0: chunked mask (the window is not used, no pooled blocks)
     float softcap;                           // > 0: score <- softcap * tanh(score / softcap)
+    int keep;                                // > 0: the first `keep` tokens are seen from everywhere (no pooled blocks, no chunks)
     int gate_head;                           // gate holds one value per head (at h) instead of one per output value (at h * vdim + e)
 };
 
@@ -246,11 +313,18 @@ DEV int wa_mod(int x, int d, int shift) { return shift >= 0 ? x & (d - 1) : x % 
 
 #define WA_MAX_V_PER_THREAD 4
 
+// The key list of a position (of a tile: from its first position's window on) is [entries in front | tokens j_lo ..]: in front stand
+// the pooled blocks, or the kept first tokens that lie in front of j_lo.
+
 // number of pooled blocks position `pos` sees
 DEV int wa_blocks_seen(int pos, int window, int pool)
 {
     const int behind = pos - window + 1;     // tokens in front of the window
     return pool > 0 && behind > 0 ? behind / pool : 0;
+}
+DEV int wa_front_entries(const WinAttnArgs& a, int pos, int j_lo)
+{
+    return a.keep > 0 ? min(a.keep, j_lo) : wa_blocks_seen(pos, a.window, a.pool);
 }
 
 // Workgroup = one (row, head); general and fp32 form.  The key list is [pooled blocks | window tokens], taken 256 at a time:
@@ -272,8 +346,8 @@ KERNEL void __launch_bounds__(256) window_attn_kernel(const WinAttnArgs a)
     const T* qr = (const T*)a.q + ((long long)r * a.H + h) * a.dim;
     for (int i = t; i < a.dim; i += 256) qv[i] = wa_ld<T>(qr + i);
     block_sync();
-    const int nb = wa_blocks_seen(pos, a.window, a.pool);
     const int j_lo = max(0, wa_first_key(pos, a.window, a.chunk));
+    const int nb = wa_front_entries(a, pos, j_lo);
     const int nkeys = nb + (pos - j_lo + 1);
     float m_run = a.sink ? a.sink[h] : -INFINITY, l_run = a.sink ? 1.0f : 0.0f;
     float acc[WA_MAX_V_PER_THREAD];
@@ -287,7 +361,7 @@ KERNEL void __launch_bounds__(256) window_attn_kernel(const WinAttnArgs a)
         {
             const int e = c0 + t;
             const T* kr;
-            if (e < nb)
+            if (e < nb && a.keep == 0)
             {
                 const int p0 = e * a.pool;
                 const long long row = (long long)bt[p0 / a.page] * a.per_page + (p0 % a.page) / a.pool;
@@ -296,7 +370,7 @@ KERNEL void __launch_bounds__(256) window_attn_kernel(const WinAttnArgs a)
             }
             else
             {
-                const int j = j_lo + (e - nb);
+                const int j = e < nb ? e : j_lo + (e - nb);
                 const long long row = (long long)bt[j / a.page] * a.page + j % a.page;
                 kr = (const T*)a.k_cache + (row * a.G + g) * a.dim;
                 voff[t] = (row * a.G + g) * (long long)a.vdim;
@@ -365,7 +439,7 @@ KERNEL void __launch_bounds__(256) window_attn_kernel(const WinAttnArgs a)
 
 // ---- bfloat16 on the matrix cores ---------------------------------------------------------------------------------------------------
 // Workgroup = one tile of <= 64 RPW consecutive positions of one sequence x one head; wave w owns RPW blocks of 16 query rows.
-// The tile's key list is [pooled blocks 0 .. NB) | tokens j_lo .. last position], NB and j_lo taken for the tile as a whole and
+// The tile's key list is [pooled blocks (or kept first tokens) 0 .. NB) | tokens j_lo .. last position], NB and j_lo taken for the tile as a whole and
 // masked per query row; it goes by in steps of 64 entries whose key and value rows are staged row-major in LDS (each entry's row is
 // looked up through the block table -- pooled rows in the pooled tensors -- one step ahead of its loads, two steps ahead of its use).
 // Scores are computed transposed, S^T = K Q^T (A = key rows from LDS, B = the wave's query rows held in registers), so that the
@@ -408,8 +482,8 @@ KERNEL void __launch_bounds__(256, 2) window_attn_mfma_kernel(const WinMfmaArgs 
     const int r0 = m.tile_row0[tile_i], n_rows = m.tile_rows[tile_i];
     const int p0 = a.row_pos[r0], p_last = p0 + n_rows - 1;
     const int* bt = a.block_table + (long long)a.row_seq[r0] * a.bt_stride;
-    const int NB = wa_blocks_seen(p_last, a.window, a.pool);
     const int j_lo = max(0, wa_first_key(p0, a.window, a.chunk));
+    const int NB = wa_front_entries(a, p_last, j_lo);
     const int total = NB + (p_last - j_lo + 1);
     const int n_tiles = (total + WM_BK - 1) / WM_BK;
     const u16* kc = (const u16*)a.k_cache; const u16* vc = (const u16*)a.v_cache;
@@ -418,13 +492,13 @@ KERNEL void __launch_bounds__(256, 2) window_attn_mfma_kernel(const WinMfmaArgs 
     // entry e of the key list -> its row in the cache (>= 0) or in the pooled tensors (-1 - row)
     auto entry_row = [&](int e) -> long long {
         e = min(e, total - 1);
-        if (e < NB)
+        if (e < NB && a.keep == 0)
         {
             const int b0 = e * a.pool;
             return -1 - ((long long)bt[wa_div(b0, a.page, a.page_shift)] * a.per_page
                          + wa_div(wa_mod(b0, a.page, a.page_shift), a.pool, a.pool_shift));
         }
-        const int j = j_lo + (e - NB);
+        const int j = e < NB ? e : j_lo + (e - NB);
         return (long long)bt[wa_div(j, a.page, a.page_shift)] * a.page + wa_mod(j, a.page, a.page_shift);
     };
 
@@ -441,13 +515,13 @@ KERNEL void __launch_bounds__(256, 2) window_attn_mfma_kernel(const WinMfmaArgs 
         const u16* qp = (const u16*)a.q + ((long long)qrow[n] * a.H + h) * DIM + 8 * g;
         #pragma unroll
         for (int kk = 0; kk < KK; kk++) qb[n][kk] = *(const u32x4*)(qp + 32 * kk);
-        my_nb[n] = wa_blocks_seen(qpos[n], a.window, a.pool);
+        my_nb[n] = a.keep > 0 ? NB : wa_blocks_seen(qpos[n], a.window, a.pool);
         my_lo[n] = wa_first_key(qpos[n], a.window, a.chunk);    // first token this query sees (may be negative)
     }
     const bool wave_live = wv * RPW * 16 < n_rows;
     // what the wave as a whole can see: blocks below wave_nb, tokens wave_lo .. wave_hi
     const int wp0 = p0 + min(wv * RPW * 16, n_rows - 1), wp1 = p0 + min(wv * RPW * 16 + RPW * 16 - 1, n_rows - 1);
-    const int wave_nb = wa_blocks_seen(wp1, a.window, a.pool), wave_lo = wa_first_key(wp0, a.window, a.chunk), wave_hi = wp1;
+    const int wave_nb = a.keep > 0 ? NB : wa_blocks_seen(wp1, a.window, a.pool), wave_lo = wa_first_key(wp0, a.window, a.chunk), wave_hi = wp1;
 
     f32x4 ot[RPW][DB];
     float m_run[RPW], l_run[RPW];
@@ -527,7 +601,7 @@ KERNEL void __launch_bounds__(256, 2) window_attn_mfma_kernel(const WinMfmaArgs 
             if (e_hi >= NB)
             {
                 const int ja = j_lo + max(k0 - NB, 0), jb = j_lo + (e_hi - NB);
-                any = any || (ja <= wave_hi && jb >= wave_lo);
+                any = any || (ja <= wave_hi && (jb >= wave_lo || ja < a.keep));
             }
             if (!wave_live || !any) continue;
         }
@@ -560,7 +634,7 @@ KERNEL void __launch_bounds__(256, 2) window_attn_mfma_kernel(const WinMfmaArgs 
                 {
                     const int e = k0 + 16 * blk + 4 * g + r;
                     const int j = j_lo + (e - NB);
-                    const bool valid = e < total && (e < NB ? e < my_nb[n] : (j <= qpos[n] && j >= my_lo[n]));
+                    const bool valid = e < total && (e < NB ? e < my_nb[n] : (j <= qpos[n] && (j >= my_lo[n] || j < a.keep)));
                     const float v = valid ? wa_soft_cap(st[n][blk][r], a.softcap) : WM_NEG_BIG;
                     sc[blk * 4 + r] = v;
                     m_loc = fmaxf(m_loc, v);
@@ -701,8 +775,8 @@ KERNEL void __launch_bounds__(256) window_attn_decode_kernel(const WinMfmaArgs m
     const int r = m.tile_row0[bid_x()];
     const int pos = a.row_pos[r];
     const int* bt = a.block_table + (long long)a.row_seq[r] * a.bt_stride;
-    const int NB = wa_blocks_seen(pos, a.window, a.pool);
     const int j_lo = max(0, wa_first_key(pos, a.window, a.chunk));
+    const int NB = wa_front_entries(a, pos, j_lo);
     const int total = NB + (pos - j_lo + 1);
     const int all_steps = (total + WD_BK - 1) / WD_BK;
     const int per_split = (all_steps + m.nsplit - 1) / m.nsplit;
@@ -711,13 +785,13 @@ KERNEL void __launch_bounds__(256) window_attn_decode_kernel(const WinMfmaArgs m
     const u16* kp = (const u16*)a.k_pool; const u16* vp = (const u16*)a.v_pool;
     auto entry_row = [&](int e) -> long long {
         e = min(e, total - 1);
-        if (e < NB)
+        if (e < NB && a.keep == 0)
         {
             const int b0 = e * a.pool;
             return -1 - ((long long)bt[wa_div(b0, a.page, a.page_shift)] * a.per_page
                          + wa_div(wa_mod(b0, a.page, a.page_shift), a.pool, a.pool_shift));
         }
-        const int j = j_lo + (e - NB);
+        const int j = e < NB ? e : j_lo + (e - NB);
         return (long long)bt[wa_div(j, a.page, a.page_shift)] * a.page + wa_mod(j, a.page, a.page_shift);
     };
     const int head = kh * hpg + h0 + min(qi, nh - 1);
@@ -972,17 +1046,17 @@ extern "C" int exl2_kv_rot_append_ex(const float* f, int ld, int q_off, int k_of
                                      void* k_cache, void* v_cache, void* k_pool, void* v_pool, const float* freq, float amp, int rot_dims,
                                      const float* vfreq, int v_rot, int interleaved, const int* row_seq, const int* row_pos,
                                      const int* block_table, int bt_stride, int page, int pool, int dtype, int rows, int heads,
-                                     int kv_heads, int dim, int vdim, void* stream);
+                                     int kv_heads, int dim, int vdim, int head_norm, float norm_eps, void* stream);
 extern "C" int exl2_window_attn_ex(const void* q, const void* k_cache, const void* v_cache, const void* k_pool, const void* v_pool,
                                    const float* sink, const float* gate, int ldg, const float* vfreq, int v_rot, int interleaved,
                                    const int* row_seq, const int* row_pos, const int* block_table, int bt_stride, int page, int pool,
-                                   void* out, int dtype, int rows, int heads, int kv_heads, int dim, int vdim, int window, int chunk,
+                                   void* out, int dtype, int rows, int heads, int kv_heads, int dim, int vdim, int window, int keep, int chunk,
                                    float softcap, int gate_head, void* stream);
 extern "C" int exl2_window_attn_tiles_ex(const void* q, const void* k_cache, const void* v_cache, const void* k_pool, const void* v_pool,
                                          const float* sink, const float* gate, int ldg, const float* vfreq, int v_rot, int interleaved,
                                          const int* row_seq, const int* row_pos, const int* block_table, int bt_stride, int page, int pool,
                                          void* out, const int* tile_row0, const int* tile_rows, int tiles, int tile_mode, float* part_o,
-                                         float* part_ml, int nsplit, int heads, int kv_heads, int dim, int vdim, int window, int chunk,
+                                         float* part_ml, int nsplit, int heads, int kv_heads, int dim, int vdim, int window, int keep, int chunk,
                                          float softcap, int gate_head, void* stream);
 
 extern "C" int exl2_kv_rot_append(const float* f, int ld, int q_off, int k_off, int v_off, void* q_out, const float* q_scale,
@@ -994,14 +1068,14 @@ extern "C" int exl2_kv_rot_append(const float* f, int ld, int q_off, int k_off, 
     EXL2_REQUIRE(k_cache && v_cache, "kv_rot_append: null operand");
     return exl2_kv_rot_append_ex(f, ld, q_off, k_off, v_off, q_out, q_scale, k_cache, v_cache, k_pool, v_pool, freq, amp, rot_dims, vfreq,
                                  v_rot, interleaved, row_seq, row_pos, block_table, bt_stride, page, pool, dtype, rows, heads, kv_heads,
-                                 dim, vdim, stream);
+                                 dim, vdim, 0, 0.0f, stream);
 }
 
 extern "C" int exl2_kv_rot_append_ex(const float* f, int ld, int q_off, int k_off, int v_off, void* q_out, const float* q_scale,
                                      void* k_cache, void* v_cache, void* k_pool, void* v_pool, const float* freq, float amp, int rot_dims,
                                      const float* vfreq, int v_rot, int interleaved, const int* row_seq, const int* row_pos,
                                      const int* block_table, int bt_stride, int page, int pool, int dtype, int rows, int heads,
-                                     int kv_heads, int dim, int vdim, void* stream)
+                                     int kv_heads, int dim, int vdim, int head_norm, float norm_eps, void* stream)
 {
     EXL2_REQUIRE(f && q_out && q_scale && freq && row_seq && row_pos && block_table, "kv_rot_append: null operand");
     EXL2_REQUIRE((k_cache == nullptr) == (v_cache == nullptr), "kv_rot_append: keys and values go to the cache together");
@@ -1011,13 +1085,21 @@ extern "C" int exl2_kv_rot_append_ex(const float* f, int ld, int q_off, int k_of
     EXL2_REQUIRE(rot_dims >= 0 && rot_dims <= dim && rot_dims % 2 == 0, "kv_rot_append: %d rotated of %d values", rot_dims, dim);
     EXL2_REQUIRE(!v_rot || (vfreq && vdim % 2 == 0), "kv_rot_append: rotated values need an even size and their frequencies");
     EXL2_REQUIRE(page > 0 && pool >= 0 && (pool == 0 || (k_pool && v_pool)), "kv_rot_append: bad paging (page %d, pool %d)", page, pool);
+    EXL2_REQUIRE(!head_norm || (!v_rot && dim - rot_dims / 2 <= 64 * RN_ITEMS && norm_eps >= 0.0f),
+                 "kv_rot_append: normed heads of %d values (at most %d pairs and single values), values not rotated", dim, 64 * RN_ITEMS);
     if (rows <= 0) return EXL2_OK;
     RotAppendArgs a;
     a.f = f; a.ld = ld; a.q_off = q_off; a.k_off = k_off; a.v_off = v_off; a.q_out = q_out; a.q_scale = q_scale; a.k_cache = k_cache;
     a.v_cache = v_cache; a.freq = freq; a.amp = amp; a.rot_dims = rot_dims; a.vfreq = vfreq; a.v_rot = v_rot; a.interleaved = interleaved;
     a.row_seq = row_seq; a.row_pos = row_pos; a.block_table = block_table; a.bt_stride = bt_stride; a.page = page;
     a.H = heads; a.G = kv_heads; a.dim = dim; a.vdim = vdim;
-    if (dtype == 0) LAUNCH(rot_append_kernel<u16>, dim3(rows), dim3(256), 0, stream, a);
+    if (head_norm)
+    {
+        const dim3 grid(rows, (heads + (k_cache ? 2 * kv_heads : 0) + 3) / 4);
+        if (dtype == 0) LAUNCH(rot_norm_append_kernel<u16>, grid, dim3(256), 0, stream, a, norm_eps);
+        else LAUNCH(rot_norm_append_kernel<float>, grid, dim3(256), 0, stream, a, norm_eps);
+    }
+    else if (dtype == 0) LAUNCH(rot_append_kernel<u16>, dim3(rows), dim3(256), 0, stream, a);
     else LAUNCH(rot_append_kernel<float>, dim3(rows), dim3(256), 0, stream, a);
     if (pool > 0)
     {
@@ -1041,17 +1123,18 @@ extern "C" int exl2_window_attn(const void* q, const void* k_cache, const void* 
                                 void* out, int dtype, int rows, int heads, int kv_heads, int dim, int vdim, int window, void* stream)
 {
     return exl2_window_attn_ex(q, k_cache, v_cache, k_pool, v_pool, sink, gate, ldg, vfreq, v_rot, interleaved, row_seq, row_pos,
-                               block_table, bt_stride, page, pool, out, dtype, rows, heads, kv_heads, dim, vdim, window, 0, 0.0f, 0, stream);
+                               block_table, bt_stride, page, pool, out, dtype, rows, heads, kv_heads, dim, vdim, window, 0, 0, 0.0f, 0, stream);
 }
 
 extern "C" int exl2_window_attn_ex(const void* q, const void* k_cache, const void* v_cache, const void* k_pool, const void* v_pool,
                                    const float* sink, const float* gate, int ldg, const float* vfreq, int v_rot, int interleaved,
                                    const int* row_seq, const int* row_pos, const int* block_table, int bt_stride, int page, int pool,
-                                   void* out, int dtype, int rows, int heads, int kv_heads, int dim, int vdim, int window, int chunk,
+                                   void* out, int dtype, int rows, int heads, int kv_heads, int dim, int vdim, int window, int keep, int chunk,
                                    float softcap, int gate_head, void* stream)
 {
     EXL2_REQUIRE(chunk >= 0 && (chunk == 0 || pool == 0), "window_attn: a chunked mask has no pooled blocks");
     EXL2_REQUIRE(softcap >= 0.0f, "window_attn: negative soft cap");
+    EXL2_REQUIRE(keep >= 0 && (keep == 0 || (chunk == 0 && pool == 0)), "window_attn: kept first tokens go with a plain window");
     EXL2_REQUIRE(q && k_cache && v_cache && row_seq && row_pos && block_table && out, "window_attn: null operand");
     EXL2_REQUIRE(dtype == 0 || dtype == 1, "window_attn: dtype must be 0 (bfloat16) or 1 (float32)");
     EXL2_REQUIRE(heads > 0 && kv_heads > 0 && heads % kv_heads == 0 && dim > 0, "window_attn: bad head shape");
@@ -1064,7 +1147,7 @@ extern "C" int exl2_window_attn_ex(const void* q, const void* k_cache, const voi
     a.vfreq = vfreq; a.v_rot = v_rot; a.interleaved = interleaved; a.row_seq = row_seq; a.row_pos = row_pos; a.block_table = block_table;
     a.bt_stride = bt_stride; a.page = page; a.pool = pool; a.per_page = pool > 0 ? (page + pool - 1) / pool : 0; a.out = out;
     a.H = heads; a.G = kv_heads; a.dim = dim; a.vdim = vdim; a.window = window; a.page_shift = a.pool_shift = -1;
-    a.chunk = chunk; a.softcap = softcap; a.gate_head = gate_head;
+    a.keep = keep; a.chunk = chunk; a.softcap = softcap; a.gate_head = gate_head;
     const size_t smem = (size_t)(dim + vdim) * 4;
     if (dtype == 0) LAUNCH(window_attn_kernel<u16>, dim3(rows, heads), dim3(256), smem, stream, a);
     else LAUNCH(window_attn_kernel<float>, dim3(rows, heads), dim3(256), smem, stream, a);
@@ -1076,7 +1159,7 @@ extern "C" int exl2_window_attn_ex(const void* q, const void* k_cache, const voi
 extern "C" int exl2_window_attn_tiles_supported(int dim, int vdim)
 {
     return (dim == vdim && (dim == 32 || dim == 64 || dim == 96 || dim == 128 || dim == 256)) || (dim == 192 && vdim == 128)
-           || (dim == 128 && vdim == 64) || (dim == 64 && vdim == 128);
+           || (dim == 128 && (vdim == 64 || vdim == 96)) || (dim == 64 && (vdim == 32 || vdim == 80 || vdim == 96 || vdim == 128));
 }
 
 /* exl2_window_attn on the matrix cores (bfloat16, head sizes of exl2_window_attn_tiles_supported; gate rows and offsets multiples
@@ -1092,18 +1175,19 @@ extern "C" int exl2_window_attn_tiles(const void* q, const void* k_cache, const 
 {
     return exl2_window_attn_tiles_ex(q, k_cache, v_cache, k_pool, v_pool, sink, gate, ldg, vfreq, v_rot, interleaved, row_seq, row_pos,
                                      block_table, bt_stride, page, pool, out, tile_row0, tile_rows, tiles, tile_mode, part_o, part_ml,
-                                     nsplit, heads, kv_heads, dim, vdim, window, 0, 0.0f, 0, stream);
+                                     nsplit, heads, kv_heads, dim, vdim, window, 0, 0, 0.0f, 0, stream);
 }
 
 extern "C" int exl2_window_attn_tiles_ex(const void* q, const void* k_cache, const void* v_cache, const void* k_pool, const void* v_pool,
                                          const float* sink, const float* gate, int ldg, const float* vfreq, int v_rot, int interleaved,
                                          const int* row_seq, const int* row_pos, const int* block_table, int bt_stride, int page, int pool,
                                          void* out, const int* tile_row0, const int* tile_rows, int tiles, int tile_mode, float* part_o,
-                                         float* part_ml, int nsplit, int heads, int kv_heads, int dim, int vdim, int window, int chunk,
+                                         float* part_ml, int nsplit, int heads, int kv_heads, int dim, int vdim, int window, int keep, int chunk,
                                          float softcap, int gate_head, void* stream)
 {
     EXL2_REQUIRE(chunk >= 0 && (chunk == 0 || pool == 0), "window_attn_tiles: a chunked mask has no pooled blocks");
     EXL2_REQUIRE(softcap >= 0.0f, "window_attn_tiles: negative soft cap");
+    EXL2_REQUIRE(keep >= 0 && (keep == 0 || (chunk == 0 && pool == 0)), "window_attn_tiles: kept first tokens go with a plain window");
     EXL2_REQUIRE(nsplit >= 1 && nsplit <= 64 && (nsplit == 1 || (tile_mode == 1 && part_o && part_ml)),
                  "window_attn_tiles: key splits (1 .. 64) need tile_mode 1 and scratch");
     EXL2_REQUIRE(q && k_cache && v_cache && row_seq && row_pos && block_table && out && tile_row0, "window_attn_tiles: null operand");
@@ -1122,7 +1206,7 @@ extern "C" int exl2_window_attn_tiles_ex(const void* q, const void* k_cache, con
     a.vfreq = vfreq; a.v_rot = v_rot; a.interleaved = interleaved; a.row_seq = row_seq; a.row_pos = row_pos; a.block_table = block_table;
     a.bt_stride = bt_stride; a.page = page; a.pool = pool; a.per_page = pool > 0 ? (page + pool - 1) / pool : 0; a.out = out;
     a.H = heads; a.G = kv_heads; a.dim = dim; a.vdim = vdim; a.window = window;
-    a.chunk = chunk; a.softcap = softcap; a.gate_head = gate_head;
+    a.keep = keep; a.chunk = chunk; a.softcap = softcap; a.gate_head = gate_head;
     a.page_shift = wa_log2_exact(page); a.pool_shift = pool > 0 ? wa_log2_exact(pool) : -1;
     m.tile_row0 = tile_row0; m.tile_rows = tile_rows; m.part_o = part_o; m.part_ml = part_ml; m.nsplit = nsplit;
     hipStream_t s = (hipStream_t)stream;
@@ -1135,6 +1219,10 @@ extern "C" int exl2_window_attn_tiles_ex(const void* q, const void* k_cache, con
         else if (dim == 256 && vdim == 256) wd_launch<256, 256>(m, tiles, s);
         else if (dim == 192 && vdim == 128) wd_launch<192, 128>(m, tiles, s);
         else if (dim == 128 && vdim == 64) wd_launch<128, 64>(m, tiles, s);
+        else if (dim == 128 && vdim == 96) wd_launch<128, 96>(m, tiles, s);
+        else if (dim == 64 && vdim == 32) wd_launch<64, 32>(m, tiles, s);
+        else if (dim == 64 && vdim == 80) wd_launch<64, 80>(m, tiles, s);
+        else if (dim == 64 && vdim == 96) wd_launch<64, 96>(m, tiles, s);
         else wd_launch<64, 128>(m, tiles, s);
         HIP_TRY(hipGetLastError());
         return EXL2_OK;
@@ -1146,6 +1234,10 @@ extern "C" int exl2_window_attn_tiles_ex(const void* q, const void* k_cache, con
     else if (dim == 256 && vdim == 256) wm_launch<256, 256>(m, tiles, s);
     else if (dim == 192 && vdim == 128) wm_launch<192, 128>(m, tiles, s);
     else if (dim == 128 && vdim == 64) wm_launch<128, 64>(m, tiles, s);
+    else if (dim == 128 && vdim == 96) wm_launch<128, 96>(m, tiles, s);
+    else if (dim == 64 && vdim == 32) wm_launch<64, 32>(m, tiles, s);
+    else if (dim == 64 && vdim == 80) wm_launch<64, 80>(m, tiles, s);
+    else if (dim == 64 && vdim == 96) wm_launch<64, 96>(m, tiles, s);
     else wm_launch<64, 128>(m, tiles, s);
     HIP_TRY(hipGetLastError());
     return EXL2_OK;

@@ -39,15 +39,24 @@ class JoinedFront:
     """ONE linear for everything that reads a layer's input: the members' projections (`member.front_part` = (weight [n, width], bias
     fp32 [n] | None), left by a module built with `joined=True`) stacked behind each other, every part starting at a multiple of four
     columns; a member learns where its columns start (`front_base`).  Plain (weight, bias) pairs may join; `bases` lists every
-    member's first column in order."""
+    member's first column in order.  A member may also leave `front_low` (weight [n, width]): the inner halves of low-rank projections,
+    which the next linear reads -- they stand behind everything else (n a multiple of eight, so that it can be read in 16-byte pieces)
+    and leave the same launch in the operand dtype, in rows of their own (`low_base` = the member's first column there)."""
 
     def __init__(self, ext, key: str, members):
-        weights, biases, self.bases, at = [], [], [], 0
+        weights, biases, self.bases, at, low = [], [], [], 0, []
+        self.low_columns = 0
         for m in members:
             w, b = m if isinstance(m, tuple) else m.front_part
             self.bases.append(at)
             if not isinstance(m, tuple):
                 m.front_base, m.front_part = at, None
+                if getattr(m, "front_low", None) is not None:
+                    if m.front_low.shape[0] % 8:
+                        raise RuntimeError(f"{key}: an inner projection of {m.front_low.shape[0]} columns")
+                    low.append(m.front_low)
+                    m.low_base, m.front_low = self.low_columns, None
+                    self.low_columns += low[-1].shape[0]
             pad = -w.shape[0] % 4
             weights += [w] + ([w.new_zeros((pad, w.shape[1]))] if pad else [])
             bias = torch.zeros((w.shape[0] + pad,), dtype=torch.float32, device=w.device)
@@ -55,15 +64,24 @@ class JoinedFront:
                 bias[:w.shape[0]] = b.to(torch.float32)
             biases.append(bias)
             at += w.shape[0] + pad
-        self.linear = DenseLinear(ext, key, torch.cat(weights, 0))
+        self.columns = at
+        if low:
+            biases.append(torch.zeros((self.low_columns,), dtype=torch.float32, device=low[0].device))
+        self.linear = DenseLinear(ext, key, torch.cat(weights + low, 0))
         self.bias = torch.cat(biases, 0).contiguous()
 
     def weight_bytes(self) -> int:
         return self.linear.weight_bytes()
 
     def forward(self, xh: torch.Tensor, rows: int, model):
-        """(fp32 rows of all members' projections, their leading dimension)"""
-        n = self.linear.out_features
+        """(fp32 rows of all members' projections, their leading dimension); with inner projections also (operand-dtype rows of those,
+        their leading dimension)"""
+        n = self.columns
+        if self.low_columns:
+            f = model.buf("layer.f", (rows, n), torch.float32)
+            low = model.buf("layer.low", (rows, self.low_columns), model.dtype)
+            self.linear.ext.dense_linear_split(xh, self.linear.weight, self.bias, f, low, rows, n)
+            return f, n, low, self.low_columns
         return self.linear.forward(xh, rows, out=model.buf("layer.f", (rows, n), torch.float32), bias=self.bias), n
 
 

@@ -781,6 +781,7 @@ class ExtC:
     EPI_SCALE, EPI_TANH, EPI_ROW_SCALED_RELU_SQUARED = 6, 7, 8        # acc * limit; tanh(acc); relu(aux[row] * acc)^2
     EPI_ROW_SCALED_SILU_SCALED, EPI_AUX_MUL = 9, 10                   # silu(aux[row] * acc) * aux[row]; acc * aux
     EPI_GELU_ERF, EPI_MUL_SIGMOID_ROW_AUX = 11, 12                    # exact gelu; acc * sigmoid(aux[row])
+    EPI_EXP_SOFTPLUS = 13                                             # exp(aux * softplus(acc)); ldaux 0: aux per column
 
     @staticmethod
     def _dense_code(dtype) -> int:
@@ -814,6 +815,20 @@ class ExtC:
             self._ptr(w_sel, torch.int32, "w_sel"), int(n_sel), self._ptr(gc, torch.int32, "grp_count"),
             self._ptr(go, torch.int32, "grp_offset"), self._ptr(gr, torch.int32, "grp_rows"), int(x_div), int(epi), float(limit),
             self._stream(y)))
+
+    def dense_linear_split(self, x, w, bias, y, y2, M: int, n2: int) -> None:
+        """x . w^T + bias on rows of x (leading dimension x.shape[-1]): columns [0, n2) into y, the ones behind into y2 (w's dtype)"""
+        N, K = w.shape
+        if x.dtype is not w.dtype or y2.dtype is not w.dtype or (y.dtype is not w.dtype and y.dtype is not torch.float32):
+            raise RuntimeError(f"dense_linear_split: x {x.dtype}, w {w.dtype}, y {y.dtype}, y2 {y2.dtype}")
+        if bias is not None and bias.numel() != N:
+            raise RuntimeError(f"dense_linear_split: bias has {bias.numel()} values, N is {N}")
+        if y.numel() < M * y.shape[-1] or y2.numel() < M * y2.shape[-1] or x.numel() < (M - 1) * x.shape[-1] + K:
+            raise RuntimeError(f"dense_linear_split: an operand holds fewer than {M} rows")
+        self.lib.check(self.lib.exl2_dense_linear_split(
+            self._ptr(x, None, "x"), self._ptr(w, None, "w"), self._ptr(bias, torch.float32, "bias"), self._ptr(y, None, "y"),
+            int(y.dtype is torch.float32), self._ptr(y2, None, "y2"), int(n2), y2.shape[-1], self._dense_code(w.dtype), int(M), int(N), int(K),
+            x.shape[-1], int(K), y.shape[-1], self._stream(y)))
 
     def embed_scale(self, table, ids, x32, xh, scale: float) -> None:
         rows, width = ids.numel(), table.shape[1]
@@ -957,8 +972,9 @@ class ExtC:
 
     def kv_rot_append(self, f, ld: int, q_off: int, k_off: int, v_off: int, q_out, q_scale, k_cache, v_cache, k_pool, v_pool, freq,
                       amp: float, rot_dims: int, vfreq, v_rot: bool, interleaved: bool, row_seq, row_pos, block_table, page: int, pool: int,
-                      rows: int, heads: int, kv_heads: int, dim: int, vdim: int) -> None:
-        dt = q_out.dtype                                         # (k_cache None: the rows bring queries only)
+                      rows: int, heads: int, kv_heads: int, dim: int, vdim: int, head_norm_eps: float | None = None) -> None:
+        """k_cache None: the rows bring queries only; head_norm_eps: query and key heads are divided by their root mean square"""
+        dt = q_out.dtype
         self.lib.check(self.lib.exl2_kv_rot_append_ex(
             self._ptr(f, torch.float32, "f"), int(ld), int(q_off), int(k_off), int(v_off), self._ptr(q_out, dt, "q_out"),
             self._ptr(q_scale, torch.float32, "q_scale"), self._ptr(k_cache, dt, "k_cache"), self._ptr(v_cache, dt, "v_cache"),
@@ -966,12 +982,13 @@ class ExtC:
             int(rot_dims), self._ptr(vfreq, torch.float32, "vfreq"), int(v_rot), int(interleaved),
             self._ptr(row_seq, torch.int32, "row_seq"), self._ptr(row_pos, torch.int32, "row_pos"),
             self._ptr(block_table, torch.int32, "block_table"), block_table.shape[-1], int(page), int(pool), self._dense_code(dt),
-            int(rows), int(heads), int(kv_heads), int(dim), int(vdim), self._stream(q_out)))
+            int(rows), int(heads), int(kv_heads), int(dim), int(vdim), int(head_norm_eps is not None), float(head_norm_eps or 0.0),
+            self._stream(q_out)))
 
     def window_attn(self, q, k_cache, v_cache, k_pool, v_pool, sink, gate, ldg: int, gate_off: int, vfreq, v_rot: bool, interleaved: bool,
                     row_seq, row_pos, block_table, page: int, pool: int, out, rows: int, heads: int, kv_heads: int, dim: int, vdim: int,
-                    window: int, chunk: int = 0, softcap: float = 0.0, gate_head: bool = False) -> None:
-        """chunk > 0: chunked mask instead of the window; softcap > 0: capped scores; gate_head: one gate value per head"""
+                    window: int, chunk: int = 0, softcap: float = 0.0, gate_head: bool = False, keep: int = 0) -> None:
+        """chunk > 0: chunked mask instead of the window; keep > 0: the first tokens stay visible; softcap > 0: capped scores; gate_head: one gate value per head"""
         dt = k_cache.dtype
         gp = None if gate is None else self._ptr(gate, torch.float32, "gate") + gate_off * 4
         self.lib.check(self.lib.exl2_window_attn_ex(
@@ -979,8 +996,8 @@ class ExtC:
             self._ptr(v_pool, dt, "v_pool"), self._ptr(sink, torch.float32, "sink"), gp, int(ldg), self._ptr(vfreq, torch.float32, "vfreq"),
             int(v_rot), int(interleaved), self._ptr(row_seq, torch.int32, "row_seq"), self._ptr(row_pos, torch.int32, "row_pos"),
             self._ptr(block_table, torch.int32, "block_table"), block_table.shape[-1], int(page), int(pool), self._ptr(out, dt, "out"),
-            self._dense_code(dt), int(rows), int(heads), int(kv_heads), int(dim), int(vdim), int(window), int(chunk), float(softcap),
-            int(gate_head), self._stream(out)))
+            self._dense_code(dt), int(rows), int(heads), int(kv_heads), int(dim), int(vdim), int(window), int(keep), int(chunk),
+            float(softcap), int(gate_head), self._stream(out)))
 
     def window_attn_tiles_supported(self, dtype, dim: int, vdim: int) -> bool:
         return dtype is torch.bfloat16 and bool(self.lib.exl2_window_attn_tiles_supported(int(dim), int(vdim)))
@@ -988,7 +1005,7 @@ class ExtC:
     def window_attn_tiles(self, q, k_cache, v_cache, k_pool, v_pool, sink, gate, ldg: int, gate_off: int, vfreq, v_rot: bool,
                           interleaved: bool, row_seq, row_pos, block_table, page: int, pool: int, out, tiles, tile_mode: int, heads: int,
                           kv_heads: int, dim: int, vdim: int, window: int, nsplit: int = 1, part_o=None, part_ml=None, chunk: int = 0,
-                          softcap: float = 0.0, gate_head: bool = False) -> None:
+                          softcap: float = 0.0, gate_head: bool = False, keep: int = 0) -> None:
         """tile_mode 64: tiles = (tile_row0 int32 [n], tile_rows int32 [n], n), runs of <= 64 consecutive positions of one sequence;
         tile_mode 1: tiles = (rows int32 [n], None, n), single decoded rows"""
         row0, nrows, n = tiles
@@ -1001,7 +1018,7 @@ class ExtC:
             self._ptr(block_table, torch.int32, "block_table"), block_table.shape[-1], int(page), int(pool), self._ptr(out, bf, "out"),
             self._ptr(row0, torch.int32, "tile_row0"), self._ptr(nrows, torch.int32, "tile_rows"), int(n), int(tile_mode),
             self._ptr(part_o, torch.float32, "part_o"), self._ptr(part_ml, torch.float32, "part_ml"), int(nsplit), int(heads),
-            int(kv_heads), int(dim), int(vdim), int(window), int(chunk), float(softcap), int(gate_head), self._stream(out)))
+            int(kv_heads), int(dim), int(vdim), int(window), int(keep), int(chunk), float(softcap), int(gate_head), self._stream(out)))
 
     # ---- scalar-gain RMS norm + token shift, sigmoid router (csrc/rowops.hip); decaying linear attention (csrc/wkv.hip) ----------------
 
@@ -1094,15 +1111,20 @@ class ExtC:
             self._stream(x32)))
 
     def embed_pair(self, table, pair, w, ids, prev_tok, row_seq, row_pos, spans, x32, buckets: int, mul_prev: int, mul_cur: int,
-                   scale: float, groups: int, eps: float) -> None:
-        """x32 = n_g(table[ids] * scale + pair[hash(previous token, token)]) w; spans = (span_row0, span_rows, n, longest span)"""
+                   scale: float, groups: int, eps: float, xh=None, xh_off: int = 0) -> None:
+        """x32 = n_g(table[ids] * scale + pair[hash(previous token, token)]) w; spans = (span_row0, span_rows, n, longest span); xh (2-D,
+        the table's dtype): a copy of the rows from column xh_off on"""
         row0, nrows, n, longest = spans
         rows, width = ids.numel(), table.shape[1]
+        ldxh = xh.shape[-1] if xh is not None else 0
+        if xh is not None and (xh_off + width > ldxh or xh.shape[0] < rows):
+            raise RuntimeError("embed_pair: the copy does not fit its buffer")
+        xhp = self._ptr(xh, table.dtype, "xh") + xh_off * xh.element_size() if xh is not None else None
         self.lib.check(self.lib.exl2_embed_pair(
             self._ptr(table, None, "table"), self._ptr(pair, table.dtype, "pair"), self._ptr(w, table.dtype, "w"),
             self._ptr(ids, torch.int32, "ids"), self._ptr(prev_tok, torch.int32, "prev_tok"), self._ptr(row_seq, torch.int32, "row_seq"),
             self._ptr(row_pos, torch.int32, "row_pos"), self._ptr(row0, torch.int32, "span_row0"), self._ptr(nrows, torch.int32, "span_rows"),
-            int(n), int(longest), self._ptr(x32, torch.float32, "x32"), self._dense_code(table.dtype), int(rows), int(width),
+            int(n), int(longest), self._ptr(x32, torch.float32, "x32"), xhp, int(ldxh), self._dense_code(table.dtype), int(rows), int(width),
             table.shape[0], int(buckets), int(mul_prev), int(mul_cur), float(scale), int(groups), float(eps), self._stream(x32)))
 
     def conv_rows(self, f, ld: int, f_off: int, w, bias, out, tail, spans, row_seq, row_pos, channels: int, taps: int,
@@ -1117,23 +1139,30 @@ class ExtC:
             self._ptr(row_seq, torch.int32, "row_seq"), self._ptr(row_pos, torch.int32, "row_pos"), self._dense_code(w.dtype), int(channels),
             int(taps), self._stream(out)))
 
-    SCAN_FORGET_WRITES, SCAN_DELTA = 0, 1
+    SCAN_FORGET_WRITES, SCAN_DELTA, SCAN_DELTA_CHANNELS = 0, 1, 2
 
     def gated_scan(self, mode: int, f, ld: int, q_off: int, k_off: int, v, ldv: int, v_off: int, norm_w, out, state, spans, row_seq, row_pos,
                    heads: int, qk_heads: int, n_key: int, n_val: int, eps: float, q_scale: float = 1.0, lower=None, gate_off: int | None = None,
-                   beta_off: int = 0, dt_off: int = 0, dt_bias=None, a_log=None, qk=None, ldqk: int = 0, o_raw=None) -> None:
+                   beta_off: int = 0, dt_off: int = 0, dt_bias=None, a_log=None, qk=None, ldqk: int = 0, o_raw=None, decay=None,
+                   ld_decay: int = 0, decay_off: int = 0, ready_gate_off: int | None = None) -> None:
         """o_raw (fp32 scratch [rows, heads * n_val]) given: the form for portions of prompts (exl2_gated_scan_cols).
         f fp32 [rows, ld]: the mixer's projections -- mode 0: q pre-activation at q_off, forget-gate pre-activation at k_off; mode 1:
         beta / decay inputs / output gate at beta_off / dt_off / gate_off, q and k in `qk` fp32 [rows, ldqk] at q_off / k_off (the
-        convolved rows).  v fp32 [rows, ldv] at v_off.  out [rows, heads * n_val] operand dtype or fp32."""
+        convolved rows); mode 2: as mode 1 with the decays per key channel at decay_off and the output gate's values at ready_gate_off of
+        `decay` fp32 [rows, ld_decay].  v fp32 [rows, ldv] at v_off.  out [rows, heads * n_val] operand dtype or fp32."""
         row0, nrows, n, _longest = spans
         pf = self._ptr(f, torch.float32, "f")
         pqk = self._ptr(qk, torch.float32, "qk") if qk is not None else pf
         lqk = int(ldqk) if qk is not None else int(ld)
-        delta = mode == self.SCAN_DELTA
+        delta, channels = mode != self.SCAN_FORGET_WRITES, mode == self.SCAN_DELTA_CHANNELS
+        gate = ((pf + gate_off * 4) if gate_off is not None else None, int(ld), 0)
+        dt = ((pf + dt_off * 4) if delta else None, int(ld))
+        if channels:
+            pd = self._ptr(decay, torch.float32, "decay")
+            gate = ((pd + ready_gate_off * 4) if ready_gate_off is not None else None, int(ld_decay), 1)
+            dt = (pd + decay_off * 4, int(ld_decay))
         head = (int(mode), pqk + q_off * 4, lqk, pqk + k_off * 4, lqk, self._ptr(v, torch.float32, "v") + v_off * 4, int(ldv),
-                (pf + gate_off * 4) if gate_off is not None else None, int(ld), (pf + beta_off * 4) if delta else None, int(ld),
-                (pf + dt_off * 4) if delta else None, int(ld), self._ptr(dt_bias, torch.float32, "dt_bias"),
+                *gate, (pf + beta_off * 4) if delta else None, int(ld), *dt, self._ptr(dt_bias, torch.float32, "dt_bias"),
                 self._ptr(a_log, torch.float32, "a_log"), self._ptr(lower, torch.float32, "lower"), self._ptr(norm_w, torch.float32, "norm_w"),
                 self._ptr(out, None, "out"), out.shape[-1], int(out.dtype is torch.float32), self._ptr(state, torch.float32, "state"),
                 self._ptr(row0, torch.int32, "span_row0"), self._ptr(nrows, torch.int32, "span_rows"), int(n),
@@ -1155,9 +1184,9 @@ class ExtC:
 
     def gated_residual(self, x32, out, rows: int, eps: float, w_in=None, y=None, y2=None, wy=None, wy2=None, ya: float = 1.0, yb: float = 1.0,
                        gates=None, ldg: int = 0, g1_off: int | None = None, g2_off: int | None = None, moe_y=None, moe_w=None, top: int = 0,
-                       table=None, ids=None, init: bool = False, row_idx=None, dtype=None) -> None:
-        """x32 += t sigmoid(g1) + sigmoid(g2) sum_k moe_w moe_y (+ table[ids]; init: x32 = table[ids]), t = y or ya n(y) wy + yb n(y2) wy2;
-        out = n(x32) w_in (out may be None).  The gates are columns g1_off / g2_off of fp32 rows ldg apart."""
+                       table=None, ids=None, init: bool = False, row_idx=None, dtype=None, mult: float = 1.0, ldo: int | None = None) -> None:
+        """x32 += mult (t sigmoid(g1) + sigmoid(g2) sum_k moe_w moe_y) (+ table[ids]; init: x32 = table[ids]), t = y or ya n(y) wy + yb n(y2) wy2;
+        out = n(x32) w_in (out may be None; w_in None: x32 itself; rows ldo apart).  The gates are columns g1_off / g2_off of fp32 rows ldg apart."""
         width = x32.shape[-1]
         wt = w_in if w_in is not None else table if table is not None else wy
         dt = dtype if dtype is not None else wt.dtype
@@ -1169,8 +1198,21 @@ class ExtC:
             self._ptr(wy2, dt, "wy2"), float(ya), float(yb), g1, g2, int(ldg), self._ptr(moe_y, torch.float32, "moe_y"),
             self._ptr(moe_w, torch.float32, "moe_w"), int(top), self._ptr(table, dt, "table"), self._ptr(ids, torch.int32, "ids"),
             table.shape[0] if table is not None else 0, int(init), self._ptr(w_in, dt, "w_in"), self._ptr(out, None, "out"),
-            int(out is not None and out.dtype is torch.float32), self._ptr(row_idx, torch.int32, "row_idx"), self._dense_code(dt), int(rows),
-            int(width), float(eps), self._stream(x32)))
+            int(out is not None and out.dtype is torch.float32), int(ldo or width), self._ptr(row_idx, torch.int32, "row_idx"),
+            self._dense_code(dt), int(rows), int(width), float(mult), float(eps), self._stream(x32)))
+
+    def moe_route_chosen(self, logits, ldl: int, logits_off: int, ids, wts, rows: int, n_total: int, top: int, scale: float = 1.0,
+                         extra: int = 0, extra_col: int = -1, groups=None) -> None:
+        """router whose weights are the softmax over the chosen logits (columns logits_off .. + n_total of fp32 rows ldl apart); extra experts
+        every token uses behind them, weighted by sigmoid(column logits_off + extra_col) (extra_col < 0: 1)"""
+        gc, go, gr = groups if groups is not None else (None, None, None)
+        if ids.numel() < rows * (top + extra) or wts.numel() < rows * (top + extra):
+            raise RuntimeError("moe_route_chosen: ids / wts smaller than rows x choices")
+        self.lib.check(self.lib.exl2_moe_route_chosen(
+            self._ptr(logits, torch.float32, "logits") + 4 * logits_off, int(ldl), self._ptr(ids, torch.int32, "ids"),
+            self._ptr(wts, torch.float32, "wts"), int(rows), int(n_total), int(top), float(scale), int(extra), int(extra_col),
+            self._ptr(gc, torch.int32, "grp_count"), self._ptr(go, torch.int32, "grp_offset"), self._ptr(gr, torch.int32, "grp_rows"),
+            self._stream(logits)))
 
     def moe_route_grouped(self, logits, ldl: int, logits_off: int, ids, wts, rows: int, n_total: int, top: int, scale: float = 1.0,
                           group_count: int = 1, group_keep: int = 1, groups=None) -> None:

@@ -5,9 +5,9 @@ bias, logits from the embedding table, optional soft cap), or pre-norm steps wit
 of every mixer (a `head` matrix, scaled logits), or sandwich-normed steps  x <- x + mult n_g(sublayer(conv_in(n_g(x) w))) w'  with
 grouped RMS norms, a short input convolution and a token-pair table beside the embedding, or layers with ONE RMS norm whose mixer and
 feed-forward stand side by side behind gates, x <- x + mixer(h) sigmoid(W_1 h + b_1) + ff(h) sigmoid(W_2 h + b_2), some of them gone
-through several times.  Mixers: latent attention, windowed /
+through several times, or plain pre-norm steps  x <- x + mult sublayer(n(x) w)  whose loop starts every pass from W [x; embedding].  Mixers: latent attention, windowed /
 chunked / plain causal attention (pooled blocks, sinks, shared keys and values), state-space scan, decaying linear attention, linear
-attention whose forget gate writes, gated delta rule, minimal gated recurrence, two mixers side by side; a stack may mix them -- each keeps what it needs between steps (pages
+attention whose forget gate writes, gated delta rule (decay per head or per key channel), minimal gated recurrence, two mixers side by side; a stack may mix them -- each keeps what it needs between steps (pages
 of keys and values, per-slot recurrent state) under one page pool.
 
 The model has ONE forward, `step(batch, cache)`: the rows of a step are a flat list of tokens, each with its sequence slot and
@@ -28,9 +28,9 @@ from .latent_attn import LatentAttention
 from .linear_attn import ForgetGateLinearAttention, GatedDeltaRule
 from .mingru import MinimalGRU
 from .mlp import DenseActMLP, DenseGatedMLP
-from .moe_mlp import ScoredMoEMLP, SigmoidMoEMLP
+from .moe_mlp import ChosenSoftmaxMoEMLP, ScoredMoEMLP, SigmoidMoEMLP
 from .parallel_mixer import ParallelMixer
-from .rmsnorm import GatedResidualNorm, PostNorm, PreLayerNorm, PreShiftRMSNorm, SandwichNorm
+from .rmsnorm import GatedResidualNorm, PostNorm, PreLayerNorm, PreRMSNorm, PreShiftRMSNorm, SandwichNorm
 from .ssm import StateSpaceMixer
 from .window_attn import WindowAttention
 from .wkv import DecayLinearAttention
@@ -85,9 +85,18 @@ def _causal_attention(model, key, idx, m, out_tag="mix.y", **kw):
 
 
 def _parallel(model, key, idx, spec):
-    """softmax attention (left) beside a recurrence (right: a state-space scan, or a minimal gated recurrence) on the same input"""
+    """softmax attention (left) beside a recurrence (right: a state-space scan, a minimal gated recurrence, or a delta rule with a decay per
+    key channel) on the same input"""
     m = spec["mixer"]
     r = m["right"]
+    if model.config.residual == "pre_rms":
+        # half the sum of both results, each normed over the model width; normed queries and keys, first tokens stay visible
+        left = _causal_attention(model, key + ".left", (idx, "left"), m["left"], out_tag="mix.y.left", joined=True, head_norm=True,
+                                 keep=int((m["left"].get("mask") or {}).get("keep_first") or 0))
+        right = GatedDeltaRule(model, key + ".right", (idx, "right"), heads=int(r["heads"]), kv_heads=int(r.get("kv_heads") or r["heads"]),
+                               dim=int(r["dim"]), vdim=int(r["vdim"]), taps=int(r["conv"]), out_tag="mix.y.right", channel_decay=True,
+                               joined=True)
+        return ParallelMixer(model, key, idx, left, right, 0.5, 0.5, out_norms=True)
     if model.config.residual == "parallel_gated":
         # half the sum of both results, each normed over the model width
         left = _causal_attention(model, key + ".left", (idx, "left"), m["left"], out_tag="mix.y.left", interleaved=True, joined=True)
@@ -114,11 +123,15 @@ def _delta_rule(model, key, idx, spec):
 def _dense_mlp(model, key, idx, spec):
     if model.config.residual == "pre_ln":                      # two matrices, squared relu between them
         return DenseActMLP(model, key, idx)
-    return DenseGatedMLP(model, key, idx)
+    return DenseGatedMLP(model, key, idx, limit=float(spec["limit"]) if spec.get("limit") is not None else None)
 
 
 def _moe_mlp(model, key, idx, spec):
     r, e = spec["router"], spec["expert"]
+    if model.config.residual == "pre_rms":                    # softmax over the chosen logits; a gated shared expert
+        shared = spec.get("shared")
+        return ChosenSoftmaxMoEMLP(model, key, idx, experts=int(r["experts"]), top=int(r["top"]), ff=int(e["ff"]),
+                                   shared_ff=int(shared["ff"]) if shared else None)
     if model.config.residual == "parallel_gated":             # sigmoid scores among the best groups weigh the experts' outputs
         gr = r.get("groups")
         return SigmoidMoEMLP(model, key, idx, experts=int(r["experts"]), top=int(r["top"]), ff=int(e["ff"]), shared_ff=None, act="gelu",
@@ -217,7 +230,8 @@ class LayeredModel:
         if tuple(self.embed.shape) != (cfg.vocab, cfg.width):
             raise RuntimeError(f"embed is {tuple(self.embed.shape)}, config says {(cfg.vocab, cfg.width)}")
         gated = cfg.residual == "parallel_gated"
-        pre = cfg.residual in ("pre_ln", "pre_rms_shift", "sandwich") or gated
+        plain = cfg.residual == "pre_rms"
+        pre = cfg.residual in ("pre_ln", "pre_rms_shift", "sandwich") or gated or plain
 
         def make_norm(name, shift=None):
             if cfg.residual == "sandwich":
@@ -228,6 +242,8 @@ class LayeredModel:
                                     cfg.norm_groups, cfg.norm_eps, cfg.residual_mult)
             if gated:
                 return GatedResidualNorm(self.ext, name, need(name), cfg.norm_eps)
+            if plain:
+                return PreRMSNorm(self.ext, name, need(name), cfg.norm_eps, cfg.residual_mult)
             if cfg.residual == "pre_rms_shift":
                 return PreShiftRMSNorm(self.ext, name, need(name), cfg.norm_eps, shift=need(shift) if shift else None)
             if pre:
@@ -253,6 +269,8 @@ class LayeredModel:
             self.layers.append((mixer, norm1, ff, norm2))
             if gated:
                 self.fronts.append(self._join_front(key, mixer, ff, need))
+            elif plain:
+                self.fronts.append((JoinedFront(self.ext, key + ".front", getattr(mixer, "front_members", [mixer])), None, None))
         for i, (mixer, *_rest) in enumerate(self.layers):
             j = getattr(mixer, "kv_from", None)
             if j is not None:
@@ -282,6 +300,13 @@ class LayeredModel:
                 self.pair_table = need("bigram")
                 if tuple(self.pair_table.shape) != (cfg.pair_embedding["buckets"] + 1, cfg.width):
                     raise RuntimeError(f"bigram is {tuple(self.pair_table.shape)}, config says {(cfg.pair_embedding['buckets'] + 1, cfg.width)}")
+        self.loop_in = None
+        if plain:
+            self.embed_norm = need("embed.norm")
+            if any(enters for _i, _p, enters in cfg.layer_runs()):
+                self.loop_in = DenseLinear(self.ext, "loop.in", need("loop.in"))
+                if tuple(self.loop_in.weight.shape) != (cfg.width, 2 * cfg.width):
+                    raise RuntimeError(f"loop.in is {tuple(self.loop_in.weight.shape)}, config says {(cfg.width, 2 * cfg.width)}")
         self.head = DenseLinear(self.ext, "head", self.embed if cfg.tied_head else need("head"))
         self.loaded = True
         return self
@@ -302,8 +327,10 @@ class LayeredModel:
     def weight_bytes(self) -> int:
         """bytes a decoded token streams (a tied output table counts once: the embedding reads one row of it)"""
         n = self.head.weight_bytes()
-        for i, _pass, _embed in self.config.layer_runs():
+        for i, _pass, embed in self.config.layer_runs():
             mixer, _n1, ff, _n2 = self.layers[i]
+            if embed and getattr(self, "loop_in", None) is not None:
+                n += self.loop_in.weight_bytes()
             n += mixer.weight_bytes() + (ff.weight_bytes() if ff is not None else 0) + (self.fronts[i][0].weight_bytes() if self.fronts else 0)
         return n
 
@@ -354,6 +381,8 @@ class LayeredModel:
             return self._step_sandwich(batch, cache)
         if cfg.residual == "parallel_gated":
             return self._step_parallel_gated(batch, cache)
+        if cfg.residual == "pre_rms":
+            return self._step_pre_rms(batch, cache)
         x32 = self.buf("x32", (rows, self.width), torch.float32)
         xh = x32 if self.dtype is torch.float32 else self.buf("xh", (rows, self.width), self.dtype)
         ext.embed_scale(self.embed, batch.ids, x32, xh, cfg.embedding_scale)
@@ -484,6 +513,43 @@ class LayeredModel:
             mix = ff.forward(xh, rows, front=front)[1] if ff is not None else None
             pending = (y, getattr(mixer, "out_norms", None), front, g1, g2, mix)
         xn = self.buf("xn", (max(batch.n_logits, 1), self.width), self.dtype)
+        if batch.logits_all_rows and batch.n_logits == rows:
+            self.final_norm.forward(x32, pending, xn, rows, dtype=self.dtype)       # the last addition and the final norm in one launch
+        else:
+            self.final_norm.forward(x32, pending, None, rows, dtype=self.dtype)
+            if batch.n_logits == 0:
+                return None
+            self.final_norm.forward(x32, None, xn, batch.n_logits, row_idx=batch.logit_rows, dtype=self.dtype)
+        return self.head.forward(xn, batch.n_logits, out=self.buf("logits", (batch.n_logits, self.vocab), f32))
+
+    def _step_pre_rms(self, batch: StepBatch, cache) -> torch.Tensor | None:
+        """x <- x + mult mixer(n(x) w1), x <- x + mult ff(n(x) w2): per layer ONE linear brings everything that reads the mixer's input, and
+        every residual addition -- two normed results of mixers side by side, a linear's output, the chosen experts' weighted rows -- runs
+        in the launch of the norm that follows it.  A loop starts every pass from W_in [x; x0], x0 the normed embedding: the embedding's
+        launch leaves x0 in the second half of that linear's input, the residual step in front of a pass leaves x in the first.  A looped
+        layer finds the memory of its pass in `cache.at_pass`.  Logits: head(n(x) w) for the wanted rows."""
+        ext, cfg, rows, f32, width = self.ext, self.config, batch.rows, torch.float32, self.width
+        x32 = self.buf("x32", (rows, width), f32)
+        xh = self.buf("xh", (rows, width), self.dtype)
+        both = self.buf("loop.x", (rows, 2 * width), self.dtype) if self.loop_in is not None else None
+        ext.embed_pair(self.embed, None, self.embed_norm, batch.ids, None, batch.row_seq, batch.row_pos, batch.spans_dev, x32, 0, 0, 0,
+                       cfg.embedding_scale, 1, cfg.norm_eps, xh=both, xh_off=width)
+        pending = None
+        for i, loop_pass, enters in cfg.layer_runs():
+            mixer, norm1, ff, norm2 = self.layers[i]
+            if enters:
+                norm1.copy_stream(x32, pending, both, rows, 2 * width, dtype=self.dtype)
+                self.loop_in.forward(both, rows, out=x32)
+                pending = None
+            norm1.forward(x32, pending, xh, rows, dtype=self.dtype)
+            front = self.fronts[i][0].forward(xh, rows, self)
+            y = mixer.forward(xh, rows, batch, cache.at_pass(loop_pass) if loop_pass else cache, front=front)
+            pending = (y, getattr(mixer, "out_norms", None), None)
+            if ff is not None:
+                norm2.forward(x32, pending, xh, rows, dtype=self.dtype)
+                y, mix = ff.forward(xh, rows)
+                pending = (y, None, mix)
+        xn = self.buf("xn", (max(batch.n_logits, 1), width), self.dtype)
         if batch.logits_all_rows and batch.n_logits == rows:
             self.final_norm.forward(x32, pending, xn, rows, dtype=self.dtype)       # the last addition and the final norm in one launch
         else:

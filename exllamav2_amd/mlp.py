@@ -43,11 +43,12 @@ class ExLlamaV2MLP:
 
 class DenseGatedMLP:
     """Gated MLP over unquantized weights: W_down(silu(W_gate h) * (W_up h)) in three launches -- the activation and the product
-    run in the up projection's epilogue (csrc/dense.hip).  Returns the sublayer's output in fp32; the residual step is the
-    caller's (pre- or post-norm)."""
+    run in the up projection's epilogue (csrc/dense.hip).  `limit`: the clamped unit W_down(a sigmoid(1.702 a) (u + 1)),
+    a = min(W_gate h, limit), u = clamp(W_up h, +-limit) instead.  Returns the sublayer's output in fp32 (`row_gate` = (fp32 rows, leading
+    dimension, column): times the sigmoid of that column, one number per row); the residual step is the caller's (pre- or post-norm)."""
 
-    def __init__(self, model, key: str, layer_idx: int):
-        self.model, self.ext, self.key, self.layer_idx = model, model.ext, key, layer_idx
+    def __init__(self, model, key: str, layer_idx: int, limit: float | None = None):
+        self.model, self.ext, self.key, self.layer_idx, self.limit = model, model.ext, key, layer_idx, limit
 
     def load(self, get):
         from .dense_linear import DenseLinear
@@ -59,11 +60,13 @@ class DenseGatedMLP:
     def weight_bytes(self) -> int:
         return self.gate.weight_bytes() + self.up.weight_bytes() + self.down.weight_bytes()
 
-    def forward(self, xh: torch.Tensor, rows: int):
-        m, ff = self.model, self.gate.out_features
+    def forward(self, xh: torch.Tensor, rows: int, row_gate=None):
+        m, ff, ext = self.model, self.gate.out_features, self.ext
         g = self.gate.forward(xh, rows, out=m.buf("ff.g", (rows, ff), torch.float32))
-        a = self.up.forward(xh, rows, out=m.buf("ff.a", (rows, ff), m.dtype), aux=g, aux_ld=ff, epi=self.ext.EPI_SILU_AUX_MUL)
-        return self.down.forward(a, rows, out=m.buf("ff.y", (rows, m.width), torch.float32)), None
+        a = self.up.forward(xh, rows, out=m.buf("ff.a", (rows, ff), m.dtype), aux=g, aux_ld=ff,
+                            epi=ext.EPI_SILU_AUX_MUL if self.limit is None else ext.EPI_CLAMPED_GLU, limit=self.limit or 0.0)
+        kw = dict(aux=row_gate[0], aux_ld=row_gate[1], aux_off=row_gate[2], epi=ext.EPI_MUL_SIGMOID_ROW_AUX) if row_gate is not None else {}
+        return self.down.forward(a, rows, out=m.buf("ff.y", (rows, m.width), torch.float32), **kw), None
 
 
 class DenseActMLP:

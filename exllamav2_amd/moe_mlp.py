@@ -224,3 +224,83 @@ class SigmoidMoEMLP:
         ext.dense_linear(a, self.down.weight, y, pairs, width, ff, ff, ff, width, swb=width * ff, **kw)
         ys = self.shared.forward(xh, rows)[0] if self.shared is not None else None
         return ys, (y, ids, wts, S)
+
+
+class ChosenSoftmaxMoEMLP:
+    """Sparse MoE whose router picks the `top` largest logits z = W_router h + b (fp32) and weighs their experts by the softmax over the
+    chosen logits alone.  Experts are gated units W_down (silu(W_gate h) * (W_up h)) whose OUTPUTS carry the weights; the weighted sum is
+    the residual step's (rmsnorm.PreRMSNorm).  A shared expert of the same form runs for every token times sigmoid(W_sg h), one number
+    per token whose projection is one more row of the router's linear: where its width is a whole multiple of the routed ones' it is cut
+    into slabs of their width (W_down (a_1 | a_2) = W_down,1 a_1 + W_down,2 a_2) that stand behind them and ride their launches as further
+    pairs of every token, otherwise it runs as a feed-forward of its own whose last linear applies the sigmoid.  Few rows: every (token,
+    choice) pair names its expert's slab; many rows: one grouped launch per projection.
+    forward returns (the shared expert's output | None, mixture)."""
+
+    PAIR_ROWS_MAX = 64
+
+    def __init__(self, model, key: str, layer_idx: int, *, experts: int, top: int, ff: int, shared_ff: int | None):
+        self.model, self.ext, self.key, self.layer_idx = model, model.ext, key, layer_idx
+        self.experts, self.top, self.ff, self.shared_ff = experts, top, ff, shared_ff or 0
+        if not 0 < top <= experts or ff <= 0 or self.shared_ff < 0:
+            raise ValueError(f"{key}: top {top} of {experts} experts of {ff}, shared {shared_ff}")
+        self.extra = self.shared_ff // ff if self.shared_ff % ff == 0 else 0      # slabs of the shared expert among the routed ones
+
+    def load(self, get):
+        from .dense_linear import DenseLinear
+        from .mlp import DenseGatedMLP
+        E, ff, width, n = self.experts, self.ff, self.model.width, self.extra
+        router, bias = get("router"), get("router.b").to(torch.float32).reshape(-1)
+        if tuple(router.shape) != (E, width) or bias.numel() != E:
+            raise RuntimeError(f"{self.key}: the router is {tuple(router.shape)} with {bias.numel()} biases for {E} experts")
+        if self.shared_ff:
+            sg = get("shared.sg").reshape(-1, width)
+            if sg.shape[0] != 1:
+                raise RuntimeError(f"{self.key}: the shared expert's gate is one number per token")
+            router, bias = torch.cat([router, sg], 0), torch.cat([bias, bias.new_zeros((1,))])
+        self.router, self.router_bias = DenseLinear(self.ext, self.key + ".router", router), bias.contiguous()
+
+        def slabs(name, cut):
+            parts = [get(f"e{e}.{name}") for e in range(E)]
+            return torch.stack(parts + ([cut(get("shared." + name), i) for i in range(n)] if n else []), 0)
+        rows_of, cols_of = (lambda w, i: w[i * ff:(i + 1) * ff]), (lambda w, i: w[:, i * ff:(i + 1) * ff])
+        if self.shared_ff and (tuple(get("shared.gate").shape) != (self.shared_ff, width) or tuple(get("shared.up").shape) != (self.shared_ff, width)
+                               or tuple(get("shared.down").shape) != (width, self.shared_ff)):
+            raise RuntimeError(f"{self.key}: the shared expert's tensors do not match its width of {self.shared_ff}")
+        self.gate = DenseLinear(self.ext, self.key + ".gate", slabs("gate", rows_of))
+        self.up = DenseLinear(self.ext, self.key + ".up", slabs("up", rows_of))
+        self.down = DenseLinear(self.ext, self.key + ".down", slabs("down", cols_of))
+        if tuple(self.gate.weight.shape) != (E + n, ff, width) or tuple(self.up.weight.shape) != (E + n, ff, width) \
+                or tuple(self.down.weight.shape) != (E + n, width, ff):
+            raise RuntimeError(f"{self.key}: tensor shapes do not match the feed-forward's sizes")
+        self.shared = None
+        if self.shared_ff and not n:
+            self.shared = DenseGatedMLP(self.model, self.key + ".shared", self.layer_idx).load(lambda name: get("shared." + name))
+        return self
+
+    def weight_bytes(self) -> int:
+        per_slab = (self.gate.weight_bytes() + self.up.weight_bytes() + self.down.weight_bytes()) // (self.experts + self.extra)
+        n = self.router.weight_bytes() + per_slab * (self.top + self.extra)
+        return n + (self.shared.weight_bytes() if self.shared is not None else 0)
+
+    def forward(self, xh: torch.Tensor, rows: int):
+        ext, m = self.ext, self.model
+        E, ff, width, per_row, S = self.experts, self.ff, m.width, self.top + self.extra, self.experts + self.extra
+        ldl = self.router.out_features
+        logits = self.router.forward(xh, rows, out=m.buf("moe.logits", (rows, ldl), torch.float32), bias=self.router_bias)
+        ids = m.buf("moe.ids", (rows, per_row), torch.int32)
+        wts = m.buf("moe.wts", (rows, per_row), torch.float32)
+        pairs = rows * per_row
+        groups = None
+        if pairs > self.PAIR_ROWS_MAX:
+            groups = (m.buf("moe.count", (S,), torch.int32), m.buf("moe.offset", (S,), torch.int32), m.buf("moe.rows", (pairs,), torch.int32))
+        ext.moe_route_chosen(logits, ldl, 0, ids, wts, rows, E, self.top, extra=self.extra, extra_col=E if self.extra else -1, groups=groups)
+        g = m.buf("moe.g", (pairs, ff), torch.float32)
+        a = m.buf("moe.a", (pairs, ff), m.dtype)
+        y = m.buf("moe.y", (pairs, width), torch.float32)
+        kw = dict(batch=S, groups=groups) if groups is not None else dict(w_sel=ids.view(-1), n_sel=S)
+        ext.dense_linear(xh, self.gate.weight, g, pairs, ff, width, width, width, ff, swb=ff * width, x_div=per_row, **kw)
+        ext.dense_linear(xh, self.up.weight, a, pairs, ff, width, width, width, ff, swb=ff * width, x_div=per_row, aux=g, ldaux=ff,
+                         epi=ext.EPI_SILU_AUX_MUL, **kw)
+        ext.dense_linear(a, self.down.weight, y, pairs, width, ff, ff, ff, width, swb=width * ff, **kw)
+        ys = self.shared.forward(xh, rows, row_gate=(logits, ldl, E))[0] if self.shared is not None else None
+        return ys, (y, ids, wts, S)

@@ -165,3 +165,36 @@ class GatedResidualNorm:
                 kw.update(moe_y=mix[0], moe_w=mix[2], top=mix[2].shape[-1])
         self.ext.gated_residual(x32, out, rows, self.eps, w_in=self.weight if out is not None else None, table=table if ids is not None else None,
                                 ids=ids, init=init, row_idx=row_idx, dtype=dtype, **kw)
+
+
+class PreRMSNorm:
+    """The norm in front of a sublayer of a plain pre-norm layer, n(x) w with n(v) = v / sqrt(mean(v^2) + eps), fused with the residual
+    addition of the sublayer BEFORE it, x <- x + mult * y: the same launch as GatedResidualNorm's without gates (csrc/rowops.hip).  y is a
+    linear's output, the weighted sum of two separately normed results (ParallelMixer with `out_norms`), the weighted rows of a token's
+    chosen experts, or a linear's output plus those.  `copy_stream` makes the addition and hands the stream itself on in the operand
+    dtype (what a linear of the stream reads) instead of a normed row."""
+
+    def __init__(self, ext, key: str, weight: torch.Tensor, eps: float, mult: float):
+        self.ext, self.key, self.weight, self.eps, self.mult = ext, key, weight.contiguous(), float(eps), float(mult)
+
+    @staticmethod
+    def _pending_args(pending) -> dict:
+        """pending: None or (sublayer result(s) | None, norms behind two halves | None, mixture | None)"""
+        kw = {}
+        if pending is not None:
+            y, norms, mix = pending
+            if norms is not None:
+                kw.update(y=y[0], ya=y[1], y2=y[2], yb=y[3], wy=norms[0], wy2=norms[1])
+            elif y is not None:
+                kw.update(y=y)
+            if mix is not None:
+                kw.update(moe_y=mix[0], moe_w=mix[2], top=mix[2].shape[-1])
+        return kw
+
+    def forward(self, x32: torch.Tensor, pending, out: torch.Tensor | None, rows: int, row_idx=None, dtype=None) -> None:
+        """out (operand dtype or fp32, [rows, width]) takes the normed rows; None: only the additions"""
+        self.ext.gated_residual(x32, out, rows, self.eps, w_in=self.weight if out is not None else None, row_idx=row_idx, dtype=dtype,
+                                mult=self.mult, **self._pending_args(pending))
+
+    def copy_stream(self, x32: torch.Tensor, pending, out: torch.Tensor, rows: int, ldo: int, dtype=None) -> None:
+        self.ext.gated_residual(x32, out, rows, self.eps, dtype=dtype, mult=self.mult, ldo=ldo, **self._pending_args(pending))

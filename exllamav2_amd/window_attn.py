@@ -17,6 +17,8 @@ pair layout, score scale, and the variants
     kv_from      the layer has no key / value projections: it attends over the rows layer `kv_from` cached, with its own queries
     conv_taps    q, k and v (biases added) pass a short causal convolution over time per channel before the rotation; the last
                  conv_taps - 1 projected rows of every sequence are kept per slot
+    keep         the first `keep` tokens stay visible however far the window has moved on (their distances are the true ones)
+    head_norm    every query and key head is divided by its root mean square over dim after the rotation (no weight, the model's eps)
     talk         the heads exchange their (capped) scores before the softmax, s_h <- sum_g T[h, g] s_g  (csrc/talk_attn.hip; a window,
                  without pooled blocks, chunks, gate or rotated values)
     joined       the projections are part of a linear the layer shares (dense_linear.JoinedFront)
@@ -73,7 +75,7 @@ class WindowAttention:
     def __init__(self, model, key: str, layer_idx: int, *, heads: int, kv_heads: int, dim: int, vdim: int, window: int, pool: int,
                  rot_base: float, rot_dims: int, rot_scaling: dict | None, scale: float, rotate_values: bool = True,
                  interleaved: bool = False, chunk: int = 0, softcap: float = 0.0, sink_one: bool = False, kv_from: int | None = None,
-                 out_tag: str = "mix.y", conv_taps: int = 0, talk: bool = False, joined: bool = False):
+                 out_tag: str = "mix.y", conv_taps: int = 0, talk: bool = False, joined: bool = False, keep: int = 0, head_norm: bool = False):
         self.model, self.ext, self.key, self.layer_idx = model, model.ext, key, layer_idx
         self.heads, self.kv_heads, self.dim, self.vdim = heads, kv_heads, dim, vdim
         self.window, self.pool, self.scale = window, pool, scale
@@ -81,10 +83,13 @@ class WindowAttention:
         self.rotate_values, self.interleaved = rotate_values, interleaved
         self.chunk, self.softcap, self.sink_one, self.kv_from = int(chunk), float(softcap), bool(sink_one), kv_from
         self.out_tag, self.conv_taps, self.talk, self.joined = out_tag, int(conv_taps), bool(talk), bool(joined)
+        self.keep, self.head_norm = int(keep), bool(head_norm)
         self.front, self.front_base = None, 0
         if heads % kv_heads or rot_dims > dim or rot_dims % 2 or (rotate_values and vdim % 2) or window <= 0 or pool < 0 \
                 or chunk < 0 or (chunk and pool) or softcap < 0:
             raise ValueError(f"{key}: inconsistent attention sizes")
+        if self.keep < 0 or (self.keep and (pool or chunk or talk)) or (self.head_norm and rotate_values):
+            raise ValueError(f"{key}: kept first tokens go with a plain window, head norms with values as they are")
         if (self.talk and (pool or chunk or rotate_values)) or (self.conv_taps and kv_from is not None):
             raise ValueError(f"{key}: head mixing goes with a plain window, a convolution with keys and values of the layer's own")
         self.tiles_ok = self.ext.window_attn_tiles_supported(model.dtype, dim, vdim) and (self.heads * vdim) % 4 == 0
@@ -190,15 +195,15 @@ class WindowAttention:
         ext.kv_rot_append(qkv, ld, at, at + self.off_k, at + self.off_v, q, self.q_scale, st.k if own else None, st.v if own else None,
                           st.k_pool if own else None, st.v_pool if own else None, self.freq, self.amp,
                           self.rot_dims, self.vfreq, self.rotate_values, self.interleaved, batch.row_seq, batch.row_pos, batch.block_table,
-                          page, self.pool if own else 0, rows, H, G, dim, vd)
+                          page, self.pool if own else 0, rows, H, G, dim, vd, head_norm_eps=m.norm_eps if self.head_norm else None)
         o = m.buf("attn.o", (rows, H * vd), m.dtype)
         if self.talk:
             self._talk(q, st, batch, page, o, rows)
             return self.o.forward(o, rows, out=m.buf(self.out_tag, (rows, m.width), f32), bias=self.o_bias)
         common = (q, st.k, st.v, st.k_pool, st.v_pool, self.sink, f if self.gated else None, ncat, base + self.off_g, self.vfreq, self.rotate_values, self.interleaved,
                   batch.row_seq, batch.row_pos, batch.block_table, page, self.pool, o)
-        var = dict(chunk=self.chunk, softcap=self.softcap, gate_head=self.gate_head)
-        reach = self.chunk or self.window                     # the most tokens a position sees
+        var = dict(chunk=self.chunk, softcap=self.softcap, gate_head=self.gate_head, keep=self.keep)
+        reach = self.chunk or self.window + self.keep         # the most tokens a position sees
         if self.tiles_ok and (batch.prompt_tiles is not None or batch.tiles1 is not None):
             # matrix-core kernels: portions of prompts as tiles of <= 64 positions x one head per workgroup, decoded tokens as one
             # row x one key / value head per workgroup (its query heads share the pass over the keys)

@@ -443,6 +443,11 @@ int exl2_dense_linear_bias(const void* x, const void* w, const float* bias, void
                            int batch, long long sxb, long long swb, long long syb, long long sauxb,
                            const int* w_sel, int n_sel, const int* grp_count, const int* grp_offset, const int* grp_rows,
                            int x_div, int epi, float limit, void* stream);
+/* y[r, n] = x[r] . w[n] + bias[n] with the columns split: n < n2 -> y (fp32 or operand dtype), n >= n2 -> y2[r * ldy2 + n - n2] in the
+   operand dtype (what a further linear reads); plain one-slab call without epilogue.  (Epilogue 13 of the other forms:
+   exp(aux softplus(acc)); ldaux = 0: one aux value per column.) */
+int exl2_dense_linear_split(const void* x, const void* w, const float* bias, void* y, int y_f32, void* y2, int n2, int ldy2,
+                            int dtype, int M, int N, int K, int ldx, int ldw, int ldy, void* stream);
 /* the pre-norm residual step: x[r] += y[r] (y nullable) on the fp32 stream, then out[r] = (x - mean) / sqrt(var + eps) * w + b in
    the operand dtype (or fp32); w == NULL: only the addition.  row_idx (nullable, no addition then): output row r is made from
    stream row row_idx[r]. */
@@ -519,24 +524,26 @@ int exl2_window_attn_tiles(const void* q, const void* k_cache, const void* v_cac
               counted from the sequence's start (pool must be 0);
    softcap > 0: score <- softcap * tanh(score / softcap) before the softmax;
    gate_head: gate holds ONE value per head (gate[r * ldg + h]) instead of one per output value;
+   keep > 0: position p also sees the sequence's first `keep` tokens, however far back (no pooled blocks, no chunks);
+   head_norm: every query and key head is divided by sqrt(mean(.^2) + norm_eps) after its rotation (values are not rotated then);
    exl2_kv_rot_append_ex with k_cache == v_cache == NULL: the rows bring queries only (a layer that attends over the keys and
    values another layer cached). */
 int exl2_kv_rot_append_ex(const float* f, int ld, int q_off, int k_off, int v_off, void* q_out, const float* q_scale,
                           void* k_cache, void* v_cache, void* k_pool, void* v_pool, const float* freq, float amp, int rot_dims,
                           const float* vfreq, int v_rot, int interleaved, const int* row_seq, const int* row_pos,
                           const int* block_table, int bt_stride, int page, int pool, int dtype, int rows, int heads,
-                          int kv_heads, int dim, int vdim, void* stream);
+                          int kv_heads, int dim, int vdim, int head_norm, float norm_eps, void* stream);
 int exl2_window_attn_ex(const void* q, const void* k_cache, const void* v_cache, const void* k_pool, const void* v_pool,
                         const float* sink, const float* gate, int ldg, const float* vfreq, int v_rot, int interleaved,
                         const int* row_seq, const int* row_pos, const int* block_table, int bt_stride, int page, int pool,
-                        void* out, int dtype, int rows, int heads, int kv_heads, int dim, int vdim, int window, int chunk,
-                        float softcap, int gate_head, void* stream);
+                        void* out, int dtype, int rows, int heads, int kv_heads, int dim, int vdim, int window, int keep,
+                        int chunk, float softcap, int gate_head, void* stream);
 int exl2_window_attn_tiles_ex(const void* q, const void* k_cache, const void* v_cache, const void* k_pool, const void* v_pool,
                               const float* sink, const float* gate, int ldg, const float* vfreq, int v_rot, int interleaved,
                               const int* row_seq, const int* row_pos, const int* block_table, int bt_stride, int page, int pool,
                               void* out, const int* tile_row0, const int* tile_rows, int tiles, int tile_mode, float* part_o,
-                              float* part_ml, int nsplit, int heads, int kv_heads, int dim, int vdim, int window, int chunk,
-                              float softcap, int gate_head, void* stream);
+                              float* part_ml, int nsplit, int heads, int kv_heads, int dim, int vdim, int window, int keep,
+                              int chunk, float softcap, int gate_head, void* stream);
 
 /* ---- pre-norm stacks with a scalar-gain RMS norm and a token shift (csrc/rowops.hip).  Further epilogues of exl2_dense_linear(_bias):
    6 acc * limit, 7 tanh(acc), 8 relu(aux[row * ldaux] * acc)^2 (ONE aux value per row). */
@@ -602,10 +609,11 @@ int exl2_sandwich_norm(float* x, const float* y, float ya, const float* y2, floa
                        int width, int groups, float eps, void* stream);
 /* x[r] = n_g(table[ids[r]] * scale + pair[(t' * mul_prev + ids[r] * mul_cur) mod buckets]) w, t' = the previous token of the row's
    sequence (the row in front within a span, else prev_tok[slot]); row `buckets` of pair at position 0.  Afterwards prev_tok holds
-   every span's last token.  pair and w nullable (no pair term / no norm). */
+   every span's last token.  pair and w nullable (no pair term / no norm).  xh (nullable): a copy of the rows in the operand dtype,
+   ldxh values apart. */
 int exl2_embed_pair(const void* table, const void* pair, const void* w, const int* ids, int* prev_tok, const int* row_seq,
                     const int* row_pos, const int* span_row0, const int* span_rows, int spans, int max_span_rows, float* x,
-                    int dtype, int rows, int width, int vocab, int buckets, int mul_prev, int mul_cur, float scale, int groups,
+                    void* xh, int ldxh, int dtype, int rows, int width, int vocab, int buckets, int mul_prev, int mul_cur, float scale, int groups,
                     float eps, void* stream);
 /* exl2_conv_silu_rows with a choice of output: residual 0: silu(conv + bias); 1: in + conv + bias; 2: conv + bias (no activation).  out fp32
    (out_f32 = 1) or the operand dtype. */
@@ -618,10 +626,11 @@ int exl2_conv_rows_ex(const float* in, int ld, const void* w, const void* bias, 
    mode 1: qq = q / sqrt(sum q^2 + 1e-6) * q_scale, kk = k / sqrt(sum k^2 + 1e-6) per head (q / k head h / (heads / qk_heads));
            b = sigmoid(beta[h]); g = exp(-exp(a_log[h]) softplus(dt[h] + dt_bias[h])); S <- g S; u = b (v - S^T kk); S <- S + kk u^T;
            o = S^T qq.
-   out = o / sqrt(mean(o^2) + eps) * norm_w (fp32 [n_val]) (* silu(gate), head h at h * n_val; nullable); [rows, ldo] operand dtype
+   mode 2: mode 1 with one decay per head and key channel, ready made: dt[h * n_key + n] multiplies row n of S (dt_bias, a_log unused).
+   out = o / sqrt(mean(o^2) + eps) * norm_w (fp32 [n_val]) (* silu(gate), or gate itself where gate_ready, head h at h * n_val; nullable); [rows, ldo] operand dtype
    (bfloat16) or fp32.  The state is read at a span's start (unless it starts at position 0) and written at its end. */
 int exl2_gated_scan(int mode, const float* q, int ldq, const float* k, int ldk, const float* v, int ldv, const float* gate,
-                    int ldg, const float* beta, int ldb, const float* dt, int lddt, const float* dt_bias, const float* a_log,
+                    int ldg, int gate_ready, const float* beta, int ldb, const float* dt, int lddt, const float* dt_bias, const float* a_log,
                     const float* lower, const float* norm_w, void* out, int ldo, int out_f32, float* state,
                     const int* span_row0, const int* span_rows, int spans, const int* row_seq, const int* row_pos, int heads,
                     int qk_heads, int n_key, int n_val, float q_scale, float eps, void* stream);
@@ -631,7 +640,7 @@ int exl2_gated_scan(int mode, const float* q, int ldq, const float* k, int ldk, 
    exl2_gated_scan_cols_supported returns 1; results agree with exl2_gated_scan to rounding. */
 int exl2_gated_scan_cols_supported(int n_key, int n_val);
 int exl2_gated_scan_cols(int mode, const float* q, int ldq, const float* k, int ldk, const float* v, int ldv, const float* gate,
-                         int ldg, const float* beta, int ldb, const float* dt, int lddt, const float* dt_bias,
+                         int ldg, int gate_ready, const float* beta, int ldb, const float* dt, int lddt, const float* dt_bias,
                          const float* a_log, const float* lower, const float* norm_w, void* out, int ldo, int out_f32,
                          float* state, const int* span_row0, const int* span_rows, int spans, const int* row_seq,
                          const int* row_pos, int rows, float* o_raw, int heads, int qk_heads, int n_key, int n_val,
@@ -641,18 +650,24 @@ int exl2_gated_scan_cols(int mode, const float* q, int ldq, const float* k, int 
    (csrc/mingru.hip), attention whose heads exchange their scores (csrc/talk_attn.hip), latent attention with a sink per head and either
    rotary layout (csrc/latent_attn.hip) */
 
-/* x[r] <- x[r] + t sigmoid(g1[r]) + sigmoid(g2[r]) sum_k moe_w[r, k] moe_y[r * top + k],  t = y[r], or ya n(y[r]) wy + yb n(y2[r]) wy2 when
+/* x[r] <- x[r] + mult (t sigmoid(g1[r]) + sigmoid(g2[r]) sum_k moe_w[r, k] moe_y[r * top + k]),  t = y[r], or ya n(y[r]) wy + yb n(y2[r]) wy2 when
    wy / wy2 are given;  x[r] <- x[r] + table[ids[r]] (ids nullable; init: x[r] = table[ids[r]], nothing is read);  then
-   out[r] = n(x[r]) w_in (out nullable), n(v) = v / sqrt(mean(v^2) + eps).  y, moe_y and the gates (fp32 rows ldg apart) are nullable.
+   out[r] = n(x[r]) w_in (out nullable; w_in nullable: x[r] itself; rows ldo apart), n(v) = v / sqrt(mean(v^2) + eps).  y, moe_y and the gates (fp32 rows ldg apart) are nullable.
    row_idx: output row r reads stream row row_idx[r] (no addition then).  Weights and table in the operand dtype. */
 int exl2_gated_residual(float* x, const float* y, const float* y2, const void* wy, const void* wy2, float ya, float yb,
                         const float* g1, const float* g2, int ldg, const float* moe_y, const float* moe_w, int top,
                         const void* table, const int* ids, int vocab, int init, const void* w_in, void* out, int out_f32,
-                        const int* row_idx, int dtype, int rows, int width, float eps, void* stream);
+                        int ldo, const int* row_idx, int dtype, int rows, int width, float mult, float eps, void* stream);
 /* exl2_moe_route_sigmoid with logits ldl apart and experts in group_count equal groups of neighbours: a group scores the sum of its two
    largest scores, only experts of the group_keep best groups can be chosen (the first of equals wins) */
 int exl2_moe_route_grouped(const float* logits, int ldl, int* ids, float* wts, int rows, int n_total, int top, float scale,
                            int group_count, int group_keep, int* grp_count, int* grp_offset, int* grp_rows, void* stream);
+/* router over logits ldl apart whose `top` largest logits choose (the first of equals wins) and whose weights are the softmax over the
+   chosen logits, times scale.  extra > 0: ids / wts are [rows, top + extra] and the last columns name the experts n_total .. n_total +
+   extra - 1 (what every token uses, stacked behind the routed ones) with weight sigmoid(logits[r * ldl + extra_col]) (extra_col < 0: 1).
+   grp_* as in exl2_moe_route_scored, over n_total + extra experts. */
+int exl2_moe_route_chosen(const float* logits, int ldl, int* ids, float* wts, int rows, int n_total, int top, float scale, int extra,
+                          int extra_col, int* grp_count, int* grp_offset, int* grp_rows, void* stream);
 /* exl2_latent_append / _attn / _attn_tiles with a choice of rotary layout (halves 0: pairs (2i, 2i + 1); 1: (i, i + rot_dims / 2)) and,
    nullable, a learned score per head (sink fp32 [heads]) that joins the softmax denominator without key or value */
 int exl2_latent_append_ex(const float* dkv, int ld, const void* norm_w, float eps, int dtype, int rows, int kv_rank, int rot,
