@@ -61,7 +61,7 @@ def parse():
     p.add_argument("--windows", type=int, default=5, help="timed windows of --steps steps (each after --warmup untimed steps from the same "
                                                            "cache position); the MEDIAN window is the reported value")
     p.add_argument("--headline-only", action="store_true", help="= --no-cpu-baseline --no-prefill --no-dropin --no-ctx-window (A/B runs)")
-    p.add_argument("--design", default=None, choices=["benolix", "tibalorn", "negilorn", "kilurax", "zevilorn"],
+    p.add_argument("--design", default=None, choices=["benolix", "tibalorn", "negilorn", "kilurax", "zevilorn", "savenex"],
                    help="instead of the headline: prefill / decode throughput of a layer-stack design at real layer sizes beside the "
                         "package's closest other model of equal size (benolix: latent attention + MoE beside the quantized Mixtral-style "
                         "stack; tibalorn: state-space + windowed attention beside a latent-attention stack; negilorn: chunked attention + decaying "

@@ -3,7 +3,7 @@ other model of the package at equal size: the latent-attention / scored-MoE stac
 expert width, expert count, depth), the state-space / windowed-attention stack beside a latent-attention stack (same width, depth,
 heads, window, feed-forward parameters), the token-shifted chunked-attention / linear-attention stack beside a state-space /
 windowed-attention stack (same width, depth, heads, reach, streamed feed-forward parameters), and so on for each later design.  Used by
-`bench.py --design benolix | tibalorn | negilorn | kilurax | zevilorn`; one JSON object per size and model."""
+`bench.py --design benolix | tibalorn | negilorn | kilurax | zevilorn | savenex`; one JSON object per size and model."""
 from __future__ import annotations
 
 import json
@@ -468,6 +468,9 @@ def sandwich_random_tensors(cfg: dict, device, seed: int = 0) -> dict:
             mat(k + ".mix.b", H, w); mat(k + ".mix.a", H, w); mat(k + ".mix.g", H * vd, w)
             vec(k + ".mix.dt_bias", H, -1.0, 0.5); vec(k + ".mix.A_log", H, -1.0, 0.5); vec(k + ".mix.norm", vd, 1.0); mat(k + ".mix.o", w, H * vd)
         ms = L["mlp"]
+        if ms["kind"] == "dense":
+            mat(k + ".mlp.gate", ms["ff"], w); mat(k + ".mlp.up", ms["ff"], w); mat(k + ".mlp.down", w, ms["ff"])
+            continue
         mat(k + ".mlp.router", ms["router"]["experts"], w)
         for n, ff in [(f"e{e}", ms["expert"]["ff"]) for e in range(ms["router"]["experts"])] + [("shared", ms["shared"]["ff"])]:
             mat(f"{k}.mlp.{n}.gate", ff, w); mat(f"{k}.mlp.{n}.up", ff, w); mat(f"{k}.mlp.{n}.down", w, ff)
@@ -625,8 +628,124 @@ def bench_gated_peer(size: str, device="cuda:0", prompt: int = 2048, ctx: int = 
     return _bench_engine(model, out, s["vocab"], prompt, ctx, decode_steps, batches)
 
 
+PLAIN_SIZES = {
+    # every layer: window attention beside a delta rule with a decay per key channel; pattern of the feed-forwards: d = dense, m = sparse
+    # with a shared expert; loop: those layers are gone through several times
+    "w2048": dict(width=2048, heads=16, kv_heads=4, dim=128, vdim=128, window=4096, keep=4, la_heads=16, la_kv_heads=8, la_dim=128, la_vdim=128,
+                  conv=4, rank=128, experts=8, top=2, expert_ff=2816, shared_ff=2816, dense_ff=8448, pattern="dmdm", loop=None, vocab=32000),
+    "w4096": dict(width=4096, heads=32, kv_heads=8, dim=128, vdim=128, window=4096, keep=4, la_heads=32, la_kv_heads=16, la_dim=128, la_vdim=128,
+                  conv=4, rank=128, experts=8, top=2, expert_ff=7168, shared_ff=7168, dense_ff=14336, pattern="dm", loop=None, vocab=32000),
+    "w2048-loop": dict(width=2048, heads=16, kv_heads=4, dim=128, vdim=128, window=4096, keep=4, la_heads=16, la_kv_heads=8, la_dim=128,
+                       la_vdim=128, conv=4, rank=128, experts=8, top=2, expert_ff=2816, shared_ff=2816, dense_ff=8448, pattern="dmd",
+                       loop={"start": 0, "stop": 2, "times": 3}, vocab=32000),
+}
+
+
+def plain_config(s: dict) -> dict:
+    m = {"left": {"dim": s["dim"], "heads": s["heads"], "kv_heads": s["kv_heads"], "vdim": s["vdim"], "scale": s["dim"] ** -0.5,
+                  "mask": {"size": s["window"], "keep_first": s["keep"]},
+                  "rot": {"base": 500000.0, "dims": s["dim"], "scaling": {"factor": 4.0}}},
+         "right": {"conv": s["conv"], "dim": s["la_dim"], "heads": s["la_heads"], "kv_heads": s["la_kv_heads"], "vdim": s["la_vdim"]}}
+    dense = {"ff": s["dense_ff"], "kind": "dense", "limit": 7.0}
+    moe = {"expert": {"ff": s["expert_ff"]}, "kind": "moe", "router": {"experts": s["experts"], "top": s["top"]}, "shared": {"ff": s["shared_ff"]}}
+    return {"architecture": "Savenex", "layers": [{"type": "parallel", "mixer": m, "mlp": dense if ch == "d" else moe} for ch in s["pattern"]],
+            "loop": s["loop"], "norm": {"eps": 1e-5}, "residual_mult": 0.7, "vocab": s["vocab"], "width": s["width"]}
+
+
+def plain_random_tensors(cfg: dict, rank: int, device, seed: int = 0) -> dict:
+    g = torch.Generator(device=device).manual_seed(seed)
+    T = {}
+
+    def mat(name, out, inp, gain=1.0):
+        T[name] = (torch.randn((out, inp), device=device, generator=g) * gain / inp ** 0.5).to(torch.bfloat16)
+
+    def vec(name, n, centre, spread=0.1):
+        T[name] = (centre + spread * torch.randn((n,), device=device, generator=g)).to(torch.bfloat16)
+
+    w = cfg["width"]
+    T["embed"] = (torch.randn((cfg["vocab"], w), device=device, generator=g) * 0.5).to(torch.bfloat16)
+    vec("embed.norm", w, 1.0); vec("final.norm", w, 1.0); mat("head", cfg["vocab"], w)
+    if cfg["loop"]:
+        mat("loop.in", w, 2 * w)
+    for i, L in enumerate(cfg["layers"]):
+        k, a, r = f"l{i}", L["mixer"]["left"], L["mixer"]["right"]
+        x, y = k + ".mix.left", k + ".mix.right"
+        vec(k + ".norm1", w, 1.0); vec(k + ".norm2", w, 1.0)
+        H, G, dim, vd = a["heads"], a["kv_heads"], a["dim"], a["vdim"]
+        mat(x + ".q", H * dim, w); mat(x + ".k", G * dim, w); mat(x + ".v", G * vd, w); mat(x + ".o", w, H * vd); vec(x + ".out", w, 1.0)
+        H, G, dim, vd = r["heads"], r["kv_heads"], r["dim"], r["vdim"]
+        for n, c in (("q", G * dim), ("k", G * dim), ("v", H * vd)):
+            mat(f"{y}.{n}", c, w)
+            T[f"{y}.{n}.conv"] = (0.5 * torch.randn((c, r["conv"]), device=device, generator=g)).to(torch.bfloat16)
+        mat(y + ".b", H, w); vec(y + ".A_log", H, -1.0, 0.5); vec(y + ".norm", vd, 1.0); mat(y + ".a1", rank, w); mat(y + ".a2", H * dim, rank)
+        vec(y + ".dt_bias", H * dim, -1.0, 0.5); mat(y + ".g1", rank, w); mat(y + ".g2", H * vd, rank); mat(y + ".o", w, H * vd); vec(y + ".out", w, 1.0)
+        ms = L["mlp"]
+        if ms["kind"] == "dense":
+            mat(k + ".mlp.gate", ms["ff"], w); mat(k + ".mlp.up", ms["ff"], w); mat(k + ".mlp.down", w, ms["ff"])
+            continue
+        mat(k + ".mlp.router", ms["router"]["experts"], w); vec(k + ".mlp.router.b", ms["router"]["experts"], 0.0); mat(k + ".mlp.shared.sg", 1, w)
+        for n, ff in [(f"e{e}", ms["expert"]["ff"]) for e in range(ms["router"]["experts"])] + [("shared", ms["shared"]["ff"])]:
+            mat(f"{k}.mlp.{n}.gate", ff, w); mat(f"{k}.mlp.{n}.up", ff, w); mat(f"{k}.mlp.{n}.down", w, ff)
+    return T
+
+
+def bench_plain(size: str, device="cuda:0", prompt: int = 2048, ctx: int = 1024, decode_steps: int = 64, batches=(1, 4)) -> dict:
+    from .config import LayeredConfig
+    from .layered import LayeredModel
+    s = PLAIN_SIZES[size]
+    cfg = plain_config(s)
+    lc = LayeredConfig.from_dict_prerms(cfg)
+    model = LayeredModel(lc, device=device, dtype=torch.bfloat16).load(plain_random_tensors(cfg, s["rank"], device))
+    out = {"design": "savenex", "size": size, "layers": len(cfg["layers"]), "layer_runs": len(lc.layer_runs()), "pattern": s["pattern"],
+           "weight_bytes_per_token": model.weight_bytes()}
+    return _bench_engine(model, out, s["vocab"], prompt, ctx, decode_steps, batches)
+
+
+def bench_plain_peer(size: str, device="cuda:0", prompt: int = 2048, ctx: int = 1024, decode_steps: int = 64, batches=(1, 4)) -> dict:
+    """the closest model of the package: a sandwich-normed stack (bfloat16, the same engine) of the same width with one layer per layer run,
+    by turns causal attention of the same heads beside a state-space scan (twice the heads of half the size) and a gated delta rule of the
+    same heads and state, the same kinds of feed-forward as much wider as it takes for a token to stream the same bytes"""
+    from .config import LayeredConfig
+    from .layered import LayeredModel
+    s = PLAIN_SIZES[size]
+    runs = LayeredConfig.from_dict_prerms(plain_config(s)).layer_runs()
+    w, H, G, dim, vd = s["width"], s["heads"], s["kv_heads"], s["dim"], s["vdim"]
+    Hr, Gr, dr, vr = s["la_heads"], s["la_kv_heads"], s["la_dim"], s["la_vdim"]
+    inner, state = Hr * vr, 128
+    attn = w * (H * dim + G * (dim + vd)) + w * H * vd
+    rule = w * (2 * Gr * dr + 2 * Hr * vr + Hr)
+    ours = len(runs) * (attn + rule + 2 * s["rank"] * w + 2 * s["rank"] * Hr * (dr + vr)) + 2 * w * w * sum(e for *_x, e in runs)
+    theirs = sum(attn + w * (3 * inner + 2 * state + 2 * Hr) if n % 2 == 0 else rule + w * (Hr + Hr * vr) for n in range(len(runs)))
+    extra = (ours - theirs) / len(runs) / (3 * w)
+    layers = []
+    for n, (i, _p, _e) in enumerate(runs):
+        if n % 2 == 0:
+            m = {"left": {"dim": dim, "heads": H, "kv_heads": G, "vdim": vd, "scale": dim ** -0.5, "rot": {"base": 500000.0, "dims": dim}},
+                 "left_scale": 1.0, "right_scale": 1.0,
+                 "right": {"conv": s["conv"], "groups": 1, "heads": 2 * Hr, "norm_groups": 1, "state": state, "vdim": vr // 2}}
+        else:
+            m = {"conv": s["conv"], "dim": dr, "heads": Hr, "kv_heads": Gr, "vdim": vr}
+        if s["pattern"][i] == "d":
+            ff = {"ff": s["dense_ff"] + int(extra) // 64 * 64, "kind": "dense"}
+        else:
+            more = int(extra / (s["top"] + 1)) // 64 * 64
+            ff = {"expert": {"ff": s["expert_ff"] + more}, "kind": "moe", "router": {"experts": s["experts"], "top": s["top"]},
+                  "shared": {"ff": s["shared_ff"] + more}}
+        layers.append({"type": "parallel" if n % 2 == 0 else "delta", "mixer": m, "mlp": ff})
+    cfg = {"architecture": "Kilurax", "canon": {"taps": 4}, "embedding": {"bigram": {"buckets": 65521, "mul_cur": 11, "mul_prev": 131}, "scale": 1.0},
+           "layers": layers, "norm": {"eps": 1e-5, "groups": 2}, "residual_mult": 0.7, "vocab": s["vocab"], "width": w}
+    model = LayeredModel(LayeredConfig.from_dict_sandwich(cfg), device=device, dtype=torch.bfloat16).load(sandwich_random_tensors(cfg, device))
+    out = {"design": "kilurax-peer", "size": size, "layers": len(layers), "weight_bytes_per_token": model.weight_bytes()}
+    return _bench_engine(model, out, s["vocab"], prompt, ctx, decode_steps, batches)
+
+
 def run(sizes, device="cuda:0", peer: bool = True, design: str = "benolix"):
     for size in sizes:
+        if design == "savenex":
+            print(json.dumps(bench_plain(size, device)), flush=True)
+            if peer:
+                print(json.dumps(bench_plain_peer(size, device)), flush=True)
+            continue
         if design == "zevilorn":
             print(json.dumps(bench_gated(size, device)), flush=True)
             if peer:

@@ -101,12 +101,15 @@ DEV float lin_epilogue(int epi, float acc, float aux, float limit)
     return acc;
 }
 
+DEV float lin_aux(const LinArgs& a, int z, long long r, int n)
+{
+    return a.aux[(long long)z * a.sauxb + r * a.ldaux + EPI_AUX_COL(a.epi, n)];
+}
+
 // bias, epilogue and store of output (row r, column n) of batch z
 template <typename T, typename TY>
-DEV void lin_store(const LinArgs& a, int z, long long r, int n, float acc)
+DEV void lin_store(const LinArgs& a, int z, long long r, int n, float acc, float aux)
 {
-    float aux = 0.0f;
-    if (EPI_READS_AUX(a.epi)) aux = a.aux[(long long)z * a.sauxb + r * a.ldaux + EPI_AUX_COL(a.epi, n)];
     const float v = lin_epilogue(a.epi, acc + (a.bias ? a.bias[n] : 0.0f), aux, a.limit);
     if (n >= a.n2) { st1<T>((T*)a.y2 + r * a.ldy2 + (n - a.n2), v); return; }
     st1<TY>((TY*)a.y + (long long)z * a.syb + r * a.ldy + n, v);
@@ -175,7 +178,7 @@ KERNEL void __launch_bounds__(256) lin_rows_kernel(const LinArgs a)
         {
             const int r = r0 + m;
             if (r >= a.M) break;
-            lin_store<T, TY>(a, z, r, n, acc[m]);
+            lin_store<T, TY>(a, z, r, n, acc[m], EPI_READS_AUX(a.epi) ? lin_aux(a, z, r, n) : 0.0f);
         }
     }
 }
@@ -242,7 +245,7 @@ KERNEL void __launch_bounds__(256) lin_tile_kernel(const LinArgs a)
         {
             const int n = n0 + tx * 4 + j;
             if (n >= a.N) continue;
-            lin_store<T, TY>(a, z, r, n, acc[i][j]);
+            lin_store<T, TY>(a, z, r, n, acc[i][j], EPI_READS_AUX(a.epi) ? lin_aux(a, z, r, n) : 0.0f);
         }
     }
 }
@@ -251,6 +254,20 @@ KERNEL void __launch_bounds__(256) lin_tile_kernel(const LinArgs a)
 // Workgroup = 4 waves = (16 * RT) rows x 256 columns; a wave owns 64 columns (4 B fragments) and RT row blocks.  Lane l of a
 // fragment holds row / column (l & 15), k = 8 (l >> 4) .. + 7 of the 32-wide step: 16 contiguous bytes of a K-contiguous row.
 // Rows and columns past the edge are clamped for the loads and dropped at the store; the K tail is masked by lane group.
+
+// aux values of a lane's 4 x 4 outputs: rows rows[0 .. 3], columns n + 16 j
+DEV void lin_block_aux(const LinArgs& a, int z, const int* rows, int n, float (&aux)[4][4])
+{
+    #pragma unroll
+    for (int r = 0; r < 4; r++)
+        #pragma unroll
+        for (int j = 0; j < 4; j++) aux[r][j] = 0.0f;
+    if (!EPI_READS_AUX(a.epi)) return;
+    #pragma unroll
+    for (int r = 0; r < 4; r++)
+        #pragma unroll
+        for (int j = 0; j < 4; j++) aux[r][j] = lin_aux(a, z, rows[r], min(n + 16 * j, a.N - 1));
+}
 
 template <typename TY, int RT>
 KERNEL void __launch_bounds__(256) lin_mfma_kernel(const LinArgs a)
@@ -299,6 +316,9 @@ KERNEL void __launch_bounds__(256) lin_mfma_kernel(const LinArgs a)
     // D: column (lane & 15) of the fragment, rows 4 (lane >> 4) + r
     #pragma unroll
     for (int i = 0; i < RT; i++)
+    {
+        float aux[4][4];                                     // all of a row block's aux values are requested before the first is used
+        lin_block_aux(a, z, rowmap + 16 * i + 4 * (lane >> 4), n0 + li, aux);
         #pragma unroll
         for (int r = 0; r < 4; r++)
         {
@@ -310,9 +330,10 @@ KERNEL void __launch_bounds__(256) lin_mfma_kernel(const LinArgs a)
             {
                 const int n = n0 + 16 * j + li;
                 if (n >= a.N) continue;
-                lin_store<u16, TY>(a, z, row, n, acc[i][j][r]);
+                lin_store<u16, TY>(a, z, row, n, acc[i][j][r], aux[r][j]);
             }
         }
+    }
 }
 
 // ---- bfloat16 on the matrix cores, 128 x 128 tiles through LDS (many rows) ------------------------------------------------------
@@ -394,6 +415,9 @@ KERNEL void __launch_bounds__(256) lin_mfma_tile_kernel(const LinArgs a)
     }
     #pragma unroll
     for (int i = 0; i < 4; i++)
+    {
+        float aux[4][4];
+        lin_block_aux(a, z, rowmap + wm + 16 * i + 4 * (lane >> 4), n0 + wn + li, aux);
         #pragma unroll
         for (int r = 0; r < 4; r++)
         {
@@ -405,9 +429,10 @@ KERNEL void __launch_bounds__(256) lin_mfma_tile_kernel(const LinArgs a)
             {
                 const int n = n0 + wn + 16 * j + li;
                 if (n >= a.N) continue;
-                lin_store<u16, TY>(a, z, row, n, acc[i][j][r]);
+                lin_store<u16, TY>(a, z, row, n, acc[i][j][r], aux[r][j]);
             }
         }
+    }
 }
 
 // ---- host -------------------------------------------------------------------------------------------------------------------

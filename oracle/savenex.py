@@ -217,3 +217,93 @@ class Oracle:
 
     def drop(self, seq):
         self.seqs.pop(seq, None)
+
+
+# ---- small random models for the tests ---------------------------------------------------------------------------------------
+
+
+def bf16_round(a):
+    u = np.asarray(a, dtype=np.float32).view(np.uint32)
+    return (((u + 0x7fff + ((u >> 16) & 1)) & 0xffff0000).astype(np.uint32)).view(np.float32)
+
+
+def left_spec(heads=4, kv_heads=2, dim=12, vdim=10, dims=8, size=9, keep=3, base=1000.0, factor=3.0, scale=None):
+    return {"dim": dim, "heads": heads, "kv_heads": kv_heads, "mask": {"keep_first": keep, "size": size},
+            "rot": {"base": base, "dims": dims, "scaling": {"factor": factor}}, "scale": scale or dim ** -0.5, "vdim": vdim}
+
+
+def right_spec(heads=4, kv_heads=2, dim=8, vdim=14, conv=3):
+    return {"conv": conv, "dim": dim, "heads": heads, "kv_heads": kv_heads, "vdim": vdim}
+
+
+def dense_spec(ff=24, limit=1.5):
+    return {"ff": ff, "kind": "dense", "limit": limit}
+
+
+def moe_spec(experts=8, top=3, ff=12, shared=24):
+    return {"expert": {"ff": ff}, "kind": "moe", "router": {"experts": experts, "top": top}, "shared": {"ff": shared} if shared else None}
+
+
+def layer(left=None, right=None, ff=None):
+    return {"type": "parallel", "mixer": {"left": left or left_spec(), "right": right or right_spec()}, "mlp": ff}
+
+
+def small_config(layers, width=32, vocab=61, eps=1e-5, mult=0.6, loop=(0, 2, 2)):
+    return {"architecture": "Savenex", "layers": layers, "loop": {"start": loop[0], "stop": loop[1], "times": loop[2]} if loop else None,
+            "norm": {"eps": eps}, "residual_mult": mult, "vocab": vocab, "width": width}
+
+
+def random_model(cfg: dict, seed: int = 0, ranks=(5, 3)) -> dict:
+    """name -> float32 array (bfloat16-representable values), shapes from the configuration; ranks = inner sizes of the low-rank pairs
+    (decay, output gate)"""
+    rng = np.random.default_rng(seed)
+    Wd, out = cfg["width"], {}
+
+    def mat(name, o, i, gain=1.0):
+        out[name] = bf16_round(rng.standard_normal((o, i)) * gain / math.sqrt(i))
+
+    def vec(name, n, centre=0.0, spread=0.1):
+        out[name] = bf16_round(centre + rng.standard_normal(n) * spread)
+
+    out["embed"] = bf16_round(rng.standard_normal((cfg["vocab"], Wd)))
+    vec("embed.norm", Wd, 1.0, 0.2)
+    if cfg.get("loop"):
+        mat("loop.in", Wd, 2 * Wd, 1.3)
+    for i, spec in enumerate(cfg["layers"]):
+        k, m = f"l{i}", spec["mixer"]
+        vec(k + ".norm1", Wd, 1.0)
+        x, a = k + ".mix.left", m["left"]
+        H, G, dim, vd = a["heads"], a["kv_heads"], a["dim"], a["vdim"]
+        mat(x + ".q", H * dim, Wd); mat(x + ".k", G * dim, Wd); mat(x + ".v", G * vd, Wd); mat(x + ".o", Wd, H * vd)
+        vec(x + ".out", Wd, 1.0, 0.2)
+        x, r = k + ".mix.right", m["right"]
+        H, G, dim, vd = r["heads"], r["kv_heads"], r["dim"], r["vdim"]
+        for s, n in (("q", G * dim), ("k", G * dim), ("v", H * vd)):
+            mat(f"{x}.{s}", n, Wd, 1.5)
+            taps = rng.standard_normal((n, r["conv"])) * 0.5
+            taps[:, -1] += 0.8
+            out[f"{x}.{s}.conv"] = bf16_round(taps)
+        mat(x + ".b", H, Wd, 2.0); vec(x + ".A_log", H, -0.5, 0.7); vec(x + ".norm", vd, 1.0, 0.2)
+        mat(x + ".a1", ranks[0], Wd); mat(x + ".a2", H * dim, ranks[0], 1.5); vec(x + ".dt_bias", H * dim, -2.0, 1.0)
+        mat(x + ".g1", ranks[1], Wd, 1.5); mat(x + ".g2", H * vd, ranks[1], 1.5); mat(x + ".o", Wd, H * vd)
+        vec(x + ".out", Wd, 1.0, 0.2)
+        ms = spec.get("mlp")
+        if ms is None:
+            continue
+        vec(k + ".norm2", Wd, 1.0)
+        f = k + ".mlp"
+
+        def gated(name, ff):
+            mat(name + ".gate", ff, Wd, 1.5); mat(name + ".up", ff, Wd, 1.5); mat(name + ".down", Wd, ff, 1.5)
+        if ms["kind"] == "dense":
+            gated(f, ms["ff"])
+        else:
+            mat(f + ".router", ms["router"]["experts"], Wd, 2.0); vec(f + ".router.b", ms["router"]["experts"], 0.0, 0.7)
+            for e in range(ms["router"]["experts"]):
+                gated(f"{f}.e{e}", ms["expert"]["ff"])
+            if ms.get("shared"):
+                gated(f + ".shared", ms["shared"]["ff"])
+                mat(f + ".shared.sg", 1, Wd, 1.5)
+    vec("final.norm", Wd, 1.0)
+    mat("head", cfg["vocab"], Wd)
+    return out
