@@ -215,6 +215,9 @@ KERNEL void __launch_bounds__(256) gated_scan_kernel(const GatedScanArgs a)
 // come as 16-byte LDS reads; otherwise every 16th, guarded
 #define GSC_ROW(i) (FULL ? j * NPT + (i) : j + GSC_KS * (i))
 
+// what a thread reads of one staged token: k (or forget gate), q and decays at its rows; v of its column, beta, the head's decay
+template <int NPT> struct GscToken { float k[NPT], q[NPT], g[NPT], v, b, gh; };
+
 template <int NPT, int MODE, bool FULL>
 KERNEL void __launch_bounds__(256) gated_scan_cols_kernel(const GatedScanArgs a, float* o_raw)
 {
@@ -343,14 +346,14 @@ KERNEL void __launch_bounds__(256) gated_scan_cols_kernel(const GatedScanArgs a,
         block_sync_lds();
         if (c0 + GSC_CHUNK < n_tok) request(c0 + GSC_CHUNK);
         float* orow = o_raw + (long long)(r0 + c0) * a.heads * P + h * P + p;
-        // (four tokens unrolled: only the state's own update chains from token to token -- the sums that close a read-out and the
-        // LDS reads of the tokens behind overlap with it; two partial sums halve each chain)
-        #pragma unroll 4
-        for (int kk = 0; kk < nc; kk++)
+        // (two tokens by turns: the LDS reads of one are in flight while the other is stepped through -- the lane exchanges keep the
+        // compiler from unrolling the loop by itself --; two partial sums halve each chain; the 16 lanes of a column keep the read-outs of
+        // 16 tokens, one each, and store them together)
+        auto load = [&](int kk, GscToken<NPT>& x)
         {
-            const float vv = s_v[kk * GSC_COLS + pl];
-            float o = 0.0f;
-            float kr[NPT], qr[NPT], gr[NPT];                     // the token's k (or forget gate), q and decays at this thread's rows
+            x.v = s_v[kk * GSC_COLS + pl];
+            if (RULE) x.b = s_b[kk];
+            if (MODE == GS_DELTA) x.gh = s_g[kk];
             if (FULL)
             {
                 #pragma unroll
@@ -358,12 +361,12 @@ KERNEL void __launch_bounds__(256) gated_scan_cols_kernel(const GatedScanArgs a,
                 {
                     const f32x4 k4 = *(const f32x4*)(s_k + kk * N + j * NPT + 4 * c), q4 = *(const f32x4*)(s_q + kk * N + j * NPT + 4 * c);
                     #pragma unroll
-                    for (int e = 0; e < 4; e++) { kr[4 * c + e] = k4[e]; qr[4 * c + e] = q4[e]; }
+                    for (int e = 0; e < 4; e++) { x.k[4 * c + e] = k4[e]; x.q[4 * c + e] = q4[e]; }
                     if (CHANNELS)
                     {
                         const f32x4 g4 = *(const f32x4*)(s_g + kk * N + j * NPT + 4 * c);
                         #pragma unroll
-                        for (int e = 0; e < 4; e++) gr[4 * c + e] = g4[e];
+                        for (int e = 0; e < 4; e++) x.g[4 * c + e] = g4[e];
                     }
                 }
             }
@@ -373,39 +376,59 @@ KERNEL void __launch_bounds__(256) gated_scan_cols_kernel(const GatedScanArgs a,
                 for (int i = 0; i < NPT; i++)
                 {
                     const int n = GSC_ROW(i);
-                    kr[i] = n < N ? s_k[kk * N + n] : 0.0f;
-                    qr[i] = n < N ? s_q[kk * N + n] : 0.0f;
-                    if (CHANNELS) gr[i] = n < N ? s_g[kk * N + n] : 0.0f;
+                    x.k[i] = n < N ? s_k[kk * N + n] : 0.0f;
+                    x.q[i] = n < N ? s_q[kk * N + n] : 0.0f;
+                    if (CHANNELS) x.g[i] = n < N ? s_g[kk * N + n] : 0.0f;
                 }
             }
+        };
+        // one token: the state moves on, the column's read-out comes back (in all of its lanes)
+        auto step = [&](const GscToken<NPT>& x) -> float
+        {
+            float o = 0.0f, o2 = 0.0f;
             if (RULE)
             {
-                const float g = CHANNELS ? 1.0f : s_g[kk];
-                float kt[2] = {0.0f, 0.0f}, o2 = 0.0f;
+                float kt[2] = {0.0f, 0.0f};
                 #pragma unroll
-                for (int i = 0; i < NPT; i++) { S[i] *= CHANNELS ? gr[i] : g; kt[i & 1] = fmaf(S[i], kr[i], kt[i & 1]); }
-                const float u = s_b[kk] * (vv - row16_allreduce_add(kt[0] + kt[1]));
+                for (int i = 0; i < NPT; i++) { S[i] *= CHANNELS ? x.g[i] : x.gh; kt[i & 1] = fmaf(S[i], x.k[i], kt[i & 1]); }
+                const float u = x.b * (x.v - row16_allreduce_add(kt[0] + kt[1]));
                 #pragma unroll
                 for (int i = 0; i < NPT; i++)
                 {
-                    S[i] = fmaf(kr[i], u, S[i]);
-                    if (i & 1) o2 = fmaf(S[i], qr[i], o2); else o = fmaf(S[i], qr[i], o);
+                    S[i] = fmaf(x.k[i], u, S[i]);
+                    if (i & 1) o2 = fmaf(S[i], x.q[i], o2); else o = fmaf(S[i], x.q[i], o);
                 }
-                o += o2;
             }
             else
             {
-                float o2 = 0.0f;
                 #pragma unroll
                 for (int i = 0; i < NPT; i++)
                 {
-                    S[i] = fmaf(kr[i], S[i] - vv, vv);           // f S + (1 - f) v (rows outside the state read f = q = 0 and are never stored)
-                    if (i & 1) o2 = fmaf(S[i], qr[i], o2); else o = fmaf(S[i], qr[i], o);
+                    S[i] = fmaf(x.k[i], S[i] - x.v, x.v);        // f S + (1 - f) v (rows outside the state read f = q = 0 and are never stored)
+                    if (i & 1) o2 = fmaf(S[i], x.q[i], o2); else o = fmaf(S[i], x.q[i], o);
                 }
-                o += o2;
             }
-            o = row16_allreduce_add(o);
-            if (owner && j == 0) orow[(long long)kk * a.heads * P] = o;
+            return row16_allreduce_add(o + o2);
+        };
+        float kept = 0.0f;
+        auto put = [&](int kk, float o)
+        {
+            kept = (kk & 15) == j ? o : kept;
+            if ((kk & 15) == 15 || kk == nc - 1)
+            {
+                const int tok = (kk & ~15) + j;
+                if (owner && tok <= kk) orow[(long long)tok * a.heads * P] = kept;
+            }
+        };
+        GscToken<NPT> ta, tb;
+        load(0, ta);
+        for (int kk = 0; kk < nc; kk += 2)
+        {
+            load(min(kk + 1, GSC_CHUNK - 1), tb);
+            put(kk, step(ta));
+            if (kk + 1 >= nc) break;
+            load(min(kk + 2, GSC_CHUNK - 1), ta);
+            put(kk + 1, step(tb));
         }
     }
     #pragma unroll
