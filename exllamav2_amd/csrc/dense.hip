@@ -101,16 +101,18 @@ DEV float lin_epilogue(int epi, float acc, float aux, float limit)
     return acc;
 }
 
-DEV float lin_aux(const LinArgs& a, int z, long long r, int n)
+DEV float lin_aux(const LinArgs& a, int epi, int z, long long r, int n)
 {
-    return a.aux[(long long)z * a.sauxb + r * a.ldaux + EPI_AUX_COL(a.epi, n)];
+    return a.aux[(long long)z * a.sauxb + r * a.ldaux + EPI_AUX_COL(epi, n)];
 }
 
-// bias, epilogue and store of output (row r, column n) of batch z
+DEV float lin_bias(const LinArgs& a, int n) { return a.bias ? a.bias[n] : 0.0f; }
+
+// epilogue and store of output (row r, column n) of batch z; acc holds the bias already
 template <typename T, typename TY>
-DEV void lin_store(const LinArgs& a, int z, long long r, int n, float acc, float aux)
+DEV void lin_store(const LinArgs& a, int epi, int z, long long r, int n, float acc, float aux)
 {
-    const float v = lin_epilogue(a.epi, acc + (a.bias ? a.bias[n] : 0.0f), aux, a.limit);
+    const float v = lin_epilogue(epi, acc, aux, a.limit);
     if (n >= a.n2) { st1<T>((T*)a.y2 + r * a.ldy2 + (n - a.n2), v); return; }
     st1<TY>((TY*)a.y + (long long)z * a.syb + r * a.ldy + n, v);
 }
@@ -178,7 +180,7 @@ KERNEL void __launch_bounds__(256) lin_rows_kernel(const LinArgs a)
         {
             const int r = r0 + m;
             if (r >= a.M) break;
-            lin_store<T, TY>(a, z, r, n, acc[m], EPI_READS_AUX(a.epi) ? lin_aux(a, z, r, n) : 0.0f);
+            lin_store<T, TY>(a, a.epi, z, r, n, acc[m] + lin_bias(a, n), EPI_READS_AUX(a.epi) ? lin_aux(a, a.epi, z, r, n) : 0.0f);
         }
     }
 }
@@ -245,7 +247,7 @@ KERNEL void __launch_bounds__(256) lin_tile_kernel(const LinArgs a)
         {
             const int n = n0 + tx * 4 + j;
             if (n >= a.N) continue;
-            lin_store<T, TY>(a, z, r, n, acc[i][j], EPI_READS_AUX(a.epi) ? lin_aux(a, z, r, n) : 0.0f);
+            lin_store<T, TY>(a, a.epi, z, r, n, acc[i][j] + lin_bias(a, n), EPI_READS_AUX(a.epi) ? lin_aux(a, a.epi, z, r, n) : 0.0f);
         }
     }
 }
@@ -256,22 +258,23 @@ KERNEL void __launch_bounds__(256) lin_tile_kernel(const LinArgs a)
 // Rows and columns past the edge are clamped for the loads and dropped at the store; the K tail is masked by lane group.
 
 // aux values of a lane's 4 x 4 outputs: rows rows[0 .. 3], columns n + 16 j
-DEV void lin_block_aux(const LinArgs& a, int z, const int* rows, int n, float (&aux)[4][4])
+DEV void lin_block_aux(const LinArgs& a, int epi, int z, const int* rows, int n, float (&aux)[4][4])
 {
     #pragma unroll
     for (int r = 0; r < 4; r++)
         #pragma unroll
         for (int j = 0; j < 4; j++) aux[r][j] = 0.0f;
-    if (!EPI_READS_AUX(a.epi)) return;
+    if (!EPI_READS_AUX(epi)) return;
     #pragma unroll
     for (int r = 0; r < 4; r++)
         #pragma unroll
-        for (int j = 0; j < 4; j++) aux[r][j] = lin_aux(a, z, rows[r], min(n + 16 * j, a.N - 1));
+        for (int j = 0; j < 4; j++) aux[r][j] = lin_aux(a, epi, z, rows[r], min(n + 16 * j, a.N - 1));
 }
 
-template <typename TY, int RT>
+template <typename TY, int RT, int EPI>
 KERNEL void __launch_bounds__(256) lin_mfma_kernel(const LinArgs a)
 {
+    const int epi = EPI >= 0 ? EPI : a.epi;
     SHARED int rowmap[16 * RT];
     const int z = bid_z();
     const int m0 = bid_y() * 16 * RT, n0 = bid_x() * 256 + wave_id() * 64;
@@ -314,11 +317,14 @@ KERNEL void __launch_bounds__(256) lin_mfma_kernel(const LinArgs a)
             for (int j = 0; j < 4; j++) acc[i][j] = mfma_16x16x32_bf16(af[i], bf[j], acc[i][j]);
     }
     // D: column (lane & 15) of the fragment, rows 4 (lane >> 4) + r
+    float bias[4];
+    #pragma unroll
+    for (int j = 0; j < 4; j++) bias[j] = lin_bias(a, min(n0 + 16 * j + li, a.N - 1));
     #pragma unroll
     for (int i = 0; i < RT; i++)
     {
         float aux[4][4];                                     // all of a row block's aux values are requested before the first is used
-        lin_block_aux(a, z, rowmap + 16 * i + 4 * (lane >> 4), n0 + li, aux);
+        lin_block_aux(a, epi, z, rowmap + 16 * i + 4 * (lane >> 4), n0 + li, aux);
         #pragma unroll
         for (int r = 0; r < 4; r++)
         {
@@ -330,7 +336,7 @@ KERNEL void __launch_bounds__(256) lin_mfma_kernel(const LinArgs a)
             {
                 const int n = n0 + 16 * j + li;
                 if (n >= a.N) continue;
-                lin_store<u16, TY>(a, z, row, n, acc[i][j][r], aux[r][j]);
+                lin_store<u16, TY>(a, epi, z, row, n, acc[i][j][r] + bias[j], aux[r][j]);
             }
         }
     }
@@ -344,9 +350,11 @@ KERNEL void __launch_bounds__(256) lin_mfma_kernel(const LinArgs a)
 
 #define LT_STRIDE 40                                         // values per staged row (32 + 8 of padding)
 
-template <typename TY>
+// EPI >= 0: that epilogue alone (64 copies of all of them are more code than the instruction cache holds); -1: a.epi's
+template <typename TY, int EPI>
 KERNEL void __launch_bounds__(256) lin_mfma_tile_kernel(const LinArgs a)
 {
+    const int epi = EPI >= 0 ? EPI : a.epi;
     SHARED __attribute__((aligned(16))) u16 As[2][128 * LT_STRIDE];
     SHARED __attribute__((aligned(16))) u16 Bs[2][128 * LT_STRIDE];
     SHARED int rowmap[128];
@@ -413,11 +421,14 @@ KERNEL void __launch_bounds__(256) lin_mfma_tile_kernel(const LinArgs a)
         block_sync();
         stage ^= 1;
     }
+    float bias[4];
+    #pragma unroll
+    for (int j = 0; j < 4; j++) bias[j] = lin_bias(a, min(n0 + wn + 16 * j + li, a.N - 1));
     #pragma unroll
     for (int i = 0; i < 4; i++)
     {
         float aux[4][4];
-        lin_block_aux(a, z, rowmap + wm + 16 * i + 4 * (lane >> 4), n0 + wn + li, aux);
+        lin_block_aux(a, epi, z, rowmap + wm + 16 * i + 4 * (lane >> 4), n0 + wn + li, aux);
         #pragma unroll
         for (int r = 0; r < 4; r++)
         {
@@ -429,7 +440,7 @@ KERNEL void __launch_bounds__(256) lin_mfma_tile_kernel(const LinArgs a)
             {
                 const int n = n0 + wn + 16 * j + li;
                 if (n >= a.N) continue;
-                lin_store<u16, TY>(a, z, row, n, acc[i][j][r], aux[r][j]);
+                lin_store<u16, TY>(a, epi, z, row, n, acc[i][j][r] + bias[j], aux[r][j]);
             }
         }
     }
@@ -459,9 +470,31 @@ static void launch_dense(const LinArgs& a, int batch, bool vec_ok, int max_rows,
     {
         if (vec_ok)
         {
-            if (max_rows <= 32) LAUNCH((lin_mfma_kernel<TY, 2>), dim3((a.N + 255) / 256, (max_rows + 31) / 32, batch), dim3(256), 0, s, a);
-            else if (max_rows <= 64) LAUNCH((lin_mfma_kernel<TY, 4>), dim3((a.N + 255) / 256, (max_rows + 63) / 64, batch), dim3(256), 0, s, a);
-            else LAUNCH((lin_mfma_tile_kernel<TY>), dim3((a.N + 127) / 128, (max_rows + 127) / 128, batch), dim3(256), 0, s, a);
+            if (max_rows <= 32)
+            {
+                const dim3 grid((a.N + 255) / 256, (max_rows + 31) / 32, batch);
+                if (a.epi == EPI_NONE) LAUNCH((lin_mfma_kernel<TY, 2, EPI_NONE>), grid, dim3(256), 0, s, a);
+                else LAUNCH((lin_mfma_kernel<TY, 2, -1>), grid, dim3(256), 0, s, a);
+            }
+            else if (max_rows <= 64)
+            {
+                const dim3 grid((a.N + 255) / 256, (max_rows + 63) / 64, batch);
+                if (a.epi == EPI_NONE) LAUNCH((lin_mfma_kernel<TY, 4, EPI_NONE>), grid, dim3(256), 0, s, a);
+                else LAUNCH((lin_mfma_kernel<TY, 4, -1>), grid, dim3(256), 0, s, a);
+            }
+            else
+            {
+                const dim3 grid((a.N + 127) / 128, (max_rows + 127) / 128, batch);
+                switch (a.epi)
+                {
+#define LIN_TILE_CASE(E) case E: LAUNCH((lin_mfma_tile_kernel<TY, E>), grid, dim3(256), 0, s, a); break
+                    LIN_TILE_CASE(EPI_NONE); LIN_TILE_CASE(EPI_MUL_SIGMOID_AUX); LIN_TILE_CASE(EPI_SILU_AUX_MUL); LIN_TILE_CASE(EPI_CLAMPED_GLU);
+                    LIN_TILE_CASE(EPI_RELU_SQUARED); LIN_TILE_CASE(EPI_ROW_SCALED_RELU_SQUARED); LIN_TILE_CASE(EPI_ROW_SCALED_SILU_SCALED);
+                    LIN_TILE_CASE(EPI_AUX_MUL); LIN_TILE_CASE(EPI_GELU_ERF); LIN_TILE_CASE(EPI_MUL_SIGMOID_ROW_AUX); LIN_TILE_CASE(EPI_EXP_SOFTPLUS);
+#undef LIN_TILE_CASE
+                    default: LAUNCH((lin_mfma_tile_kernel<TY, -1>), grid, dim3(256), 0, s, a);
+                }
+            }
             return;
         }
     }
