@@ -67,7 +67,8 @@ def parse():
                         "stack; tibalorn: state-space + windowed attention beside a latent-attention stack; negilorn: chunked attention + decaying "
                         "linear attention + sigmoid MoE beside a state-space / windowed-attention stack; kilurax: attention beside a state-space scan, "
                         "forget-gate linear attention and gated delta rule behind sandwich norms beside a negilorn stack; zevilorn: head-mixing attention, "
-                        "latent attention and window attention beside a minimal gated recurrence in gated parallel layers beside a negilorn stack; "
+                        "latent attention and window attention beside a minimal gated recurrence in gated parallel layers beside a negilorn stack; savenex: "
+                        "window attention with kept first tokens beside a delta rule with a decay per key channel beside a kilurax stack; "
                         "exllamav2_amd/bench_layered.py); one JSON line each")
     p.add_argument("--design-sizes", default="w2048,w4096")
     p.add_argument("--design-no-peer", action="store_true", help="--design: skip the peer model")
